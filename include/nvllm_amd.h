@@ -129,6 +129,38 @@ typedef struct nvllm_latent_config {
  * dkv.norm, uk, uv, o}, l<i>.mlp.{gate, up, down}. */
 int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_config* cfg, const nvllm_latent_layer* layers, nvllm_model** out);
 
+/* ---- hybrid decoders: every layer has one of three token mixers and optionally a squared-ReLU feed-forward; sublayers read the
+ * residual stream itself and are normed on their output, x += residual_mult * norm(sublayer(x)).  Norm weights of layers and of the
+ * output are stored minus norm_offset.  Loading, pool, step, sampling and decode are the same API as the Qwen3 model's; recurrent
+ * state lives in the sequence's slot, and a step that asks for a sequence shorter than what was processed starts it again. */
+#define NVLLM_MIXER_ATTENTION 0 /* grouped-query attention, distance bias instead of positions */
+#define NVLLM_MIXER_LINEAR 1    /* S = decay_h S + k v^T, o = S^T q; silu inputs, one output norm over all heads, output gate */
+#define NVLLM_MIXER_DELTA 2     /* gated delta rule with a decay per key channel, short convolutions, output norm per head, output gate */
+typedef struct nvllm_hybrid_layer {
+    int32_t mixer;
+    int32_t heads, kv_heads, dim, vdim; /* per head: query/key and value size; kv_heads divides heads */
+    int32_t ff;                         /* feed-forward width, 0 = the layer has none */
+    /* attention */
+    double scale;                       /* of q . k; q and k are RMS-normed over the whole projection before */
+    int32_t bias_rows;                  /* rows of the distance table (0: no bias): half of them exact, the rest logarithmic up to bias_max */
+    double bias_max;
+    int32_t sink;                       /* 1: the softmax denominator has one more term exp(0) */
+    int32_t v_mix;                      /* 1: values are mixed with those of the first layer that has this set */
+    /* NVLLM_MIXER_LINEAR */
+    const double* decay;                /* [heads], read by the create call only */
+    /* NVLLM_MIXER_DELTA */
+    int32_t conv_taps, decay_rank, gate_rank;
+} nvllm_hybrid_layer;
+typedef struct nvllm_hybrid_config {
+    int32_t vocab_size, width, num_layers;
+    double norm_eps, embed_scale, residual_mult, norm_offset;
+    int32_t f32;                        /* 0: bf16 weights, hi + lo planes, f16 cache; 1: every product and the cache in f32 */
+} nvllm_hybrid_config;
+/* Tensor names for nvllm_model_load_tensor: embed, head, final.norm and, per layer, l<i>.norm1, l<i>.norm2, l<i>.mlp.{up, down},
+ * l<i>.mix.o and by mixer: attention l<i>.mix.{q, k, v} with .b, .{q, k}.norm, .rel, .vmix (a scalar); linear l<i>.mix.{q, k, v, g,
+ * norm}; delta l<i>.mix.{q, k, v} with .conv, .{b, A_log, a1, a2, dt_bias, g1, g2, norm}. */
+int nvllm_model_create_hybrid(nvllm_ctx* ctx, const nvllm_hybrid_config* cfg, const nvllm_hybrid_layer* layers, nvllm_model** out);
+
 /* ---- KV block pool (the real allocation the reference's stub BlockManager lacks,
  *      src/engine/block_manager.rs:24-29,64-98).  block_size must be 256 (src/engine/sequence.rs:35).
  *      max_batched_tokens bounds the rows processed per internal chunk (prefill is chunked). */

@@ -54,6 +54,24 @@ class LatentConfigC(C.Structure):
     ]
 
 
+class HybridLayerC(C.Structure):
+    """nvllm_hybrid_layer"""
+
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "vdim", "ff")] + [
+        ("scale", C.c_double), ("bias_rows", C.c_int32), ("bias_max", C.c_double), ("sink", C.c_int32), ("v_mix", C.c_int32),
+        ("decay", C.POINTER(C.c_double)), ("conv_taps", C.c_int32), ("decay_rank", C.c_int32), ("gate_rank", C.c_int32),
+    ]
+
+
+class HybridConfigC(C.Structure):
+    """nvllm_hybrid_config"""
+
+    _fields_ = [(n, C.c_int32) for n in ("vocab_size", "width", "num_layers")] + [
+        (n, C.c_double) for n in ("norm_eps", "embed_scale", "residual_mult", "norm_offset")] + [("f32", C.c_int32)]
+
+
+MIXER_ATTENTION, MIXER_LINEAR, MIXER_DELTA = 0, 1, 2  # NVLLM_MIXER_*
+
 _vp, _fp = C.c_void_p, C.c_void_p  # device pointers travel as integers
 _SIGS = {
     "nvllm_last_error": (C.c_char_p, [_vp]),
@@ -70,6 +88,7 @@ _SIGS = {
     "nvllm_timer_stop": (C.c_int, [_vp, C.POINTER(C.c_float)]),
     "nvllm_model_create": (C.c_int, [_vp, C.POINTER(Qwen3ConfigC), C.POINTER(_vp)]),
     "nvllm_model_create_latent": (C.c_int, [_vp, C.POINTER(LatentConfigC), C.POINTER(LatentLayerC), C.POINTER(_vp)]),
+    "nvllm_model_create_hybrid": (C.c_int, [_vp, C.POINTER(HybridConfigC), C.POINTER(HybridLayerC), C.POINTER(_vp)]),
     "nvllm_model_destroy": (C.c_int, [_vp]),
     "nvllm_model_load_tensor": (C.c_int, [_vp, C.c_char_p, C.c_void_p, C.c_int, C.POINTER(C.c_int64), C.c_int]),
     "nvllm_model_fill_synthetic": (C.c_int, [_vp, C.c_uint64]),

@@ -9,8 +9,7 @@ from dataclasses import dataclass, field
 import numpy as np
 
 from . import _lib
-from .causal_lm import CausalLM, checkpoint_files, read_safetensors
-from .context import Context
+from .causal_lm import LayeredCausalLM, random_matrix
 
 GLU_ALPHA = 1.702  # gate slope of the feed-forward's sigmoid
 GLU_SHIFT = 1.0    # added to the clamped up branch
@@ -107,6 +106,9 @@ class BerevikConfig:
                 out[p + "mlp.down"] = (w, mlp.ff)
         return out
 
+    def random_tensor(self, name, shape, rng):
+        return np.ones(shape, np.float32) if len(shape) == 1 else random_matrix(shape, rng)
+
     def to_c(self, f32):
         c = _lib.LatentConfigC(self.vocab_size, self.hidden_size, len(self.layers), self.loop_start, self.loop_stop, self.loop_times,
                                self.norm_eps, self.embed_scale, self.logit_softcap, int(f32))
@@ -119,51 +121,11 @@ class BerevikConfig:
         return c, ls
 
 
-class BerevikForCausalLM(CausalLM):
-    """dtype "bfloat16": products on bf16 hi + lo activation planes, f16 latent cache (the serving mode); "float32": every product
-    and the cache in f32.  What the design computes in 32-bit (norms, rotation, scores, softmax, residual) is so in both."""
+class BerevikForCausalLM(LayeredCausalLM):
+    """Both dtypes of LayeredCausalLM.  What the design computes in 32-bit (norms, rotation, scores, softmax, residual) is so in both."""
 
-    DTYPES = ("bfloat16", "float32")
+    CONFIG = BerevikConfig
 
-    def __init__(self, cfg, ctx=None, dtype="bfloat16"):
-        if dtype not in self.DTYPES:
-            raise ValueError(f"dtype {dtype!r} unsupported ({', '.join(self.DTYPES)})")
-        self.cfg, self.dtype = cfg, dtype
-        self.ctx = ctx or Context(0)
-        h = C.c_void_p()
-        cc, layers = cfg.to_c(dtype == "float32")
-        _lib.check(_lib.lib().nvllm_model_create_latent(self.ctx.h, C.byref(cc), layers, C.byref(h)), self.ctx.h)
-        self.h = h
-
-    @classmethod
-    def from_dir(cls, model_dir, ctx=None, dtype="bfloat16"):
-        m = cls(BerevikConfig.from_dir(model_dir), ctx, dtype)
-        for path in checkpoint_files(model_dir):
-            for name, arr, code in read_safetensors(path):
-                m.load_tensor(name, arr, code)
-        m.finalize()
-        return m
-
-    @classmethod
-    def from_state_dict(cls, cfg, tensors, ctx=None, dtype="bfloat16"):
-        """tensors: name -> ndarray, float32 or bf16 bits as uint16 (full shapes)"""
-        m = cls(cfg, ctx, dtype)
-        for name, arr in tensors.items():
-            m.load_tensor(name, np.asarray(arr))
-        m.finalize()
-        return m
-
-    @classmethod
-    def from_random(cls, cfg, seed=0, ctx=None, dtype="bfloat16"):
-        """random weights of the configured shapes (benchmarks): matrices of unit output variance, norm weights 1"""
-        rng = np.random.default_rng(seed)
-        m = cls(cfg, ctx, dtype)
-        for name, shape in cfg.tensor_shapes().items():
-            if len(shape) == 1:
-                m.load_tensor(name, np.ones(shape, np.float32))
-            else:  # bf16 bits: random sign and mantissa, exponent of 1 / sqrt(fan-in)
-                e = 127 - max(1, int(round(0.5 * np.log2(shape[1]))))
-                bits = rng.integers(0, 1 << 16, shape, dtype=np.uint16)
-                m.load_tensor(name, (bits & np.uint16(0x807F)) | np.uint16(e << 7))
-        m.finalize()
-        return m
+    def _create(self, cfg, f32, out):
+        cc, layers = cfg.to_c(f32)
+        return _lib.lib().nvllm_model_create_latent(self.ctx.h, C.byref(cc), layers, out)

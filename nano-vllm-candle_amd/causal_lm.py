@@ -9,18 +9,28 @@ import struct
 import numpy as np
 
 from . import _lib
+from .context import Context
+
+
+def _safetensors_header(path):
+    with open(path, "rb") as f:
+        n = struct.unpack("<Q", f.read(8))[0]
+        header = json.loads(f.read(n))
+    header.pop("__metadata__", None)
+    return header, 8 + n
+
+
+def tensor_shapes(model_dir):
+    """name -> shape of every tensor of a checkpoint directory"""
+    return {name: tuple(meta["shape"]) for path in checkpoint_files(model_dir) for name, meta in _safetensors_header(path)[0].items()}
 
 
 def read_safetensors(path):
     """Minimal safetensors reader (header JSON + raw little-endian data, memory-mapped): yields
     (name, np.ndarray view, dtype code).  Executes nothing from the file.  BF16 tensors come back as uint16."""
-    with open(path, "rb") as f:
-        n = struct.unpack("<Q", f.read(8))[0]
-        header = json.loads(f.read(n))
-    data = np.memmap(path, dtype=np.uint8, mode="r", offset=8 + n)
+    header, start = _safetensors_header(path)
+    data = np.memmap(path, dtype=np.uint8, mode="r", offset=start)
     for name, meta in header.items():
-        if name == "__metadata__":
-            continue
         b, e = meta["data_offsets"]
         dt = meta["dtype"]
         if dt == "BF16":
@@ -49,7 +59,7 @@ def checkpoint_files(model_dir):
 
 
 class CausalLM:
-    """Base of Qwen3ForCausalLM and BerevikForCausalLM: a native model handle and the calls on it"""
+    """Base of the model classes: a native model handle and the calls on it"""
 
     cfg = None
     ctx = None
@@ -64,7 +74,7 @@ class CausalLM:
             code = _lib.DTYPE_BF16 if arr.dtype == np.uint16 else _lib.DTYPE_F32
             if code == _lib.DTYPE_F32:
                 arr = np.ascontiguousarray(arr, np.float32)
-        arr = np.ascontiguousarray(arr)
+        arr = np.ascontiguousarray(arr).reshape(arr.shape)  # ascontiguousarray makes a scalar one-dimensional
         shape = (C.c_int64 * arr.ndim)(*arr.shape)
         _lib.check(_lib.lib().nvllm_model_load_tensor(self.h, name.encode(), arr.ctypes.data_as(C.c_void_p), code, shape,
                                                       arr.ndim), self.ctx.h)
@@ -167,7 +177,7 @@ class CausalLM:
         _lib.check(_lib.lib().nvllm_decode_collect(self.h, buf.ctypes.data_as(C.POINTER(C.c_uint32))), self.ctx.h)
         return buf
 
-    PROF_KINDS = {"attn": 1, "gemm": 2, "norm": 3, "qk": 4, "silu": 5, "lm_head": 6, "empty": 7}
+    PROF_KINDS = {"attn": 1, "gemm": 2, "norm": 3, "qk": 4, "silu": 5, "lm_head": 6, "empty": 7, "recur": 8}
 
     def profile_kernel(self, kind):
         """HIP-event bracketing of one kernel class on the library stream (None/0 = off)"""
@@ -208,3 +218,58 @@ class CausalLM:
             self.close()
         except Exception:
             pass
+
+
+class LayeredCausalLM(CausalLM):
+    """Base of the models built from layer descriptions.  dtype "bfloat16": products on bf16 hi + lo activation planes, f16 cache (the
+    serving mode); "float32": every product and the cache in f32.  A subclass names its CONFIG (with from_dir, tensor_shapes and
+    random_tensor) and creates the native handle from it."""
+
+    DTYPES = ("bfloat16", "float32")
+    CONFIG = None
+
+    def __init__(self, cfg, ctx=None, dtype="bfloat16"):
+        if dtype not in self.DTYPES:
+            raise ValueError(f"dtype {dtype!r} unsupported ({', '.join(self.DTYPES)})")
+        self.cfg, self.dtype = cfg, dtype
+        self.ctx = ctx or Context(0)
+        h = C.c_void_p()
+        _lib.check(self._create(cfg, dtype == "float32", C.byref(h)), self.ctx.h)
+        self.h = h
+
+    def _create(self, cfg, f32, out):
+        raise NotImplementedError
+
+    @classmethod
+    def from_dir(cls, model_dir, ctx=None, dtype="bfloat16"):
+        m = cls(cls.CONFIG.from_dir(model_dir), ctx, dtype)
+        for path in checkpoint_files(model_dir):
+            for name, arr, code in read_safetensors(path):
+                m.load_tensor(name, arr, code)
+        m.finalize()
+        return m
+
+    @classmethod
+    def from_state_dict(cls, cfg, tensors, ctx=None, dtype="bfloat16"):
+        """tensors: name -> ndarray, float32 or bf16 bits as uint16 (full shapes)"""
+        m = cls(cfg, ctx, dtype)
+        for name, arr in tensors.items():
+            m.load_tensor(name, np.asarray(arr))
+        m.finalize()
+        return m
+
+    @classmethod
+    def from_random(cls, cfg, seed=0, ctx=None, dtype="bfloat16"):
+        """random weights of the configured shapes (benchmarks)"""
+        rng = np.random.default_rng(seed)
+        m = cls(cfg, ctx, dtype)
+        for name, shape in cfg.tensor_shapes().items():
+            m.load_tensor(name, cfg.random_tensor(name, shape, rng))
+        m.finalize()
+        return m
+
+
+def random_matrix(shape, rng):
+    """bf16 bits of unit output variance: random sign and mantissa, exponent of 1 / sqrt(fan-in)"""
+    e = 127 - max(1, int(round(0.5 * np.log2(shape[1]))))
+    return (rng.integers(0, 1 << 16, shape, dtype=np.uint16) & np.uint16(0x807F)) | np.uint16(e << 7)

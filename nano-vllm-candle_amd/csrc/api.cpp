@@ -22,7 +22,7 @@
 #include "../../include/nvllm_amd.h"
 #include "../../include/nvllm_amd_debug.h"
 #include "kernels.h"
-#include "model.h"
+#include "decoder.h"
 #include "synth_device.h"
 
 // ---------------------------------------------------------------------------------------------------
@@ -441,7 +441,7 @@ extern "C" int nvllm_model_create(nvllm_ctx* ctx, const nvllm_qwen3_config* cfg,
 }
 
 static void free_kv(nvllm_model* m) {
-    if (m->lat) latent_free_kv(m);
+    if (m->dec) m->dec->free_kv();
     for (auto p : m->kcache) (void)hipFree(p);
     for (auto p : m->vcache) (void)hipFree(p);
     for (auto p : m->vlocache) (void)hipFree(p);
@@ -464,7 +464,7 @@ extern "C" int nvllm_model_destroy(nvllm_model* m) {
     (void)hipSetDevice(m->ctx->device);
     (void)hipStreamSynchronize(m->ctx->stream);
     free_kv(m);
-    if (m->lat) latent_destroy(m);
+    m->dec.reset();
     if (m->pin_ids) (void)hipHostFree(m->pin_ids);
     for (hipEvent_t e : m->pend_ev) if (e) (void)hipEventDestroy(e);
     for (hipEvent_t e : m->prof_ev) (void)hipEventDestroy(e);
@@ -538,7 +538,7 @@ extern "C" int nvllm_model_load_tensor(nvllm_model* m, const char* hf_name, cons
     if (!m || !hf_name || !host_data || !shape) return fail(m ? m->ctx : nullptr, NVLLM_EINVAL, "NULL argument");
     nvllm_ctx* ctx = m->ctx;
     if (dtype != NVLLM_DTYPE_F32 && dtype != NVLLM_DTYPE_BF16) return fail(ctx, NVLLM_EINVAL, "dtype %d unsupported", dtype);
-    if (m->lat) return latent_load_tensor(m, hf_name, host_data, dtype, shape, ndim);
+    if (m->dec) return m->dec->load_tensor(m, hf_name, host_data, dtype, shape, ndim);
     Target t;
     if (!resolve(m, hf_name, t)) return fail(ctx, NVLLM_EINVAL, "unknown tensor name '%s'", hf_name);
     int64_t rows = ndim == 2 ? shape[0] : 1, cols = ndim == 2 ? shape[1] : (ndim == 1 ? shape[0] : -1);
@@ -625,7 +625,7 @@ extern "C" int nvllm_tp_shard(const nvllm_qwen3_config* cfg, int tp_size, int tp
 
 extern "C" int nvllm_model_fill_synthetic_profile(nvllm_model* m, uint64_t seed, int profile) {
     if (!m) return NVLLM_EINVAL;
-    if (m->lat) return fail(m->ctx, NVLLM_EINVAL, "the synthetic generator covers Qwen3 tensors only: load the latent model's tensors");
+    if (m->dec) return fail(m->ctx, NVLLM_EINVAL, "the synthetic generator covers Qwen3 tensors only: load the model's tensors");
     if (profile != 0 && profile != 1) return fail(m->ctx, NVLLM_EINVAL, "synthetic profile %d unknown (0 benign, 1 heavy)", profile);
     HIPCHK(m->ctx, hipSetDevice(m->ctx->device));
     int rc = synth_one(m, "model.embed_tokens.weight", seed, profile);
@@ -648,7 +648,7 @@ extern "C" int nvllm_model_finalize(nvllm_model* m) {
     if (!m) return NVLLM_EINVAL;
     nvllm_ctx* ctx = m->ctx;
     HIPCHK(ctx, hipSetDevice(ctx->device));
-    if (m->lat) return latent_finalize(m);
+    if (m->dec) return m->dec->finalize(m);
     char name[160];
     if (!m->loaded.count("model.embed_tokens.weight")) return fail(ctx, NVLLM_ESTATE, "missing tensor model.embed_tokens.weight");
     if (!m->loaded.count("model.norm.weight")) return fail(ctx, NVLLM_ESTATE, "missing tensor model.norm.weight");
@@ -668,7 +668,7 @@ extern "C" int nvllm_model_finalize(nvllm_model* m) {
 
 extern "C" int64_t nvllm_model_weight_bytes(const nvllm_model* m) {
     if (!m) return 0;
-    if (m->lat) return latent_weight_bytes(m);
+    if (m->dec) return m->dec->weight_bytes();
     int64_t b = (int64_t)m->lm_head.bytes() + (int64_t)m->H * 4;
     for (const auto& w : m->layers)
         b += (int64_t)(w.qkv.bytes() + w.o.bytes() + w.gu.bytes() + w.down.bytes()) + (int64_t)(2 * m->H + 2 * m->hd) * 4;
@@ -817,7 +817,7 @@ extern "C" int nvllm_kv_alloc(nvllm_model* m, int num_blocks, int block_size, in
     if (rc) return rc;
     m->h_stage_bytes = (R * 24 + (size_t)max_seqs * 4) * sizeof(int) + 256;
     HIPCHK(ctx, hipHostMalloc(&m->h_stage, m->h_stage_bytes, hipHostMallocDefault));
-    rc = m->lat ? latent_kv_alloc(m) : qwen3_kv_alloc(m);
+    rc = m->dec ? m->dec->kv_alloc(m) : qwen3_kv_alloc(m);
     if (rc) { m->num_blocks = 0; return rc; }
     HIPCHK(ctx, hipStreamSynchronize(ctx->stream));
     return NVLLM_OK;
@@ -826,11 +826,14 @@ extern "C" int nvllm_kv_alloc(nvllm_model* m, int num_blocks, int block_size, in
 extern "C" int nvllm_kv_num_free_blocks(const nvllm_model* m) { return m ? (int)m->free_blocks.size() : 0; }
 extern "C" int64_t nvllm_kv_bytes_per_token(const nvllm_model* m) {
     if (!m) return 0;
-    if (m->lat) return latent_kv_bytes_per_token(m);
+    if (m->dec) return m->dec->kv_bytes_per_token();
     const int64_t v_bytes = m->vlocache.empty() ? 2 : 3;  // 24-bit V: + one residual byte per element
     const int64_t k_bytes = m->klocache.empty() ? 2 : 3;
     return (int64_t)m->kv_l * m->hd * (k_bytes + v_bytes) * m->L;
 }
+
+nvllm_model::nvllm_model() = default;
+nvllm_model::~nvllm_model() = default;
 
 static void release_seq(nvllm_model* m, SeqState& s) {
     for (int b : s.blocks)
@@ -1185,7 +1188,7 @@ int gemm_slabs(nvllm_model* m, const bf16_bits* xh, const bf16_bits* xl, int ldx
 
 // rows R (ids/pos/slot/tiles already on the device), n_last rows listed in d_last_rows -> logits rows
 static int forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n_last, int logits_row0) {
-    if (m->lat) return latent_forward_chunk(m, R, n_tiles, qt, n_last, logits_row0);
+    if (m->dec) return m->dec->forward_chunk(m, R, n_tiles, qt, n_last, logits_row0);
     FusedPlan fp;
     if (fused_plan(m, R, fp)) return forward_chunk_fused(m, fp, R, n_tiles, qt, n_last, logits_row0);
     nvllm_ctx* ctx = m->ctx;
@@ -1591,6 +1594,7 @@ static int step_impl(nvllm_model* m, int n_seqs, const int64_t* seq_ids, const u
     }
     // sequence bookkeeping + block allocation (the part BlockManager::allocate/may_append leave undone)
     std::vector<int> start(n_seqs);
+    const bool recurrent = m->dec && m->dec->recurrent();
     int new_slots = 0;
     for (int i = 0; i < n_seqs; ++i) if (!m->seqs.count(seq_ids[i])) ++new_slots;
     if (new_slots > (int)m->free_slots.size()) return fail(ctx, NVLLM_ENOMEM, "no free sequence slots (max_seqs %d)", m->max_seqs);
@@ -1607,12 +1611,15 @@ static int step_impl(nvllm_model* m, int n_seqs, const int64_t* seq_ids, const u
         SeqState& s = it->second;
         if (s.cached >= lens[i]) {  // nothing new: recompute the last token
             s.cached = lens[i] - 1;
-            if (std::max(0, s.cached - m->widest_window + 1) < s.released * kBlockTokens) release_seq(m, s);  // ... or everything
+            if (recurrent) release_seq(m, s);
+            else if (std::max(0, s.cached - m->widest_window + 1) < s.released * kBlockTokens) release_seq(m, s);  // ... or everything
         }
         start[i] = s.cached;
         int rc = ensure_blocks(m, s, lens[i]);
         if (rc) return rc;
     }
+    // carried state moves on with the rows: if this step fails, the sequences start again
+    if (recurrent) for (int i = 0; i < n_seqs; ++i) m->seqs[seq_ids[i]].cached = 0;
     HIPCHK(ctx, hipMemcpyAsync(m->d_block_tables, m->h_block_tables.data(), m->h_block_tables.size() * 4, hipMemcpyHostToDevice, ctx->stream));
     m->want_logits = last_logits != nullptr || temperatures != nullptr || score != nullptr;  // sampling reads the last-row logits on the device
     m->cur_n = n_seqs;
@@ -1623,8 +1630,8 @@ static int step_impl(nvllm_model* m, int n_seqs, const int64_t* seq_ids, const u
     bool all_single = true;
     for (int i = 0; i < n_seqs; ++i) if (lens[i] - start[i] != 1) all_single = false;
     const int qt = all_single ? 1 : 2;
-    const int tpt = m->lat ? (qt == 1 ? 1 : kLatentTileRows) : attn_tokens_per_tile(m->gqa, qt);
-    const bool tile_groups = qt == 2 && !m->lat && m->vlocache.empty();
+    const int tpt = m->dec ? m->dec->tile_rows(qt) : attn_tokens_per_tile(m->gqa, qt);
+    const bool tile_groups = qt == 2 && !m->dec && m->vlocache.empty();
     const int32_t* want_next = score ? score->want_pos : nullptr;
     std::vector<int> head_rows;  // rows the head runs on, in output order: every sequence's last one, or the wanted ones
     for (int i = 0; i < n_seqs; ++i) {
@@ -1664,10 +1671,10 @@ static int step_impl(nvllm_model* m, int n_seqs, const int64_t* seq_ids, const u
         for (; hr < head_rows.size() && head_rows[hr] < r0 + R; ++hr) last_local.push_back(head_rows[hr] - r0);
         int rc = upload_chunk(m, p, r0, R, 0, (int)p.tile_row0.size(), last_local);
         if (rc) return rc;
-        if (m->lat) {
+        if (m->dec) {
             std::vector<int> local(p.tile_row0);
             for (int& x : local) x -= r0;
-            rc = latent_plan_chunk(m, p.pos.data() + r0, p.slot.data() + r0, row_seq.data() + r0, R, local.data(), (int)local.size(), qt);
+            rc = m->dec->plan_chunk(m, p.pos.data() + r0, p.slot.data() + r0, row_seq.data() + r0, R, local.data(), (int)local.size(), qt);
             if (rc) return rc;
         }
         rc = forward_chunk(m, R, (int)p.tile_row0.size(), qt, (int)last_local.size(), score ? 0 : logits_row);
@@ -1717,7 +1724,7 @@ static int step_impl(nvllm_model* m, int n_seqs, const int64_t* seq_ids, const u
         release_unseen(m, st);
     }
     int64_t kv_bytes = kv_read_tokens * nvllm_kv_bytes_per_token(m);
-    if (m->lat) { kv_bytes = 0; for (int i = 0; i < n_seqs; ++i) kv_bytes += latent_kv_read_bytes(m, lens[i]); }
+    if (m->dec) { kv_bytes = 0; for (int i = 0; i < n_seqs; ++i) kv_bytes += m->dec->kv_read_bytes(lens[i]); }
     m->last_bytes = nvllm_model_weight_bytes(m) + kv_bytes +
                     (last_logits ? (int64_t)4 * n_seqs * m->cfg.vocab_size : 0);
     return NVLLM_OK;
@@ -1767,8 +1774,13 @@ static int decode_core(nvllm_model* m) {
     m->cur_n = n;
     m->cur_max_len = *std::max_element(m->last_lens.begin(), m->last_lens.end()) + 1;
     set_attn_split(m, n, m->cur_max_len);
+    const bool recurrent = m->dec && m->dec->recurrent();
+    if (recurrent) for (int64_t id : m->last_ids) m->seqs[id].cached = 0;  // until the step is on the stream
     int rc = forward_chunk(m, n, n, 1, n, 0);
-    if (rc) return rc;
+    if (rc) {
+        if (recurrent) m->last_ids.clear();  // carried state may have moved on: no step continues from here
+        return rc;
+    }
     int64_t kv_bytes = 0;
     const int64_t per_token = nvllm_kv_bytes_per_token(m);
     for (int i = 0; i < n; ++i) {
@@ -1776,7 +1788,7 @@ static int decode_core(nvllm_model* m) {
         SeqState& st = m->seqs[m->last_ids[i]];
         st.cached = m->last_lens[i];
         release_unseen(m, st);
-        kv_bytes += m->lat ? latent_kv_read_bytes(m, m->last_lens[i]) : m->last_lens[i] * per_token;
+        kv_bytes += m->dec ? m->dec->kv_read_bytes(m->last_lens[i]) : m->last_lens[i] * per_token;
     }
     m->last_bytes = nvllm_model_weight_bytes(m) + kv_bytes;
     return NVLLM_OK;
@@ -1861,6 +1873,7 @@ extern "C" int nvllm_debug_set_option(nvllm_model* m, const char* name, int valu
     if (!strcmp(name, "latent_plain")) { m->opt_latent_plain = value; return NVLLM_OK; }
     if (!strcmp(name, "tile_fuse_qk")) { m->opt_tile_fuse_qk = value; return NVLLM_OK; }
     if (!strcmp(name, "tile_min_wgs")) { m->opt_tile_min_wgs = value; return NVLLM_OK; }  // <= 0: never use the tile GEMM
+    if (m->dec && m->dec->option(name, value) == 0) return NVLLM_OK;
     return fail(m->ctx, NVLLM_EINVAL, "unknown option '%s'", name);
 }
 
@@ -1893,6 +1906,7 @@ extern "C" int nvllm_debug_get_counter(nvllm_model* m, const char* name, int64_t
         *value = !strcmp(name, "kv_f16_saturated") ? (int64_t)h[0] : (int64_t)(h[1] & 0xFFFFu);
         return NVLLM_OK;
     }
+    if (m->dec && m->dec->counter(name, value) == 0) return NVLLM_OK;
     return fail(m->ctx, NVLLM_EINVAL, "unknown counter '%s'", name);
 }
 
@@ -1925,7 +1939,7 @@ extern "C" int nvllm_debug_stamps_read(nvllm_model* m, int launch, uint64_t* out
 }
 
 extern "C" int nvllm_profile_kernel(nvllm_model* m, int kind) {
-    if (!m || kind < 0 || kind > PROF_EMPTY) return NVLLM_EINVAL;
+    if (!m || kind < 0 || kind > PROF_RECUR) return NVLLM_EINVAL;
     HIPCHK(m->ctx, hipStreamSynchronize(m->ctx->stream));
     m->prof_kind = kind;
     m->prof_used = 0;

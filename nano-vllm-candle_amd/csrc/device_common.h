@@ -59,6 +59,9 @@ __device__ __forceinline__ float soft_cap(float v, float cap) {
     return cap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(__expf(2.0f * z) + 1.0f));
 }
 
+// log(1 + e^x) without overflow
+__device__ __forceinline__ float softplusf(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+
 // 16 bytes of a stream that THIS CU reads once per launch (a sequence's K/V in decode): non-temporal, so the lines do not
 // displace what other kernels re-read from L2 / Infinity Cache (`global_load_dwordx4 ... nt`; guide, nt-weights row)
 __device__ __forceinline__ uint4 ld_stream16(const void* p) {
@@ -211,6 +214,59 @@ __device__ __forceinline__ void load_slabs8(float (&x)[8], const float* p, int l
         if (j < left)
             for (int sl = 0; sl < n_slabs; ++sl) x[j] += p[(size_t)sl * stride + j];
     }
+}
+
+// s += the n partial sums of one float4, four independent loads per trip (clamped index, masked sum)
+__device__ __forceinline__ void add_slabs(float4& s, const float* p, int n, int64_t stride) {
+    for (int sl0 = 0; sl0 < n; sl0 += 4) {
+        float4 t[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) t[u] = *reinterpret_cast<const float4*>(p + (size_t)min(sl0 + u, n - 1) * stride);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+            if (sl0 + u < n) { s.x += t[u].x; s.y += t[u].y; s.z += t[u].z; s.w += t[u].w; }
+    }
+}
+// one element of them
+__device__ __forceinline__ float slab_elem(const float* p, int n_slabs, int64_t stride) {
+    float v = p[0];
+    for (int sl0 = 1; sl0 < n_slabs; sl0 += 4) {  // four independent loads per trip (clamped index, masked sum)
+        float t[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) t[u] = p[(size_t)min(sl0 + u, n_slabs - 1) * stride];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) v += sl0 + u < n_slabs ? t[u] : 0.f;
+    }
+    return v;
+}
+
+// four consecutive columns of one row (only the first `left` exist) as bf16 hi / lo, row-major or fragment order
+__device__ __forceinline__ void put_planes4(uint16_t* ph, uint16_t* pl, int row, int col, int left, int ld, int packed, const f32x4& v) {
+    uint16_t h[4], l[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) split_bf16(v[r], h[r], l[r]);
+    if (left >= 4 && (col & 3) == 0) {
+        const size_t o = packed ? xpack_off(row, col, ld >> 5) : (size_t)row * ld + col;
+        *reinterpret_cast<uint2*>(ph + o) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
+        *reinterpret_cast<uint2*>(pl + o) = make_uint2(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16));
+        return;
+    }
+    for (int r = 0; r < 4 && r < left; ++r) {
+        const size_t o = packed ? xpack_off(row, col + r, ld >> 5) : (size_t)row * ld + col + r;
+        ph[o] = h[r];
+        pl[o] = l[r];
+    }
+}
+
+// sum over the workgroup; red: one float per wave
+__device__ __forceinline__ float block_sum(float v, float* red, int n_waves) {
+    v = wave_sum(v);
+    __syncthreads();  // red may still be read from an earlier sum
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    v = 0.f;
+    for (int q = 0; q < n_waves; ++q) v += red[q];
+    return v;
 }
 
 typedef const __attribute__((address_space(1))) void* gptr_t;

@@ -1,5 +1,5 @@
 // Latent-attention decoders (compressed K/V: every token caches one latent vector and one rotated key part shared by all
-// heads): launchers of latent_ops.hip / latent_attn.hip and the model half of latent_model.cpp.
+// heads): launchers of latent_ops.hip / latent_attn.hip / latent_prefill.hip.
 #pragma once
 #include "kernels.h"
 
@@ -27,7 +27,10 @@ struct AddNormArgs {
     const int* row_idx = nullptr;      // input row of output row r (outputs are compact)
     int W = 0, ldr = 0, ldx = 0;
     float eps = 0.f;
+    const float* post_w = nullptr;
+    float post_mult = 1.f;
     const float* w[2] = {nullptr, nullptr};  // nullptr: output k absent
+    int raw = 0;                       // output 0 is s itself (w[0] unused)
     bf16_bits* xh[2] = {nullptr, nullptr};
     bf16_bits* xl[2] = {nullptr, nullptr};
     float* y[2] = {nullptr, nullptr};
@@ -72,6 +75,7 @@ hipError_t launch_latent_cache(const LatentRowsArgs& a, int rows, hipStream_t s)
 // ---- per-head products and 32-bit products -------------------------------------------------------------------------------
 // y[r][h][n] = sum_k x[r][h][k] W[h][n][k]: x f32 (element strides), W packed per head (N % 16 == 0, K % 32 == 0).
 // exact = 0: x as bf16 hi + lo, 16x16x32 bf16 MFMA; exact = 1: everything in f32 (16x16x4 f32 MFMA, weights widened).
+// decay_rate set (f32 output): head 0 leaves exp(-decay_rate[n] softplus(y + decay_bias[n])), every other head sigmoid(y).
 // Output: f32 with strides, or bf16 hi/lo planes [rows][ld] at column h * n_valid + n (n < n_valid).
 struct HeadGemmArgs {
     const float* x = nullptr;
@@ -80,6 +84,8 @@ struct HeadGemmArgs {
     int64_t w_head = 0;            // uint4 per head
     int N = 0, K = 0, heads = 1, M = 0, n_valid = 0;
     int exact = 0;
+    const float* decay_rate = nullptr;
+    const float* decay_bias = nullptr;
     float* y = nullptr;            // columns >= n_valid are not written
     int64_t y_row = 0, y_head = 0;
     bf16_bits* yh = nullptr;
@@ -184,18 +190,3 @@ hipError_t launch_logits_finish(const float* in, int n_slabs, int64_t slab_strid
                                 float* logits, int64_t ld_out, hipStream_t s);
 
 }  // namespace nvllm
-
-// ---- model half (latent_model.cpp), called by the shared step / pool code of api.cpp -------------------------------------
-struct nvllm_model;
-struct LatentModel;
-int latent_load_tensor(nvllm_model* m, const char* name, const void* data, int dtype, const int64_t* shape, int ndim);
-int latent_finalize(nvllm_model* m);
-int latent_kv_alloc(nvllm_model* m);
-void latent_free_kv(nvllm_model* m);
-void latent_destroy(nvllm_model* m);
-int64_t latent_weight_bytes(const nvllm_model* m);
-int64_t latent_kv_bytes_per_token(const nvllm_model* m);
-int64_t latent_kv_read_bytes(const nvllm_model* m, int len);  // cache bytes a decode step reads for a sequence of len tokens
-// metadata of the chunk about to run beyond the q-tiles (rows r0 .. r0 + R of pos / slot / seq; tiles already uploaded)
-int latent_plan_chunk(nvllm_model* m, const int* pos, const int* slot, const int* seq, int R, const int* tile_row0, int n_tiles, int qt);
-int latent_forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n_last, int logits_row0);

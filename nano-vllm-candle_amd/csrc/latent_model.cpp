@@ -10,7 +10,7 @@
 #include <cstring>
 #include <map>
 
-#include "model.h"
+#include "decoder.h"
 
 struct LatentLayer {
     nvllm_latent_layer c{};
@@ -36,7 +36,7 @@ struct RopeTable {
     float *cos = nullptr, *sin = nullptr;
 };
 
-struct LatentModel {
+struct LatentModel : DecoderImpl {
     nvllm_latent_config cfg{};
     std::vector<LatentLayer> layers;
     std::vector<int> order;            // layer of every run (a looped layer runs several times, each with its own cache)
@@ -56,9 +56,20 @@ struct LatentModel {
     struct Segment { int pos0, n; };
     std::vector<Segment> segments;
     float *y1 = nullptr, *y2 = nullptr, *ctx_f = nullptr, *act_f = nullptr;                   // 32-bit mode
-};
 
-static int up(int v, int q) { return (v + q - 1) / q * q; }
+    ~LatentModel() override;
+    int load_tensor(nvllm_model* m, const char* name, const void* data, int dtype, const int64_t* shape, int ndim) override;
+    int finalize(nvllm_model* m) override;
+    int kv_alloc(nvllm_model* m) override;
+    void free_kv() override;
+    int64_t weight_bytes() const override;
+    int64_t kv_bytes_per_token() const override;
+    int64_t kv_read_bytes(int len) const override;
+    int tile_rows(int qt) const override { return qt == 1 ? 1 : kLatentTileRows; }
+    int plan_chunk(nvllm_model* m, const int* pos, const int* slot, const int* seq, int R, const int* tile_row0, int n_tiles, int qt) override;
+    int forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n_last, int logits_row0) override;
+};
+static LatentModel& latent(const nvllm_model* m) { return *static_cast<LatentModel*>(m->dec.get()); }
 
 extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_config* cfg, const nvllm_latent_layer* layers, nvllm_model** out) {
     if (!ctx || !cfg || !layers || !out) return fail(ctx, NVLLM_EINVAL, "NULL argument");
@@ -81,8 +92,8 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
     HIPCHK(ctx, hipSetDevice(ctx->device));
     nvllm_model* m = new nvllm_model();
     m->ctx = ctx;
-    m->lat = new LatentModel();
-    LatentModel& L = *m->lat;
+    m->dec = std::make_unique<LatentModel>();
+    LatentModel& L = latent(m);
     L.cfg = c;
     m->H = c.width; m->V_l = c.vocab_size / tp; m->kv_l = 1;
     m->cfg.vocab_size = c.vocab_size; m->cfg.hidden_size = c.width; m->cfg.max_position_embeddings = 1 << 30;
@@ -152,8 +163,8 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
     return NVLLM_OK;
 }
 
-void latent_free_kv(nvllm_model* m) {
-    LatentModel& L = *m->lat;
+void LatentModel::free_kv() {
+    LatentModel& L = *this;
     for (void* p : L.cache) if (p) (void)hipFree(p);
     L.cache.clear();
     void* ptrs[] = {L.slabs2, L.q, L.qlat, L.olat, L.part_o, L.part_ml, L.tap, L.kx, L.vx, L.d_exp, L.d_tile_exp, L.x2h, L.x2l, L.y1, L.y2, L.ctx_f, L.act_f};
@@ -173,54 +184,19 @@ void latent_free_kv(nvllm_model* m) {
     }
 }
 
-void latent_destroy(nvllm_model* m) {
-    LatentModel& L = *m->lat;
+LatentModel::~LatentModel() {
+    LatentModel& L = *this;
+    free_kv();
     (void)hipFree(L.embed); (void)hipFree(L.head.data); (void)hipFree(L.final_norm);
     for (LatentLayer& w : L.layers) {
         for (PackedW* p : {&w.qkv, &w.ukt, &w.ukx, &w.uv, &w.uvx, &w.o, &w.gu, &w.down}) (void)hipFree(p->data);
         (void)hipFree(w.norm1); (void)hipFree(w.norm2); (void)hipFree(w.dkv_norm);
     }
-    delete m->lat;
-    m->lat = nullptr;
 }
 
 // ---------------------------------------------------------------------------------------------------
 // weights
 // ---------------------------------------------------------------------------------------------------
-// bf16 view of a host tensor
-struct HostMat {
-    const void* p;
-    int dtype;
-    int64_t cols;
-    uint16_t at(int64_t r, int64_t c) const {
-        const int64_t i = r * cols + c;
-        return dtype == NVLLM_DTYPE_F32 ? host_f32_to_bf16(((const float*)p)[i]) : ((const uint16_t*)p)[i];
-    }
-    float f32(int64_t i) const {
-        if (dtype == NVLLM_DTYPE_F32) return ((const float*)p)[i];
-        const uint32_t u = (uint32_t)((const uint16_t*)p)[i] << 16;
-        float f;
-        memcpy(&f, &u, 4);
-        return f;
-    }
-};
-
-// rows [row0, row0 + rows) of w <- elem(r, c), c < cols (columns beyond are zero)
-template <typename F>
-static int put_rows(nvllm_ctx* ctx, const PackedW& w, int row0, int rows, int cols, int ileave, F elem) {
-    std::vector<uint16_t> tmp((size_t)rows * w.K, 0);
-    for (int r = 0; r < rows; ++r)
-        for (int c = 0; c < cols; ++c) tmp[(size_t)r * w.K + c] = elem(r, c);
-    bf16_bits* d = nullptr;
-    HIPCHK(ctx, hipMalloc((void**)&d, tmp.size() * 2));
-    hipError_t e = hipMemcpyAsync(d, tmp.data(), tmp.size() * 2, hipMemcpyHostToDevice, ctx->stream);
-    if (e == hipSuccess) e = launch_pack_rows(w, row0, rows, d, w.K, ileave, ctx->stream);
-    if (e == hipSuccess) e = hipStreamSynchronize(ctx->stream);
-    (void)hipFree(d);
-    HIPCHK(ctx, e);
-    return NVLLM_OK;
-}
-
 // weights of the expanded form: `size` rows per head as f16, scaled by the power of two that brings the largest entry of the
 // (bf16-valued) matrix to [2^14, 2^15); *unscale undoes it
 static int put_expand(nvllm_ctx* ctx, const PackedW& w, float* unscale, const HostMat& h, int64_t head0, int heads, int size, int size_p, int kr) {
@@ -248,9 +224,9 @@ static int put_expand(nvllm_ctx* ctx, const PackedW& w, float* unscale, const Ho
 static const char* const kMixTensors[] = {"norm1", "mix.q", "mix.dkv", "mix.dkv.norm", "mix.uk", "mix.uv", "mix.o"};
 static const char* const kMlpTensors[] = {"norm2", "mlp.gate", "mlp.up", "mlp.down"};
 
-int latent_load_tensor(nvllm_model* m, const char* name, const void* data, int dtype, const int64_t* shape, int ndim) {
+int LatentModel::load_tensor(nvllm_model* m, const char* name, const void* data, int dtype, const int64_t* shape, int ndim) {
     nvllm_ctx* ctx = m->ctx;
-    LatentModel& L = *m->lat;
+    LatentModel& L = latent(m);
     const int rank = ctx->tp_rank;
     if (ndim != 1 && ndim != 2) return fail(ctx, NVLLM_EINVAL, "tensor '%s' has %d dimensions", name, ndim);
     const int64_t rows = ndim == 2 ? shape[0] : 1, cols = shape[ndim - 1];
@@ -322,17 +298,17 @@ int latent_load_tensor(nvllm_model* m, const char* name, const void* data, int d
     return NVLLM_OK;
 }
 
-int latent_finalize(nvllm_model* m) {
+int LatentModel::finalize(nvllm_model* m) {
     nvllm_ctx* ctx = m->ctx;
     for (const char* s : {"embed", "head", "final.norm"})
         if (!m->loaded.count(s)) return fail(ctx, NVLLM_ESTATE, "missing tensor %s", s);
     char name[96];
-    for (int l = 0; l < m->lat->cfg.num_layers; ++l) {
+    for (int l = 0; l < latent(m).cfg.num_layers; ++l) {
         for (const char* s : kMixTensors) {
             snprintf(name, sizeof name, "l%d.%s", l, s);
             if (!m->loaded.count(name)) return fail(ctx, NVLLM_ESTATE, "missing tensor %s", name);
         }
-        if (m->lat->layers[l].ff)
+        if (latent(m).layers[l].ff)
             for (const char* s : kMlpTensors) {
                 snprintf(name, sizeof name, "l%d.%s", l, s);
                 if (!m->loaded.count(name)) return fail(ctx, NVLLM_ESTATE, "missing tensor %s", name);
@@ -342,8 +318,8 @@ int latent_finalize(nvllm_model* m) {
     return NVLLM_OK;
 }
 
-int64_t latent_weight_bytes(const nvllm_model* m) {
-    const LatentModel& L = *m->lat;
+int64_t LatentModel::weight_bytes() const {
+    const LatentModel& L = *this;
     int64_t b = (int64_t)L.head.bytes() + (int64_t)L.cfg.width * 4;
     for (int l : L.order) {
         const LatentLayer& w = L.layers[l];
@@ -352,16 +328,18 @@ int64_t latent_weight_bytes(const nvllm_model* m) {
     }
     return b;
 }
-int64_t latent_kv_bytes_per_token(const nvllm_model* m) {
+int64_t LatentModel::kv_bytes_per_token() const {
+    const LatentModel& L = *this;
     int64_t b = 0;
-    for (int l : m->lat->order) b += (int64_t)(m->lat->layers[l].rank_p + m->lat->layers[l].rot_p) * (m->lat->cfg.f32 ? 4 : 2);
+    for (int l : L.order) b += (int64_t)(L.layers[l].rank_p + L.layers[l].rot_p) * (L.cfg.f32 ? 4 : 2);
     return b;
 }
-int64_t latent_kv_read_bytes(const nvllm_model* m, int len) {
+int64_t LatentModel::kv_read_bytes(int len) const {
+    const LatentModel& L = *this;
     int64_t b = 0;
-    for (int l : m->lat->order) {
-        const LatentLayer& w = m->lat->layers[l];
-        b += (int64_t)(w.rank_p + w.rot_p) * (m->lat->cfg.f32 ? 4 : 2) * (w.c.window > 0 ? std::min(len, w.c.window) : len);
+    for (int l : L.order) {
+        const LatentLayer& w = L.layers[l];
+        b += (int64_t)(w.rank_p + w.rot_p) * (L.cfg.f32 ? 4 : 2) * (w.c.window > 0 ? std::min(len, w.c.window) : len);
     }
     return b;
 }
@@ -369,9 +347,9 @@ int64_t latent_kv_read_bytes(const nvllm_model* m, int len) {
 // ---------------------------------------------------------------------------------------------------
 // cache and step buffers (pool sizes are set, the shared buffers exist)
 // ---------------------------------------------------------------------------------------------------
-int latent_kv_alloc(nvllm_model* m) {
+int LatentModel::kv_alloc(nvllm_model* m) {
     nvllm_ctx* ctx = m->ctx;
-    LatentModel& L = *m->lat;
+    LatentModel& L = latent(m);
     hipStream_t s = ctx->stream;
     const bool f32 = L.cfg.f32 != 0;
     const size_t R = m->max_rows, R16 = (R + 15) / 16 * 16;
@@ -461,115 +439,11 @@ int latent_kv_alloc(nvllm_model* m) {
 }
 
 // ---------------------------------------------------------------------------------------------------
-// products
-// ---------------------------------------------------------------------------------------------------
-enum { P_GENERIC = 0, P_ROW, P_STREAM, P_TILE };
-struct ProductPlan {
-    int kind = P_GENERIC;
-    int packed = 0;     // input planes in fragment order
-    int max_split = 1;  // K slabs that fit the slab buffer
-};
-
-// y = x.W^T left as f32 slabs
-static ProductPlan plan_product(const nvllm_model* m, int R, const PackedW& w) {
-    ProductPlan p;
-    const size_t one = (size_t)R * w.N;
-    p.max_split = (int)std::max<size_t>(1, std::min<size_t>(8, m->slab_floats / one));
-    const int tmin = m->opt_tile_min_wgs;
-    if (tmin > 0 && R > kFusedMaxRows) {
-        const int ks = gemm_tile_splits(R, w.N, w.K, tmin, std::min(p.max_split, R <= 512 ? 8 : 4));
-        if (ks > 0) { p.kind = P_TILE; p.packed = 1; p.max_split = std::min(p.max_split, R <= 512 ? 8 : 4); return p; }
-    }
-    const int ss = gemm_stream_splits(R, w.N, w.K);
-    if (ss > 0 && (size_t)ss * one <= m->slab_floats) { p.kind = P_STREAM; p.packed = 1; return p; }
-    if (R <= kFusedMaxRows && gemm_rowpar_ok(w.N, w.K, 2, R) && (size_t)gemm_rowpar_splits(w.N, w.K, 2, R) * one <= m->slab_floats) {
-        p.kind = P_ROW;
-        p.packed = R >= 16 && gemm_rowdir_ok(w.N, w.K, 2, R);
-    }
-    return p;
-}
-static int run_product(nvllm_model* m, const ProductPlan& p, const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, float* out, int R, int* n_slabs) {
-    hipStream_t s = m->ctx->stream;
-    if (p.kind == P_TILE) {
-        PROF(m, PROF_GEMM, launch_gemm_tile(xh, xl, w, R, 0, out, nullptr, nullptr, 0, m->opt_tile_min_wgs, p.max_split, n_slabs, s));
-        ++m->tile_launches;
-    } else if (p.kind == P_STREAM) {
-        PROF(m, PROF_GEMM, launch_gemm_stream(xh, xl, w.K, w, out, R, p.packed, s));
-        *n_slabs = gemm_stream_splits(R, w.N, w.K);
-    } else if (p.kind == P_ROW) {
-        RowParArgs a;
-        a.xh = xh; a.xl = xl; a.ldx = w.K; a.out = out; a.M = R; a.x_packed = p.packed;
-        PROF(m, PROF_GEMM, launch_gemm_rowpar(a, w, 2, s));
-        *n_slabs = gemm_rowpar_splits(w.N, w.K, 2, R);
-    } else {
-        GemmPlan g = plan_gemm(R, w.N, w.K, p.max_split);
-        PROF(m, PROF_GEMM, launch_gemm(g, xh, xl, w.K, w, out, R, s));
-        *n_slabs = g.n_split;
-    }
-    return NVLLM_OK;
-}
-
-// gate/up + activation as hi/lo planes: fused into the product where a kernel has the epilogue, else slabs + one row kernel
-struct GluPlan {
-    int kind = P_GENERIC;  // P_STREAM: slabs + activation kernel on a product plan
-    int packed = 0, out_packed_ok = 0;
-    ProductPlan slabs;
-};
-static GluPlan plan_glu(const nvllm_model* m, int R, const PackedW& w, bool want_packed_out) {
-    GluPlan g;
-    const int tmin = m->opt_tile_min_wgs;
-    if (tmin > 0 && R > kFusedMaxRows && gemm_tile_ok(R, w.N, w.K, 2, tmin)) { g.kind = P_TILE; g.packed = 1; g.out_packed_ok = 1; return g; }
-    if (R <= kFusedMaxRows && gemm_rowpar_ok(w.N, w.K, 1, R)) {
-        g.kind = P_ROW;
-        const bool dir = gemm_rowdir_ok(w.N, w.K, 1, R);
-        g.packed = R >= 16 && dir;
-        g.out_packed_ok = dir;
-        return g;
-    }
-    if (gemm_stream_splits(R, w.N, w.K) > 0 || want_packed_out) {
-        g.kind = P_STREAM;
-        g.slabs = plan_product(m, R, w);
-        g.packed = g.slabs.packed;
-        g.out_packed_ok = 1;
-    }
-    return g;
-}
-static int run_glu(nvllm_model* m, const GluPlan& g, const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int R, const GluSpec& spec,
-                   bf16_bits* oh, bf16_bits* ol, int out_packed) {
-    hipStream_t s = m->ctx->stream;
-    if (g.kind == P_TILE) {
-        PROF(m, PROF_GEMM, launch_gemm_tile(xh, xl, w, R, 2, nullptr, oh, ol, out_packed, m->opt_tile_min_wgs, 1, nullptr, s, spec));
-        ++m->tile_launches;
-    } else if (g.kind == P_ROW) {
-        RowParArgs a;
-        a.xh = xh; a.xl = xl; a.ldx = w.K; a.oh = oh; a.ol = ol; a.M = R; a.x_packed = g.packed; a.o_packed = out_packed; a.glu = spec;
-        PROF(m, PROF_GEMM, launch_gemm_rowpar(a, w, 1, s));
-    } else if (g.kind == P_STREAM) {
-        int ns = 1;
-        int rc = run_product(m, g.slabs, xh, xl, w, m->slabs, R, &ns);
-        if (rc) return rc;
-        PROF(m, PROF_SILU, launch_silu_mul_interleaved(m->slabs, ns, (int64_t)R * w.N, R, w.N / 2, oh, ol, out_packed, s, spec));
-    } else {
-        GemmPlan p = plan_gemm_swiglu(R, w.N, w.K);
-        PROF(m, PROF_GEMM, launch_gemm_swiglu(p, xh, xl, w.K, w, R, oh, ol, nullptr, s, spec));
-    }
-    return NVLLM_OK;
-}
-
-// 32-bit product of row-major f32 rows
-static int exact_product(nvllm_model* m, const float* x, const PackedW& w, float* out, int R) {
-    HeadGemmArgs a;
-    a.x = x; a.x_row = w.K; a.w = w.data; a.N = a.n_valid = w.N; a.K = w.K; a.M = R; a.exact = 1; a.y = out; a.y_row = w.N;
-    PROF(m, PROF_GEMM, launch_head_gemm(a, m->ctx->stream));
-    return NVLLM_OK;
-}
-
-// ---------------------------------------------------------------------------------------------------
 // forward over one chunk of rows
 // ---------------------------------------------------------------------------------------------------
-int latent_plan_chunk(nvllm_model* m, const int* pos, const int* slot, const int* seq, int R, const int* tile_row0, int n_tiles, int qt) {
+int LatentModel::plan_chunk(nvllm_model* m, const int* pos, const int* slot, const int* seq, int R, const int* tile_row0, int n_tiles, int qt) {
     nvllm_ctx* ctx = m->ctx;
-    LatentModel& L = *m->lat;
+    LatentModel& L = latent(m);
     L.exp_n = 0;
     L.segments.clear();
     if (qt == 1 || !L.exp_cap || m->opt_latent_plain || m->opt_latent_absorb == 1) return NVLLM_OK;
@@ -598,7 +472,7 @@ int latent_plan_chunk(nvllm_model* m, const int* pos, const int* slot, const int
 
 // products per head: expansion + expanded attention against absorbing + absorbed attention + carrying values back
 static bool latent_expanded_pays(const nvllm_model* m, const LatentLayer& w, int R) {
-    const LatentModel& L = *m->lat;
+    const LatentModel& L = latent(m);
     if (!w.expands || !L.exp_n) return false;
     if (m->opt_latent_absorb == -1) return true;
     double pairs = 0, tokens = 0;
@@ -614,7 +488,7 @@ static bool latent_expanded_pays(const nvllm_model* m, const LatentLayer& w, int
 
 static int latent_attention(nvllm_model* m, const LatentLayer& w, void* cache_data, const float* qkv, int n_slabs, int R, int n_tiles, int qt, int ctx_packed) {
     nvllm_ctx* ctx = m->ctx;
-    LatentModel& L = *m->lat;
+    LatentModel& L = latent(m);
     hipStream_t s = ctx->stream;
     const bool f32 = L.cfg.f32 != 0;
     const int dq = w.dim_p + w.rot_p;
@@ -700,9 +574,9 @@ static int latent_attention(nvllm_model* m, const LatentLayer& w, void* cache_da
     return NVLLM_OK;
 }
 
-int latent_forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n_last, int logits_row0) {
+int LatentModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n_last, int logits_row0) {
     nvllm_ctx* ctx = m->ctx;
-    LatentModel& L = *m->lat;
+    LatentModel& L = latent(m);
     hipStream_t s = ctx->stream;
     const bool f32 = L.cfg.f32 != 0, tp = ctx->tp_size > 1;
     m->tap_rows = R;
@@ -779,29 +653,5 @@ int latent_forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n_last,
     nf.w[0] = L.final_norm;
     if (f32) nf.y[0] = L.y1; else { nf.xh[0] = m->xh; nf.xl[0] = m->xl; }
     PROF(m, PROF_NORM, launch_add_norm(nf, n_last, s));
-    const int tps = ctx->tp_size;
-    uint32_t* ids_dst = tps == 1 ? m->d_next + logits_row0 : m->d_next + m->cur_n + (size_t)ctx->tp_rank * m->cur_n + logits_row0;
-    float* val_dst = tps == 1 ? nullptr : m->d_maxval + (size_t)ctx->tp_rank * m->cur_n + logits_row0;
-    float* lg = m->logits + (size_t)logits_row0 * m->V_l;
-    const float cap = (float)L.cfg.logit_softcap;
-    if (!f32 && m->V_l % 16 == 0) {
-        RowNorm rn;
-        rn.softcap = cap;
-        GemmPlan pl = plan_lmhead(n_last, m->V_l, L.Kw);
-        PROF(m, PROF_LMHEAD, launch_gemm_argmax(pl, m->xh, m->xl, L.Kw, L.head, m->want_logits ? lg : nullptr, n_last, m->part_val, m->part_idx, &rn, s));
-        const int parts = gemm_argmax_parts(pl, m->V_l);
-        if (pl.lm_nt > 0) HIPCHK(ctx, launch_argmax_rows(m->part_val, m->part_idx, parts, n_last, ids_dst, val_dst, s));
-        else HIPCHK(ctx, launch_argmax_parts(m->part_val, m->part_idx, parts, n_last, m->argmax_scratch, ids_dst, val_dst, s));
-        return NVLLM_OK;
-    }
-    int ns = 1, rc = NVLLM_OK;
-    if (f32) rc = exact_product(m, L.y1, L.head, m->slabs, n_last);
-    else {
-        ProductPlan ph;  // row-major planes, one slab
-        rc = run_product(m, ph, m->xh, m->xl, L.head, m->slabs, n_last, &ns);
-    }
-    if (rc) return rc;
-    HIPCHK(ctx, launch_logits_finish(m->slabs, ns, (int64_t)n_last * L.Vp, L.Vp, n_last, m->V_l, cap, lg, m->V_l, s));
-    HIPCHK(ctx, launch_argmax(lg, n_last, m->V_l, m->V_l, ids_dst, val_dst, s));
-    return NVLLM_OK;
+    return output_head(m, L.head, L.Kw, L.Vp, f32 ? L.y1 : nullptr, (float)L.cfg.logit_softcap, n_last, logits_row0);
 }

@@ -12,27 +12,15 @@ namespace nvllm {
 // ---------------------------------------------------------------------------------------------------
 constexpr int kAddNormMax = 8192;  // widest row
 
-// s += the n partial sums of one float4, four independent loads per trip (clamped index, masked sum)
-__device__ __forceinline__ void add_slabs(float4& s, const float* p, int n, int64_t stride) {
-    for (int sl0 = 0; sl0 < n; sl0 += 4) {
-        float4 t[4];
-#pragma unroll
-        for (int u = 0; u < 4; ++u) t[u] = *reinterpret_cast<const float4*>(p + (size_t)min(sl0 + u, n - 1) * stride);
-#pragma unroll
-        for (int u = 0; u < 4; ++u)
-            if (sl0 + u < n) { s.x += t[u].x; s.y += t[u].y; s.z += t[u].z; s.w += t[u].w; }
-    }
-}
-
 // BS = 256, or 1024 for few wide rows (decode): every thread's loads are then in flight at once
-template <int BS>
+template <int BS, bool POST>
 __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
     constexpr int NV = kAddNormMax / 4 / BS;
     __shared__ float red[BS / 64];
     const int r = blockIdx.x;
     const int src = a.row_idx ? a.row_idx[r] : r;
     const int nv4 = a.ldr >> 2;
-    float4 cache[NV];
+    float4 cache[NV], res[POST ? NV : 1];
     float ss = 0.f;
 #pragma unroll
     for (int c = 0; c < NV; ++c) {
@@ -47,23 +35,35 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
                 if (a.in) add_slabs(s, a.in + (size_t)src * a.ldr + (size_t)i * 4, a.n_slabs, a.slab_stride);
                 if (a.in2) add_slabs(s, a.in2 + (size_t)src * a.ldr + (size_t)i * 4, a.n_slabs2, a.slab_stride2);
             }
-            if (a.residual_in) {
-                const float4 t = *reinterpret_cast<const float4*>(a.residual_in + (size_t)src * a.ldr + (size_t)i * 4);
-                s.x += t.x; s.y += t.y; s.z += t.z; s.w += t.w;
+            float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (a.residual_in) t = *reinterpret_cast<const float4*>(a.residual_in + (size_t)src * a.ldr + (size_t)i * 4);
+            if constexpr (POST) {
+                res[c] = t;
+            } else {
+                if (a.residual_in) { s.x += t.x; s.y += t.y; s.z += t.z; s.w += t.w; }
+                if (a.residual_out) *reinterpret_cast<float4*>(a.residual_out + (size_t)src * a.ldr + (size_t)i * 4) = s;
             }
+            cache[c] = s;
+            ss += s.x * s.x + s.y * s.y + s.z * s.z + s.w * s.w;
+        }
+    }
+    if constexpr (POST) {
+        const float f = a.post_mult / sqrtf(block_sum(ss, red, BS / 64) / (float)a.W + a.eps);
+        ss = 0.f;
+#pragma unroll
+        for (int c = 0; c < NV; ++c) {
+            const int i = threadIdx.x + c * BS;
+            if (i >= nv4) continue;
+            const float4 w = *reinterpret_cast<const float4*>(a.post_w + (size_t)i * 4);
+            float4 s = cache[c];
+            s.x = res[c].x + (s.x * f) * w.x; s.y = res[c].y + (s.y * f) * w.y; s.z = res[c].z + (s.z * f) * w.z; s.w = res[c].w + (s.w * f) * w.w;
             if (a.residual_out) *reinterpret_cast<float4*>(a.residual_out + (size_t)src * a.ldr + (size_t)i * 4) = s;
             cache[c] = s;
             ss += s.x * s.x + s.y * s.y + s.z * s.z + s.w * s.w;
         }
     }
-    if (!a.w[0] && !a.w[1]) return;
-    ss = wave_sum(ss);
-    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
-    __syncthreads();
-    ss = 0.f;
-#pragma unroll
-    for (int q = 0; q < BS / 64; ++q) ss += red[q];
-    const float rinv = 1.0f / sqrtf(ss / (float)a.W + a.eps);
+    if (!a.w[0] && !a.w[1] && !a.raw) return;
+    const float rinv = a.w[0] || a.w[1] ? 1.0f / sqrtf(block_sum(ss, red, BS / 64) / (float)a.W + a.eps) : 1.f;
     const int no4 = a.ldx >> 2;
 #pragma unroll
     for (int c = 0; c < NV; ++c) {
@@ -72,9 +72,13 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
         const float4 s = i < nv4 ? cache[c] : make_float4(0.f, 0.f, 0.f, 0.f);
 #pragma unroll
         for (int k = 0; k < 2; ++k) {
-            if (!a.w[k]) continue;
-            const float4 w = *reinterpret_cast<const float4*>(a.w[k] + (size_t)i * 4);
-            const float y0 = (s.x * rinv) * w.x, y1 = (s.y * rinv) * w.y, y2 = (s.z * rinv) * w.z, y3 = (s.w * rinv) * w.w;
+            const bool raw = k == 0 && a.raw;
+            if (!a.w[k] && !raw) continue;
+            float y0 = s.x, y1 = s.y, y2 = s.z, y3 = s.w;
+            if (!raw) {
+                const float4 w = *reinterpret_cast<const float4*>(a.w[k] + (size_t)i * 4);
+                y0 = (s.x * rinv) * w.x; y1 = (s.y * rinv) * w.y; y2 = (s.z * rinv) * w.z; y3 = (s.w * rinv) * w.w;
+            }
             if (a.y[k]) *reinterpret_cast<float4*>(a.y[k] + (size_t)r * a.ldx + (size_t)i * 4) = make_float4(y0, y1, y2, y3);
             if (a.xh[k]) {
                 uint16_t h0, h1, h2, h3, l0, l1, l2, l3;
@@ -89,10 +93,10 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
 
 // prompt chunks whose outputs are planes in fragment order: one workgroup = 16 rows, lane (grp, l15) owns row l15's eight consecutive
 // columns of k-tiles wave, wave + 16, ...  Reads are whole 128-byte lines, every plane store one contiguous KiB per wave.
-template <int IT>
+template <int IT, bool POST>
 __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, int rows) {
     constexpr int NW = 16;
-    __shared__ float red[NW][16];
+    __shared__ float red[POST ? 2 : 1][NW][16];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, grp = lane >> 4;
     const int KT = a.ldr >> 5, row = blockIdx.x * 16 + l15, rowc = min(row, rows - 1);
     float v[IT][8];
@@ -116,9 +120,9 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
             };
             if (a.in) for (int sl = 0; sl < a.n_slabs; ++sl) add(a.in + (size_t)sl * a.slab_stride + off);
             if (a.in2) for (int sl = 0; sl < a.n_slabs2; ++sl) add(a.in2 + (size_t)sl * a.slab_stride2 + off);
-            if (a.residual_in) add(a.residual_in + off);
+            if (!POST && a.residual_in) add(a.residual_in + off);
         }
-        if (a.residual_out && row < rows) {
+        if (!POST && a.residual_out && row < rows) {
             *reinterpret_cast<float4*>(a.residual_out + off) = s0;
             *reinterpret_cast<float4*>(a.residual_out + off + 4) = s1;
         }
@@ -127,26 +131,55 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
 #pragma unroll
         for (int e = 0; e < 8; ++e) ss += v[i][e] * v[i][e];
     }
-    ss += __shfl_xor(ss, 16);
-    ss += __shfl_xor(ss, 32);
-    if (grp == 0) red[wave][l15] = ss;
-    __syncthreads();
-    ss = 0.f;
+    auto row_rinv = [&](float (&rd)[NW][16]) {
+        ss += __shfl_xor(ss, 16);
+        ss += __shfl_xor(ss, 32);
+        if (grp == 0) rd[wave][l15] = ss;
+        __syncthreads();
+        ss = 0.f;
 #pragma unroll
-    for (int q = 0; q < NW; ++q) ss += red[q][l15];
-    const float rinv = 1.0f / sqrtf(ss / (float)a.W + a.eps);
+        for (int q = 0; q < NW; ++q) ss += rd[q][l15];
+        return 1.0f / sqrtf(ss / (float)a.W + a.eps);
+    };
+    if constexpr (POST) {
+        const float f = row_rinv(red[1]) * a.post_mult;
+        ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < IT; ++i) {
+            const int kt = wave + i * NW;
+            if (kt >= KT) continue;
+            const size_t col = (size_t)kt * 32 + grp * 8, off = (size_t)rowc * a.ldr + col;
+            float4 s0 = *reinterpret_cast<const float4*>(a.residual_in + off), s1 = *reinterpret_cast<const float4*>(a.residual_in + off + 4);
+            const float4 w0 = *reinterpret_cast<const float4*>(a.post_w + col), w1 = *reinterpret_cast<const float4*>(a.post_w + col + 4);
+            s0.x += (v[i][0] * f) * w0.x; s0.y += (v[i][1] * f) * w0.y; s0.z += (v[i][2] * f) * w0.z; s0.w += (v[i][3] * f) * w0.w;
+            s1.x += (v[i][4] * f) * w1.x; s1.y += (v[i][5] * f) * w1.y; s1.z += (v[i][6] * f) * w1.z; s1.w += (v[i][7] * f) * w1.w;
+            if (a.residual_out && row < rows) {
+                *reinterpret_cast<float4*>(a.residual_out + off) = s0;
+                *reinterpret_cast<float4*>(a.residual_out + off + 4) = s1;
+            }
+            v[i][0] = s0.x; v[i][1] = s0.y; v[i][2] = s0.z; v[i][3] = s0.w;
+            v[i][4] = s1.x; v[i][5] = s1.y; v[i][6] = s1.z; v[i][7] = s1.w;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss += v[i][e] * v[i][e];
+        }
+    }
+    const float rinv = a.w[0] || a.w[1] ? row_rinv(red[0]) : 1.f;
 #pragma unroll
     for (int i = 0; i < IT; ++i) {
         const int kt = wave + i * NW;
         if (kt >= KT) continue;
 #pragma unroll
         for (int k = 0; k < 2; ++k) {
-            if (!a.w[k]) continue;
-            const float4 w0 = *reinterpret_cast<const float4*>(a.w[k] + kt * 32 + grp * 8), w1 = *reinterpret_cast<const float4*>(a.w[k] + kt * 32 + grp * 8 + 4);
-            const float wv[8] = {w0.x, w0.y, w0.z, w0.w, w1.x, w1.y, w1.z, w1.w};
+            const bool raw = k == 0 && a.raw;
+            if (!a.w[k] && !raw) continue;
+            float wv[8];
+            if (!raw) {
+                const float4 w0 = *reinterpret_cast<const float4*>(a.w[k] + kt * 32 + grp * 8), w1 = *reinterpret_cast<const float4*>(a.w[k] + kt * 32 + grp * 8 + 4);
+                wv[0] = w0.x; wv[1] = w0.y; wv[2] = w0.z; wv[3] = w0.w; wv[4] = w1.x; wv[5] = w1.y; wv[6] = w1.z; wv[7] = w1.w;
+            }
             uint16_t h[8], l[8];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) split_bf16((v[i][e] * rinv) * wv[e], h[e], l[e]);
+            for (int e = 0; e < 8; ++e) split_bf16(raw ? v[i][e] : (v[i][e] * rinv) * wv[e], h[e], l[e]);
             const size_t o = ((size_t)blockIdx.x * KT + kt) * 64 + lane;
             reinterpret_cast<uint4*>(a.xh[k])[o] = make_uint4(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16), h[4] | ((uint32_t)h[5] << 16), h[6] | ((uint32_t)h[7] << 16));
             reinterpret_cast<uint4*>(a.xl[k])[o] = make_uint4(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16), l[4] | ((uint32_t)l[5] << 16), l[6] | ((uint32_t)l[7] << 16));
@@ -155,37 +188,34 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
 }
 
 hipError_t launch_add_norm(const AddNormArgs& a, int rows, hipStream_t s) {
-    if (a.ldr % 16 || a.ldr > kAddNormMax || ((a.w[0] || a.w[1]) && (a.ldx % 16 || a.ldx < a.ldr || a.ldx > kAddNormMax)))
+    if (a.ldr % 16 || a.ldr > kAddNormMax || ((a.w[0] || a.w[1] || a.raw) && (a.ldx % 16 || a.ldx < a.ldr || a.ldx > kAddNormMax)))
         return hipErrorInvalidValue;
     if (rows <= 0) return hipSuccess;
-    bool packed = a.w[0] && a.ldr == a.ldx && a.ldr % 32 == 0 && !a.row_idx;
-    for (int k = 0; k < 2; ++k) packed &= !a.w[k] || (a.packed[k] && a.xh[k] && !a.y[k]);
-    if (packed && rows >= 512 && a.ldr <= 4096) {
-        const int kt = a.ldr / 32, tiles = (rows + 15) / 16;
-        if (kt <= 32) add_norm_rows16_kernel<2><<<tiles, 1024, 0, s>>>(a, rows);
-        else if (kt <= 64) add_norm_rows16_kernel<4><<<tiles, 1024, 0, s>>>(a, rows);
-        else add_norm_rows16_kernel<8><<<tiles, 1024, 0, s>>>(a, rows);
-        return hipGetLastError();
-    }
-    if (rows <= 128 && a.ldr >= 2048) add_norm_kernel<1024><<<rows, 1024, 0, s>>>(a);
-    else add_norm_kernel<256><<<rows, 256, 0, s>>>(a);
+    const bool post = a.post_w != nullptr, any = a.w[0] || a.w[1] || a.raw;
+    if (a.raw && a.w[0]) return hipErrorInvalidValue;
+    bool packed = any && a.ldr == a.ldx && a.ldr % 32 == 0 && !a.row_idx && (!post || a.residual_in);
+    for (int k = 0; k < 2; ++k) packed &= !(a.w[k] || (k == 0 && a.raw)) || (a.packed[k] && a.xh[k] && !a.y[k]);
+    auto launch = [&](auto P) {
+        constexpr bool POST = decltype(P)::value;
+        if (packed && rows >= 512 && a.ldr <= 4096) {
+            const int kt = a.ldr / 32, tiles = (rows + 15) / 16;
+            if (kt <= 32) add_norm_rows16_kernel<2, POST><<<tiles, 1024, 0, s>>>(a, rows);
+            else if (kt <= 64) add_norm_rows16_kernel<4, POST><<<tiles, 1024, 0, s>>>(a, rows);
+            else add_norm_rows16_kernel<8, POST><<<tiles, 1024, 0, s>>>(a, rows);
+        } else if (rows <= 128 && a.ldr >= 2048) {
+            add_norm_kernel<1024, POST><<<rows, 1024, 0, s>>>(a);
+        } else {
+            add_norm_kernel<256, POST><<<rows, 256, 0, s>>>(a);
+        }
+    };
+    if (post) launch(std::true_type{});
+    else launch(std::false_type{});
     return hipGetLastError();
 }
 
 // ---------------------------------------------------------------------------------------------------
 // rows of the q / latent projection: one wave per (row, head); head index `heads` = the latent part
 // ---------------------------------------------------------------------------------------------------
-__device__ __forceinline__ float slab_elem(const float* p, int n_slabs, int64_t stride) {
-    float v = p[0];
-    for (int sl0 = 1; sl0 < n_slabs; sl0 += 4) {  // four independent loads per trip (clamped index, masked sum)
-        float t[4];
-#pragma unroll
-        for (int u = 0; u < 4; ++u) t[u] = p[(size_t)min(sl0 + u, n_slabs - 1) * stride];
-#pragma unroll
-        for (int u = 0; u < 4; ++u) v += sl0 + u < n_slabs ? t[u] : 0.f;
-    }
-    return v;
-}
 __device__ __forceinline__ void cache_put(const LatentCache& c, size_t block_base, int t, int d, float v) {
     const size_t o = block_base + k_packed_offset(t, d, c.D());
     if (c.f32) reinterpret_cast<float*>(c.data)[o] = v;
@@ -313,24 +343,6 @@ hipError_t launch_latent_rows(const LatentRowsArgs& a, int rows, hipStream_t s) 
     return hipGetLastError();
 }
 
-// four consecutive columns of one row (only the first `left` exist) as bf16 hi / lo, row-major or fragment order
-__device__ __forceinline__ void put_planes4(uint16_t* ph, uint16_t* pl, int row, int col, int left, int ld, int packed, const f32x4& v) {
-    uint16_t h[4], l[4];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) split_bf16(v[r], h[r], l[r]);
-    if (left >= 4 && (col & 3) == 0) {
-        const size_t o = packed ? xpack_off(row, col, ld >> 5) : (size_t)row * ld + col;
-        *reinterpret_cast<uint2*>(ph + o) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
-        *reinterpret_cast<uint2*>(pl + o) = make_uint2(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16));
-        return;
-    }
-    for (int r = 0; r < 4 && r < left; ++r) {
-        const size_t o = packed ? xpack_off(row, col + r, ld >> 5) : (size_t)row * ld + col + r;
-        ph[o] = h[r];
-        pl[o] = l[r];
-    }
-}
-
 // ---------------------------------------------------------------------------------------------------
 // per-head products: wave = NT n-tiles x MT m-tiles of one head, fragments straight from memory
 // ---------------------------------------------------------------------------------------------------
@@ -400,7 +412,18 @@ __global__ void __launch_bounds__(256) head_gemm_kernel(HeadGemmArgs a) {
         for (int b = 0; b < MT; ++b) {
             const int row = m0 + b * 16 + l15;
             if (row >= a.M) continue;
-            const f32x4 v = acc[n][b];
+            f32x4 v = acc[n][b];
+            if (a.decay_rate) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    if (head == 0) {
+                        const int f = min(f0 + r, a.n_valid - 1);
+                        v[r] = expf(-a.decay_rate[f] * softplusf(v[r] + a.decay_bias[f]));
+                    } else {
+                        v[r] = 1.0f / (1.0f + expf(-v[r]));
+                    }
+                }
+            }
             if (a.y) {
                 float* o = a.y + (size_t)row * a.y_row + (size_t)head * a.y_head + f0;
                 if (whole && ((a.y_row | a.y_head) & 3) == 0) *reinterpret_cast<float4*>(o) = make_float4(v[0], v[1], v[2], v[3]);

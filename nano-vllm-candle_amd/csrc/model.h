@@ -92,9 +92,13 @@ struct SeqState {
     int released = 0;  // leading blocks given back because no window reaches them (blocks[i] = -1)
 };
 
+struct DecoderImpl;  // decoder.h
+
 struct nvllm_model {
+    nvllm_model();
+    ~nvllm_model();
     nvllm_ctx* ctx = nullptr;
-    LatentModel* lat = nullptr;  // latent-attention decoder (latent_model.cpp); nullptr: Qwen3
+    std::unique_ptr<DecoderImpl> dec;  // a decoder built from layer descriptions; nullptr: Qwen3
     nvllm_qwen3_config cfg{};
     int H = 0, hd = 0, L = 0, nh_l = 0, kv_l = 0, I_l = 0, V_l = 0, gqa = 1;
     bf16_bits* embed = nullptr;  // [V][H] row-major bf16 (gather table, replicated)
@@ -195,7 +199,7 @@ constexpr size_t kStampStride = (size_t)1024 * 16 * 8;  // u64 per launch: [<= 1
 #define STAMPS(args_, m_) do { } while (0)
 #endif
 
-enum { PROF_ATTN = 1, PROF_GEMM = 2, PROF_NORM = 3, PROF_QK = 4, PROF_SILU = 5, PROF_LMHEAD = 6, PROF_EMPTY = 7 };
+enum { PROF_ATTN = 1, PROF_GEMM = 2, PROF_NORM = 3, PROF_QK = 4, PROF_SILU = 5, PROF_LMHEAD = 6, PROF_EMPTY = 7, PROF_RECUR = 8 };
 
 // bracket one launch with HIP events on the library stream when its class is being profiled
 #define PROF(m_, kind_, expr_)                                                           \

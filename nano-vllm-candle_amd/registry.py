@@ -3,10 +3,12 @@ import json
 import os
 
 from .berevik import BerevikForCausalLM
+from .gopunex import GopunexForCausalLM
 from .qwen3 import Qwen3ForCausalLM
 
 MODELS = {
     "Berevik": BerevikForCausalLM,
+    "Gopunex": GopunexForCausalLM,
     "Qwen3ForCausalLM": Qwen3ForCausalLM,
 }
 
