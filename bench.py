@@ -73,6 +73,11 @@ def parse():
     ap.add_argument("--berevik-window", type=int, default=1 << 20, help="attention window of the --berevik layers")
     ap.add_argument("--berevik-batch", type=int, default=64)
     ap.add_argument("--berevik-prompt", type=int, default=1024)
+    ap.add_argument("--gopunex", nargs="*", metavar="SIZE", default=None,
+                    help="instead of the headline: the Gopunex design beside Qwen3 layers of equal size (bench_gopunex.py; sizes 1k 2k 4k, default all)")
+    ap.add_argument("--gopunex-mixers", nargs="+", default=None, help="attention, channel_delta, lightning, mixed (default all)")
+    ap.add_argument("--gopunex-batch", type=int, default=64)
+    ap.add_argument("--gopunex-prompt", type=int, default=1024)
     ap.add_argument("--option", action="append", default=[], metavar="NAME=VALUE",
                     help="A/B aid: nvllm_debug_set_option on the headline model before kv_alloc (repeatable)")
     ap.add_argument("--launch-timeout", type=float, default=1500.0, help="plain `python bench.py --gpus N`: overall limit of the rank processes")
@@ -327,6 +332,11 @@ def live_traffic(a, dom_kernel):
 
 def main():
     a = parse()
+    if a.gopunex is not None:
+        import bench_gopunex
+
+        bench_gopunex.main(a.gopunex or None, batch=a.gopunex_batch, prompt=a.gopunex_prompt, mixers=a.gopunex_mixers or bench_gopunex.MIXERS)
+        return
     if a.berevik is not None:
         import bench_berevik
 

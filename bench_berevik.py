@@ -24,7 +24,7 @@ def berevik_config(pkg, z, vocab, window):
     return pkg.BerevikConfig(vocab, z["width"], [(mix, GatedMlpConfig(z["ff"], 7.0))] * z["layers"], 1e-6, 1.0, 30.0)
 
 
-def measure(model, batch, prompt, steps, rng, vocab):
+def measure(model, batch, prompt, steps, rng, vocab, classes=CLASSES):
     model.kv_alloc(batch * -(-(prompt + 4 * steps + 64) // 256), batch, max_batched_tokens=8192)
     toks = [rng.integers(0, vocab, prompt, dtype=np.uint32) for _ in range(batch)]
     ids = list(range(batch))
@@ -38,7 +38,7 @@ def measure(model, batch, prompt, steps, rng, vocab):
         best = min(best, time.perf_counter() - t0)
     out["prefill_ms"], out["prefill_tokens_per_s"] = best * 1e3, batch * prompt / best
     out["prefill_class_ms"] = {}
-    for c in CLASSES:
+    for c in classes:
         model.profile_kernel(c)
         model.step(ids, toks, True)
         ms, n = model.profile_read()
@@ -57,7 +57,7 @@ def measure(model, batch, prompt, steps, rng, vocab):
     dt = (time.perf_counter() - t0) / steps
     out["decode_ms_per_step"], out["decode_tokens_per_s"] = dt * 1e3, batch / dt
     out["decode_class_ms"] = {}
-    for c in CLASSES:
+    for c in classes:
         model.profile_kernel(c)
         for _ in range(4):
             model.decode_next(False)

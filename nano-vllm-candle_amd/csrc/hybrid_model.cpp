@@ -318,7 +318,7 @@ int HybridModel::load_tensor(nvllm_model* m, const char* name, const void* data,
                         for (int d = 0; d < w.n_bias; ++d) t[(size_t)n * w.n_bias + d] = (float)(h.f32((int64_t)w.bucket[d] * H + h0 + n) * 1.4426950408889634);
                     rc = put(w.table, t);
                 }
-            } else if (w.c.v_mix && !strcmp(s, "vmix")) {
+            } else if (!strcmp(s, "vmix")) {  // unused where nothing is mixed
                 if (!(rc = want(1, 1, 0))) rc = put(w.vmix, {h.f32(0)});
             } else return fail(ctx, NVLLM_EINVAL, "%s", unknown.c_str());
         } else if (!w.delta()) {

@@ -2,7 +2,6 @@
 batches, window edges, block and slot reuse, greedy generation through the engine -- in both precisions."""
 import json
 import os
-import struct
 import subprocess
 import sys
 
@@ -11,6 +10,7 @@ import pytest
 
 from oracle import berevik_oracle as B
 from tests.berevik_util import CONFIGS, EVEN, MIXED, TOL, beacon_weights, config, layer, row_err, sharp_weights
+from tests.util import write_checkpoint
 
 pytestmark = pytest.mark.gpu
 DTYPES = ("bfloat16", "float32")
@@ -321,18 +321,6 @@ def test_two_ranks_match_one(dtype):
     for lg, nxt in res:
         assert row_err(lg, ref) < TOL[dtype]
         assert nxt == int(ref[1].argmax())
-
-
-def write_checkpoint(path, cfg, w):
-    header, blobs, at = {}, [], 0
-    for k, v in w.items():
-        b = (np.ascontiguousarray(v, np.float32).view(np.uint32) >> 16).astype("<u2").tobytes()
-        header[k] = {"dtype": "BF16", "shape": list(v.shape), "data_offsets": [at, at + len(b)]}
-        blobs.append(b)
-        at += len(b)
-    h = json.dumps(header).encode()
-    (path / "model.safetensors").write_bytes(struct.pack("<Q", len(h)) + h + b"".join(blobs))
-    (path / "config.json").write_text(json.dumps(cfg))
 
 
 @pytest.mark.parametrize("dtype", DTYPES)

@@ -1,3 +1,6 @@
+import json
+import struct
+
 import numpy as np
 
 
@@ -165,3 +168,16 @@ def random_calls(m, om, cfg, seed, iters, NB, MS, lock=None, max_new=2, lens_men
     assert m.free_blocks() == NB
     assert len(ties) <= max(3, ops // 20), ties  # ties are rare by construction
     return ops, worst
+
+
+def write_checkpoint(path, cfg, w):
+    """config.json and a bf16 model.safetensors of a layered model in directory `path`"""
+    header, blobs, at = {}, [], 0
+    for k, v in w.items():
+        b = (np.ascontiguousarray(v, np.float32).view(np.uint32) >> 16).astype("<u2").tobytes()
+        header[k] = {"dtype": "BF16", "shape": list(v.shape), "data_offsets": [at, at + len(b)]}
+        blobs.append(b)
+        at += len(b)
+    h = json.dumps(header).encode()
+    (path / "model.safetensors").write_bytes(struct.pack("<Q", len(h)) + h + b"".join(blobs))
+    (path / "config.json").write_text(json.dumps(cfg))
