@@ -153,6 +153,20 @@ __device__ __forceinline__ void q_frag(const float* p, bool valid, f16x8& h, f16
     }
 }
 
+// weights of eight tokens as f16 hi (rounded towards zero) + lo: 21 bits together
+__device__ __forceinline__ void split_weights(const float (&pa)[4], const float (&pb)[4], f16x8& h, f16x8& l) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const float x = i < 2 ? pa[2 * i] : pb[2 * i - 4], y = i < 2 ? pa[2 * i + 1] : pb[2 * i - 3];
+        const auto hi = __builtin_amdgcn_cvt_pkrtz(x, y);
+        const auto lo = __builtin_amdgcn_cvt_pkrtz(x - (float)hi[0], y - (float)hi[1]);
+        h[2 * i] = (_Float16)hi[0];
+        h[2 * i + 1] = (_Float16)hi[1];
+        l[2 * i] = (_Float16)lo[0];
+        l[2 * i + 1] = (_Float16)lo[1];
+    }
+}
+
 // ---------------------------------------------------------------------------------------------------
 // decode: one workgroup = one token x up to 16 heads of one group x a range of 32-token tiles; four waves take alternate tiles
 // ---------------------------------------------------------------------------------------------------
@@ -236,17 +250,14 @@ __global__ void __launch_bounds__(256) bias_decode_kernel(BiasAttnArgs a) {
         const float mn = fmaxf(m, mt), alpha = __builtin_amdgcn_exp2f(m - mn);
         m = mn;
         f16x8 P, Pl;
-        float ps = 0.f;
+        float ps = 0.f, pa[4], pb[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const float pa = tokA + r <= pos ? __builtin_amdgcn_exp2f(sa[r] - mn) : 0.f;
-            const float pb = tokB + r <= pos ? __builtin_amdgcn_exp2f(sb[r] - mn) : 0.f;
-            ps += pa + pb;
-            P[r] = (_Float16)pa;
-            P[4 + r] = (_Float16)pb;
-            Pl[r] = (_Float16)(pa - (float)P[r]);
-            Pl[4 + r] = (_Float16)(pb - (float)P[4 + r]);
+            pa[r] = tokA + r <= pos ? __builtin_amdgcn_exp2f(sa[r] - mn) : 0.f;
+            pb[r] = tokB + r <= pos ? __builtin_amdgcn_exp2f(sb[r] - mn) : 0.f;
+            ps += pa[r] + pb[r];
         }
+        split_weights(pa, pb, P, Pl);
         lsum = lsum * alpha + ps;
         if (__any(alpha != 1.0f)) {
 #pragma unroll
@@ -359,14 +370,15 @@ hipError_t launch_bias_decode(const BiasAttnArgs& a, int rows, int parts, hipStr
 
 // ---------------------------------------------------------------------------------------------------
 // prompt chunks: one workgroup = 128 (token, head of the group) rows of one sequence; four waves of two 16-row tiles share the
-// 32-token K and V tiles staged in LDS (two buffers, the next tile in flight in registers)
+// 32-token K and V tiles, copied straight into LDS (two buffers, the next tile in flight)
 // ---------------------------------------------------------------------------------------------------
 template <int DC, int VC>
 __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, int bias_lds) {
     constexpr int MT = 2, F = 2 * DC + VC, NL = (F + 3) / 4;  // fragments per tile, per wave
     __shared__ __attribute__((aligned(16))) uint4 buf[2][F * 64];
     extern __shared__ float tab[];  // [gqa][n_bias] when bias_lds
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, grp = lane >> 4;
+    const int lane = threadIdx.x & 63, l15 = lane & 15, grp = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int tile = a.tile_order ? a.tile_order[blockIdx.x] : blockIdx.x;
     const int gqa = a.heads / a.kv.kv, kvh = blockIdx.y / gqa, f0 = (blockIdx.y % gqa) * 128;
     const int row0 = a.tile_row0[tile], total = a.tile_nrows[tile] * gqa, slot = a.tile_slot[tile];
@@ -378,23 +390,18 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
     const _Float16* kd = reinterpret_cast<const _Float16*>(a.kv.k);
     const _Float16* vd = reinterpret_cast<const _Float16*>(a.kv.v);
     const int far = a.n_bias - 1;
-    uint4 pre[NL];
-    auto fetch = [&](int t) {
+    // fragments of tile t straight into LDS, a KiB per wave and copy
+    auto stage = [&](int t, uint4* b) {
         const size_t blk = (size_t)bt[t >> 3] * a.kv.kv + kvh;
         const uint4* kp = reinterpret_cast<const uint4*>(kd + blk * (kBlockTokens * DC * 32) + (size_t)(t & 7) * (2 * DC * 512));
-        const uint4* vp = reinterpret_cast<const uint4*>(vd + blk * (kBlockTokens * VC * 16) + (size_t)(t & 7) * (VC * 512));
+        const uint4* vp = reinterpret_cast<const uint4*>(vd + blk * (kBlockTokens * VC * 16) + (size_t)(t & 7) * (VC * 512)) - 2 * DC * 64;
 #pragma unroll
         for (int i = 0; i < NL; ++i) {
-            const int f = min(wave + i * 4, F - 1);
-            pre[i] = f < 2 * DC ? kp[f * 64 + lane] : vp[(f - 2 * DC) * 64 + lane];
+            const int f = wave + i * 4;
+            if (F % 4 == 0 || f < F) __builtin_amdgcn_global_load_lds((gptr_t)((f < 2 * DC ? kp : vp) + f * 64 + lane), (lptr_t)(b + f * 64), 16, 0, 0);
         }
     };
-    auto park = [&](uint4* b) {
-#pragma unroll
-        for (int i = 0; i < NL; ++i)
-            if (wave + i * 4 < F) b[(wave + i * 4) * 64 + lane] = pre[i];
-    };
-    fetch(0);
+    stage(0, buf[0]);
     if (bias_lds)
         for (int i = threadIdx.x; i < gqa * a.n_bias; i += 256) tab[i] = a.bias[(size_t)kvh * gqa * a.n_bias + i];
     int my_pos[MT];
@@ -426,11 +433,10 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
 #pragma unroll
         for (int d = 0; d < VC; ++d) o[u][d] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    park(buf[0]);
-    __syncthreads();
+    dma_publish_barrier();
     for (int t = 0; t < nt; ++t) {
         const uint4* b = buf[t & 1];
-        if (t + 1 < nt) fetch(t + 1);
+        if (t + 1 < nt) stage(t + 1, buf[(t + 1) & 1]);  // its last readers have passed the barrier of the previous tile
         const int tokA = (t << 5) + grp * 4, tokB = tokA + 16;
         f32x4 sa[MT], sb[MT];
         if (a.n_bias && pmin - (t << 5) - 31 < far) {  // some distance below the last bucket
@@ -474,18 +480,15 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
             mt = fmaxf(mt, __shfl_xor(mt, 32));
             const float mn = fmaxf(m[u], mt), alpha = __builtin_amdgcn_exp2f(m[u] - mn);
             m[u] = mn;
-            float ps = 0.f;
+            float ps = 0.f, pa[4], pb[4];
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 // a row that sees nothing of any tile so far has mn = -1e30: its masked scores would count as exp2(0)
-                const float pa = edge && tokA + r > my_pos[u] ? 0.f : __builtin_amdgcn_exp2f(sa[u][r] - mn);
-                const float pb = edge && tokB + r > my_pos[u] ? 0.f : __builtin_amdgcn_exp2f(sb[u][r] - mn);
-                ps += pa + pb;
-                P[u][r] = (_Float16)pa;
-                P[u][4 + r] = (_Float16)pb;
-                Pl[u][r] = (_Float16)(pa - (float)P[u][r]);
-                Pl[u][4 + r] = (_Float16)(pb - (float)P[u][4 + r]);
+                pa[r] = edge && tokA + r > my_pos[u] ? 0.f : __builtin_amdgcn_exp2f(sa[u][r] - mn);
+                pb[r] = edge && tokB + r > my_pos[u] ? 0.f : __builtin_amdgcn_exp2f(sb[u][r] - mn);
+                ps += pa[r] + pb[r];
             }
+            split_weights(pa, pb, P[u], Pl[u]);
             lsum[u] = lsum[u] * alpha + ps;
             if (__any(alpha != 1.0f)) {
 #pragma unroll
@@ -501,8 +504,7 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
                 o[u][d] = __builtin_amdgcn_mfma_f32_16x16x32_f16(v, Pl[u], o[u][d], 0, 0, 0);
             }
         }
-        if (t + 1 < nt) park(buf[(t + 1) & 1]);
-        __syncthreads();
+        dma_publish_barrier();
     }
 #pragma unroll
     for (int u = 0; u < MT; ++u) {

@@ -44,6 +44,11 @@ __device__ __forceinline__ float max3_raw(float a, float b, float c) {
 // rcp(inf) = 0, i.e. -0 for very negative gates; no NaN.  The fine-seam op keeps the division.
 __device__ __forceinline__ float silu_mul(float g, float u) { return (g * __builtin_amdgcn_rcpf(1.0f + __expf(-g))) * u; }
 
+__device__ __forceinline__ float relu2(float x) {
+    x = fmaxf(x, 0.f);
+    return x * x;
+}
+
 // any GluSpec (uniform branch: the plain form costs nothing extra)
 __device__ __forceinline__ float glu_mul(float g, float u, const GluSpec& s) {
     if (s.limit <= 0.f) return silu_mul(g, u);

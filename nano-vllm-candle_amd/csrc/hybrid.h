@@ -109,8 +109,6 @@ struct RecurArgs {
     const int* pos = nullptr;        // position 0: the state starts at zero
     float* o = nullptr;              // [rows][heads][vdim_p]
 };
-hipError_t launch_recurrence(const RecurArgs& a, hipStream_t s);
-
 // RMS norm of o over one head or over all heads, times weight and gate, as context planes / f32 rows [rows][ld], column head * vdim
 struct GatedNormArgs {
     const float* o = nullptr;        // [rows][heads][vdim_p]
@@ -129,6 +127,8 @@ struct GatedNormArgs {
     int ld = 0, packed = 0;
 };
 hipError_t launch_gated_norm(const GatedNormArgs& a, int rows, hipStream_t s);
+// norm (nullable): decode with per-head norms, the gated output norm in the same launch (o is not written)
+hipError_t launch_recurrence(const RecurArgs& a, const GatedNormArgs* norm, hipStream_t s);
 
 // rows after the q / k / v / gate projection of the constant-decay recurrence: silu(q, k, v), sigmoid(gate)
 struct LinearRowsArgs {

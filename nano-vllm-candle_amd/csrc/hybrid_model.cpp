@@ -593,7 +593,11 @@ int HybridModel::recurrence(nvllm_model* m, HybridLayer& w, int ns, int R, int q
         gn.gate = g; gn.gate_row = (int64_t)w.heads * w.vdim_p;
         gn.whole = 1; gn.all = w.c.heads * w.c.vdim;
     }
-    PROF(m, PROF_RECUR, launch_recurrence(rc, s));
+    if (seg.single && !gn.whole) {
+        PROF(m, PROF_RECUR, launch_recurrence(rc, &gn, s));
+        return NVLLM_OK;
+    }
+    PROF(m, PROF_RECUR, launch_recurrence(rc, nullptr, s));
     if (gn.whole && ctx->tp_size > 1) {  // the norm runs over every rank's heads (padding columns are zero)
         const int n = w.heads * w.vdim_p, c0[2] = {0, 0}, nn[2] = {n, 0};
         HIPCHK(ctx, launch_rows_ssq(out, 1, 0, n, nullptr, c0, nn, R, ssq, s));
@@ -666,9 +670,14 @@ int HybridModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
         if (!rc) rc = product(m, po, ctx_f, m->ctxh, m->ctxl, w.o, R, &ns);
         if (!rc) rc = add(ns, w.norm1, w.ff ? &pu : last ? nullptr : &pnext);
         if (!rc && w.ff) {
-            rc = product(m, pu, y, m->xh, m->xl, w.up, R, &ns);
-            if (rc) return rc;
-            PROF(m, PROF_SILU, launch_relu2(m->slabs, ns, (int64_t)R * w.ff_p, R, w.ff_p, f32 ? nullptr : m->xh2, f32 ? nullptr : m->xl2, pd.packed, f32 ? act_f : nullptr, s));
+            if (pu.kind == P_TILE && gemm_tile_ok(R, w.ff_p, Kw, 4, m->opt_tile_min_wgs)) {
+                PROF(m, PROF_GEMM, launch_gemm_tile(m->xh, m->xl, w.up, R, 4, nullptr, m->xh2, m->xl2, pd.packed, m->opt_tile_min_wgs, 1, nullptr, s));
+                ++m->tile_launches;
+            } else {
+                rc = product(m, pu, y, m->xh, m->xl, w.up, R, &ns);
+                if (rc) return rc;
+                PROF(m, PROF_SILU, launch_relu2(m->slabs, ns, (int64_t)R * w.ff_p, R, w.ff_p, f32 ? nullptr : m->xh2, f32 ? nullptr : m->xl2, pd.packed, f32 ? act_f : nullptr, s));
+            }
             rc = product(m, pd, act_f, m->xh2, m->xl2, w.down, R, &ns);
             if (!rc) rc = add(ns, w.norm2, last ? nullptr : &pnext);
         }

@@ -19,9 +19,7 @@ __global__ void __launch_bounds__(256) relu2_kernel(const float* __restrict__ in
         const int r = (int)(i / (F >> 2)), c = (int)(i % (F >> 2)) * 4;
         float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
         add_slabs(s, in + (size_t)r * F + c, n_slabs, slab_stride);
-        f32x4 v = {fmaxf(s.x, 0.f), fmaxf(s.y, 0.f), fmaxf(s.z, 0.f), fmaxf(s.w, 0.f)};
-#pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] *= v[e];
+        const f32x4 v = {relu2(s.x), relu2(s.y), relu2(s.z), relu2(s.w)};
         if (y) *reinterpret_cast<float4*>(y + (size_t)r * F + c) = make_float4(v[0], v[1], v[2], v[3]);
         if (hi) put_planes4(hi, lo, r, c, 4, F, packed, v);
     }

@@ -187,7 +187,7 @@ hipError_t launch_qk_norm_rope_kvwrite(const QkvArgs& a, int rows, hipStream_t s
 
 // ---- prefill GEMM (tile_gemm.hip): 256 x 256/192 output tile, both operands in fragment order -------------------
 // x planes in xpack_off order; mode 0: out f32 [M][N]; mode 2: w = interleaved gate/up, act hi/lo [M][N/2] (row-major or
-// xpack_off order).  min_wgs: smallest grid the kernel is used for (a 256-row tile needs many rows to fill 256 CUs).
+// xpack_off order); mode 4: squared ReLU as hi/lo planes [M][N].  min_wgs: smallest grid the kernel is used for (a 256-row tile needs many rows to fill 256 CUs).
 // hipErrorNotSupported = shape not covered.
 bool gemm_tile_ok(int M, int N, int K, int mode, int min_wgs);
 // mode 0 with n_slabs != nullptr may split K (narrow outputs, 128-row blocks): out = [*n_slabs][M][N], up to max_split slabs

@@ -153,23 +153,101 @@ __global__ void __launch_bounds__(256) recurrence_kernel(RecurArgs a) {
     state_io<R4>(S, st, lane, true);
 }
 
-bool recur_ok(int dim, int vdim) { return dim >= 1 && dim <= 512 && vdim >= 1; }
+// ---------------------------------------------------------------------------------------------------
+// decode: one workgroup = one (row, head); a wave takes every fourth block of eight columns, four blocks' state in flight.  With
+// NORM (per-head norms) the gated output norm follows in the same launch.
+// ---------------------------------------------------------------------------------------------------
+template <int R4, bool DELTA, bool NORM>
+__global__ void __launch_bounds__(256) recurrence_decode_kernel(RecurArgs a, GatedNormArgs n) {
+    constexpr int DP = R4 * 64, NB = R4 <= 2 ? 4 : 1;
+    extern __shared__ float o_lds[];  // [vdim_p], NORM
+    __shared__ float red[4];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, p = lane & 15, cg = lane >> 4;
+    const int head = blockIdx.x, row = blockIdx.y, slot = a.seg.slot[row], qh = head / (a.heads / a.q_heads), blocks = a.vdim_p / 8;
+    const bool fresh = a.pos[row] == 0;
+    float* st = a.state + ((size_t)slot * a.heads + head) * DP * a.vdim_p;
+    float4 k[R4], q[R4], g[R4];
+    const float4* kp = reinterpret_cast<const float4*>(a.k + ((size_t)row * a.q_heads + qh) * DP) + p;
+    const float4* qp = reinterpret_cast<const float4*>(a.q + ((size_t)row * a.q_heads + qh) * DP) + p;
+    const float4* gp = reinterpret_cast<const float4*>(DELTA ? a.g + (size_t)row * a.g_row + (size_t)head * DP : a.k) + p;
+    const float* vp = a.v + ((size_t)row * a.heads + head) * a.vdim_p + cg * 2;
+#pragma unroll
+    for (int r = 0; r < R4; ++r) {
+        k[r] = kp[r * 16];
+        q[r] = qp[r * 16];
+        g[r] = DELTA ? gp[r * 16] : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+    const float decay = DELTA ? 1.f : a.decay[head], beta = DELTA ? a.beta[(size_t)row * a.heads + head] : 0.f;
+    for (int b0 = wave; b0 < blocks; b0 += 4 * NB) {
+        float S[NB][R4][2][4];
+        float2 v[NB];
+#pragma unroll
+        for (int u = 0; u < NB; ++u) {
+            const int b = min(b0 + u * 4, blocks - 1);
+            state_io<R4>(S[u], st + (size_t)b * 8 * DP, lane, false);
+            v[u] = *reinterpret_cast<const float2*>(vp + b * 8);
+        }
+#pragma unroll
+        for (int u = 0; u < NB; ++u) {
+            const int b = b0 + u * 4;
+            if (b >= blocks) continue;
+            if (fresh) {
+#pragma unroll
+                for (int r = 0; r < R4; ++r)
+#pragma unroll
+                    for (int c = 0; c < 2; ++c)
+#pragma unroll
+                        for (int i = 0; i < 4; ++i) S[u][r][c][i] = 0.f;
+            }
+            const float2 o = recur_token<R4, DELTA>(S[u], k, q, g, decay, v[u], beta);
+            state_io<R4>(S[u], st + (size_t)b * 8 * DP, lane, true);
+            if (p == 0) {
+                if (NORM) *reinterpret_cast<float2*>(o_lds + b * 8 + cg * 2) = o;
+                else *reinterpret_cast<float2*>(a.o + ((size_t)row * a.heads + head) * a.vdim_p + b * 8 + cg * 2) = o;
+            }
+        }
+    }
+    if constexpr (NORM) {
+        __syncthreads();
+        float ss = 0.f;
+        for (int e = threadIdx.x; e < n.vdim; e += 256) ss += o_lds[e] * o_lds[e];
+        const float rinv = 1.0f / sqrtf(block_sum(ss, red, 4) / (float)n.vdim + n.eps);
+        const float* gate = n.gate + (size_t)row * n.gate_row + (size_t)head * n.gate_head;
+        for (int e = threadIdx.x; e < n.vdim; e += 256) {
+            const float x = (o_lds[e] * rinv) * n.weight[e] * gate[e];
+            const int col = head * n.vdim + e;
+            if (n.of) n.of[(size_t)row * n.ld + col] = x;
+            if (n.oh) {
+                const size_t at = n.packed ? xpack_off(row, col, n.ld >> 5) : (size_t)row * n.ld + col;
+                split_bf16(x, n.oh[at], n.ol[at]);
+            }
+        }
+    }
+}
 
+bool recur_ok(int dim, int vdim) { return dim >= 1 && dim <= 512 && vdim >= 1 && vdim <= 8192; }
+
+template <int R4, bool DELTA>
+static void recurrence_t(const RecurArgs& a, const GatedNormArgs* norm, hipStream_t s) {
+    if (!a.seg.single) recurrence_kernel<R4, DELTA><<<dim3(a.heads * (a.vdim_p / 32), a.seg.count), 256, 0, s>>>(a);
+    else if (norm) recurrence_decode_kernel<R4, DELTA, true><<<dim3(a.heads, a.seg.count), 256, (size_t)a.vdim_p * 4, s>>>(a, *norm);
+    else recurrence_decode_kernel<R4, DELTA, false><<<dim3(a.heads, a.seg.count), 256, 0, s>>>(a, GatedNormArgs());
+}
 template <bool DELTA>
-static hipError_t recurrence_launch(const RecurArgs& a, hipStream_t s) {
-    const dim3 grid(a.heads * (a.vdim_p / 32), a.seg.count);
+static hipError_t recurrence_launch(const RecurArgs& a, const GatedNormArgs* norm, hipStream_t s) {
     switch (a.dim_p / 64) {
-#define NVLLM_RC(R_) case R_: recurrence_kernel<R_, DELTA><<<grid, 256, 0, s>>>(a); break;
+#define NVLLM_RC(R_) case R_: recurrence_t<R_, DELTA>(a, norm, s); break;
         NVLLM_RC(1) NVLLM_RC(2) NVLLM_RC(3) NVLLM_RC(4) NVLLM_RC(5) NVLLM_RC(6) NVLLM_RC(7) NVLLM_RC(8)
 #undef NVLLM_RC
         default: return hipErrorNotSupported;
     }
     return hipGetLastError();
 }
-hipError_t launch_recurrence(const RecurArgs& a, hipStream_t s) {
+hipError_t launch_recurrence(const RecurArgs& a, const GatedNormArgs* norm, hipStream_t s) {
     if (a.dim_p % 64 || a.vdim_p % 32 || a.q_heads < 1 || a.heads % a.q_heads || (a.g && !a.beta) || (!a.g && !a.decay) || (a.g_row & 3)) return hipErrorInvalidValue;
+    if (norm && (!a.seg.single || norm->whole || norm->heads != a.heads || norm->vdim_p != a.vdim_p || norm->heads * norm->vdim > norm->ld)) return hipErrorInvalidValue;
     if (a.seg.count <= 0) return hipSuccess;
-    return a.g ? recurrence_launch<true>(a, s) : recurrence_launch<false>(a, s);
+    return a.g ? recurrence_launch<true>(a, norm, s) : recurrence_launch<false>(a, norm, s);
 }
 
 }  // namespace nvllm

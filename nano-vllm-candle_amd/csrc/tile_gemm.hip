@@ -18,6 +18,7 @@
 //     operand re-reads hit that XCD's L2.
 // MODE 0: f32 [M][N].  MODE 2: W is the gate/up matrix interleaved in 16-row tiles; the epilogue writes
 // silu(gate)*up as hi/lo planes [M][N/2] (row-major or xpack_off order) -- SiluAndMul, activation.rs:13-18.
+// MODE 4: squared ReLU of every feature as hi/lo planes [M][N].
 // MODE 3 (NTW = 8, head_dim 128): W is the fused QKV matrix, so a wave's 64 rows x 128 features are 64 tokens of ONE
 // head and the epilogue is the whole of qwen3.rs:208-234 on registers: RMS norm over the head (q_norm / k_norm BEFORE
 // RoPE), half-split RoPE (rotary_embedding.rs:82-107: features d and d+64 sit in the same lane, accumulators j and j+4),
@@ -35,7 +36,7 @@ struct TileArgs {
     const uint4* xl = nullptr;
     const uint4* wp = nullptr;  // [N/16][KT][64] uint4
     float* out = nullptr;       // MODE 0
-    uint16_t* act_hi = nullptr; // MODE 2
+    uint16_t* act_hi = nullptr; // MODE 2, 4
     uint16_t* act_lo = nullptr;
     int act_packed = 0;
     GluSpec glu;                // MODE 2
@@ -376,6 +377,23 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
                 }
             }
         }
+    } else if constexpr (MODE == 4) {
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+            const int row = row0 + b * 16 + l15;
+            if (row < a.M) {
+#pragma unroll
+                for (int j = 0; j < NTW; ++j) {
+                    const int f0 = (nt0 + j) * 16 + grp * 4;
+                    uint16_t h[4], l[4];
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) split_bf16(relu2(acc[j][b][r]), h[r], l[r]);
+                    const size_t xo = a.act_packed ? xpack_off(row, f0, a.N >> 5) : (size_t)row * a.N + f0;
+                    *reinterpret_cast<uint2*>(a.act_hi + xo) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
+                    *reinterpret_cast<uint2*>(a.act_lo + xo) = make_uint2(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16));
+                }
+            }
+        }
     } else {
         static_assert(MODE != 2 || NTW % 2 == 0, "gate and up tiles of a feature live in one wave");
         const int I = a.N >> 1;
@@ -464,6 +482,7 @@ hipError_t launch_gemm_tile(const bf16_bits* xh, const bf16_bits* xl, const Pack
     const TileShape t = tile_shape(M, w.N, w.K, mode, min_wgs, n_slabs ? max_split : 1);
     if (!t.ntw) return hipErrorNotSupported;
     if (mode == 2 && act_packed && (w.N / 2) % 32 != 0) return hipErrorNotSupported;
+    if (mode == 4 && act_packed && w.N % 32 != 0) return hipErrorNotSupported;
     TileArgs a;
     a.xh = reinterpret_cast<const uint4*>(xh); a.xl = reinterpret_cast<const uint4*>(xl); a.wp = w.data;
     a.out = out; a.act_hi = act_hi; a.act_lo = act_lo; a.act_packed = act_packed; a.glu = glu;
@@ -476,6 +495,10 @@ hipError_t launch_gemm_tile(const bf16_bits* xh, const bf16_bits* xl, const Pack
     if (mode == 2) {
         if (t.wn == 4) return tile_launch_t<4, 4, 2>(a, 1, s);
         return t.ntw == 8 ? tile_launch_t<8, 2, 2>(a, 1, s) : tile_launch_t<6, 2, 2>(a, 1, s);
+    }
+    if (mode == 4) {
+        if (t.wn == 4) return tile_launch_t<4, 4, 4>(a, 1, s);
+        return t.ntw == 8 ? tile_launch_t<8, 2, 4>(a, 1, s) : tile_launch_t<6, 2, 4>(a, 1, s);
     }
     return hipErrorInvalidValue;
 }
