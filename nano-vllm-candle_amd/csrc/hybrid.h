@@ -130,6 +130,23 @@ hipError_t launch_gated_norm(const GatedNormArgs& a, int rows, hipStream_t s);
 // norm (nullable): decode with per-head norms, the gated output norm in the same launch (o is not written)
 hipError_t launch_recurrence(const RecurArgs& a, const GatedNormArgs* norm, hipStream_t s);
 
+// prompt chunks: the same recurrences in pieces of 16 tokens (recurrent_chunk.hip); a sequence's pieces follow each other
+constexpr int kPiece = 16;
+struct PieceArgs {
+    const int* row0 = nullptr;       // first row and number of rows of every piece
+    const int* n = nullptr;
+    const int* seg_piece0 = nullptr; // [segments + 1] first piece of every segment
+    int count = 0;
+    float* pair = nullptr;           // scratch per (piece, head): [16][16]
+    float* qt = nullptr;             // delta rule: [16][dim_p] decayed queries,
+    float* wt = nullptr;             // [16][dim_p] solved keys,
+    float* kt = nullptr;             // [dim_p][16] keys decayed to the piece's end,
+    float* decay = nullptr;          // [dim_p] decays of the whole piece
+};
+bool piece_scan_ok(int dim_p);
+// v is overwritten for the delta rule
+hipError_t launch_piece_scan(const RecurArgs& a, const PieceArgs& c, hipStream_t s);
+
 // rows after the q / k / v / gate projection of the constant-decay recurrence: silu(q, k, v), sigmoid(gate)
 struct LinearRowsArgs {
     const float* in = nullptr;       // columns: heads * dim query, heads * dim key, heads * vdim value, heads * vdim gate

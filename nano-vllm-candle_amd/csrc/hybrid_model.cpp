@@ -44,7 +44,10 @@ struct HybridModel : DecoderImpl {
     float *q = nullptr, *k = nullptr, *v = nullptr, *g = nullptr, *beta = nullptr, *gate_in = nullptr, *out = nullptr, *v_first = nullptr, *ssq = nullptr;
     float *part_o = nullptr, *part_ml = nullptr;
     float *y = nullptr, *ctx_f = nullptr, *act_f = nullptr;  // 32-bit mode
-    int *d_seg = nullptr, *h_seg = nullptr, n_seg = 0;       // first row, rows, slot of every segment of the chunk
+    int *d_seg = nullptr, *h_seg = nullptr, n_seg = 0;       // first row, rows, slot, first piece of every segment of the chunk
+    int *d_piece = nullptr, n_piece = 0, piece_cap = 0;      // first row, rows of every 16-token piece (staged behind h_seg)
+    float *pc_pair = nullptr, *pc_q = nullptr, *pc_w = nullptr, *pc_k = nullptr, *pc_decay = nullptr;
+    int opt_scan = 0;                                        // recurrences: token by token in prompt chunks too
     int opt_plain = 0;                                       // attention: the plain kernel instead of the matrix-core ones
 
     ~HybridModel() override;
@@ -60,8 +63,9 @@ struct HybridModel : DecoderImpl {
     int plan_chunk(nvllm_model* m, const int* pos, const int* slot, const int* seq, int R, const int* tile_row0, int n_tiles, int qt) override;
     int forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n_last, int logits_row0) override;
     int option(const char* name, int value) override {
-        if (strcmp(name, "bias_attn_plain")) return 1;
-        opt_plain = value;
+        if (!strcmp(name, "bias_attn_plain")) opt_plain = value;
+        else if (!strcmp(name, "recur_scan")) opt_scan = value;
+        else return 1;
         return 0;
     }
     int product(nvllm_model* m, const ProductPlan& p, const float* f, const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int R, int* ns) {
@@ -216,14 +220,15 @@ void HybridModel::free_kv() {
         w.kc = w.vc = nullptr;
         w.state = w.history = nullptr;
     }
-    for (float** p : {&q, &k, &v, &g, &beta, &gate_in, &out, &v_first, &ssq, &part_o, &part_ml, &y, &ctx_f, &act_f}) {
+    for (float** p : {&q, &k, &v, &g, &beta, &gate_in, &out, &v_first, &ssq, &part_o, &part_ml, &y, &ctx_f, &act_f, &pc_pair, &pc_q, &pc_w, &pc_k, &pc_decay}) {
         if (*p) (void)hipFree(*p);
         *p = nullptr;
     }
     if (d_seg) (void)hipFree(d_seg);
     if (h_seg) (void)hipHostFree(h_seg);
-    d_seg = h_seg = nullptr;
-    n_seg = 0;
+    if (d_piece) (void)hipFree(d_piece);
+    d_seg = h_seg = d_piece = nullptr;
+    n_seg = n_piece = 0;
 }
 
 HybridModel::~HybridModel() {
@@ -485,8 +490,19 @@ int HybridModel::kv_alloc(nvllm_model* m) {
         for (bf16_bits** p : {&m->ctxh, &m->ctxl}) if (!rc) rc = zalloc((void**)p, R16 * kc * 2);
         if (ffp) for (bf16_bits** p : {&m->xh2, &m->xl2}) if (!rc) rc = zalloc((void**)p, R16 * ffp * 2);
     }
-    if (!rc) rc = dmalloc(ctx, &d_seg, (size_t)3 * m->max_seqs);
-    if (!rc) HIPCHK(ctx, hipHostMalloc((void**)&h_seg, (size_t)3 * m->max_seqs * sizeof(int), hipHostMallocDefault));
+    piece_cap = (int)(R / kPiece) + m->max_seqs;
+    size_t ph = 0, pd = 0, pdd = 0;  // heads, channels of the layers that run in pieces, channels of the delta rule's
+    for (const HybridLayer& w : layers)
+        if (!w.attention() && piece_scan_ok(w.dim_p)) {
+            ph = std::max<size_t>(ph, w.heads);
+            if (w.delta()) pdd = std::max<size_t>(pdd, (size_t)w.heads * w.dim_p);
+        }
+    pd = pdd * kPiece;
+    struct { float** p; size_t n; } pieces[] = {{&pc_pair, ph * kPiece * kPiece}, {&pc_q, pd}, {&pc_w, pd}, {&pc_k, pd}, {&pc_decay, pdd}};
+    for (auto& b : pieces) if (!rc && b.n) rc = dmalloc(ctx, b.p, (size_t)piece_cap * b.n);
+    if (!rc) rc = dmalloc(ctx, &d_seg, (size_t)4 * m->max_seqs + 1);
+    if (!rc) rc = dmalloc(ctx, &d_piece, (size_t)2 * piece_cap);
+    if (!rc) HIPCHK(ctx, hipHostMalloc((void**)&h_seg, ((size_t)4 * m->max_seqs + 1 + 2 * piece_cap) * sizeof(int), hipHostMallocDefault));
     m->rope_len = (int)std::min<int64_t>((int64_t)m->max_blocks * kBlockTokens, 1 << 20);  // positions a block table covers
     return rc;
 }
@@ -496,17 +512,22 @@ int HybridModel::kv_alloc(nvllm_model* m) {
 // ---------------------------------------------------------------------------------------------------
 int HybridModel::plan_chunk(nvllm_model* m, const int*, const int* slot, const int* seq, int R, const int*, int, int qt) {
     nvllm_ctx* ctx = m->ctx;
-    n_seg = 0;
+    n_seg = n_piece = 0;
     if (qt == 1) return NVLLM_OK;
     const int cap = m->max_seqs;
+    int *h_piece0 = h_seg + 3 * cap, *h_row0 = h_seg + 4 * cap + 1, *h_n = h_row0 + piece_cap;
     for (int r = 0; r < R; ++n_seg) {
         int e = r;
         while (e < R && seq[e] == seq[r]) ++e;
         h_seg[n_seg] = r; h_seg[cap + n_seg] = e - r; h_seg[2 * cap + n_seg] = slot[r];
+        h_piece0[n_seg] = n_piece;
+        for (; r < e; r += kPiece, ++n_piece) { h_row0[n_piece] = r; h_n[n_piece] = std::min(kPiece, e - r); }
         r = e;
     }
+    h_piece0[n_seg] = n_piece;
     // the staging buffer is free: the tile upload before this call waited for the stream
-    HIPCHK(ctx, hipMemcpyAsync(d_seg, h_seg, (size_t)3 * cap * sizeof(int), hipMemcpyHostToDevice, ctx->stream));
+    HIPCHK(ctx, hipMemcpyAsync(d_seg, h_seg, ((size_t)4 * cap + 1) * sizeof(int), hipMemcpyHostToDevice, ctx->stream));
+    HIPCHK(ctx, hipMemcpyAsync(d_piece, h_row0, (size_t)2 * piece_cap * sizeof(int), hipMemcpyHostToDevice, ctx->stream));
     return NVLLM_OK;
 }
 
@@ -597,7 +618,15 @@ int HybridModel::recurrence(nvllm_model* m, HybridLayer& w, int ns, int R, int q
         PROF(m, PROF_RECUR, launch_recurrence(rc, &gn, s));
         return NVLLM_OK;
     }
-    PROF(m, PROF_RECUR, launch_recurrence(rc, nullptr, s));
+    // in pieces of 16 tokens unless most of them would be padding
+    if (!seg.single && !opt_scan && piece_scan_ok(w.dim_p) && R >= 4 * n_seg && n_piece <= 65535) {
+        PieceArgs pc;
+        pc.row0 = d_piece; pc.n = d_piece + piece_cap; pc.seg_piece0 = d_seg + 3 * m->max_seqs; pc.count = n_piece;
+        pc.pair = pc_pair; pc.qt = pc_q; pc.wt = pc_w; pc.kt = pc_k; pc.decay = pc_decay;
+        PROF(m, PROF_RECUR, launch_piece_scan(rc, pc, s));
+    } else {
+        PROF(m, PROF_RECUR, launch_recurrence(rc, nullptr, s));
+    }
     if (gn.whole && ctx->tp_size > 1) {  // the norm runs over every rank's heads (padding columns are zero)
         const int n = w.heads * w.vdim_p, c0[2] = {0, 0}, nn[2] = {n, 0};
         HIPCHK(ctx, launch_rows_ssq(out, 1, 0, n, nullptr, c0, nn, R, ssq, s));

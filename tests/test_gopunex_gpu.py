@@ -173,6 +173,25 @@ def test_state_carries_far(dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["mixed", "even", "wide", "state"])
+def test_recurrences_token_by_token_and_in_pieces(name, dtype):
+    # prompt portions in pieces of 16 tokens and by the scan, each continuing from the state the other left
+    cfg = CONFIGS[name]
+    w = sharp_weights(cfg, 17)
+    toks = tokens(260, cfg["vocab"], 3)
+    ref = G.forward(cfg, w, toks)
+    m = make(cfg, w, dtype)
+    for sid, scans in enumerate(([1] * 6, [0] * 6, [0, 1, 0, 1, 0, 1])):
+        at, got = 0, []
+        for n, scan in zip((17, 64, 33, 5, 80, 61), scans):
+            m.set_option("recur_scan", scan)
+            got.append(m.step_score([sid], [toks[:at + n]], False, [list(range(at, at + n))]))
+            at += n
+        assert at == 260 and row_err(np.concatenate(got), ref) < TOL[dtype], scans
+        m.seq_free(sid)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 def test_decays_of_every_strength(dtype):
     # rates from exp(-12) to exp(6) and strongly varying step sizes: decays that underflow within a token beside some that never do
     cfg = config([delta(heads=8, kv=4, dim=32, vdim=32, ff=0)], vocab=60)
