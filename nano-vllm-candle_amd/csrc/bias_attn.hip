@@ -369,22 +369,23 @@ hipError_t launch_bias_decode(const BiasAttnArgs& a, int rows, int parts, hipStr
 }
 
 // ---------------------------------------------------------------------------------------------------
-// prompt chunks: one workgroup = 128 (token, head of the group) rows of one sequence; four waves of two 16-row tiles share the
+// prompt chunks: one workgroup = 128 (token, head of the group) rows of one sequence (64 for the widest heads, whose accumulators
+// would not stay in registers: a fragment spilled while its read is in flight would be lost); four waves of MT 16-row tiles share the
 // 32-token K and V tiles, copied straight into LDS (two buffers, the next tile in flight)
 // ---------------------------------------------------------------------------------------------------
-template <int DC, int VC>
+template <int DC, int VC, int MT>
 __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, int bias_lds) {
-    constexpr int MT = 2, F = 2 * DC + VC, NL = (F + 3) / 4;  // fragments per tile, per wave
+    constexpr int RW = 64 * MT, F = 2 * DC + VC, NL = (F + 3) / 4;  // fragments per tile, per wave
     __shared__ __attribute__((aligned(16))) uint4 buf[2][F * 64];
     extern __shared__ float tab[];  // [gqa][n_bias] when bias_lds
     const int lane = threadIdx.x & 63, l15 = lane & 15, grp = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int tile = a.tile_order ? a.tile_order[blockIdx.x] : blockIdx.x;
-    const int gqa = a.heads / a.kv.kv, kvh = blockIdx.y / gqa, f0 = (blockIdx.y % gqa) * 128;
+    const int gqa = a.heads / a.kv.kv, per = gqa * (kBiasTileRows / RW), kvh = blockIdx.y / per, f0 = (blockIdx.y % per) * RW;
     const int row0 = a.tile_row0[tile], total = a.tile_nrows[tile] * gqa, slot = a.tile_slot[tile];
     if (f0 >= total) return;
     const int pos0 = a.pos[row0];
-    const int pmin = pos0 + f0 / gqa, pmax = pos0 + min(f0 + 127, total - 1) / gqa;
+    const int pmin = pos0 + f0 / gqa, pmax = pos0 + min(f0 + RW - 1, total - 1) / gqa;
     const int nt = (pmax >> 5) + 1;
     const int* bt = a.block_tables + (size_t)slot * a.max_blocks;
     const _Float16* kd = reinterpret_cast<const _Float16*>(a.kv.k);
@@ -434,27 +435,54 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
         for (int d = 0; d < VC; ++d) o[u][d] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
     dma_publish_barrier();
+    const uint32_t tab0 = lds_address(tab);
     for (int t = 0; t < nt; ++t) {
-        const uint4* b = buf[t & 1];
+        const uint32_t b = lds_address(buf[t & 1]) + lane * 16;
         if (t + 1 < nt) stage(t + 1, buf[(t + 1) & 1]);  // its last readers have passed the barrier of the previous tile
         const int tokA = (t << 5) + grp * 4, tokB = tokA + 16;
         f32x4 sa[MT], sb[MT];
+        constexpr int KG = DC < 4 ? DC : 4;  // chunks of K in flight
+        f16x8 ka[KG], kb[KG];
+        auto read_k = [&](int c0) {
+#pragma unroll
+            for (int c = 0; c < KG; ++c)
+                if (c0 + c < DC) {
+                    NVLLM_LDS_READ128(ka[c], b + c0 * 1024, c * 1024);
+                    NVLLM_LDS_READ128(kb[c], b + c0 * 1024, (DC + c) * 1024);
+                }
+        };
         if (a.n_bias && pmin - (t << 5) - 31 < far) {  // some distance below the last bucket
 #pragma unroll
             for (int u = 0; u < MT; ++u)
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     const int na = max(0, min(my_pos[u] - tokA - r, far)), nb = max(0, min(my_pos[u] - tokB - r, far));
-                    sa[u][r] = bias_lds ? tab[hd[u] * a.n_bias + na] : bias[u][na];
-                    sb[u][r] = bias_lds ? tab[hd[u] * a.n_bias + nb] : bias[u][nb];
+                    float xa, xb;
+                    if (bias_lds) {
+                        NVLLM_LDS_READ32(xa, tab0 + (uint32_t)(hd[u] * a.n_bias + na) * 4u);
+                        NVLLM_LDS_READ32(xb, tab0 + (uint32_t)(hd[u] * a.n_bias + nb) * 4u);
+                    } else {
+                        xa = bias[u][na];
+                        xb = bias[u][nb];
+                    }
+                    sa[u][r] = xa;
+                    sb[u][r] = xb;
                 }
+            read_k(0);
+            NVLLM_LDS_WAIT(2 * KG - 2);
         } else {
+            read_k(0);
 #pragma unroll
             for (int u = 0; u < MT; ++u) sa[u] = sb[u] = f32x4{b_far[u], b_far[u], b_far[u], b_far[u]};
+            NVLLM_LDS_WAIT(2 * KG - 2);
         }
 #pragma unroll
         for (int c = 0; c < DC; ++c) {
-            const f16x8 fa = __builtin_bit_cast(f16x8, b[c * 64 + lane]), fb = __builtin_bit_cast(f16x8, b[(DC + c) * 64 + lane]);
+            if (c % KG == 0 && c) { read_k(c); NVLLM_LDS_WAIT(2 * KG - 2); }
+            if (c % KG == 1) NVLLM_LDS_WAIT(KG > 2 ? 2 * KG - 4 : 0);
+            if (c % KG == 2) NVLLM_LDS_WAIT(KG > 3 ? 2 * KG - 6 : 0);
+            if (c % KG == 3) NVLLM_LDS_WAIT(0);
+            const f16x8 fa = ka[c % KG], fb = kb[c % KG];
 #pragma unroll
             for (int u = 0; u < MT; ++u) {
                 sa[u] = __builtin_amdgcn_mfma_f32_16x16x32_f16(fa, qh[u][c], sa[u], 0, 0, 0);
@@ -462,7 +490,15 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
                 sa[u] = __builtin_amdgcn_mfma_f32_16x16x32_f16(fa, ql[u][c], sa[u], 0, 0, 0);
                 sb[u] = __builtin_amdgcn_mfma_f32_16x16x32_f16(fb, ql[u][c], sb[u], 0, 0, 0);
             }
+            __builtin_amdgcn_sched_barrier(0);
         }
+        constexpr int VG = VC < 8 ? VC : 8;  // value tiles in flight
+        f16x8 vf[VG];
+        auto read_v = [&](int d0) {
+#pragma unroll
+            for (int d = 0; d < VG; ++d) NVLLM_LDS_READ128(vf[d], b + d0 * 1024, (2 * DC + d) * 1024);
+        };
+        read_v(0);
         const bool edge = (t << 5) + 31 > pmin;  // some row does not see the whole tile
         f16x8 P[MT], Pl[MT];
 #pragma unroll
@@ -496,13 +532,19 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
             }
         }
 #pragma unroll
-        for (int d = 0; d < VC; ++d) {
-            const f16x8 v = __builtin_bit_cast(f16x8, b[(2 * DC + d) * 64 + lane]);
+        for (int d0 = 0; d0 < VC; d0 += VG) {
+            if (d0) read_v(d0);
 #pragma unroll
-            for (int u = 0; u < MT; ++u) {
-                o[u][d] = __builtin_amdgcn_mfma_f32_16x16x32_f16(v, P[u], o[u][d], 0, 0, 0);
-                o[u][d] = __builtin_amdgcn_mfma_f32_16x16x32_f16(v, Pl[u], o[u][d], 0, 0, 0);
+            for (int d = 0; d < VG; ++d) {
+                if (d == 0) NVLLM_LDS_WAIT(VG / 2);
+                if (d == VG / 2) NVLLM_LDS_WAIT(0);
+#pragma unroll
+                for (int u = 0; u < MT; ++u) {
+                    o[u][d0 + d] = __builtin_amdgcn_mfma_f32_16x16x32_f16(vf[d], P[u], o[u][d0 + d], 0, 0, 0);
+                    o[u][d0 + d] = __builtin_amdgcn_mfma_f32_16x16x32_f16(vf[d], Pl[u], o[u][d0 + d], 0, 0, 0);
+                }
             }
+            __builtin_amdgcn_sched_barrier(0);
         }
         dma_publish_barrier();
     }
@@ -530,14 +572,15 @@ hipError_t launch_bias_prefill(const BiasAttnArgs& a, int n_tiles, hipStream_t s
     const int gqa = a.heads / a.kv.kv;
     const int bias_lds = a.n_bias && (size_t)gqa * a.n_bias <= 6144;
     const size_t lds = bias_lds ? (size_t)gqa * a.n_bias * 4 : 0;
-    const dim3 grid(n_tiles, a.kv.kv * gqa * (kBiasTileRows / 128));
 #define NVLLM_BA_P(K_, V_)                                                                                           \
     {                                                                                                                \
+        constexpr int MT_ = K_ > 4 || V_ > 8 ? 1 : 2;                                                                \
+        const dim3 grid(n_tiles, a.kv.kv * gqa * (kBiasTileRows / (64 * MT_)));                                      \
         if (lds + 2 * (2 * K_ + V_) * 1024 > 64 * 1024) {                                                            \
             static std::atomic<uint64_t> done{0};                                                                    \
-            ensure_dyn_lds(reinterpret_cast<const void*>(bias_prefill_kernel<K_, V_>), 24 * 1024, done);             \
+            ensure_dyn_lds(reinterpret_cast<const void*>(bias_prefill_kernel<K_, V_, MT_>), 24 * 1024, done);             \
         }                                                                                                            \
-        bias_prefill_kernel<K_, V_><<<grid, 256, lds, s>>>(a, bias_lds);                                             \
+        bias_prefill_kernel<K_, V_, MT_><<<grid, 256, lds, s>>>(a, bias_lds);                                             \
     }
     NVLLM_BA(NVLLM_BA_P)
 #undef NVLLM_BA_P

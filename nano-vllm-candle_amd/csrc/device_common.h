@@ -81,6 +81,21 @@ __device__ __forceinline__ float wave_sum(float v) {
     return v;
 }
 
+// sum over the 16 lanes of a DPP row, in every lane
+__device__ __forceinline__ float row16_sum(float v) {
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x128, 0xf, 0xf, false));  // row_ror:8
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x124, 0xf, 0xf, false));  // row_ror:4
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x122, 0xf, 0xf, false));  // row_ror:2
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x121, 0xf, 0xf, false));  // row_ror:1
+    return v;
+}
+// sum over the wave without LDS traffic, as a uniform value
+__device__ __forceinline__ float wave_sum_uniform(float v) {
+    const int x = __builtin_bit_cast(int, row16_sum(v));
+    return (__builtin_bit_cast(float, __builtin_amdgcn_readlane(x, 0)) + __builtin_bit_cast(float, __builtin_amdgcn_readlane(x, 16))) +
+           (__builtin_bit_cast(float, __builtin_amdgcn_readlane(x, 32)) + __builtin_bit_cast(float, __builtin_amdgcn_readlane(x, 48)));
+}
+
 // rinv[row] of a deferred RMSNorm (see RowNorm); 1 when the activations were normalised by the producer
 __device__ __forceinline__ float rownorm_rinv(const RowNorm& rn, int row) {
     if (!rn.ssq) return 1.0f;
@@ -289,6 +304,18 @@ typedef __attribute__((address_space(3))) void* lptr_t;
 #else
 #define NVLLM_STAMP(args_, idx_) do { } while (0)
 #endif
+
+// LDS reads beside an LDS-DMA in flight: hipcc waits for every outstanding global_load_lds before an ordinary LDS read (it cannot
+// tell the buffers apart), which serialises the copy with the compute it should hide behind.  These reads are inline asm with counted
+// waits: LDS returns in order, so LDS_WAIT(n) leaves at most the n youngest outstanding (anything else in flight only makes it wait longer).
+#define NVLLM_LDS_READ128(DST_, ADDR_, OFF_) asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(DST_) : "v"(ADDR_), "n"(OFF_))
+#define NVLLM_LDS_READ32(DST_, ADDR_) asm volatile("ds_read_b32 %0, %1" : "=v"(DST_) : "v"(ADDR_))
+#define NVLLM_LDS_WAIT(N_)                                             \
+    do {                                                               \
+        asm volatile("s_waitcnt lgkmcnt(%0)" ::"n"(N_) : "memory");    \
+        __builtin_amdgcn_sched_barrier(0);                             \
+    } while (0)
+__device__ __forceinline__ uint32_t lds_address(const void* p) { return (uint32_t)(uintptr_t)(lptr_t)p; }
 
 // Barrier that PUBLISHES LDS-DMA data (global_load_lds): every wave first waits for its own DMA to land, then joins the
 // barrier; only then may any wave ds_read fragments another wave staged.  __syncthreads() alone is not enough: hipcc

@@ -1,7 +1,7 @@
 // Decoders whose layers mix tokens by recurrence or by attention with a distance bias (hybrid_model.cpp): launchers of
 // hybrid_ops.hip (row kernels), recurrent.hip (carried-state scans) and bias_attn.hip (grouped-query attention).
 #pragma once
-#include "kernels.h"
+#include "latent.h"
 
 namespace nvllm {
 
@@ -135,16 +135,16 @@ constexpr int kPiece = 16;
 struct PieceArgs {
     const int* row0 = nullptr;       // first row and number of rows of every piece
     const int* n = nullptr;
-    const int* seg_piece0 = nullptr; // [segments + 1] first piece of every segment
+    const int* seg_piece0 = nullptr; // first piece of every segment
     int count = 0;
-    float* pair = nullptr;           // scratch per (piece, head): [16][16]
+    float* pair = nullptr;           // scratch per (piece, head): [16][16] decayed products of queries and keys,
+    float* kt = nullptr;             // [dim_p][16] keys decayed to the piece's end;
     float* qt = nullptr;             // delta rule: [16][dim_p] decayed queries,
     float* wt = nullptr;             // [16][dim_p] solved keys,
-    float* kt = nullptr;             // [dim_p][16] keys decayed to the piece's end,
     float* decay = nullptr;          // [dim_p] decays of the whole piece
 };
 bool piece_scan_ok(int dim_p);
-// v is overwritten for the delta rule
+// q, k and v hold kPiece more rows than the chunk (anything finite); v is overwritten for the delta rule
 hipError_t launch_piece_scan(const RecurArgs& a, const PieceArgs& c, hipStream_t s);
 
 // rows after the q / k / v / gate projection of the constant-decay recurrence: silu(q, k, v), sigmoid(gate)
@@ -184,6 +184,8 @@ struct DeltaRowsArgs {
 };
 constexpr float kUnitNormEps = 1e-6f;
 hipError_t launch_delta_rows(const DeltaRowsArgs& a, int rows, hipStream_t s);
+// gate_in -> decays and output gates (HeadGemmArgs with decay_rate set)
+hipError_t launch_delta_gates(const HeadGemmArgs& a, hipStream_t s);
 // the history half of it for chunks with longer segments (after launch_delta_rows)
 hipError_t launch_delta_history(const DeltaRowsArgs& a, hipStream_t s);
 

@@ -476,7 +476,7 @@ int HybridModel::kv_alloc(nvllm_model* m) {
     if (!rc) rc = dmalloc(ctx, &m->slabs, m->slab_floats);
     if (!rc) rc = dmalloc(ctx, &m->red, R * ldr);
     struct { float** p; size_t n; } bufs[] = {{&q, nq}, {&k, nk}, {&v, nv}, {&g, ng}, {&beta, nb}, {&gate_in, nin}, {&out, no}, {&v_first, nvf}};
-    for (auto& b : bufs) if (!rc && b.n) rc = zalloc((void**)b.p, R * b.n * 4);
+    for (auto& b : bufs) if (!rc && b.n) rc = zalloc((void**)b.p, (R + kPiece) * b.n * 4);  // pieces read past the last row
     if (!rc) rc = dmalloc(ctx, &ssq, R * 2);
     if (!rc && po && !f32) rc = dmalloc(ctx, &part_o, po);
     if (!rc && pm && !f32) rc = dmalloc(ctx, &part_ml, pm);
@@ -491,18 +491,18 @@ int HybridModel::kv_alloc(nvllm_model* m) {
         if (ffp) for (bf16_bits** p : {&m->xh2, &m->xl2}) if (!rc) rc = zalloc((void**)p, R16 * ffp * 2);
     }
     piece_cap = (int)(R / kPiece) + m->max_seqs;
-    size_t ph = 0, pd = 0, pdd = 0;  // heads, channels of the layers that run in pieces, channels of the delta rule's
+    size_t ph = 0, pd = 0, pdd = 0;  // heads, channels of the layers that run in pieces, channels of the delta rule's alone
     for (const HybridLayer& w : layers)
         if (!w.attention() && piece_scan_ok(w.dim_p)) {
             ph = std::max<size_t>(ph, w.heads);
+            pd = std::max<size_t>(pd, (size_t)w.heads * w.dim_p);
             if (w.delta()) pdd = std::max<size_t>(pdd, (size_t)w.heads * w.dim_p);
         }
-    pd = pdd * kPiece;
-    struct { float** p; size_t n; } pieces[] = {{&pc_pair, ph * kPiece * kPiece}, {&pc_q, pd}, {&pc_w, pd}, {&pc_k, pd}, {&pc_decay, pdd}};
+    struct { float** p; size_t n; } pieces[] = {{&pc_pair, ph * kPiece * kPiece}, {&pc_k, pd * kPiece}, {&pc_q, pdd * kPiece}, {&pc_w, pdd * kPiece}, {&pc_decay, pdd}};
     for (auto& b : pieces) if (!rc && b.n) rc = dmalloc(ctx, b.p, (size_t)piece_cap * b.n);
-    if (!rc) rc = dmalloc(ctx, &d_seg, (size_t)4 * m->max_seqs + 1);
+    if (!rc) rc = dmalloc(ctx, &d_seg, (size_t)4 * m->max_seqs);
     if (!rc) rc = dmalloc(ctx, &d_piece, (size_t)2 * piece_cap);
-    if (!rc) HIPCHK(ctx, hipHostMalloc((void**)&h_seg, ((size_t)4 * m->max_seqs + 1 + 2 * piece_cap) * sizeof(int), hipHostMallocDefault));
+    if (!rc) HIPCHK(ctx, hipHostMalloc((void**)&h_seg, ((size_t)4 * m->max_seqs + 2 * piece_cap) * sizeof(int), hipHostMallocDefault));
     m->rope_len = (int)std::min<int64_t>((int64_t)m->max_blocks * kBlockTokens, 1 << 20);  // positions a block table covers
     return rc;
 }
@@ -515,7 +515,7 @@ int HybridModel::plan_chunk(nvllm_model* m, const int*, const int* slot, const i
     n_seg = n_piece = 0;
     if (qt == 1) return NVLLM_OK;
     const int cap = m->max_seqs;
-    int *h_piece0 = h_seg + 3 * cap, *h_row0 = h_seg + 4 * cap + 1, *h_n = h_row0 + piece_cap;
+    int *h_piece0 = h_seg + 3 * cap, *h_row0 = h_seg + 4 * cap, *h_n = h_row0 + piece_cap;
     for (int r = 0; r < R; ++n_seg) {
         int e = r;
         while (e < R && seq[e] == seq[r]) ++e;
@@ -524,9 +524,8 @@ int HybridModel::plan_chunk(nvllm_model* m, const int*, const int* slot, const i
         for (; r < e; r += kPiece, ++n_piece) { h_row0[n_piece] = r; h_n[n_piece] = std::min(kPiece, e - r); }
         r = e;
     }
-    h_piece0[n_seg] = n_piece;
     // the staging buffer is free: the tile upload before this call waited for the stream
-    HIPCHK(ctx, hipMemcpyAsync(d_seg, h_seg, ((size_t)4 * cap + 1) * sizeof(int), hipMemcpyHostToDevice, ctx->stream));
+    HIPCHK(ctx, hipMemcpyAsync(d_seg, h_seg, (size_t)4 * cap * sizeof(int), hipMemcpyHostToDevice, ctx->stream));
     HIPCHK(ctx, hipMemcpyAsync(d_piece, h_row0, (size_t)2 * piece_cap * sizeof(int), hipMemcpyHostToDevice, ctx->stream));
     return NVLLM_OK;
 }
@@ -601,7 +600,7 @@ int HybridModel::recurrence(nvllm_model* m, HybridLayer& w, int ns, int R, int q
         ga.x = gate_in; ga.x_row = 2 * w.rank_p; ga.x_head = w.rank_p;
         ga.w = w.gates.data; ga.w_head = (int64_t)w.Ng * w.rank_p / 8; ga.N = ga.n_valid = w.Ng; ga.K = w.rank_p; ga.heads = 2; ga.M = R; ga.exact = cfg.f32;
         ga.y = g; ga.y_row = 2 * w.Ng; ga.y_head = w.Ng; ga.decay_rate = w.rate; ga.decay_bias = w.dt;
-        PROF(m, PROF_GEMM, launch_head_gemm(ga, s));
+        PROF(m, PROF_GEMM, launch_delta_gates(ga, s));
         rc.g = g; rc.g_row = 2 * w.Ng; rc.beta = beta;
         gn.gate = g + w.Ng; gn.gate_row = 2 * w.Ng;
     } else {

@@ -232,10 +232,91 @@ __global__ void __launch_bounds__(256) delta_rows_kernel(DeltaRowsArgs a) {
     for (int d = lane; d < n; d += 64)
         for (int i = 0; i < a.taps - 1; ++i) next[(size_t)i * channels + c0 + d] = past_input(a, p, row, a.taps - 2 - i, c0 + d, channels);
 }
+// prompt chunks: one wave per (16 rows, unit), the convolution's window in registers
+template <int TAPS, int NE>
+__global__ void __launch_bounds__(256) delta_rows16_kernel(DeltaRowsArgs a, int rows) {
+    const int lane = threadIdx.x & 63, unit = blockIdx.y * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int row0 = blockIdx.x * 16, row1 = min(row0 + 16, rows);
+    const int channels = 2 * a.kv * a.dim + a.heads * a.vdim;
+    if (unit > 2 * a.kv + a.heads) return;
+    if (unit == 2 * a.kv + a.heads) {
+        const int per = a.heads + 2 * a.rank_p;
+        for (int i = lane; i < (row1 - row0) * per; i += 64) {
+            const int row = row0 + i / per, c = i % per;
+            const float x = slab_elem(a.in + (size_t)row * a.ld + channels + c, a.n_slabs, a.slab_stride);
+            if (c < a.heads) a.beta[(size_t)row * a.heads + c] = sigmoidf(x);
+            else a.gate_in[(size_t)row * 2 * a.rank_p + c - a.heads] = x;
+        }
+        return;
+    }
+    const bool qk = unit < 2 * a.kv;
+    const int n = qk ? a.dim : a.vdim, n_p = qk ? a.dim_p : a.vdim_p;
+    const int c0 = qk ? unit * a.dim : 2 * a.kv * a.dim + (unit - 2 * a.kv) * a.vdim;
+    const int hd = qk ? unit % a.kv : unit - 2 * a.kv, hs = qk ? a.kv : a.heads;
+    float* out = (qk ? (unit < a.kv ? a.q : a.k) : a.v) + (size_t)hd * n_p;
+    const float unit_scale = unit < a.kv ? a.q_scale : 1.f;
+    for (int d0 = 0; d0 < n_p; d0 += 64 * NE) {  // once for q and k (dim_p = 64 NE): their norm needs the whole head
+        float w[TAPS][NE], x[TAPS][NE];
+#pragma unroll
+        for (int e = 0; e < NE; ++e) {
+            const int d = d0 + e * 64 + lane;
+#pragma unroll
+            for (int i = 0; i < TAPS; ++i) w[i][e] = d < n ? a.conv[(size_t)i * channels + c0 + d] : 0.f;
+        }
+        for (int row = row0; row < row1; ++row) {
+            const int slot = a.slot[row];
+            const bool start = row == 0 || a.slot[row - 1] != slot;
+            if (row == row0 || start) {
+                const RowPast p = row_past(a, row);
+#pragma unroll
+                for (int j = 1; j < TAPS; ++j)
+#pragma unroll
+                    for (int e = 0; e < NE; ++e) {
+                        const int d = d0 + e * 64 + lane;
+                        x[TAPS - 1 - j][e] = d < n ? past_input(a, p, row, j, c0 + d, channels) : 0.f;
+                    }
+            } else {
+#pragma unroll
+                for (int i = 0; i < TAPS - 1; ++i)
+#pragma unroll
+                    for (int e = 0; e < NE; ++e) x[i][e] = x[i + 1][e];
+            }
+            const float* in = a.in + (size_t)row * a.ld + c0;
+            float y[NE], ss = 0.f;
+#pragma unroll
+            for (int e = 0; e < NE; ++e) {
+                const int d = d0 + e * 64 + lane;
+                x[TAPS - 1][e] = d < n ? slab_elem(in + d, a.n_slabs, a.slab_stride) : 0.f;
+                float t = 0.f;
+#pragma unroll
+                for (int i = 0; i < TAPS; ++i) t += x[i][e] * w[i][e];
+                y[e] = t * sigmoidf(t);
+                ss += y[e] * y[e];
+            }
+            const float f = qk ? unit_scale / sqrtf(wave_sum_uniform(ss) + kUnitNormEps) : 1.f;
+#pragma unroll
+            for (int e = 0; e < NE; ++e)
+                if (d0 + e * 64 + lane < n_p) out[(size_t)row * hs * n_p + d0 + e * 64 + lane] = y[e] * f;
+        }
+    }
+}
+template <int NE>
+static bool delta_rows16(const DeltaRowsArgs& a, int rows, hipStream_t s) {
+    const dim3 grid((rows + 15) / 16, (2 * a.kv + a.heads + 1 + 3) / 4);
+    if (a.taps == 4) delta_rows16_kernel<4, NE><<<grid, 256, 0, s>>>(a, rows);
+    else if (a.taps == 3) delta_rows16_kernel<3, NE><<<grid, 256, 0, s>>>(a, rows);
+    else if (a.taps == 2) delta_rows16_kernel<2, NE><<<grid, 256, 0, s>>>(a, rows);
+    else return false;
+    return true;
+}
 hipError_t launch_delta_rows(const DeltaRowsArgs& a, int rows, hipStream_t s) {
-    if (a.dim_p % 4 || a.vdim_p % 4 || a.taps < 1 || 2 * a.kv * a.dim + a.heads * (a.vdim + 1) + 2 * a.rank_p > a.ld) return hipErrorInvalidValue;
+    if (a.dim_p % 64 || a.vdim_p % 4 || a.taps < 1 || 2 * a.kv * a.dim + a.heads * (a.vdim + 1) + 2 * a.rank_p > a.ld) return hipErrorInvalidValue;
     if (a.dim_p > 512) return hipErrorNotSupported;
     if (rows <= 0) return hipSuccess;
+    if (!a.seg.single && rows >= 64) {
+        const bool done = a.dim_p == 64 ? delta_rows16<1>(a, rows, s) : a.dim_p == 128 ? delta_rows16<2>(a, rows, s) : a.dim_p == 256 ? delta_rows16<4>(a, rows, s) : false;
+        if (done) return hipGetLastError();
+    }
     const dim3 grid(rows, (2 * a.kv + a.heads + 1 + 3) / 4);
     if (a.dim_p <= 64) delta_rows_kernel<1><<<grid, 256, 0, s>>>(a);
     else if (a.dim_p <= 128) delta_rows_kernel<2><<<grid, 256, 0, s>>>(a);
@@ -273,6 +354,78 @@ hipError_t launch_delta_history(const DeltaRowsArgs& a, hipStream_t s) {
 }
 
 // ---------------------------------------------------------------------------------------------------
+// second step of the gate projections over prompt chunks: one workgroup = 64 rows x a slice of one gate's features; the rows' operand
+// is built once in LDS as bf16 hi + lo fragments, each wave streams its share of the weight fragments
+// ---------------------------------------------------------------------------------------------------
+template <int KT>
+__global__ void __launch_bounds__(256) delta_gates_kernel(HeadGemmArgs a) {
+    __shared__ __attribute__((aligned(16))) uint4 xs[2 * 4 * KT * 64];  // [plane][row tile][k-tile][lane]
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, grp = lane >> 4;
+    const int row0 = blockIdx.x * 64, head = blockIdx.y;
+    for (int i = wave; i < 4 * KT; i += 4) {
+        const int row = min(row0 + (i / KT) * 16 + l15, a.M - 1);
+        const float* p = a.x + (size_t)row * a.x_row + (size_t)head * a.x_head + (i % KT) * 32 + grp * 8;
+        float x[8];
+        *reinterpret_cast<float4*>(&x[0]) = *reinterpret_cast<const float4*>(p);
+        *reinterpret_cast<float4*>(&x[4]) = *reinterpret_cast<const float4*>(p + 4);
+        bf16x8 h, l;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            h[j] = (__bf16)x[j];
+            l[j] = (__bf16)(x[j] - (float)h[j]);
+        }
+        xs[i * 64 + lane] = __builtin_bit_cast(uint4, h);
+        xs[(4 * KT + i) * 64 + lane] = __builtin_bit_cast(uint4, l);
+    }
+    __syncthreads();
+    const uint4* w = a.w + (size_t)head * a.w_head;
+    const int ntiles = a.N >> 4;
+    for (int nt = blockIdx.z * 4 + wave; nt < ntiles; nt += 4 * gridDim.z) {
+        uint4 wf[KT];
+#pragma unroll
+        for (int k = 0; k < KT; ++k) wf[k] = w[((size_t)nt * KT + k) * 64 + lane];
+        f32x4 acc[4];
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+            acc[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int k = 0; k < KT; ++k) {
+                const bf16x8 wv = __builtin_bit_cast(bf16x8, wf[k]);
+                acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv, __builtin_bit_cast(bf16x8, xs[(b * KT + k) * 64 + lane]), acc[b], 0, 0, 0);
+                acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv, __builtin_bit_cast(bf16x8, xs[((4 + b) * KT + k) * 64 + lane]), acc[b], 0, 0, 0);
+            }
+        }
+        const int f0 = nt * 16 + grp * 4;
+        float4 rate = make_float4(0.f, 0.f, 0.f, 0.f), dt = rate;
+        if (head == 0) {
+            rate = *reinterpret_cast<const float4*>(a.decay_rate + f0);
+            dt = *reinterpret_cast<const float4*>(a.decay_bias + f0);
+        }
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+            const int row = row0 + b * 16 + l15;
+            const f32x4 v = acc[b];
+            float4 o;
+            if (head == 0) o = make_float4(expf(-rate.x * softplusf(v[0] + dt.x)), expf(-rate.y * softplusf(v[1] + dt.y)),
+                                           expf(-rate.z * softplusf(v[2] + dt.z)), expf(-rate.w * softplusf(v[3] + dt.w)));
+            else o = make_float4(sigmoidf(v[0]), sigmoidf(v[1]), sigmoidf(v[2]), sigmoidf(v[3]));
+            if (row < a.M) *reinterpret_cast<float4*>(a.y + (size_t)row * a.y_row + (size_t)head * a.y_head + f0) = o;
+        }
+    }
+}
+hipError_t launch_delta_gates(const HeadGemmArgs& a, hipStream_t s) {
+    const int kt = a.K / 32;
+    if (a.exact || a.M < 512 || kt > 4 || a.N % 16 || a.K % 32 || a.x_row % 4 || a.x_head % 4 || a.y_row % 4 || a.y_head % 4 || a.n_valid != a.N || !a.decay_rate)
+        return launch_head_gemm(a, s);
+    const dim3 grid((a.M + 63) / 64, a.heads, std::max(1, std::min(8, a.N / 16 / 16)));
+    if (kt == 1) delta_gates_kernel<1><<<grid, 256, 0, s>>>(a);
+    else if (kt == 2) delta_gates_kernel<2><<<grid, 256, 0, s>>>(a);
+    else if (kt == 3) delta_gates_kernel<3><<<grid, 256, 0, s>>>(a);
+    else delta_gates_kernel<4><<<grid, 256, 0, s>>>(a);
+    return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------------------------------
 // gated output norm: one wave per (row, head), or one workgroup per row when the norm runs over all heads
 // ---------------------------------------------------------------------------------------------------
 template <bool WHOLE>
@@ -281,24 +434,50 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(GatedNormArgs a, int ro
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int row = WHOLE ? blockIdx.x : (blockIdx.x * 4 + wave) / a.heads, head0 = WHOLE ? 0 : (blockIdx.x * 4 + wave) % a.heads;
     if (row >= rows) return;  // WHOLE: one row per workgroup, never taken
-    const float* o = a.o + (size_t)row * a.heads * a.vdim_p;
-    const int n = WHOLE ? a.heads * a.vdim : a.vdim, t0 = WHOLE ? threadIdx.x : lane;
+    const float* o = a.o + ((size_t)row * a.heads + head0) * a.vdim_p;
+    const float* gate = a.gate + (size_t)row * a.gate_row + (size_t)head0 * a.gate_head;
     constexpr int step = WHOLE ? 256 : 64;
+    const int t0 = WHOLE ? threadIdx.x : lane;
+    const float n = WHOLE ? (float)a.all : (float)a.vdim;
+    if ((a.vdim & 3) == 0) {  // four values of one head per thread; padding columns of o are zero
+        const int n4 = WHOLE ? a.heads * (a.vdim_p >> 2) : a.vdim_p >> 2;
+        float ss = 0.f;
+        if (WHOLE && a.ssq) {
+            ss = a.ssq[row * 2];
+        } else {
+            for (int i = t0; i < n4; i += step) {
+                const float4 x = reinterpret_cast<const float4*>(o)[i];
+                ss += x.x * x.x + x.y * x.y + x.z * x.z + x.w * x.w;
+            }
+            ss = WHOLE ? block_sum(ss, red, 4) : wave_sum_uniform(ss);
+        }
+        const float rinv = 1.0f / sqrtf(ss / n + a.eps);
+        for (int i = t0; i < n4; i += step) {
+            const int h = WHOLE ? i * 4 / a.vdim_p : 0, e = i * 4 - h * a.vdim_p, col = (head0 + h) * a.vdim + e;
+            if (e >= a.vdim) continue;
+            const float4 x = reinterpret_cast<const float4*>(o)[i], g = *reinterpret_cast<const float4*>(gate + (size_t)h * a.gate_head + e);
+            const float4 w = *reinterpret_cast<const float4*>(a.weight + (WHOLE ? col : e));
+            const f32x4 v = {(x.x * rinv) * w.x * g.x, (x.y * rinv) * w.y * g.y, (x.z * rinv) * w.z * g.z, (x.w * rinv) * w.w * g.w};
+            if (a.of) *reinterpret_cast<float4*>(a.of + (size_t)row * a.ld + col) = make_float4(v[0], v[1], v[2], v[3]);
+            if (a.oh) put_planes4(a.oh, a.ol, row, col, 4, a.ld, a.packed, v);
+        }
+        return;
+    }
+    const int cnt = WHOLE ? a.heads * a.vdim : a.vdim;
     float ss = 0.f;
     if (WHOLE && a.ssq) {
         ss = a.ssq[row * 2];
     } else {
-        for (int i = t0; i < n; i += step) {
+        for (int i = t0; i < cnt; i += step) {
             const int h = WHOLE ? i / a.vdim : 0, e = i - h * a.vdim;
-            const float v = o[(head0 + h) * a.vdim_p + e];
+            const float v = o[h * a.vdim_p + e];
             ss += v * v;
         }
-        ss = WHOLE ? block_sum(ss, red, 4) : wave_sum(ss);
+        ss = WHOLE ? block_sum(ss, red, 4) : wave_sum_uniform(ss);
     }
-    const float rinv = 1.0f / sqrtf(ss / (float)(WHOLE ? a.all : n) + a.eps);
-    const float* gate = a.gate + (size_t)row * a.gate_row;
-    for (int i = t0; i < n; i += step) {
-        const int h = head0 + (WHOLE ? i / a.vdim : 0), e = WHOLE ? i - h * a.vdim : i, col = h * a.vdim + e;
+    const float rinv = 1.0f / sqrtf(ss / n + a.eps);
+    for (int i = t0; i < cnt; i += step) {
+        const int h = WHOLE ? i / a.vdim : 0, e = i - h * a.vdim, col = (head0 + h) * a.vdim + e;
         const float v = (o[h * a.vdim_p + e] * rinv) * a.weight[i] * gate[h * a.gate_head + e];
         if (a.of) a.of[(size_t)row * a.ld + col] = v;
         if (a.oh) {
@@ -308,7 +487,7 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(GatedNormArgs a, int ro
     }
 }
 hipError_t launch_gated_norm(const GatedNormArgs& a, int rows, hipStream_t s) {
-    if (a.heads * a.vdim > a.ld || (!a.oh && !a.of) || (a.whole && a.all < 1)) return hipErrorInvalidValue;
+    if (a.heads * a.vdim > a.ld || (!a.oh && !a.of) || (a.whole && a.all < 1) || a.vdim_p % 4 || a.gate_head % 4 || a.gate_row % 4) return hipErrorInvalidValue;
     if (rows <= 0) return hipSuccess;
     if (a.whole) gated_norm_kernel<true><<<rows, 256, 0, s>>>(a, rows);
     else gated_norm_kernel<false><<<(rows * a.heads + 3) / 4, 256, 0, s>>>(a, rows);

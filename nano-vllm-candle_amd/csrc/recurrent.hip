@@ -11,15 +11,6 @@
 
 namespace nvllm {
 
-// sum over the 16 lanes of a DPP row, in every lane
-__device__ __forceinline__ float row16_sum(float v) {
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x128, 0xf, 0xf, false));  // row_ror:8
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x124, 0xf, 0xf, false));  // row_ror:4
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x122, 0xf, 0xf, false));  // row_ror:2
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x121, 0xf, 0xf, false));  // row_ror:1
-    return v;
-}
-
 // one token on the wave's registers
 template <int R4, bool DELTA>
 __device__ __forceinline__ float2 recur_token(float (&S)[R4][2][4], const float4 (&k)[R4], const float4 (&q)[R4], const float4 (&g)[R4], float decay,

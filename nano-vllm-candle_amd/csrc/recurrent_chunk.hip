@@ -18,13 +18,6 @@
 
 namespace nvllm {
 
-__device__ __forceinline__ float row16_sum(float v) {
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x128, 0xf, 0xf, false));
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x124, 0xf, 0xf, false));
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x122, 0xf, 0xf, false));
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x121, 0xf, 0xf, false));
-    return v;
-}
 __device__ __forceinline__ int token_slot(int j) { return ((j & 3) << 2) | (j >> 2); }  // place of token j among a row's 16: lane group, register
 
 // ---------------------------------------------------------------------------------------------------
@@ -173,7 +166,7 @@ __global__ void __launch_bounds__(64) delta_pieces_kernel(RecurArgs a, PieceArgs
     }
 }
 
-// constant decays: decay^(i - j) q_i . k_j, j <= i; one wave per (piece, head)
+// constant decays: decay^(i - j) q_i . k_j (j <= i) and the keys decayed to the piece's end; one wave per (piece, head)
 template <int R4>
 __global__ void __launch_bounds__(64) linear_pieces_kernel(RecurArgs a, PieceArgs c) {
     constexpr int DP = R4 * 64;
@@ -181,6 +174,20 @@ __global__ void __launch_bounds__(64) linear_pieces_kernel(RecurArgs a, PieceArg
     const int head = blockIdx.x, piece = blockIdx.y, row0 = c.row0[piece], n = c.n[piece], qh = head / (a.heads / a.q_heads);
     const float* q = a.q + ((size_t)(row0 + min(l15, n - 1)) * a.q_heads + qh) * DP + grp * 4;
     const float* k = a.k + ((size_t)(row0 + min(l15, n - 1)) * a.q_heads + qh) * DP + grp * 4;
+    const size_t ph = (size_t)piece * a.heads + head;
+    const float decay = a.decay[head];
+    float p[16];
+    p[0] = 1.f;
+#pragma unroll
+    for (int i = 1; i < 16; ++i) p[i] = p[i - 1] * decay;
+    auto power = [&](int e) {
+        float f = 0.f;
+#pragma unroll
+        for (int x = 0; x < 16; ++x) f = e == x ? p[x] : f;
+        return f;
+    };
+    const float end = l15 < n ? power(n - 1 - l15) : 0.f;
+    float* kt = c.kt + ph * (16 * DP) + token_slot(l15);
     f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
     for (int t = 0; t < R4 * 4; ++t) {
@@ -189,20 +196,17 @@ __global__ void __launch_bounds__(64) linear_pieces_kernel(RecurArgs a, PieceArg
         acc[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, acc[t & 1], 0, 0, 0);
         acc[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, y.z, acc[t & 1], 0, 0, 0);
         acc[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, acc[t & 1], 0, 0, 0);
+        float* o = kt + (t * 16 + grp * 4) * 16;
+        o[0] = y.x * end;
+        o[16] = y.y * end;
+        o[32] = y.z * end;
+        o[48] = y.w * end;
     }
-    const float decay = a.decay[head];
-    float* o = c.pair + ((size_t)piece * a.heads + head) * 256;
-    float p[16];
-    p[0] = 1.f;
-#pragma unroll
-    for (int i = 1; i < 16; ++i) p[i] = p[i - 1] * decay;
+    float* o = c.pair + ph * 256;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         const int i = grp * 4 + r, j = l15;
-        float f = 0.f;
-#pragma unroll
-        for (int x = 0; x < 16; ++x) f = i - j == x ? p[x] : f;
-        o[i * 16 + token_slot(j)] = i < n && j < n ? (acc[0][r] + acc[1][r]) * f : 0.f;
+        o[i * 16 + token_slot(j)] = i < n && j <= i ? (acc[0][r] + acc[1][r]) * power(i - j) : 0.f;
     }
 }
 
@@ -212,7 +216,7 @@ __global__ void __launch_bounds__(64) linear_pieces_kernel(RecurArgs a, PieceArg
 template <int R4, bool DELTA, int NW>
 __global__ void __launch_bounds__(64 * NW) piece_scan_kernel(RecurArgs a, PieceArgs c) {
     constexpr int DP = R4 * 64, T = DP / 16, ROW = DP / 4;  // float4 per row of a [16][DP] operand
-    // float4 slots of a stage: Q, K (transposed and decayed for the delta rule), pair, then W and the decays
+    // float4 slots of a stage: Q, K (transposed and decayed), pair, then W and the decays of the delta rule
     constexpr int oQ = 0, oK = 16 * ROW, oP = 32 * ROW, oW = oP + 64, oG = oW + 16 * ROW, N4 = DELTA ? oG + ROW : oW;
     constexpr int NI = (N4 + 64 * NW - 1) / (64 * NW);
     constexpr int SLOTS = NI * 64 * NW;
@@ -220,41 +224,63 @@ __global__ void __launch_bounds__(64 * NW) piece_scan_kernel(RecurArgs a, PieceA
     const int lane = threadIdx.x & 63, l15 = lane & 15, grp = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int blocks = (a.vdim_p + 16 * NW - 1) / (16 * NW), head = blockIdx.x / blocks, col0 = ((blockIdx.x % blocks) * NW + wave) * 16;
-    const int sg = blockIdx.y, slot = a.seg.slot[sg], p0 = c.seg_piece0[sg], p1 = c.seg_piece0[sg + 1];
+    const int sg = blockIdx.y, slot = a.seg.slot[sg], p0 = c.seg_piece0[sg];
     const int qh = head / (a.heads / a.q_heads);
     const bool live = col0 < a.vdim_p;
     const int col = min(col0, a.vdim_p - 16) + l15;
-    // rows of Q, W (and K of the constant decays) are stored with their float4 units permuted by the token: reads of one unit of 16 tokens,
-    // and of one channel of 4 tokens, fall on different banks
-    auto source = [&](int piece, int row0, int n, int x) -> const float4* {
-        const size_t ph = (size_t)piece * a.heads + head;
-        if (x < oP) {
-            const int y = x < oK ? x : x - oK, tok = y / ROW, unit = (y % ROW) ^ token_slot(tok);
-            if (!DELTA) return reinterpret_cast<const float4*>((x < oK ? a.q : a.k) + ((size_t)(row0 + min(tok, n - 1)) * a.q_heads + qh) * DP) + unit;
-            return x < oK ? reinterpret_cast<const float4*>(c.qt + ph * (16 * DP)) + tok * ROW + unit : reinterpret_cast<const float4*>(c.kt + ph * (16 * DP)) + y;
+    // Rows of Q and W are stored with their float4 units permuted by the token: reads of one unit of 16 tokens fall on different banks.
+    // Every copy of a stage has a uniform base that moves on by a
+    // constant per piece and a lane offset that stays; a last piece of fewer rows reads on into rows that meet zero weights.
+    const int first = a.seg.row0[sg], rows = a.seg.n[sg];
+    const size_t ph = (size_t)p0 * a.heads + head, lin = ((size_t)first * a.q_heads + qh) * ROW;
+    const float4* src[NI];
+    int move[NI];
+    uint32_t off[NI];
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+        const int x0 = (i * NW + wave) * 64, x = x0 + lane;
+        const float4* base = reinterpret_cast<const float4*>(c.pair) + ph * 64;
+        int mv = a.heads * 64, o = min(x - oP, 63);
+        if (x0 < oP) {
+            const bool isq = x0 < oK;
+            const int y = isq ? x : x - oK, tok = y / ROW, unit = (y % ROW) ^ token_slot(tok);
+            if (!DELTA && isq) {
+                base = reinterpret_cast<const float4*>(a.q) + lin;
+                mv = 16 * a.q_heads * ROW;
+                o = tok * a.q_heads * ROW + unit;
+            } else {
+                base = reinterpret_cast<const float4*>(isq ? c.qt : c.kt) + ph * (16 * ROW);
+                mv = a.heads * 16 * ROW;
+                o = isq ? tok * ROW + unit : y;
+            }
+        } else if (DELTA && x0 >= oG) {
+            base = reinterpret_cast<const float4*>(c.decay) + ph * ROW;
+            mv = a.heads * ROW;
+            o = min(x - oG, ROW - 1);
+        } else if (DELTA && x0 >= oW) {
+            const int y = x - oW, tok = y / ROW;
+            base = reinterpret_cast<const float4*>(c.wt) + ph * (16 * ROW);
+            mv = a.heads * 16 * ROW;
+            o = tok * ROW + ((y % ROW) ^ token_slot(tok));
         }
-        if (x < oW || !DELTA) return reinterpret_cast<const float4*>(c.pair + ph * 256) + min(x - oP, 63);
-        if (x < oG) {
-            const int tok = (x - oW) / ROW, unit = ((x - oW) % ROW) ^ token_slot(tok);
-            return reinterpret_cast<const float4*>(c.wt + ph * (16 * DP)) + tok * ROW + unit;
-        }
-        return reinterpret_cast<const float4*>(c.decay + ph * DP) + min(x - oG, ROW - 1);
-    };
-    auto stage = [&](int piece, float4* b) {
-        const int row0 = c.row0[piece], n = c.n[piece];
+        src[i] = base;
+        move[i] = mv;
+        off[i] = (uint32_t)o * 16u;
+    }
+    auto stage = [&](float4* b) {  // the next piece
 #pragma unroll
         for (int i = 0; i < NI; ++i) {
-            const int x0 = (i * NW + wave) * 64;
-            __builtin_amdgcn_global_load_lds((gptr_t)source(piece, row0, n, x0 + lane), (lptr_t)(b + x0), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((gptr_t)(reinterpret_cast<const char*>(src[i]) + off[i]), (lptr_t)(b + (i * NW + wave) * 64), 16, 0, 0);
+            src[i] += move[i];
         }
     };
-    stage(p0, buf[0]);
+    stage(buf[0]);
     f32x4 S[T];
     float* st = a.state + ((size_t)slot * a.heads + head) * DP * a.vdim_p;
     auto state_at = [&](int t) {  // channels 16 t + 4 grp .. + 3 of column col
         return reinterpret_cast<f32x4*>(st) + ((size_t)((col >> 3) * R4 + (t >> 2)) * 2 + (col & 1)) * 64 + ((col & 7) >> 1) * 16 + (t & 3) * 4 + grp;
     };
-    const bool fresh = a.pos[c.row0[p0]] == 0;
+    const bool fresh = a.pos[first] == 0;
 #pragma unroll
     for (int t = 0; t < T; ++t) S[t] = fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *state_at(t);
     const float decay = DELTA ? 1.f : a.decay[head];
@@ -263,49 +289,65 @@ __global__ void __launch_bounds__(64 * NW) piece_scan_kernel(RecurArgs a, PieceA
         d4 = (decay * decay) * (decay * decay);
         for (int i = 0; i < grp; ++i) pw_lo *= decay;
     }
+    const float rest16 = (d4 * d4) * (d4 * d4);
     float v[4];
-    auto load_v = [&](int piece) {
-        const int row0 = c.row0[piece], n = c.n[piece];
+    const int hv = a.heads * a.vdim_p;
+    const float* vp = a.v + (size_t)(first + grp) * hv + (size_t)head * a.vdim_p + col;
+    float* op = a.o + (size_t)(first + grp) * hv + (size_t)head * a.vdim_p + col;
+    auto load_v = [&]() {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) v[r] = a.v[((size_t)(row0 + min(4 * r + grp, n - 1)) * a.heads + head) * a.vdim_p + col];
+        for (int r = 0; r < 4; ++r) v[r] = vp[(size_t)(4 * r) * hv];
+        vp += (size_t)16 * hv;
     };
-    load_v(p0);
+    load_v();
     const int tok = token_slot(l15);  // token of this lane's operand rows
+    uint32_t qa[T];  // LDS addresses in the first buffer
+#pragma unroll
+    for (int t = 0; t < T; ++t) qa[t] = lds_address(buf[0]) + (uint32_t)(tok * ROW + ((4 * t + grp) ^ l15)) * 16u;  // token_slot(tok) == l15
+    const uint32_t ka = lds_address(buf[0]) + (uint32_t)(l15 * 4 + grp) * 16u, ga = lds_address(buf[0]) + (uint32_t)grp * 16u;
+    const uint32_t pa = lds_address(buf[0]) + (uint32_t)(tok * 4 + grp) * 16u;
     dma_publish_barrier();
-    for (int pc = p0; pc < p1; ++pc) {
-        const float4* b = buf[(pc - p0) & 1];
-        const int row0 = c.row0[pc], n = c.n[pc];
+    for (int row = 0, cur = 0; row < rows; row += 16, cur ^= 1) {
+        const uint32_t b = (uint32_t)cur * (SLOTS * 16u);
+        const int n = min(16, rows - row);
+        const bool more = row + 16 < rows;
         f32x4 u;
 #pragma unroll
         for (int r = 0; r < 4; ++r) u[r] = 4 * r + grp < n ? v[r] : 0.f;
-        if (pc + 1 < p1) {
-            stage(pc + 1, buf[(pc - p0 + 1) & 1]);
-            load_v(pc + 1);
+        if (more) {
+            stage(buf[cur ^ 1]);
+            load_v();
         }
+        // W S and Q S: two state tiles' operands in flight ahead of the ones in use
         f32x4 qs[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}}, ws[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+        f32x4 xq[4], xw[4], xk[4], xg[4], pr;
+        auto read_qw = [&](int t) {
+            NVLLM_LDS_READ128(xq[t & 3], qa[t] + b, oQ * 16);
+            if constexpr (DELTA) NVLLM_LDS_READ128(xw[t & 3], qa[t] + b, oW * 16);
+        };
+        auto read_kg = [&](int t) {
+            NVLLM_LDS_READ128(xk[t & 3], ka + b + t * 1024, oK * 16);
+            if constexpr (DELTA) NVLLM_LDS_READ128(xg[t & 3], ga + b + t * 64, oG * 16);
+        };
+        constexpr int PER = DELTA ? 2 : 1;  // reads per tile
+        read_qw(0); read_qw(1);
 #pragma unroll
-        for (int t = 0; t < T; ++t) {
-            const int unit = (4 * t + grp) ^ l15;  // token_slot(tok) == l15
-            const float4 x = b[oQ + tok * ROW + unit];
-            if constexpr (DELTA) {
-                const float4 w = b[oW + tok * ROW + unit];
-                ws[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(w.x, S[t][0], ws[t & 1], 0, 0, 0);
-                qs[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, S[t][0], qs[t & 1], 0, 0, 0);
-                ws[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(w.y, S[t][1], ws[t & 1], 0, 0, 0);
-                qs[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, S[t][1], qs[t & 1], 0, 0, 0);
-                ws[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(w.z, S[t][2], ws[t & 1], 0, 0, 0);
-                qs[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, S[t][2], qs[t & 1], 0, 0, 0);
-                ws[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(w.w, S[t][3], ws[t & 1], 0, 0, 0);
-                qs[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, S[t][3], qs[t & 1], 0, 0, 0);
-            } else {
-                qs[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, S[t][0], qs[t & 1], 0, 0, 0);
-                qs[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, S[t][1], qs[t & 1], 0, 0, 0);
-                qs[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, S[t][2], qs[t & 1], 0, 0, 0);
-                qs[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, S[t][3], qs[t & 1], 0, 0, 0);
-            }
+        for (int t = 0; t < T; t += 2) {
+            if (t + 2 < T) { read_qw(t + 2); read_qw(t + 3); }
+            else { NVLLM_LDS_READ128(pr, pa + b, oP * 16); read_kg(0); read_kg(1); }
+            if (t + 2 < T) NVLLM_LDS_WAIT(2 * PER);
+            else NVLLM_LDS_WAIT(2 * PER + 1);
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int x = 0; x < 2; ++x) {
+                    if constexpr (DELTA) ws[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(xw[(t + x) & 3][i], S[t + x][i], ws[x], 0, 0, 0);
+                    qs[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(xq[(t + x) & 3][i], S[t + x][i], qs[x], 0, 0, 0);
+                }
+            __builtin_amdgcn_sched_barrier(0);
         }
         f32x4 o;
-        float pw = pw_lo * decay, rest = 1.f;  // decay^(i + 1) of token i = grp; decay^(n - 1 - i) below
+        float rest = rest16;
         if constexpr (DELTA) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
@@ -313,52 +355,44 @@ __global__ void __launch_bounds__(64 * NW) piece_scan_kernel(RecurArgs a, PieceA
                 o[r] = qs[0][r] + qs[1][r];
             }
         } else {
+            float pw = pw_lo * decay;  // decay^(i + 1) of token i = grp
 #pragma unroll
             for (int r = 0; r < 4; ++r, pw *= d4) o[r] = (qs[0][r] + qs[1][r]) * pw;
+            if (n < 16) {
+                rest = 1.f;
+                for (int i = 0; i < n; ++i) rest *= decay;
+            }
         }
-        const float4 pr = b[oP + tok * 4 + grp];
-        o = __builtin_amdgcn_mfma_f32_16x16x4f32(pr.x, u[0], o, 0, 0, 0);
-        o = __builtin_amdgcn_mfma_f32_16x16x4f32(pr.y, u[1], o, 0, 0, 0);
-        o = __builtin_amdgcn_mfma_f32_16x16x4f32(pr.z, u[2], o, 0, 0, 0);
-        o = __builtin_amdgcn_mfma_f32_16x16x4f32(pr.w, u[3], o, 0, 0, 0);
-        if constexpr (!DELTA) {
-            // rows of u times decay^(n - 1 - i), the state times decay^n
-            float up[4];
+#pragma unroll
+        for (int t = 0; t < T; t += 2) {
+            if (t + 2 < T) { read_kg(t + 2); read_kg(t + 3); NVLLM_LDS_WAIT(2 * PER); }
+            else NVLLM_LDS_WAIT(0);
+#pragma unroll
+            for (int x = 0; x < 2; ++x)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) S[t + x][r] *= DELTA ? xg[(t + x) & 3][r] : rest;
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                float f = 1.f;
-                for (int i = 4 * r + grp; i < n - 1; ++i) f *= decay;
-                up[r] = f;
+                if (t == 0) o = __builtin_amdgcn_mfma_f32_16x16x4f32(pr[r], u[r], o, 0, 0, 0);
+#pragma unroll
+                for (int x = 0; x < 2; ++x) S[t + x] = __builtin_amdgcn_mfma_f32_16x16x4f32(xk[(t + x) & 3][r], u[r], S[t + x], 0, 0, 0);
             }
-            for (int i = 0; i < n; ++i) rest *= decay;
-#pragma unroll
-            for (int r = 0; r < 4; ++r) u[r] *= up[r];
+            __builtin_amdgcn_sched_barrier(0);
         }
+        if (more && live) {
 #pragma unroll
-        for (int t = 0; t < T; ++t) {
-            float kx[4];
-            if constexpr (DELTA) {
-                const float4 g = b[oG + t * 4 + grp], k = b[oK + (t * 16 + l15) * 4 + grp];
-                S[t][0] *= g.x; S[t][1] *= g.y; S[t][2] *= g.z; S[t][3] *= g.w;
-                kx[0] = k.x; kx[1] = k.y; kx[2] = k.z; kx[3] = k.w;
-            } else {
-                const float* kb = reinterpret_cast<const float*>(b + oK);
+            for (int r = 0; r < 4; ++r) op[(size_t)(4 * r) * hv] = o[r];
+            op += (size_t)16 * hv;
+            // the next piece has landed everywhere; the four stores may still be on their way
+            asm volatile("s_waitcnt vmcnt(4)\n\ts_barrier" ::: "memory");
+        } else {
+            if (live) {
 #pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    S[t][r] *= rest;
-                    const int j = 4 * r + grp;
-                    kx[r] = kb[(j * ROW + ((4 * t + (l15 >> 2)) ^ token_slot(j))) * 4 + (l15 & 3)];
-                }
+                for (int r = 0; r < 4; ++r)
+                    if (4 * r + grp < n) op[(size_t)(4 * r) * hv] = o[r];
             }
-#pragma unroll
-            for (int r = 0; r < 4; ++r) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(kx[r], u[r], S[t], 0, 0, 0);
+            asm volatile("s_waitcnt vmcnt(0)\n\ts_barrier" ::: "memory");
         }
-        if (live) {
-#pragma unroll
-            for (int r = 0; r < 4; ++r)
-                if (4 * r + grp < n) a.o[((size_t)(row0 + 4 * r + grp) * a.heads + head) * a.vdim_p + col] = o[r];
-        }
-        dma_publish_barrier();
     }
     if (live) {
 #pragma unroll
@@ -381,7 +415,7 @@ static void piece_scan_t(const RecurArgs& a, const PieceArgs& c, hipStream_t s) 
     else piece_scan_kernel<R4, DELTA, 1><<<grid, 64, 0, s>>>(a, c);
 }
 hipError_t launch_piece_scan(const RecurArgs& a, const PieceArgs& c, hipStream_t s) {
-    if (!piece_scan_ok(a.dim_p) || a.vdim_p % 16 || a.seg.single || !c.pair || (a.g && (!c.qt || !c.wt || !c.kt || !c.decay || !a.beta)) || (!a.g && !a.decay)) return hipErrorInvalidValue;
+    if (!piece_scan_ok(a.dim_p) || a.vdim_p % 16 || a.seg.single || !c.pair || !c.kt || (a.g && (!c.qt || !c.wt || !c.decay || !a.beta)) || (!a.g && !a.decay)) return hipErrorInvalidValue;
     if (c.count > 65535) return hipErrorNotSupported;
     if (a.seg.count <= 0 || c.count <= 0) return hipSuccess;
     switch (a.dim_p / 64) {
