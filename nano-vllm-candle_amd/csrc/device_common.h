@@ -238,6 +238,11 @@ __device__ __forceinline__ void load_slabs8(float (&x)[8], const float* p, int l
 
 // s += the n partial sums of one float4, four independent loads per trip (clamped index, masked sum)
 __device__ __forceinline__ void add_slabs(float4& s, const float* p, int n, int64_t stride) {
+    if (n == 1) {
+        const float4 t = *reinterpret_cast<const float4*>(p);
+        s.x += t.x; s.y += t.y; s.z += t.z; s.w += t.w;
+        return;
+    }
     for (int sl0 = 0; sl0 < n; sl0 += 4) {
         float4 t[4];
 #pragma unroll

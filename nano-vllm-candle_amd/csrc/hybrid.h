@@ -144,7 +144,7 @@ struct PieceArgs {
     float* decay = nullptr;          // [dim_p] decays of the whole piece
 };
 bool piece_scan_ok(int dim_p);
-// q, k and v hold kPiece more rows than the chunk (anything finite); v is overwritten for the delta rule
+// q, k, v, g and beta hold kPiece more rows than the chunk (anything finite); v is overwritten for the delta rule
 hipError_t launch_piece_scan(const RecurArgs& a, const PieceArgs& c, hipStream_t s);
 
 // rows after the q / k / v / gate projection of the constant-decay recurrence: silu(q, k, v), sigmoid(gate)

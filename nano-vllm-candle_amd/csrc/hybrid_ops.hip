@@ -56,7 +56,7 @@ __device__ __forceinline__ void sum_row(float* x, const float* in, int n, int n_
 
 __global__ void __launch_bounds__(256) attn_rows_kernel(AttnRowsArgs a) {
     extern __shared__ __attribute__((aligned(16))) float xr[];
-    __shared__ float red[4];
+    __shared__ float red[8];
     const int row = blockIdx.x;
     const int nq = a.heads * a.kv.dim, nk = a.kv.kv * a.kv.dim, nv = a.kv.kv * a.kv.vdim;
     sum_row(xr, a.in + (size_t)row * a.ld, (nq + nk + nv + 3) & ~3, a.n_slabs, a.slab_stride, a.bias);
@@ -68,17 +68,61 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(AttnRowsArgs a) {
     } else {
         for (int c = threadIdx.x; c < nq; c += 256) sq += xr[c] * xr[c];
         for (int c = threadIdx.x; c < nk; c += 256) sk += xr[nq + c] * xr[nq + c];
-        sq = block_sum(sq, red, 4);
-        sk = block_sum(sk, red, 4);
+        sq = wave_sum_uniform(sq);
+        sk = wave_sum_uniform(sk);
+        if ((threadIdx.x & 63) == 0) { red[threadIdx.x >> 6] = sq; red[4 + (threadIdx.x >> 6)] = sk; }
+        __syncthreads();
+        sq = (red[0] + red[1]) + (red[2] + red[3]);
+        sk = (red[4] + red[5]) + (red[6] + red[7]);
     }
     const float rq = 1.0f / sqrtf(sq / (float)a.q_all + a.eps), rk = 1.0f / sqrtf(sk / (float)a.k_all + a.eps);
     float* q = a.q + (size_t)row * a.heads * a.kv.dim_p;
+    const int pos = a.pos[row], t = pos & (kBlockTokens - 1);
+    const size_t blk = (size_t)a.block_tables[(size_t)a.slot[row] * a.max_blocks + pos / kBlockTokens] * a.kv.kv;
+    if (((a.kv.dim | a.kv.vdim) & 3) == 0) {  // four columns of one head per thread
+        const int d4 = a.kv.dim_p >> 2, k4 = a.kv.dim >> 2, v4 = a.kv.vdim >> 2;
+        for (int i = threadIdx.x; i < a.heads * d4; i += 256) {
+            const int h = i / d4, d = (i - h * d4) * 4, c = h * a.kv.dim + d;
+            float4 y = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (d < a.kv.dim) {
+                const float4 x = *reinterpret_cast<const float4*>(xr + c), w = *reinterpret_cast<const float4*>(a.qn + c);
+                y = make_float4((x.x * rq) * w.x * a.q_scale, (x.y * rq) * w.y * a.q_scale, (x.z * rq) * w.z * a.q_scale, (x.w * rq) * w.w * a.q_scale);
+            }
+            reinterpret_cast<float4*>(q)[i] = y;
+        }
+        for (int i = threadIdx.x; i < a.kv.kv * k4; i += 256) {
+            const int h = i / k4, d = (i - h * k4) * 4, c = h * a.kv.dim + d;
+            const float4 x = *reinterpret_cast<const float4*>(xr + nq + c), w = *reinterpret_cast<const float4*>(a.kn + c);
+            const float y[4] = {(x.x * rk) * w.x, (x.y * rk) * w.y, (x.z * rk) * w.z, (x.w * rk) * w.w};
+            const size_t o = (blk + h) * kBlockTokens * a.kv.dim_p + k_packed_offset(t, d, a.kv.dim_p);
+            if (a.kv.f32) *reinterpret_cast<float4*>(reinterpret_cast<float*>(a.kv.k) + o) = make_float4(y[0], y[1], y[2], y[3]);
+            else {
+                typedef __attribute__((ext_vector_type(4))) _Float16 f16x4;
+                *reinterpret_cast<f16x4*>(reinterpret_cast<_Float16*>(a.kv.k) + o) = f16x4{f16_sat(y[0]), f16_sat(y[1]), f16_sat(y[2]), f16_sat(y[3])};
+            }
+        }
+        const float lam = a.mix == 2 ? a.lambda[0] : 0.f;
+        for (int i = threadIdx.x; i < a.kv.kv * v4; i += 256) {
+            const int h = i / v4, d = (i - h * v4) * 4, c = h * a.kv.vdim + d;
+            float4 x = *reinterpret_cast<const float4*>(xr + nq + nk + c);
+            float4* vf = reinterpret_cast<float4*>(a.v_first + (size_t)row * nv + c);
+            if (a.mix == 1) *vf = x;
+            if (a.mix == 2) {
+                const float4 f = *vf;
+                x = make_float4((1.0f - lam) * x.x + lam * f.x, (1.0f - lam) * x.y + lam * f.y, (1.0f - lam) * x.z + lam * f.z, (1.0f - lam) * x.w + lam * f.w);
+            }
+            const size_t o = (blk + h) * kBlockTokens * a.kv.vdim_p + v_packed_offset(t, d, a.kv.vdim_p);  // neighbouring dimensions are 8 apart
+            kv_put(a.kv.v, a.kv.f32, o, x.x);
+            kv_put(a.kv.v, a.kv.f32, o + 8, x.y);
+            kv_put(a.kv.v, a.kv.f32, o + 16, x.z);
+            kv_put(a.kv.v, a.kv.f32, o + 24, x.w);
+        }
+        return;
+    }
     for (int i = threadIdx.x; i < a.heads * a.kv.dim_p; i += 256) {
         const int h = i / a.kv.dim_p, d = i - h * a.kv.dim_p, c = h * a.kv.dim + d;
         q[i] = d < a.kv.dim ? (xr[c] * rq) * a.qn[c] * a.q_scale : 0.f;
     }
-    const int pos = a.pos[row], t = pos & (kBlockTokens - 1);
-    const size_t blk = (size_t)a.block_tables[(size_t)a.slot[row] * a.max_blocks + pos / kBlockTokens] * a.kv.kv;
     for (int c = threadIdx.x; c < nk; c += 256) {
         const int h = c / a.kv.dim, d = c - h * a.kv.dim;
         kv_put(a.kv.k, a.kv.f32, (blk + h) * kBlockTokens * a.kv.dim_p + k_packed_offset(t, d, a.kv.dim_p), (xr[nq + c] * rk) * a.kn[c]);
@@ -92,12 +136,101 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(AttnRowsArgs a) {
         kv_put(a.kv.v, a.kv.f32, (blk + h) * kBlockTokens * a.kv.vdim_p + v_packed_offset(t, d, a.kv.vdim_p), v);
     }
 }
+// prompt chunks: a wave per row, four rows per workgroup, the row in registers; values meet in LDS, so that four consecutive tokens of
+// one dimension, neighbours in the cache, are one store
+template <int NI>
+__global__ void __launch_bounds__(256) attn_rows4_kernel(AttnRowsArgs a, int rows) {
+    extern __shared__ __attribute__((aligned(16))) float vs[];  // [4][nv]
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int row0 = blockIdx.x * 4, row = min(row0 + wave, rows - 1);
+    const int nq = a.heads * a.kv.dim, nk = a.kv.kv * a.kv.dim, nv = a.kv.kv * a.kv.vdim, n = nq + nk + nv;
+    const float* in = a.in + (size_t)row * a.ld;
+    float4 x[NI];
+    float sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+        const int c = (lane + i * 64) * 4;
+        x[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (c < n) {
+            if (a.bias) x[i] = *reinterpret_cast<const float4*>(a.bias + c);
+            add_slabs(x[i], in + c, a.n_slabs, a.slab_stride);
+        }
+        const float ss = x[i].x * x[i].x + x[i].y * x[i].y + x[i].z * x[i].z + x[i].w * x[i].w;
+        if (c < nq) sq += ss;
+        else if (c < nq + nk) sk += ss;
+    }
+    sq = a.ssq ? a.ssq[row * 2] : wave_sum_uniform(sq);
+    sk = a.ssq ? a.ssq[row * 2 + 1] : wave_sum_uniform(sk);
+    const float rq = 1.0f / sqrtf(sq / (float)a.q_all + a.eps), rk = 1.0f / sqrtf(sk / (float)a.k_all + a.eps);
+    const int pos = a.pos[row], t = pos & (kBlockTokens - 1);
+    const int* bt = a.block_tables + (size_t)a.slot[row] * a.max_blocks;
+    const size_t blk = (size_t)bt[pos / kBlockTokens] * a.kv.kv;
+    const float lam = a.mix == 2 ? a.lambda[0] : 0.f;
+    const bool live = row0 + wave < rows;
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+        const int c = (lane + i * 64) * 4;
+        if (!live || c >= n) continue;
+        if (c < nq) {
+            const float4 w = *reinterpret_cast<const float4*>(a.qn + c);
+            const int h = c / a.kv.dim, d = c - h * a.kv.dim;
+            *reinterpret_cast<float4*>(a.q + ((size_t)row * a.heads + h) * a.kv.dim_p + d) =
+                make_float4((x[i].x * rq) * w.x * a.q_scale, (x[i].y * rq) * w.y * a.q_scale, (x[i].z * rq) * w.z * a.q_scale, (x[i].w * rq) * w.w * a.q_scale);
+        } else if (c < nq + nk) {
+            const float4 w = *reinterpret_cast<const float4*>(a.kn + c - nq);
+            const int h = (c - nq) / a.kv.dim, d = c - nq - h * a.kv.dim;
+            typedef __attribute__((ext_vector_type(4))) _Float16 f16x4;
+            *reinterpret_cast<f16x4*>(reinterpret_cast<_Float16*>(a.kv.k) + (blk + h) * kBlockTokens * a.kv.dim_p + k_packed_offset(t, d, a.kv.dim_p)) =
+                f16x4{f16_sat((x[i].x * rk) * w.x), f16_sat((x[i].y * rk) * w.y), f16_sat((x[i].z * rk) * w.z), f16_sat((x[i].w * rk) * w.w)};
+        } else {
+            float4 v = x[i];
+            float4* vf = reinterpret_cast<float4*>(a.v_first + (size_t)row * nv + c - nq - nk);
+            if (a.mix == 1) *vf = v;
+            if (a.mix == 2) {
+                const float4 f = *vf;
+                v = make_float4((1.0f - lam) * v.x + lam * f.x, (1.0f - lam) * v.y + lam * f.y, (1.0f - lam) * v.z + lam * f.z, (1.0f - lam) * v.w + lam * f.w);
+            }
+            *reinterpret_cast<float4*>(vs + (size_t)wave * nv + c - nq - nk) = v;
+        }
+    }
+    for (int d = a.kv.dim + lane; d < a.kv.dim_p; d += 64)
+        if (live)
+            for (int h = 0; h < a.heads; ++h) a.q[((size_t)row * a.heads + h) * a.kv.dim_p + d] = 0.f;
+    __syncthreads();
+    const int p0 = a.pos[row0], s0 = a.slot[row0];
+    bool together = row0 + 4 <= rows && (p0 & 3) == 0;
+    for (int r = 1; r < 4; ++r) together = together && a.slot[min(row0 + r, rows - 1)] == s0;
+    _Float16* v = reinterpret_cast<_Float16*>(a.kv.v);
+    if (together) {
+        typedef __attribute__((ext_vector_type(4))) _Float16 f16x4;
+        const size_t b0 = (size_t)a.block_tables[(size_t)s0 * a.max_blocks + p0 / kBlockTokens] * a.kv.kv;
+        for (int c = threadIdx.x; c < nv; c += 256) {
+            const int h = c / a.kv.vdim, d = c - h * a.kv.vdim;
+            *reinterpret_cast<f16x4*>(v + (b0 + h) * kBlockTokens * a.kv.vdim_p + v_packed_offset(p0 & (kBlockTokens - 1), d, a.kv.vdim_p)) =
+                f16x4{f16_sat(vs[c]), f16_sat(vs[nv + c]), f16_sat(vs[2 * nv + c]), f16_sat(vs[3 * nv + c])};
+        }
+    } else if (live) {
+        for (int c = lane; c < nv; c += 64) {
+            const int h = c / a.kv.vdim, d = c - h * a.kv.vdim;
+            v[(blk + h) * kBlockTokens * a.kv.vdim_p + v_packed_offset(t, d, a.kv.vdim_p)] = f16_sat(vs[(size_t)wave * nv + c]);
+        }
+    }
+}
+
 hipError_t launch_attn_rows(const AttnRowsArgs& a, int rows, hipStream_t s) {
     const int n = a.heads * a.kv.dim + a.kv.kv * (a.kv.dim + a.kv.vdim);
     if (a.kv.dim_p % 32 || a.kv.vdim_p % 16 || n > a.ld || a.ld % 4 || (a.mix && !a.v_first) || (a.mix == 2 && !a.lambda)) return hipErrorInvalidValue;
     const size_t lds = ((size_t)n + 4) * 4;
     if (lds > 64 * 1024) return hipErrorNotSupported;
     if (rows <= 0) return hipSuccess;
+    const size_t lds4 = (size_t)4 * a.kv.kv * a.kv.vdim * 4;
+    if (rows >= 64 && !a.kv.f32 && ((a.kv.dim | a.kv.vdim) & 3) == 0 && (a.slab_stride & 3) == 0 && n <= 24 * 256 && lds4 <= 64 * 1024) {
+        const int wgs = (rows + 3) / 4;
+        if (n <= 8 * 256) attn_rows4_kernel<8><<<wgs, 256, lds4, s>>>(a, rows);
+        else if (n <= 16 * 256) attn_rows4_kernel<16><<<wgs, 256, lds4, s>>>(a, rows);
+        else attn_rows4_kernel<24><<<wgs, 256, lds4, s>>>(a, rows);
+        return hipGetLastError();
+    }
     attn_rows_kernel<<<rows, 256, lds, s>>>(a);
     return hipGetLastError();
 }
@@ -255,6 +388,9 @@ __global__ void __launch_bounds__(256) delta_rows16_kernel(DeltaRowsArgs a, int 
     const int hd = qk ? unit % a.kv : unit - 2 * a.kv, hs = qk ? a.kv : a.heads;
     float* out = (qk ? (unit < a.kv ? a.q : a.k) : a.v) + (size_t)hd * n_p;
     const float unit_scale = unit < a.kv ? a.q_scale : 1.f;
+    bool plain = row0 + 16 <= rows && row0 >= TAPS - 1 && a.n_slabs == 1;
+    if (plain)
+        for (int r = -(TAPS - 1); r < 15; ++r) plain &= a.slot[row0 + r] == a.slot[row0 + 15];
     for (int d0 = 0; d0 < n_p; d0 += 64 * NE) {  // once for q and k (dim_p = 64 NE): their norm needs the whole head
         float w[TAPS][NE], x[TAPS][NE];
 #pragma unroll
@@ -262,6 +398,34 @@ __global__ void __launch_bounds__(256) delta_rows16_kernel(DeltaRowsArgs a, int 
             const int d = d0 + e * 64 + lane;
 #pragma unroll
             for (int i = 0; i < TAPS; ++i) w[i][e] = d < n ? a.conv[(size_t)i * channels + c0 + d] : 0.f;
+        }
+        if (plain) {  // one sequence, its window inside the chunk: every load of the block is in flight at once
+            float z[15 + TAPS][NE];
+            const float* in = a.in + (size_t)(row0 - (TAPS - 1)) * a.ld + c0;
+#pragma unroll
+            for (int r = 0; r < 15 + TAPS; ++r)
+#pragma unroll
+                for (int e = 0; e < NE; ++e) {
+                    const int d = d0 + e * 64 + lane;
+                    z[r][e] = d < n ? in[(size_t)r * a.ld + d] : 0.f;
+                }
+#pragma unroll
+            for (int r = 0; r < 16; ++r) {
+                float y[NE], ss = 0.f;
+#pragma unroll
+                for (int e = 0; e < NE; ++e) {
+                    float t = 0.f;
+#pragma unroll
+                    for (int i = 0; i < TAPS; ++i) t += z[r + i][e] * w[i][e];
+                    y[e] = t * sigmoidf(t);
+                    ss += y[e] * y[e];
+                }
+                const float f = qk ? unit_scale / sqrtf(wave_sum_uniform(ss) + kUnitNormEps) : 1.f;
+#pragma unroll
+                for (int e = 0; e < NE; ++e)
+                    if (d0 + e * 64 + lane < n_p) out[(size_t)(row0 + r) * hs * n_p + d0 + e * 64 + lane] = y[e] * f;
+            }
+            continue;
         }
         for (int row = row0; row < row1; ++row) {
             const int slot = a.slot[row];
@@ -380,10 +544,17 @@ __global__ void __launch_bounds__(256) delta_gates_kernel(HeadGemmArgs a) {
     __syncthreads();
     const uint4* w = a.w + (size_t)head * a.w_head;
     const int ntiles = a.N >> 4;
+    uint4 wn[KT];  // the next tile's weights
+    auto fetch = [&](int nt) {
+#pragma unroll
+        for (int k = 0; k < KT; ++k) wn[k] = w[((size_t)min(nt, ntiles - 1) * KT + k) * 64 + lane];
+    };
+    fetch(blockIdx.z * 4 + wave);
     for (int nt = blockIdx.z * 4 + wave; nt < ntiles; nt += 4 * gridDim.z) {
         uint4 wf[KT];
 #pragma unroll
-        for (int k = 0; k < KT; ++k) wf[k] = w[((size_t)nt * KT + k) * 64 + lane];
+        for (int k = 0; k < KT; ++k) wf[k] = wn[k];
+        fetch(nt + 4 * gridDim.z);
         f32x4 acc[4];
 #pragma unroll
         for (int b = 0; b < 4; ++b) {

@@ -30,9 +30,11 @@ __global__ void __launch_bounds__(64) delta_pieces_kernel(RecurArgs a, PieceArgs
     const int lane = threadIdx.x, dg = lane & 15, jg = lane >> 4;
     const int head = blockIdx.x, piece = blockIdx.y, row0 = c.row0[piece], n = c.n[piece], qh = head / (a.heads / a.q_heads);
     const size_t ph = (size_t)piece * a.heads + head;
-    auto k_row = [&](int i) { return a.k + ((size_t)(row0 + min(i, n - 1)) * a.q_heads + qh) * DP; };
-    auto q_row = [&](int i) { return a.q + ((size_t)(row0 + min(i, n - 1)) * a.q_heads + qh) * DP; };
-    auto g_row = [&](int i) { return a.g + (size_t)(row0 + min(i, n - 1)) * a.g_row + (size_t)head * DP; };
+    // rows past the piece's last one hold something finite that is masked
+    const float* kb = a.k + ((size_t)row0 * a.q_heads + qh) * DP;
+    const float* qb = a.q + ((size_t)row0 * a.q_heads + qh) * DP;
+    const float* gb = a.g + (size_t)row0 * a.g_row + (size_t)head * DP;
+    const int ks = a.q_heads * DP, gs = (int)a.g_row;
     // A and B: lane (jg, dg) carries t_j of tokens j = 4 s + jg for the channels 64 r + 4 dg + e
     {
         float t[4][R4 * 4], all[R4 * 4];
@@ -46,9 +48,9 @@ __global__ void __launch_bounds__(64) delta_pieces_kernel(RecurArgs a, PieceArgs
         auto load = [&](int i) {
 #pragma unroll
             for (int r = 0; r < R4; ++r) {
-                kn[r] = *reinterpret_cast<const float4*>(k_row(i) + r * 64 + dg * 4);
-                qn[r] = *reinterpret_cast<const float4*>(q_row(i) + r * 64 + dg * 4);
-                gn[r] = *reinterpret_cast<const float4*>(g_row(i) + r * 64 + dg * 4);
+                kn[r] = *reinterpret_cast<const float4*>(kb + i * ks + (r * 64 + dg * 4));
+                qn[r] = *reinterpret_cast<const float4*>(qb + i * ks + (r * 64 + dg * 4));
+                gn[r] = *reinterpret_cast<const float4*>(gb + i * gs + (r * 64 + dg * 4));
             }
         };
         load(0);
@@ -107,62 +109,51 @@ __global__ void __launch_bounds__(64) delta_pieces_kernel(RecurArgs a, PieceArgs
     // forward substitution, one column per lane: W for the channels, V' for the values
     float beta[16];
 #pragma unroll
-    for (int i = 0; i < 16; ++i) beta[i] = i < n ? a.beta[(size_t)(row0 + min(i, n - 1)) * a.heads + head] : 0.f;
-    auto solve = [&](float (&y)[2][16]) {
+    for (int i = 0; i < 16; ++i) beta[i] = i < n ? a.beta[(size_t)(row0 + i) * a.heads + head] : 0.f;
+    auto solve = [&](float (&y)[16]) {
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
-            float ai[16];
+            float s = y[i];
 #pragma unroll
             for (int x = 0; x < 4; ++x) {
-                const float4 v = *reinterpret_cast<const float4*>(&A[i * 16 + x * 4]);
-                ai[x] = v.x; ai[4 + x] = v.y; ai[8 + x] = v.z; ai[12 + x] = v.w;
+                if (x > 0 && x >= i) continue;
+                const float4 v = *reinterpret_cast<const float4*>(&A[i * 16 + x * 4]);  // tokens x, 4 + x, 8 + x, 12 + x
+                if (x < i) s -= v.x * y[x];
+                if (4 + x < i) s -= v.y * y[4 + x];
+                if (8 + x < i) s -= v.z * y[8 + x];
+                if (12 + x < i) s -= v.w * y[12 + x];
             }
-#pragma unroll
-            for (int u = 0; u < 2; ++u) {
-                float s = y[u][i];
-#pragma unroll
-                for (int j = 0; j < 16; ++j)
-                    if (j < i) s -= ai[j] * y[u][j];
-                y[u][i] = beta[i] * s;
-            }
+            y[i] = beta[i] * s;
         }
     };
-    for (int d0 = lane; d0 < DP; d0 += 128) {
-        float y[2][16];
+#pragma unroll 1
+    for (int d = lane; d < DP; d += 64) {
+        float y[16], f = 1.f;
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-            const int d = min(d0 + u * 64, DP - 64 + lane);
-            float f = 1.f;
-#pragma unroll
-            for (int i = 0; i < 16; ++i) {
-                const float g = g_row(i)[d], k = k_row(i)[d], q = q_row(i)[d];
-                f *= i < n ? g : 1.f;
-                y[u][i] = i < n ? k * f : 0.f;
-                if (d0 + u * 64 < DP) c.qt[(ph * 16 + i) * DP + d] = i < n ? q * f : 0.f;
-            }
+        for (int i = 0; i < 16; ++i) {
+            const float g = gb[i * gs + d], k = kb[i * ks + d], q = qb[i * ks + d];
+            f *= i < n ? g : 1.f;
+            y[i] = i < n ? k * f : 0.f;
+            c.qt[(ph * 16 + i) * DP + d] = i < n ? q * f : 0.f;
         }
         solve(y);
 #pragma unroll
-        for (int u = 0; u < 2; ++u)
-            if (d0 + u * 64 < DP) {
-#pragma unroll
-                for (int i = 0; i < 16; ++i) c.wt[(ph * 16 + i) * DP + d0 + u * 64] = y[u][i];
-            }
+        for (int i = 0; i < 16; ++i) c.wt[(ph * 16 + i) * DP + d] = y[i];
     }
     float* v = const_cast<float*>(a.v) + ((size_t)row0 * a.heads + head) * a.vdim_p;
-    const size_t vs = (size_t)a.heads * a.vdim_p;
-    for (int e0 = lane; e0 < a.vdim_p; e0 += 128) {
-        float y[2][16];
+    const int vs = a.heads * a.vdim_p;
+#pragma unroll 1
+    for (int e = lane; e < a.vdim_p; e += 64) {
+        float y[16];
 #pragma unroll
-        for (int u = 0; u < 2; ++u)
-#pragma unroll
-            for (int i = 0; i < 16; ++i) y[u][i] = i < n && e0 + u * 64 < a.vdim_p ? v[i * vs + e0 + u * 64] : 0.f;
+        for (int i = 0; i < 16; ++i) {
+            const float x = v[i * vs + e];
+            y[i] = i < n ? x : 0.f;
+        }
         solve(y);
 #pragma unroll
-        for (int u = 0; u < 2; ++u)
-#pragma unroll
-            for (int i = 0; i < 16; ++i)
-                if (i < n && e0 + u * 64 < a.vdim_p) v[i * vs + e0 + u * 64] = y[u][i];
+        for (int i = 0; i < 16; ++i)
+            if (i < n) v[i * vs + e] = y[i];
     }
 }
 
