@@ -380,8 +380,8 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
     extern __shared__ float tab[];  // [gqa][n_bias] when bias_lds
     const int lane = threadIdx.x & 63, l15 = lane & 15, grp = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const int tile = a.tile_order ? a.tile_order[blockIdx.x] : blockIdx.x;
-    const int gqa = a.heads / a.kv.kv, per = gqa * (kBiasTileRows / RW), kvh = blockIdx.y / per, f0 = (blockIdx.y % per) * RW;
+    const int tile = a.tile_order ? a.tile_order[blockIdx.y] : blockIdx.y;  // every head's longest tiles start first
+    const int gqa = a.heads / a.kv.kv, per = gqa * (kBiasTileRows / RW), kvh = blockIdx.x / per, f0 = (blockIdx.x % per) * RW;
     const int row0 = a.tile_row0[tile], total = a.tile_nrows[tile] * gqa, slot = a.tile_slot[tile];
     if (f0 >= total) return;
     const int pos0 = a.pos[row0];
@@ -568,6 +568,7 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
 
 hipError_t launch_bias_prefill(const BiasAttnArgs& a, int n_tiles, hipStream_t s) {
     if (!matrix_core_ok(a)) return hipErrorInvalidValue;
+    if (n_tiles > 65535) return hipErrorNotSupported;
     if (n_tiles <= 0) return hipSuccess;
     const int gqa = a.heads / a.kv.kv;
     const int bias_lds = a.n_bias && (size_t)gqa * a.n_bias <= 6144;
@@ -575,7 +576,7 @@ hipError_t launch_bias_prefill(const BiasAttnArgs& a, int n_tiles, hipStream_t s
 #define NVLLM_BA_P(K_, V_)                                                                                           \
     {                                                                                                                \
         constexpr int MT_ = K_ > 4 || V_ > 8 ? 1 : 2;                                                                \
-        const dim3 grid(n_tiles, a.kv.kv * gqa * (kBiasTileRows / (64 * MT_)));                                      \
+        const dim3 grid(a.kv.kv * gqa * (kBiasTileRows / (64 * MT_)), n_tiles);                                      \
         if (lds + 2 * (2 * K_ + V_) * 1024 > 64 * 1024) {                                                            \
             static std::atomic<uint64_t> done{0};                                                                    \
             ensure_dyn_lds(reinterpret_cast<const void*>(bias_prefill_kernel<K_, V_, MT_>), 24 * 1024, done);             \

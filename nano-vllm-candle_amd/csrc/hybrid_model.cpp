@@ -701,6 +701,10 @@ int HybridModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
             if (pu.kind == P_TILE && gemm_tile_ok(R, w.ff_p, Kw, 4, m->opt_tile_min_wgs)) {
                 PROF(m, PROF_GEMM, launch_gemm_tile(m->xh, m->xl, w.up, R, 4, nullptr, m->xh2, m->xl2, pd.packed, m->opt_tile_min_wgs, 1, nullptr, s));
                 ++m->tile_launches;
+            } else if (pu.kind == P_ROW && gemm_rowdir_ok(w.ff_p, Kw, 3, R)) {
+                RowParArgs ua;
+                ua.xh = m->xh; ua.xl = m->xl; ua.ldx = Kw; ua.oh = m->xh2; ua.ol = m->xl2; ua.M = R; ua.x_packed = pu.packed; ua.o_packed = pd.packed;
+                PROF(m, PROF_GEMM, launch_gemm_rowpar(ua, w.up, 3, s));
             } else {
                 rc = product(m, pu, y, m->xh, m->xl, w.up, R, &ns);
                 if (rc) return rc;

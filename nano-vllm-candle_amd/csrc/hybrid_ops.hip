@@ -54,9 +54,11 @@ __device__ __forceinline__ void sum_row(float* x, const float* in, int n, int n_
     }
 }
 
-__global__ void __launch_bounds__(256) attn_rows_kernel(AttnRowsArgs a) {
+// BS = 1024 for the few rows of a decode step: every thread's loads are in flight at once
+template <int BS>
+__global__ void __launch_bounds__(BS) attn_rows_kernel(AttnRowsArgs a) {
     extern __shared__ __attribute__((aligned(16))) float xr[];
-    __shared__ float red[8];
+    __shared__ float red[2 * BS / 64];
     const int row = blockIdx.x;
     const int nq = a.heads * a.kv.dim, nk = a.kv.kv * a.kv.dim, nv = a.kv.kv * a.kv.vdim;
     sum_row(xr, a.in + (size_t)row * a.ld, (nq + nk + nv + 3) & ~3, a.n_slabs, a.slab_stride, a.bias);
@@ -66,14 +68,15 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(AttnRowsArgs a) {
         sq = a.ssq[row * 2];
         sk = a.ssq[row * 2 + 1];
     } else {
-        for (int c = threadIdx.x; c < nq; c += 256) sq += xr[c] * xr[c];
-        for (int c = threadIdx.x; c < nk; c += 256) sk += xr[nq + c] * xr[nq + c];
+        for (int c = threadIdx.x; c < nq; c += BS) sq += xr[c] * xr[c];
+        for (int c = threadIdx.x; c < nk; c += BS) sk += xr[nq + c] * xr[nq + c];
         sq = wave_sum_uniform(sq);
         sk = wave_sum_uniform(sk);
-        if ((threadIdx.x & 63) == 0) { red[threadIdx.x >> 6] = sq; red[4 + (threadIdx.x >> 6)] = sk; }
+        if ((threadIdx.x & 63) == 0) { red[threadIdx.x >> 6] = sq; red[BS / 64 + (threadIdx.x >> 6)] = sk; }
         __syncthreads();
-        sq = (red[0] + red[1]) + (red[2] + red[3]);
-        sk = (red[4] + red[5]) + (red[6] + red[7]);
+        sq = sk = 0.f;
+#pragma unroll
+        for (int w = 0; w < BS / 64; ++w) { sq += red[w]; sk += red[BS / 64 + w]; }
     }
     const float rq = 1.0f / sqrtf(sq / (float)a.q_all + a.eps), rk = 1.0f / sqrtf(sk / (float)a.k_all + a.eps);
     float* q = a.q + (size_t)row * a.heads * a.kv.dim_p;
@@ -81,7 +84,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(AttnRowsArgs a) {
     const size_t blk = (size_t)a.block_tables[(size_t)a.slot[row] * a.max_blocks + pos / kBlockTokens] * a.kv.kv;
     if (((a.kv.dim | a.kv.vdim) & 3) == 0) {  // four columns of one head per thread
         const int d4 = a.kv.dim_p >> 2, k4 = a.kv.dim >> 2, v4 = a.kv.vdim >> 2;
-        for (int i = threadIdx.x; i < a.heads * d4; i += 256) {
+        for (int i = threadIdx.x; i < a.heads * d4; i += BS) {
             const int h = i / d4, d = (i - h * d4) * 4, c = h * a.kv.dim + d;
             float4 y = make_float4(0.f, 0.f, 0.f, 0.f);
             if (d < a.kv.dim) {
@@ -90,7 +93,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(AttnRowsArgs a) {
             }
             reinterpret_cast<float4*>(q)[i] = y;
         }
-        for (int i = threadIdx.x; i < a.kv.kv * k4; i += 256) {
+        for (int i = threadIdx.x; i < a.kv.kv * k4; i += BS) {
             const int h = i / k4, d = (i - h * k4) * 4, c = h * a.kv.dim + d;
             const float4 x = *reinterpret_cast<const float4*>(xr + nq + c), w = *reinterpret_cast<const float4*>(a.kn + c);
             const float y[4] = {(x.x * rk) * w.x, (x.y * rk) * w.y, (x.z * rk) * w.z, (x.w * rk) * w.w};
@@ -102,7 +105,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(AttnRowsArgs a) {
             }
         }
         const float lam = a.mix == 2 ? a.lambda[0] : 0.f;
-        for (int i = threadIdx.x; i < a.kv.kv * v4; i += 256) {
+        for (int i = threadIdx.x; i < a.kv.kv * v4; i += BS) {
             const int h = i / v4, d = (i - h * v4) * 4, c = h * a.kv.vdim + d;
             float4 x = *reinterpret_cast<const float4*>(xr + nq + nk + c);
             float4* vf = reinterpret_cast<float4*>(a.v_first + (size_t)row * nv + c);
@@ -119,16 +122,16 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(AttnRowsArgs a) {
         }
         return;
     }
-    for (int i = threadIdx.x; i < a.heads * a.kv.dim_p; i += 256) {
+    for (int i = threadIdx.x; i < a.heads * a.kv.dim_p; i += BS) {
         const int h = i / a.kv.dim_p, d = i - h * a.kv.dim_p, c = h * a.kv.dim + d;
         q[i] = d < a.kv.dim ? (xr[c] * rq) * a.qn[c] * a.q_scale : 0.f;
     }
-    for (int c = threadIdx.x; c < nk; c += 256) {
+    for (int c = threadIdx.x; c < nk; c += BS) {
         const int h = c / a.kv.dim, d = c - h * a.kv.dim;
         kv_put(a.kv.k, a.kv.f32, (blk + h) * kBlockTokens * a.kv.dim_p + k_packed_offset(t, d, a.kv.dim_p), (xr[nq + c] * rk) * a.kn[c]);
     }
     const float lam = a.mix == 2 ? a.lambda[0] : 0.f;
-    for (int c = threadIdx.x; c < nv; c += 256) {
+    for (int c = threadIdx.x; c < nv; c += BS) {
         const int h = c / a.kv.vdim, d = c - h * a.kv.vdim;
         float v = xr[nq + nk + c];
         if (a.mix == 1) a.v_first[(size_t)row * nv + c] = v;
@@ -224,14 +227,15 @@ hipError_t launch_attn_rows(const AttnRowsArgs& a, int rows, hipStream_t s) {
     if (lds > 64 * 1024) return hipErrorNotSupported;
     if (rows <= 0) return hipSuccess;
     const size_t lds4 = (size_t)4 * a.kv.kv * a.kv.vdim * 4;
-    if (rows >= 64 && !a.kv.f32 && ((a.kv.dim | a.kv.vdim) & 3) == 0 && (a.slab_stride & 3) == 0 && n <= 24 * 256 && lds4 <= 64 * 1024) {
+    if (rows > 128 && !a.kv.f32 && ((a.kv.dim | a.kv.vdim) & 3) == 0 && (a.slab_stride & 3) == 0 && n <= 24 * 256 && lds4 <= 64 * 1024) {
         const int wgs = (rows + 3) / 4;
         if (n <= 8 * 256) attn_rows4_kernel<8><<<wgs, 256, lds4, s>>>(a, rows);
         else if (n <= 16 * 256) attn_rows4_kernel<16><<<wgs, 256, lds4, s>>>(a, rows);
         else attn_rows4_kernel<24><<<wgs, 256, lds4, s>>>(a, rows);
         return hipGetLastError();
     }
-    attn_rows_kernel<<<rows, 256, lds, s>>>(a);
+    if (rows <= 128 && n > 1024) attn_rows_kernel<1024><<<rows, 1024, lds, s>>>(a);
+    else attn_rows_kernel<256><<<rows, 256, lds, s>>>(a);
     return hipGetLastError();
 }
 

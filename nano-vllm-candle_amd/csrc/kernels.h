@@ -302,7 +302,7 @@ bool gemm_rowdir_ok(int N, int K, int epi, int M);
 bool gemm_rowpar_ok(int N, int K, int epi, int M);
 int gemm_rowpar_splits(int N, int K, int epi, int M);  // f32 slabs the plain epilogue leaves (1 = complete sums)
 int gemm_rowpar_groups(int N, int K);
-// epi: 0 residual + next-norm prep, 1 SwiGLU, 2 plain f32 output
+// epi: 0 residual + next-norm prep, 1 SwiGLU, 2 plain f32 output, 3 squared ReLU as planes oh / ol (register-direct kernel only)
 hipError_t launch_gemm_rowpar(const RowParArgs& a, const PackedW& w, int epi, hipStream_t s);
 
 // ---- SwiGLU -----------------------------------------------------------------------------------------

@@ -1157,6 +1157,16 @@ __global__ void __launch_bounds__(NWK * 64) gemm_rowdir_kernel(RowParArgs a, con
             *reinterpret_cast<uint2*>(a.oh + o) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
             *reinterpret_cast<uint2*>(a.ol + o) = make_uint2(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16));
         }
+    } else if constexpr (EPI == 3) {
+        if (fin && row < M) {
+            uint16_t h[4], l[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) split_bf16(relu2(sum[r]), h[r], l[r]);
+            const int f0 = ntile * 16 + grp * 4;
+            const size_t o = a.o_packed ? xpack_off(row, f0, N >> 5) : (size_t)row * N + f0;
+            *reinterpret_cast<uint2*>(a.oh + o) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
+            *reinterpret_cast<uint2*>(a.ol + o) = make_uint2(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16));
+        }
     } else {
         if (fin && row < M)
             *reinterpret_cast<float4*>(a.out + (size_t)row * N + (size_t)ntile * 16 + grp * 4) = make_float4(sum[0], sum[1], sum[2], sum[3]);
@@ -1200,7 +1210,7 @@ struct RowParShape { int mt, nwn, nwk, tpw, ph, ns; };
 //   big matrices (>= 24 MB): all rows (up to 64) in one workgroup so every weight byte crosses L2 once, K sliced
 //   into <= 1024-deep pieces over blockIdx.y (plain epilogue only: the slices leave f32 slabs).
 static bool rowpar_shape(int N, int K, int epi, int M, RowParShape& sh) {
-    if (N % 16 || K % 32) return false;
+    if (N % 16 || K % 32 || epi == 3) return false;
     const int KT = K / 32, ntiles = N / 16;
     const bool big = (size_t)N * K * 2 >= (size_t)24 << 20 && M > 16;
     static const int tpws[] = {8, 12, 16};
@@ -1269,7 +1279,7 @@ static hipError_t rowdir_dispatch(const RowDirShape& d, const RowParArgs& a, con
 #define NVLLM_RD(NT_, TK_) if (d.nt == NT_ && d.tk == TK_) return rowdir_launch_t<NT_, 16, TK_, EPI>(a, w, s);
     if constexpr (EPI == 0) { NVLLM_RD(1, 2) NVLLM_RD(1, 4) NVLLM_RD(1, 6) NVLLM_RD(1, 8) NVLLM_RD(2, 2) NVLLM_RD(2, 4) NVLLM_RD(2, 6) NVLLM_RD(4, 2) NVLLM_RD(4, 4) }
     if constexpr (EPI == 1) { NVLLM_RD(6, 2) NVLLM_RD(4, 2) NVLLM_RD(4, 4) NVLLM_RD(2, 2) NVLLM_RD(2, 4) NVLLM_RD(2, 6) NVLLM_RD(2, 8) }
-    if constexpr (EPI == 2) { NVLLM_RD(4, 2) NVLLM_RD(4, 4) NVLLM_RD(2, 6) NVLLM_RD(2, 8) NVLLM_RD(1, 2) NVLLM_RD(1, 4) NVLLM_RD(1, 6) NVLLM_RD(1, 8) }
+    if constexpr (EPI >= 2) { NVLLM_RD(4, 2) NVLLM_RD(4, 4) NVLLM_RD(2, 6) NVLLM_RD(2, 8) NVLLM_RD(1, 2) NVLLM_RD(1, 4) NVLLM_RD(1, 6) NVLLM_RD(1, 8) }
 #undef NVLLM_RD
     return hipErrorNotSupported;
 }
@@ -1310,6 +1320,7 @@ hipError_t launch_gemm_rowpar(const RowParArgs& a, const PackedW& w, int epi, hi
         if (epi == 0) return rowdir_dispatch<0>(d, a, w, s);
         if (epi == 1) return rowdir_dispatch<1>(d, a, w, s);
         if (epi == 2) return rowdir_dispatch<2>(d, a, w, s);
+        if (epi == 3 && a.oh && (!a.o_packed || w.N % 32 == 0)) return rowdir_dispatch<3>(d, a, w, s);
         return hipErrorInvalidValue;
     }
     if (a.x_packed || a.o_packed) return hipErrorNotSupported;  // packed planes: register-direct kernel only
