@@ -8,7 +8,7 @@ import numpy as np
 
 from bench_berevik import HBM_GBS, MFMA_TFLOPS, measure, rooflines
 
-VALU_TFLOPS = 78.6  # f32 vector rate without packed instructions: 256 CUs x 128 flop x 2.4 GHz
+F32_TFLOPS = 157.3  # f32 matrix rate: the recurrences are computed in 32-bit
 
 # width, heads (all of 128), kv heads of the attention layers and of the Qwen3 twin, feed-forward width of the twin (two thirds of a
 # two-matrix feed-forward of equal parameters), layers
@@ -39,11 +39,11 @@ def gopunex_config(pkg, z, kind, vocab):
 
 
 def recurrence_rooflines(r, z, kind, batch, prompt):
-    """decode: the state read and written once over HBM; prefill: the token recurrence's own multiply-adds over the f32 vector rate"""
+    """decode: the state read and written once over HBM; prefill: the token recurrence's own operations over the f32 matrix rate"""
     elems = z["heads"] * 128 * 128
     r["decode_recur_hbm_frac"] = round(z["layers"] * batch * elems * 8 / (r["decode_class_ms"]["recur"][0] * 1e-3) / 1e9 / HBM_GBS, 4)
     flops = (7 if kind == "channel_delta" else 5) * elems
-    r["prefill_recur_valu_frac"] = round(z["layers"] * batch * prompt * flops / (r["prefill_class_ms"]["recur"][0] * 1e-3) / 1e12 / VALU_TFLOPS, 4)
+    r["prefill_recur_f32_frac"] = round(z["layers"] * batch * prompt * flops / (r["prefill_class_ms"]["recur"][0] * 1e-3) / 1e12 / F32_TFLOPS, 4)
 
 
 def main(sizes=None, batch=64, prompt=1024, steps=32, vocab=32768, mixers=MIXERS, with_qwen=True):

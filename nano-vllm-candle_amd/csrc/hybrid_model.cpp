@@ -76,7 +76,7 @@ struct HybridModel : DecoderImpl {
     int recurrence(nvllm_model* m, HybridLayer& w, int ns, int R, int qt, int ctx_packed);
 };
 
-constexpr int kDecodeWgs = 1024;  // workgroups the split of a decode step's context aims at
+constexpr int kDecodeWgs = 512;  // workgroups the split of a decode step's context aims at
 
 // row of the distance table
 static int distance_bucket(int n, int rows, double far) {

@@ -44,7 +44,11 @@ SIZES = config([attn(heads=4, kv=2, dim=d, vdim=v, ff=0, v_mix=False) for d, v i
 # no attention at all
 STATE = config([delta(), light(ff=0), delta(heads=2, kv=2, conv=3)])
 
-CONFIGS = {"mixed": MIXED, "even": EVEN, "one": ONE, "wide": WIDE, "sizes": SIZES, "state": STATE}
+# key sizes whose padding is no power of two, and above what runs in pieces
+KEYS = config([delta(heads=2, kv=2, dim=190, vdim=40, conv=3, ff=0), light(heads=2, dim=140, vdim=96, ff=0), delta(heads=1, kv=1, dim=400, vdim=50),
+               light(heads=1, dim=512, vdim=17, decay=[0.95])], width=100, vocab=64)
+
+CONFIGS = {"mixed": MIXED, "even": EVEN, "one": ONE, "wide": WIDE, "sizes": SIZES, "state": STATE, "keys": KEYS}
 TOL = {"bfloat16": 4e-3, "float32": 3e-5}
 
 

@@ -72,7 +72,8 @@ def test_missing_library_raises(monkeypatch, tmp_path):
 
 def _kernel_resources():
     out = {}
-    for name in ("kernel_resources.txt", "kernel_resources_tile.txt", "kernel_resources_latent.txt", "kernel_resources_latent_prefill.txt"):
+    for name in ("kernel_resources.txt", "kernel_resources_tile.txt", "kernel_resources_latent.txt", "kernel_resources_latent_prefill.txt", "kernel_resources_bias_attn.txt",
+                 "kernel_resources_recurrent.txt", "kernel_resources_recurrent_chunk.txt"):
         path = os.path.join(ROOT, "nano-vllm-candle_amd", name)
         if not os.path.exists(path):
             pytest.skip(name + " missing: rebuild the library (make -C nano-vllm-candle_amd/csrc)")
@@ -122,3 +123,19 @@ def test_latent_attention_kernels_stay_in_registers():
         assert r["ScratchSize [bytes/lane]"] == 0, (n, r)
         if "latent_attn_kernel" in n or "latent_prefill_kernel" in n:
             assert r["Occupancy [waves/SIMD]"] >= 2, (n, r)
+
+
+def test_bias_attention_and_recurrence_kernels_stay_in_registers():
+    # prompt kernels read LDS by inline asm: a destination spilled while its read is in flight would lose the data, so no instance may
+    # use scratch; the token-by-token scan may for key sizes above 256
+    res = _kernel_resources()
+    for part, count in (("bias_prefill_kernel", 20), ("bias_decode_kernel", 20), ("piece_scan_kernel", 24), ("delta_pieces_kernel", 4)):
+        hits = {n: r for n, r in res.items() if part in n}
+        assert len(hits) == count, (part, len(hits))
+        for n, r in hits.items():
+            assert r["ScratchSize [bytes/lane]"] == 0, (n, r)
+    for n, r in res.items():
+        if "bias_prefill_kernelILi4ELi8" in n or "bias_decode_kernelILi4ELi8" in n:
+            assert r["Occupancy [waves/SIMD]"] >= 2, (n, r)
+        if "recurrence_decode_kernelILi2" in n:
+            assert r["Occupancy [waves/SIMD]"] >= 4 and r["ScratchSize [bytes/lane]"] == 0, (n, r)

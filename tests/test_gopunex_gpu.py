@@ -81,7 +81,7 @@ def test_one_mechanism(what, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["mixed", "even", "wide", "one", "sizes"])
+@pytest.mark.parametrize("name", ["mixed", "even", "wide", "one", "sizes", "keys"])
 def test_portions_and_decoding_equal_the_whole_prompt(name, dtype):
     cfg = CONFIGS[name]
     w = sharp_weights(cfg, 1)
@@ -173,7 +173,7 @@ def test_state_carries_far(dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["mixed", "even", "wide", "state"])
+@pytest.mark.parametrize("name", ["mixed", "even", "wide", "state", "keys"])
 def test_recurrences_token_by_token_and_in_pieces(name, dtype):
     # prompt portions in pieces of 16 tokens and by the scan, each continuing from the state the other left
     cfg = CONFIGS[name]
