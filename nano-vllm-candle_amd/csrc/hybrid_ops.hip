@@ -301,7 +301,8 @@ hipError_t launch_linear_rows(const LinearRowsArgs& a, int rows, hipStream_t s) 
 }
 
 // ---------------------------------------------------------------------------------------------------
-// delta rule: one wave per (row, unit); units = q heads, k heads, v heads, then one for beta and the gate inputs
+// delta rule: one wave per (row, unit); units = q heads, k heads, v heads, then one for beta and the gate inputs.  The form for any
+// size of prompt chunk first, then those of decode and of long chunks.
 // ---------------------------------------------------------------------------------------------------
 // what a row sees of the tokens before its chunk: rows back to its segment's start, then the slot's history
 struct RowPast {
@@ -313,8 +314,7 @@ __device__ __forceinline__ RowPast row_past(const DeltaRowsArgs& a, int row) {
     RowPast p;
     p.slot = a.slot[row];
     const int pos = a.pos[row];
-    if (!a.seg.single)
-        while (p.in_chunk < a.taps - 1 && row - p.in_chunk - 1 >= 0 && a.slot[row - p.in_chunk - 1] == p.slot) ++p.in_chunk;
+    while (p.in_chunk < a.taps - 1 && row - p.in_chunk - 1 >= 0 && a.slot[row - p.in_chunk - 1] == p.slot) ++p.in_chunk;
     p.pos0 = pos - p.in_chunk;
     return p;
 }
@@ -360,15 +360,75 @@ __global__ void __launch_bounds__(256) delta_rows_kernel(DeltaRowsArgs a) {
         for (int h = lane; h < a.heads; h += 64) a.beta[(size_t)row * a.heads + h] = sigmoidf(slab_elem(in + h, a.n_slabs, a.slab_stride));
         for (int i = lane; i < 2 * a.rank_p; i += 64) a.gate_in[(size_t)row * 2 * a.rank_p + i] = slab_elem(in + a.heads + i, a.n_slabs, a.slab_stride);
     }
-    if (!a.seg.single || a.taps < 2) return;
-    // decode: the next half of the history = this half moved on by one token
-    const int pos = a.pos[row];
-    const int c0 = unit < 2 * a.kv ? unit * a.dim : 2 * a.kv * a.dim + (unit - 2 * a.kv) * a.vdim;
-    const int n = unit < 2 * a.kv ? a.dim : unit < 2 * a.kv + a.heads ? a.vdim : 0;
-    float* next = a.history + ((size_t)((pos + 1) & 1) * a.slots + p.slot) * (a.taps - 1) * channels;
-    for (int d = lane; d < n; d += 64)
-        for (int i = 0; i < a.taps - 1; ++i) next[(size_t)i * channels + c0 + d] = past_input(a, p, row, a.taps - 2 - i, c0 + d, channels);
 }
+
+// decode: every input is read once, for the convolution and for the history's next half (this half moved on by one token)
+template <int TAPS, int NE>
+__global__ void __launch_bounds__(256) delta_rows_decode_kernel(DeltaRowsArgs a) {
+    const int lane = threadIdx.x & 63, row = blockIdx.x, unit = blockIdx.y * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int channels = 2 * a.kv * a.dim + a.heads * a.vdim;
+    if (unit > 2 * a.kv + a.heads) return;
+    if (unit == 2 * a.kv + a.heads) {
+        const float* in = a.in + (size_t)row * a.ld + channels;
+        for (int i = lane; i < a.heads + 2 * a.rank_p; i += 64) {
+            const float x = slab_elem(in + i, a.n_slabs, a.slab_stride);
+            if (i < a.heads) a.beta[(size_t)row * a.heads + i] = sigmoidf(x);
+            else a.gate_in[(size_t)row * 2 * a.rank_p + i - a.heads] = x;
+        }
+        return;
+    }
+    const int slot = a.slot[row], pos = a.pos[row];
+    const bool qk = unit < 2 * a.kv;
+    const int n = qk ? a.dim : a.vdim, n_p = qk ? a.dim_p : a.vdim_p;
+    const int c0 = qk ? unit * a.dim : 2 * a.kv * a.dim + (unit - 2 * a.kv) * a.vdim;
+    const int hd = qk ? unit % a.kv : unit - 2 * a.kv, hs = qk ? a.kv : a.heads;
+    float* out = (qk ? (unit < a.kv ? a.q : a.k) : a.v) + ((size_t)row * hs + hd) * n_p;
+    const float* in = a.in + (size_t)row * a.ld + c0;
+    const float* past = a.history + ((size_t)(pos & 1) * a.slots + slot) * (TAPS - 1) * channels + c0;
+    float* next = a.history + ((size_t)((pos + 1) & 1) * a.slots + slot) * (TAPS - 1) * channels + c0;
+    for (int d0 = 0; d0 < n_p; d0 += 64 * NE) {  // once for q and k (dim_p <= 64 NE): their norm needs the whole head
+        float x[TAPS][NE], y[NE], ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < NE; ++e) {
+            const int d = min(d0 + e * 64 + lane, n - 1);
+            x[TAPS - 1][e] = slab_elem(in + d, a.n_slabs, a.slab_stride);
+#pragma unroll
+            for (int i = 0; i < TAPS - 1; ++i) {
+                const float h = past[(size_t)i * channels + d];
+                x[i][e] = pos >= TAPS - 1 - i ? h : 0.f;
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < NE; ++e) {
+            const int d = d0 + e * 64 + lane;
+            float t = 0.f;
+#pragma unroll
+            for (int i = 0; i < TAPS; ++i) t += x[i][e] * a.conv[(size_t)i * channels + c0 + min(d, n - 1)];
+            y[e] = d < n ? t * sigmoidf(t) : 0.f;
+            ss += y[e] * y[e];
+            if (d < n) {
+#pragma unroll
+                for (int i = 0; i < TAPS - 1; ++i) next[(size_t)i * channels + d] = x[i + 1][e];
+            }
+        }
+        const float f = qk ? (unit < a.kv ? a.q_scale : 1.f) / sqrtf(wave_sum_uniform(ss) + kUnitNormEps) : 1.f;
+#pragma unroll
+        for (int e = 0; e < NE; ++e)
+            if (d0 + e * 64 + lane < n_p) out[d0 + e * 64 + lane] = y[e] * f;
+    }
+}
+template <int NE>
+static bool delta_rows_decode(const DeltaRowsArgs& a, int rows, hipStream_t s) {
+    const dim3 grid(rows, (2 * a.kv + a.heads + 1 + 3) / 4);
+    switch (a.taps) {
+#define NVLLM_DD(T_) case T_: delta_rows_decode_kernel<T_, NE><<<grid, 256, 0, s>>>(a); return true;
+        NVLLM_DD(1) NVLLM_DD(2) NVLLM_DD(3) NVLLM_DD(4) NVLLM_DD(5) NVLLM_DD(6) NVLLM_DD(7) NVLLM_DD(8)
+        NVLLM_DD(9) NVLLM_DD(10) NVLLM_DD(11) NVLLM_DD(12) NVLLM_DD(13) NVLLM_DD(14) NVLLM_DD(15) NVLLM_DD(16)
+#undef NVLLM_DD
+    }
+    return false;
+}
+
 // prompt chunks: one wave per (16 rows, unit), the convolution's window in registers
 template <int TAPS, int NE>
 __global__ void __launch_bounds__(256) delta_rows16_kernel(DeltaRowsArgs a, int rows) {
@@ -485,6 +545,11 @@ hipError_t launch_delta_rows(const DeltaRowsArgs& a, int rows, hipStream_t s) {
         const bool done = a.dim_p == 64 ? delta_rows16<1>(a, rows, s) : a.dim_p == 128 ? delta_rows16<2>(a, rows, s) : a.dim_p == 256 ? delta_rows16<4>(a, rows, s) : false;
         if (done) return hipGetLastError();
     }
+    if (a.seg.single) {
+        const bool done = a.dim_p <= 64 ? delta_rows_decode<1>(a, rows, s) : a.dim_p <= 128 ? delta_rows_decode<2>(a, rows, s)
+                        : a.dim_p <= 256 ? delta_rows_decode<4>(a, rows, s) : delta_rows_decode<8>(a, rows, s);
+        return done ? hipGetLastError() : hipErrorNotSupported;
+    }
     const dim3 grid(rows, (2 * a.kv + a.heads + 1 + 3) / 4);
     if (a.dim_p <= 64) delta_rows_kernel<1><<<grid, 256, 0, s>>>(a);
     else if (a.dim_p <= 128) delta_rows_kernel<2><<<grid, 256, 0, s>>>(a);
@@ -525,11 +590,29 @@ hipError_t launch_delta_history(const DeltaRowsArgs& a, hipStream_t s) {
 // second step of the gate projections over prompt chunks: one workgroup = 64 rows x a slice of one gate's features; the rows' operand
 // is built once in LDS as bf16 hi + lo fragments, each wave streams its share of the weight fragments
 // ---------------------------------------------------------------------------------------------------
+// exp(x) for decays and gates: the argument's rounding costs |x| 2^-24 of the result
+__device__ __forceinline__ float exp_fast(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
+// log(1 + e^z) = max(z, 0) + log1p(e^-|z|) with log1p(t) = log(u) t / (u - 1), u = 1 + t rounded: the quotient undoes u's rounding
+__device__ __forceinline__ float softplus_fast(float z) {
+    const float t = exp_fast(-fabsf(z)), u = 1.0f + t, d = u - 1.0f;
+    const float l = __builtin_amdgcn_logf(u) * 0.6931471805599453f;
+    return fmaxf(z, 0.f) + (d == 0.f ? t : l * (t * __builtin_amdgcn_rcpf(d)));
+}
+__device__ __forceinline__ float sigmoid_fast(float x) { return __builtin_amdgcn_rcpf(1.0f + exp_fast(-x)); }
+
 template <int KT>
 __global__ void __launch_bounds__(256) delta_gates_kernel(HeadGemmArgs a) {
     __shared__ __attribute__((aligned(16))) uint4 xs[2 * 4 * KT * 64];  // [plane][row tile][k-tile][lane]
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, grp = lane >> 4;
     const int row0 = blockIdx.x * 64, head = blockIdx.y;
+    const uint4* w = a.w + (size_t)head * a.w_head;
+    const int ntiles = a.N >> 4;
+    uint4 wn[KT];  // the next tile's weights
+    auto fetch = [&](int nt) {
+#pragma unroll
+        for (int k = 0; k < KT; ++k) wn[k] = w[((size_t)min(nt, ntiles - 1) * KT + k) * 64 + lane];
+    };
+    fetch(blockIdx.z * 4 + wave);
     for (int i = wave; i < 4 * KT; i += 4) {
         const int row = min(row0 + (i / KT) * 16 + l15, a.M - 1);
         const float* p = a.x + (size_t)row * a.x_row + (size_t)head * a.x_head + (i % KT) * 32 + grp * 8;
@@ -546,14 +629,6 @@ __global__ void __launch_bounds__(256) delta_gates_kernel(HeadGemmArgs a) {
         xs[(4 * KT + i) * 64 + lane] = __builtin_bit_cast(uint4, l);
     }
     __syncthreads();
-    const uint4* w = a.w + (size_t)head * a.w_head;
-    const int ntiles = a.N >> 4;
-    uint4 wn[KT];  // the next tile's weights
-    auto fetch = [&](int nt) {
-#pragma unroll
-        for (int k = 0; k < KT; ++k) wn[k] = w[((size_t)min(nt, ntiles - 1) * KT + k) * 64 + lane];
-    };
-    fetch(blockIdx.z * 4 + wave);
     for (int nt = blockIdx.z * 4 + wave; nt < ntiles; nt += 4 * gridDim.z) {
         uint4 wf[KT];
 #pragma unroll
@@ -581,18 +656,21 @@ __global__ void __launch_bounds__(256) delta_gates_kernel(HeadGemmArgs a) {
             const int row = row0 + b * 16 + l15;
             const f32x4 v = acc[b];
             float4 o;
-            if (head == 0) o = make_float4(expf(-rate.x * softplusf(v[0] + dt.x)), expf(-rate.y * softplusf(v[1] + dt.y)),
-                                           expf(-rate.z * softplusf(v[2] + dt.z)), expf(-rate.w * softplusf(v[3] + dt.w)));
-            else o = make_float4(sigmoidf(v[0]), sigmoidf(v[1]), sigmoidf(v[2]), sigmoidf(v[3]));
+            if (head == 0) o = make_float4(exp_fast(-rate.x * softplus_fast(v[0] + dt.x)), exp_fast(-rate.y * softplus_fast(v[1] + dt.y)),
+                                           exp_fast(-rate.z * softplus_fast(v[2] + dt.z)), exp_fast(-rate.w * softplus_fast(v[3] + dt.w)));
+            else o = make_float4(sigmoid_fast(v[0]), sigmoid_fast(v[1]), sigmoid_fast(v[2]), sigmoid_fast(v[3]));
             if (row < a.M) *reinterpret_cast<float4*>(a.y + (size_t)row * a.y_row + (size_t)head * a.y_head + f0) = o;
         }
     }
 }
 hipError_t launch_delta_gates(const HeadGemmArgs& a, hipStream_t s) {
     const int kt = a.K / 32;
-    if (a.exact || a.M < 512 || kt > 4 || a.N % 16 || a.K % 32 || a.x_row % 4 || a.x_head % 4 || a.y_row % 4 || a.y_head % 4 || a.n_valid != a.N || !a.decay_rate)
+    if (a.exact || kt > 4 || a.N % 16 || a.K % 32 || a.x_row % 4 || a.x_head % 4 || a.y_row % 4 || a.y_head % 4 || a.n_valid != a.N || !a.decay_rate)
         return launch_head_gemm(a, s);
-    const dim3 grid((a.M + 63) / 64, a.heads, std::max(1, std::min(8, a.N / 16 / 16)));
+    if (a.M <= 0) return hipSuccess;
+    // eight slices per row block for prompt chunks, for few rows one tile per wave
+    const int blocks = (a.M + 63) / 64, tiles = a.N / 16;
+    const dim3 grid(blocks, a.heads, std::max(1, std::min((tiles + 3) / 4, std::max(8, 256 / (blocks * a.heads)))));
     if (kt == 1) delta_gates_kernel<1><<<grid, 256, 0, s>>>(a);
     else if (kt == 2) delta_gates_kernel<2><<<grid, 256, 0, s>>>(a);
     else if (kt == 3) delta_gates_kernel<3><<<grid, 256, 0, s>>>(a);
