@@ -18,7 +18,7 @@ struct DecoderImpl {
     virtual int64_t kv_read_bytes(int len) const = 0;  // cache (and state) bytes a decode step moves for a sequence of len tokens
     virtual int tile_rows(int qt) const = 0;           // rows of a q-tile (qt = 1: decode)
     virtual bool recurrent() const { return false; }   // carries state that cannot step back: such a step starts the sequence again
-    // metadata of the chunk about to run beyond the q-tiles (R rows; tiles already uploaded); also called for rebuilt decode batches
+    // metadata of the chunk about to run beyond the q-tiles (R rows; tiles already uploaded); decode continued on the device needs none
     virtual int plan_chunk(nvllm_model* m, const int* pos, const int* slot, const int* seq, int R, const int* tile_row0, int n_tiles, int qt) = 0;
     virtual int forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n_last, int logits_row0) = 0;
     virtual int option(const char* name, int value) { (void)name; (void)value; return 1; }        // 0: taken
