@@ -109,24 +109,45 @@ int64_t nvllm_model_weight_bytes(const nvllm_model* m);
  * (src/tp.rs:59-65; src/layers/linear.rs:80-89,201-210 only work for rank 0). */
 int nvllm_tp_shard(const nvllm_qwen3_config* cfg, int tp_size, int tp_rank, const char* hf_name, int64_t out_region[4]);
 
-/* ---- latent-attention decoders: layers of windowed latent attention beside a gated feed-forward (parallel branches, two
- * norms), an optional looped range of layers, scaled embeddings and a soft-capped head.  Everything below the create call
- * (loading, pool, step, sampling, decode) is the same API as the Qwen3 model's. */
+/* ---- latent-attention decoders: layers of parallel branches -- a token mixer (windowed latent attention or a selective scan) beside a
+ * feed-forward (gated, or routed experts) -- each with a norm of its own or both on one norm, an optional looped range of layers, scaled
+ * embeddings and a soft-capped head.  Everything below the create call (loading, pool, step, sampling, decode) is the same API as the
+ * Qwen3 model's; the state of a scan lives in the sequence's slot, and a step that asks for a sequence shorter than what was processed
+ * starts it again. */
+#define NVLLM_LATENT_ATTENTION 0
+#define NVLLM_SELECTIVE_SCAN 1  /* x: short convolution + silu; S = exp(dt A) S + dt x B^T, y = S C + D x, gated by silu(z) */
+#define NVLLM_GLU_CLAMPED 0     /* g = min(g, limit), u = clamp(u), y = g sigmoid(alpha g) (u + shift) */
+#define NVLLM_GLU_GELU 1        /* tanh form of gelu(g) times u */
 typedef struct nvllm_latent_layer {
+    int32_t mixer;                              /* NVLLM_LATENT_ATTENTION or NVLLM_SELECTIVE_SCAN */
     int32_t heads, dim, rot_dim, vdim, kv_rank; /* per head: unrotated, rotated query/key and value sizes; latent size */
     int32_t window;                             /* visible positions including the token itself; <= 0: all earlier ones */
-    double rot_base, scale;                     /* rotation base (rotate-half over the whole rotated part), score scale */
-    int32_t ff;                                 /* feed-forward width, 0 = the layer has none */
-    double glu_limit, glu_alpha, glu_shift;     /* g = min(g, limit), u = clamp(u), y = g sigmoid(alpha g) (u + shift) */
+    int32_t q_rank;                             /* > 0: queries go through a normed latent of this size */
+    int32_t kv_from;                            /* >= 0: reads the cache of that earlier layer (no latent projection of its own); < 0: its own */
+    int32_t sink;                               /* one learned term per head in the softmax's denominator */
+    int32_t rot_pairs;                          /* 0: dimension i turns with i + rot_dim / 2; 1: 2 i with 2 i + 1 */
+    double rot_base, scale;                     /* rotation base (over the whole rotated part), score scale */
+    double yarn_factor, yarn_original, yarn_fast, yarn_slow; /* YaRN scaling of the rotation; factor <= 0: none */
+    int32_t inner, state, conv_taps, dt_rank;   /* selective scan: channels, states per channel, taps of the convolution, rank of the step sizes */
+    int32_t ff;                                 /* gated feed-forward width, 0 = the layer has none */
+    int32_t glu;                                /* NVLLM_GLU_* */
+    double glu_limit, glu_alpha, glu_shift;
+    int32_t experts, top;                       /* routed feed-forward (ff = 0): experts and how many a token uses; 0: none */
+    int32_t expert_ff, shared_ff;               /* widths of an expert and of the shared, sigmoid-gated one (0: none); squared ReLU */
+    int32_t expert_weight_in;                   /* 1: the sigmoid score multiplies the expert's input, 0: its output */
 } nvllm_latent_layer;
+#define NVLLM_NORM_RMS 0
+#define NVLLM_NORM_LAYER 1  /* mean taken off first */
 typedef struct nvllm_latent_config {
     int32_t vocab_size, width, num_layers;
     int32_t loop_start, loop_stop, loop_times;  /* layers [start, stop) are passed through loop_times times before the rest; <= 1: no loop */
     double norm_eps, embed_scale, logit_softcap; /* softcap <= 0: none */
+    int32_t norm, one_norm;                     /* NVLLM_NORM_*; 1: both branches of a layer read norm1 */
     int32_t f32;                                /* 0: bf16 weights, hi + lo planes, f16 cache; 1: every product and the cache in f32 */
 } nvllm_latent_config;
-/* Tensor names for nvllm_model_load_tensor: embed, head, final.norm and, per layer, l<i>.norm1, l<i>.norm2, l<i>.mix.{q, dkv,
- * dkv.norm, uk, uv, o}, l<i>.mlp.{gate, up, down}. */
+/* Tensor names for nvllm_model_load_tensor: embed, head, final.norm and, per layer, l<i>.norm1, l<i>.norm2 (unless one_norm),
+ * l<i>.mix.{q (or dq, dq.norm, uq), dkv, dkv.norm (unless kv_from >= 0), uk, uv, sink, o} or l<i>.mix.{in, conv, conv.b, x, dt, dt.b, A_log,
+ * D, o}, and l<i>.mlp.{gate, up, down} or l<i>.mlp.{router, e<k>.up, e<k>.down, shared.up, shared.down, shared.sg}. */
 int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_config* cfg, const nvllm_latent_layer* layers, nvllm_model** out);
 
 /* ---- hybrid decoders: every layer has one of three token mixers and optionally a squared-ReLU feed-forward; sublayers read the

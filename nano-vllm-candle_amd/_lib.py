@@ -40,18 +40,18 @@ class Qwen3ConfigC(C.Structure):
 class LatentLayerC(C.Structure):
     """nvllm_latent_layer"""
 
-    _fields_ = [(n, C.c_int32) for n in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "window")] + [
-        ("rot_base", C.c_double), ("scale", C.c_double), ("ff", C.c_int32),
-        ("glu_limit", C.c_double), ("glu_alpha", C.c_double), ("glu_shift", C.c_double),
-    ]
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "dim", "rot_dim", "vdim", "kv_rank", "window", "q_rank", "kv_from", "sink", "rot_pairs")] + [
+        (n, C.c_double) for n in ("rot_base", "scale", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow")] + [
+        (n, C.c_int32) for n in ("inner", "state", "conv_taps", "dt_rank", "ff", "glu")] + [
+        (n, C.c_double) for n in ("glu_limit", "glu_alpha", "glu_shift")] + [
+        (n, C.c_int32) for n in ("experts", "top", "expert_ff", "shared_ff", "expert_weight_in")]
 
 
 class LatentConfigC(C.Structure):
     """nvllm_latent_config"""
 
     _fields_ = [(n, C.c_int32) for n in ("vocab_size", "width", "num_layers", "loop_start", "loop_stop", "loop_times")] + [
-        ("norm_eps", C.c_double), ("embed_scale", C.c_double), ("logit_softcap", C.c_double), ("f32", C.c_int32),
-    ]
+        (n, C.c_double) for n in ("norm_eps", "embed_scale", "logit_softcap")] + [(n, C.c_int32) for n in ("norm", "one_norm", "f32")]
 
 
 class HybridLayerC(C.Structure):
@@ -70,6 +70,9 @@ class HybridConfigC(C.Structure):
         (n, C.c_double) for n in ("norm_eps", "embed_scale", "residual_mult", "norm_offset")] + [("f32", C.c_int32)]
 
 
+LATENT_ATTENTION, SELECTIVE_SCAN = 0, 1
+GLU_CLAMPED, GLU_GELU = 0, 1
+NORM_RMS, NORM_LAYER = 0, 1
 MIXER_ATTENTION, MIXER_LINEAR, MIXER_DELTA = 0, 1, 2  # NVLLM_MIXER_*
 
 _vp, _fp = C.c_void_p, C.c_void_p  # device pointers travel as integers

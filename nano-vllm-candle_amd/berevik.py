@@ -111,11 +111,11 @@ class BerevikConfig:
 
     def to_c(self, f32):
         c = _lib.LatentConfigC(self.vocab_size, self.hidden_size, len(self.layers), self.loop_start, self.loop_stop, self.loop_times,
-                               self.norm_eps, self.embed_scale, self.logit_softcap, int(f32))
+                               self.norm_eps, self.embed_scale, self.logit_softcap, _lib.NORM_RMS, 0, int(f32))
         ls = (_lib.LatentLayerC * max(len(self.layers), 1))()
         for l, (m, mlp) in zip(ls, self.layers):
             l.heads, l.dim, l.rot_dim, l.vdim, l.kv_rank, l.window = m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank, m.window
-            l.rot_base, l.scale = m.rot_base, m.scale
+            l.rot_base, l.scale, l.kv_from = m.rot_base, m.scale, -1
             if mlp is not None:
                 l.ff, l.glu_limit, l.glu_alpha, l.glu_shift = mlp.ff, mlp.limit, mlp.alpha, mlp.shift
         return c, ls

@@ -1,6 +1,7 @@
 // What the decoders built from layer descriptions share on the host side: the interface api.cpp drives them through, reading of host
 // tensors into packed weights, matrix products with the kernel that fits the row count, the output head.
 #pragma once
+#include <algorithm>
 #include <cstring>
 #include <string>
 
@@ -60,6 +61,19 @@ static int put_rows(nvllm_ctx* ctx, const PackedW& w, int row0, int rows, int co
     (void)hipFree(d);
     HIPCHK(ctx, e);
     return NVLLM_OK;
+}
+
+// weights and vectors on the device, zero until loaded (padding stays zero)
+static inline int alloc_packed(nvllm_ctx* ctx, PackedW& w, int N, int K) {
+    w.N = N; w.K = K;
+    HIPCHK(ctx, hipMalloc((void**)&w.data, w.bytes()));
+    HIPCHK(ctx, hipMemsetAsync(w.data, 0, w.bytes(), ctx->stream));
+    return NVLLM_OK;
+}
+static inline int alloc_vec(nvllm_ctx* ctx, float** p, size_t n) {
+    int rc = dmalloc(ctx, p, n);
+    if (!rc) HIPCHK(ctx, hipMemsetAsync(*p, 0, std::max<size_t>(n * 4, 16), ctx->stream));
+    return rc;
 }
 
 // ---- products ---------------------------------------------------------------------------------------------------------------

@@ -49,9 +49,15 @@ __device__ __forceinline__ float relu2(float x) {
     return x * x;
 }
 
+// 1 / 2 (1 + tanh a) = 1 / (1 + e^-2a): -2a of the tanh form of GELU
+__device__ __forceinline__ float gelu_arg(float g) { return -1.5957691216057308f * (g + 0.044715f * g * g * g); }
+
 // any GluSpec (uniform branch: the plain form costs nothing extra)
 __device__ __forceinline__ float glu_mul(float g, float u, const GluSpec& s) {
-    if (s.limit <= 0.f) return silu_mul(g, u);
+    if (s.limit <= 0.f) {
+        if (!s.gelu) return silu_mul(g, u);
+        return g * __builtin_amdgcn_rcpf(1.0f + __expf(gelu_arg(g))) * u;
+    }
     g = fminf(g, s.limit);
     u = fminf(fmaxf(u, -s.limit), s.limit);
     return (g * __builtin_amdgcn_rcpf(1.0f + __expf(-s.alpha * g))) * (u + s.shift);

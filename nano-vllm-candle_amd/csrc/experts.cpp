@@ -1,0 +1,130 @@
+// Host half of routed feed-forwards: see experts.h.
+#include "experts.h"
+
+#include <algorithm>
+
+int ExpertsBlock::create(nvllm_ctx* ctx, int experts_, int top_, int ff_, int shared_, int W_, int Kw_, int ldr_) {
+    const int tp = ctx->tp_size;
+    experts = experts_; top = top_; ff_all = ff_; shared_all = shared_; W = W_; Kw = Kw_; ldr = ldr_;
+    ff = ff_all / tp; sh = shared_all / tp; ff_p = up(ff, 128); sh_p = sh ? up(sh, 128) : 0;
+    Nr = up(experts + (sh ? 1 : 0), 16);
+    int rc = alloc_packed(ctx, router, Nr, Kw);
+    if (!rc) rc = alloc_packed(ctx, wup, experts * ff_p, Kw);
+    if (!rc) rc = alloc_packed(ctx, down, experts * ldr, ff_p);
+    if (!rc && sh) rc = alloc_packed(ctx, sup, sh_p, Kw);
+    if (!rc && sh) rc = alloc_packed(ctx, sdown, ldr, sh_p);
+    return rc;
+}
+void ExpertsBlock::destroy() {
+    for (PackedW* p : {&router, &wup, &down, &sup, &sdown}) (void)hipFree(p->data);
+}
+
+int ExpertsBlock::load(nvllm_model* m, const char* name, const char* s, const HostMat& h, int64_t rows, int64_t cols) {
+    nvllm_ctx* ctx = m->ctx;
+    const int64_t f0 = (int64_t)ctx->tp_rank * ff, s0 = (int64_t)ctx->tp_rank * sh;
+    auto want = [&](int64_t r, int64_t c) -> int {
+        if (rows == r && cols == c) return NVLLM_OK;
+        return fail(ctx, NVLLM_EINVAL, "tensor '%s': shape mismatch (got %lld x %lld, want %lld x %lld)", name, (long long)rows, (long long)cols, (long long)r, (long long)c);
+    };
+    auto put_up = [&](const PackedW& w, int row0, int64_t all, int n, int64_t r0) -> int {
+        int rc = want(all, W);
+        return rc ? rc : put_rows(ctx, w, row0, n, W, -1, [&](int r, int c) { return h.at(r0 + r, c); });
+    };
+    auto put_down = [&](const PackedW& w, int row0, int64_t all, int n, int64_t c0) -> int {
+        int rc = want(W, all);
+        return rc ? rc : put_rows(ctx, w, row0, W, n, -1, [&](int r, int c) { return h.at(r, c0 + c); });
+    };
+    if (!strcmp(s, "router")) return put_up(router, 0, experts, experts, 0);
+    if (sh && !strcmp(s, "shared.sg")) return put_up(router, experts, 1, 1, 0);
+    if (sh && !strcmp(s, "shared.up")) return put_up(sup, 0, shared_all, sh, s0);
+    if (sh && !strcmp(s, "shared.down")) return put_down(sdown, 0, shared_all, sh, s0);
+    int e = -1, off = 0;
+    if (sscanf(s, "e%d.%n", &e, &off) == 1 && off && e >= 0 && e < experts) {
+        if (!strcmp(s + off, "up")) return put_up(wup, e * ff_p, ff_all, ff, f0);
+        if (!strcmp(s + off, "down")) return put_down(down, e * ldr, ff_all, ff, f0);
+    }
+    return 1;
+}
+std::vector<std::string> ExpertsBlock::tensors() const {
+    std::vector<std::string> t = {"router"};
+    for (int e = 0; e < experts; ++e)
+        for (const char* s : {".up", ".down"}) t.push_back("e" + std::to_string(e) + s);
+    if (sh) for (const char* s : {"shared.up", "shared.down", "shared.sg"}) t.push_back(s);
+    return t;
+}
+size_t ExpertsBlock::step_bytes() const { return router.bytes() + (wup.bytes() + down.bytes()) / std::max(1, experts) * top + sup.bytes() + sdown.bytes(); }
+
+constexpr int kTileAlign = 256;  // rows of the widest tile a group starts at
+
+void ExpertsScratch::reserve(const ExpertsBlock& e, size_t R) {
+    const size_t per = e.top + 1;
+    cap = (int)std::max<size_t>(cap, (R * per + (size_t)(e.experts + 1) * kTileAlign + kTileAlign - 1) / kTileAlign * kTileAlign);
+    lda = std::max({lda, e.ff_p, e.sh_p});
+    n_rows = R;
+    n_z = std::max(n_z, R * e.Nr);
+    n_top = std::max(n_top, R * e.top);
+    n_place = std::max(n_place, R * per);
+    n_out = std::max<size_t>(n_out, e.ldr);
+    n_in = std::max<size_t>(n_in, e.Kw);
+}
+int ExpertsScratch::alloc(nvllm_ctx* ctx, bool f32) {
+    if (!cap) return NVLLM_OK;
+    int rc = dmalloc(ctx, &z, n_z);
+    if (!rc) rc = dmalloc(ctx, &score, n_top);
+    if (!rc) rc = dmalloc(ctx, &chosen, n_top);
+    if (!rc) rc = dmalloc(ctx, &gate, n_rows);
+    if (!rc) rc = dmalloc(ctx, &place, n_place);
+    for (float** p : {&pre, &post}) if (!rc) rc = dmalloc(ctx, p, cap);
+    if (!rc) rc = dmalloc(ctx, &src, cap);
+    if (!rc) rc = dmalloc(ctx, &tile_group, cap / 16);
+    if (!rc) rc = dmalloc(ctx, &out, (size_t)cap * n_out);
+    if (f32) {
+        if (!rc) rc = dmalloc(ctx, &act_f, (size_t)cap * lda);
+    } else {
+        for (bf16_bits** p : {&ah, &al}) if (!rc) rc = dmalloc(ctx, p, (size_t)cap * lda);
+        for (bf16_bits** p : {&gh, &gl}) if (!rc) rc = dmalloc(ctx, p, (size_t)cap * n_in);
+    }
+    return rc;
+}
+void ExpertsScratch::release() {
+    for (void* p : {(void*)z, (void*)score, (void*)gate, (void*)pre, (void*)post, (void*)out, (void*)act_f, (void*)chosen, (void*)place, (void*)src, (void*)tile_group, (void*)ah,
+                    (void*)al, (void*)gh, (void*)gl})
+        if (p) (void)hipFree(p);
+    *this = ExpertsScratch();
+}
+
+int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_bits* xh, const bf16_bits* xl, int packed, const float* y, int R, BranchSum* out) {
+    nvllm_ctx* ctx = m->ctx;
+    hipStream_t s = ctx->stream;
+    const bool f32 = y != nullptr;
+    GroupGemmArgs in;  // of rows
+    in.xh = xh; in.xl = xl; in.xf = y; in.ldx = e.Kw; in.x_packed = packed; in.x_rows = R;
+    GroupGemmArgs rg = in;
+    rg.w = e.router.data; rg.N = e.Nr; rg.K = e.Kw; rg.align = R > 64 ? 64 : 16; rg.out = x.z; rg.ldo = e.Nr;
+    PROF(m, PROF_GEMM, launch_group_gemm(rg, s));
+    RouteArgs ra;
+    ra.z = x.z; ra.ld = e.Nr; ra.rows = R; ra.experts = e.experts; ra.top = e.top; ra.weight_in = e.weight_in;
+    ra.gate_col = e.sh ? e.experts : -1;
+    ra.shared_group = e.sh > 0;
+    ra.align = R * e.top >= 32 * e.experts ? 64 : 16;
+    ra.cap = x.cap;
+    ra.chosen = x.chosen; ra.score = x.score; ra.gate = x.gate; ra.place = x.place; ra.src = x.src; ra.pre = x.pre; ra.post = x.post; ra.tile_group = x.tile_group;
+    PROF(m, PROF_QK, launch_route(ra, s));
+    const int64_t longest = (int64_t)R * e.top + (int64_t)std::min(e.experts, R * e.top) * (ra.align - 1) + (ra.shared_group ? R + ra.align - 1 : 0);
+    GroupGemmArgs ga = in;
+    ga.src = x.src; ga.w = e.wup.data; ga.w_group = (int64_t)e.ff_p * e.Kw / 8; ga.N = e.ff_p; ga.K = e.Kw;
+    if (ra.shared_group) { ga.ws = e.sup.data; ga.last = e.experts; ga.Ns = e.sh_p; ga.Ks = e.Kw; }
+    ga.tile_group = x.tile_group; ga.align = ra.align; ga.tiles = (int)(longest / ra.align); ga.pre = x.pre; ga.post = x.post; ga.relu2 = 1;
+    ga.ldo = x.lda;
+    if (f32) ga.out = x.act_f;
+    else { ga.oh = x.ah; ga.ol = x.al; }
+    PROF(m, PROF_GEMM, launch_group_gemm(ga, s));
+    GroupGemmArgs gd;
+    gd.xh = x.ah; gd.xl = x.al; gd.xf = f32 ? x.act_f : nullptr; gd.ldx = x.lda; gd.x_packed = 1; gd.x_rows = x.cap;
+    gd.w = e.down.data; gd.w_group = (int64_t)e.ldr * e.ff_p / 8; gd.N = e.ldr; gd.K = e.ff_p;
+    if (ra.shared_group) { gd.ws = e.sdown.data; gd.last = e.experts; gd.Ns = e.ldr; gd.Ks = e.sh_p; }
+    gd.tile_group = x.tile_group; gd.align = ra.align; gd.tiles = ga.tiles; gd.out = x.out; gd.ldo = e.ldr;
+    PROF(m, PROF_GEMM, launch_group_gemm(gd, s));
+    out->gather = x.out; out->gather_row = x.place; out->n_gather = e.top + ra.shared_group;
+    return NVLLM_OK;
+}

@@ -4,6 +4,7 @@
 
 #include "device_common.h"
 #include "hybrid.h"
+#include "short_conv.h"
 
 namespace nvllm {
 
@@ -304,27 +305,6 @@ hipError_t launch_linear_rows(const LinearRowsArgs& a, int rows, hipStream_t s) 
 // delta rule: one wave per (row, unit); units = q heads, k heads, v heads, then one for beta and the gate inputs.  The form for any
 // size of prompt chunk first, then those of decode and of long chunks.
 // ---------------------------------------------------------------------------------------------------
-// what a row sees of the tokens before its chunk: rows back to its segment's start, then the slot's history
-struct RowPast {
-    int in_chunk = 0;  // earlier rows of the same sequence in this chunk, at most taps - 1
-    int pos0 = 0;      // position of the segment's first row (valid when in_chunk < taps - 1)
-    int slot = 0;
-};
-__device__ __forceinline__ RowPast row_past(const DeltaRowsArgs& a, int row) {
-    RowPast p;
-    p.slot = a.slot[row];
-    const int pos = a.pos[row];
-    while (p.in_chunk < a.taps - 1 && row - p.in_chunk - 1 >= 0 && a.slot[row - p.in_chunk - 1] == p.slot) ++p.in_chunk;
-    p.pos0 = pos - p.in_chunk;
-    return p;
-}
-// raw input of channel c, j tokens before the row
-__device__ __forceinline__ float past_input(const DeltaRowsArgs& a, const RowPast& p, int row, int j, int c, int channels) {
-    if (j <= p.in_chunk) return slab_elem(a.in + (size_t)(row - j) * a.ld + c, a.n_slabs, a.slab_stride);
-    const int back = j - p.in_chunk;  // tokens before the segment
-    if (back > p.pos0) return 0.f;
-    return a.history[((((size_t)(p.pos0 & 1) * a.slots + p.slot) * (a.taps - 1)) + (a.taps - 1 - back)) * channels + c];
-}
 __device__ __forceinline__ float conv_silu(const DeltaRowsArgs& a, const RowPast& p, int row, int c, int channels) {
     float y = 0.f;
     for (int i = 0; i < a.taps; ++i) y += past_input(a, p, row, a.taps - 1 - i, c, channels) * a.conv[(size_t)i * channels + c];
@@ -558,31 +538,11 @@ hipError_t launch_delta_rows(const DeltaRowsArgs& a, int rows, hipStream_t s) {
     return hipGetLastError();
 }
 
-// one thread per (segment, channel): everything the segment leaves behind is read before it is written
-constexpr int kMaxTaps = 16;
-__global__ void __launch_bounds__(256) delta_history_kernel(DeltaRowsArgs a) {
-    const int channels = 2 * a.kv * a.dim + a.heads * a.vdim;
-    const int c = blockIdx.x * 256 + threadIdx.x, sg = blockIdx.y;
-    if (c >= channels) return;
-    const int row = a.seg.row0[sg] + a.seg.n[sg] - 1;
-    RowPast p;
-    p.slot = a.seg.slot[sg];
-    p.in_chunk = a.seg.n[sg] - 1;
-    p.pos0 = a.pos[a.seg.row0[sg]];
-    float x[kMaxTaps - 1];
-#pragma unroll
-    for (int i = 0; i < kMaxTaps - 1; ++i)
-        if (i < a.taps - 1) x[i] = past_input(a, p, row, a.taps - 2 - i, c, channels);
-    float* next = a.history + ((size_t)((a.pos[row] + 1) & 1) * a.slots + p.slot) * (a.taps - 1) * channels;
-#pragma unroll
-    for (int i = 0; i < kMaxTaps - 1; ++i)
-        if (i < a.taps - 1) next[(size_t)i * channels + c] = x[i];
-}
 hipError_t launch_delta_history(const DeltaRowsArgs& a, hipStream_t s) {
     if (a.seg.single || a.taps > kMaxTaps) return hipErrorInvalidValue;
     if (a.taps < 2 || a.seg.count <= 0) return hipSuccess;
     const int channels = 2 * a.kv * a.dim + a.heads * a.vdim;
-    delta_history_kernel<<<dim3((channels + 255) / 256, a.seg.count), 256, 0, s>>>(a);
+    conv_history_kernel<<<dim3((channels + 255) / 256, a.seg.count), 256, 0, s>>>(a, channels);
     return hipGetLastError();
 }
 

@@ -69,9 +69,11 @@ struct RowNorm {
 };
 
 // Gated activation of a gate/up projection: g' = min(g, limit), u' = clamp(u, -limit, limit), y = g' sigmoid(alpha g') (u' + shift).
-// limit <= 0: plain SwiGLU, y = g sigmoid(g) u (alpha, shift ignored).
+// limit <= 0: plain SwiGLU, y = g sigmoid(g) u, or with gelu set the tanh form of GELU, y = g / 2 (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))) u
+// (alpha, shift ignored).
 struct GluSpec {
     float limit = 0.f, alpha = 1.f, shift = 0.f;
+    int gelu = 0;
 };
 
 // ---- GEMM: out[ks][M][N] = x[M][K-slice ks] . W[N][K-slice ks]^T  (f32 slabs, ks < n_split) ------

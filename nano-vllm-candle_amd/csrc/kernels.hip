@@ -2557,7 +2557,7 @@ __global__ void __launch_bounds__(256) silu_mul_interleaved_kernel(const float* 
             for (int q = 0; q < 4; ++q) {
                 const bool cl = glu.limit > 0.f;
                 const float a = cl ? fminf(gv[q], glu.limit) : gv[q], b = cl ? fminf(fmaxf(uv[q], -glu.limit), glu.limit) + glu.shift : uv[q];
-                r4[q] = a / (1.0f + expf(cl ? -glu.alpha * a : -a)) * b;
+                r4[q] = a / (1.0f + expf(cl ? -glu.alpha * a : glu.gelu ? gelu_arg(a) : -a)) * b;
             }
             *reinterpret_cast<float4*>(y + (size_t)r * I + c) = make_float4(r4[0], r4[1], r4[2], r4[3]);
         }

@@ -8,7 +8,7 @@ namespace nvllm {
 constexpr int kLatentTileRows = 128;  // rows of one q-tile of a prompt chunk (a decode tile is one row)
 constexpr int kLatentMaxParts = 64;   // split-KV partitions per row
 
-// ---- residual add + up to two RMSNorms of the same row ----------------------------------------------------------------
+// ---- residual add + up to two norms of the same row ---------------------------------------------------------------------
 // s = sum of the partial sums in / in2 (or embed[id] * embed_scale) (+ residual); residual_out = s;
 // output k = s / sqrt(mean(s^2) + eps) * w[k], as bf16 hi/lo planes and/or f32.  Rows are W wide, stored with stride ldr
 // (multiple of 16, zeros beyond W); planes / y have stride ldx (zeros beyond W).
@@ -19,6 +19,10 @@ struct AddNormArgs {
     const float* in2 = nullptr;        // a second product's partial sums (the other branch of a parallel layer)
     int n_slabs2 = 1;
     int64_t slab_stride2 = 0;
+    const float* in2_scale = nullptr;  // [rows] factor of in2
+    const float* gather = nullptr;     // more summands: rows gather_row[r][0 .. n_gather) of a [*][ldr] array
+    const int* gather_row = nullptr;
+    int n_gather = 0;
     const uint32_t* ids = nullptr;
     const bf16_bits* embed = nullptr;  // [vocab][ldr]
     float embed_scale = 1.f;
@@ -30,6 +34,7 @@ struct AddNormArgs {
     const float* post_w = nullptr;
     float post_mult = 1.f;
     const float* w[2] = {nullptr, nullptr};  // nullptr: output k absent
+    int center = 0;                    // layer norm: the mean is taken off before the root mean square and the weight
     int raw = 0;                       // output 0 is s itself (w[0] unused)
     bf16_bits* xh[2] = {nullptr, nullptr};
     bf16_bits* xl[2] = {nullptr, nullptr};
@@ -49,12 +54,15 @@ struct LatentCache {
 };
 
 // ---- rows after the q / latent projection: split, norm, rotate, cache write ---------------------------------------------
-// qkv row: [heads][dim + rot] query, then rank + rot of the latent projection.  Writes q [rows][heads][dim_p + rot_p] f32
+// qkv row: [heads][dim + rot] query; kv row: rank + rot of the latent projection (kv nullptr: the rows write no cache).  Writes q [rows][heads][dim_p + rot_p] f32
 // (scaled; unrotated part, then rotated part; zero padded) and the token's latent and key part into the cache.
 struct LatentRowsArgs {
     const float* qkv = nullptr;
     int n_slabs = 1, ldq = 0;
     int64_t slab_stride = 0;
+    const float* kv = nullptr;
+    int kv_slabs = 1, ldkv = 0;
+    int64_t kv_stride = 0;
     int heads = 0, dim = 0, dim_p = 0;
     float scale = 1.f;             // score scale * log2(e)
     const float* norm_w = nullptr; // [rank]
@@ -72,10 +80,27 @@ hipError_t launch_latent_rows(const LatentRowsArgs& a, int rows, hipStream_t s);
 // the cache half of it alone (the expanded prompt kernel splits and rotates the query itself)
 hipError_t launch_latent_cache(const LatentRowsArgs& a, int rows, hipStream_t s);
 
+// query latents: RMS norm of the first `rank` columns of the input projection, as planes / f32 rows [rows][ldx]; kv (kv.kv set): the rows'
+// latents and key parts into the cache
+struct QueryLatentArgs {
+    const float* in = nullptr;
+    int n_slabs = 1, ld = 0;
+    int64_t slab_stride = 0;
+    int rank = 0, ldx = 0;
+    const float* norm_w = nullptr;
+    float eps = 0.f;
+    bf16_bits* xh = nullptr;
+    bf16_bits* xl = nullptr;
+    float* y = nullptr;
+    int packed = 0;
+};
+hipError_t launch_query_latent(const QueryLatentArgs& a, const LatentRowsArgs& kv, int rows, hipStream_t s);
+
 // ---- per-head products and 32-bit products -------------------------------------------------------------------------------
 // y[r][h][n] = sum_k x[r][h][k] W[h][n][k]: x f32 (element strides), W packed per head (N % 16 == 0, K % 32 == 0).
 // exact = 0: x as bf16 hi + lo, 16x16x32 bf16 MFMA; exact = 1: everything in f32 (16x16x4 f32 MFMA, weights widened).
-// decay_rate set (f32 output): head 0 leaves exp(-decay_rate[n] softplus(y + decay_bias[n])), every other head sigmoid(y).
+// decay_bias set (f32 output): softplus(y + decay_bias[n]); decay_rate too: head 0 leaves exp(-decay_rate[n] softplus(y + decay_bias[n])),
+// every other head sigmoid(y).
 // Output: f32 with strides, or bf16 hi/lo planes [rows][ld] at column h * n_valid + n (n < n_valid).
 struct HeadGemmArgs {
     const float* x = nullptr;
@@ -111,6 +136,7 @@ struct LatentAttnArgs {
     const int* slot = nullptr;     // per row
     int single = 0;                // every q-tile is one row, tile i = row i
     int heads = 0, window = 0;     // window <= 0: causal without a window
+    const float* sink = nullptr;   // [heads] one more term 2^sink of every denominator; nullptr: none
     float* out = nullptr;          // [rows][heads][rank_p]
     // split-KV: workgroup z covers part_tiles 32-token tiles counted from the first visible tile of its q-tile
     int part_tiles = 0, max_parts = 1;
@@ -175,6 +201,7 @@ struct LatentPrefillArgs {
     const int* tile_order = nullptr; // longest context first
     const int* pos = nullptr;
     int n_tiles = 0, heads = 0, window = 0;
+    const float* sink = nullptr;   // as in LatentAttnArgs
     int dim_p = 0, vdim = 0, vdim_p = 0;
     bf16_bits* oh = nullptr;       // context planes [rows][ld], column head * vdim
     bf16_bits* ol = nullptr;

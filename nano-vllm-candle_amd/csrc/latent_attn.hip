@@ -197,8 +197,13 @@ __global__ void __launch_bounds__(256 * S, 2) latent_attn_kernel(LatentAttnArgs 
     for (int w = 0; w < 4; ++w) ms = fmaxf(ms, ml[w][0][l15]);
 #pragma unroll
     for (int w = 0; w < 4; ++w) lt += ml[w][1][l15] * __builtin_amdgcn_exp2f(ml[w][0][l15] - ms);
-    const float f = __builtin_amdgcn_exp2f(m - ms);
     const int n_parts = a.part_tiles ? (t_hi - t_lo + a.part_tiles - 1) / a.part_tiles : 1;
+    if (a.sink && n_parts == 1) {  // parts: the sink joins where they are combined
+        const float sk = a.sink[head], mn = fmaxf(ms, sk);
+        lt = lt * __builtin_amdgcn_exp2f(ms - mn) + __builtin_amdgcn_exp2f(sk - mn);
+        ms = mn;
+    }
+    const float f = __builtin_amdgcn_exp2f(m - ms);
     const float scale = n_parts > 1 ? 1.0f : 1.0f / lt;
     const size_t rh = (size_t)(row0 + tok) * a.heads + head;
     float* dst = n_parts > 1 ? a.part_o + (rh * a.max_parts + blockIdx.z) * (KC * 32) : a.out + rh * (KC * 32);

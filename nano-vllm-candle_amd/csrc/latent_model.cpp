@@ -1,7 +1,8 @@
 // Latent-attention decoders behind the C ABI: weights in MFMA tile layout, latent cache and step buffers, the forward of one
 // chunk of rows.  Sequences, blocks, slots, scheduling of chunks, sampling and decode pipelining are the shared code of api.cpp.
 //
-// A layer adds two branches of the same x:  x <- x + W_o attn(norm1 x) + W_down glu(norm2 x).
+// A layer adds two branches of the same x:  x <- x + W_o mixer(norm1 x) + ff(norm2 x), norm2 possibly being norm1.  The mixer is latent
+// attention or a selective scan (scan_mixer.h), the feed-forward gated or routed to experts (experts.h).
 // Mixed precision (the serving mode): products run on bf16 hi + lo planes (16 bits of the activation) with f32 accumulation,
 // the cache is f16; residual, norms, rotation, scores and softmax are f32.  32-bit mode: every product and the cache in f32.
 #include <algorithm>
@@ -11,17 +12,26 @@
 #include <map>
 
 #include "decoder.h"
+#include "experts.h"
+#include "scan_mixer.h"
 
 struct LatentLayer {
     nvllm_latent_layer c{};
     int heads = 0, ff = 0;                       // this rank's share
     int dim_p = 0, rank_p = 0, rot_p = 0, vdim_p = 0, ff_p = 0;
-    int Nq = 0, Kc = 0;                          // q + latent projection rows (padded), context width (padded)
+    int Nq = 0, Kc = 0;                          // q (+ latent) projection rows (padded), context width (padded)
+    int Nd = 0, Kq = 0;                          // query latents: rows of the first projection (padded), width of the second (padded)
+    PackedW dq;                                  // query latents: the first projection, then the latent projection unless kv_from
     PackedW qkv, ukt, uv, o, gu, down;           // per head: ukt [rank_p x dim_p], uv [vdim_p x rank_p]
     bool expands = false;                        // prompt chunks may run the expanded form
     PackedW ukx, uvx;                            // its weights, f16 times 1 / scale: [dim_p x rank_p], [vdim_p x rank_p] per head
     float ukx_scale = 1.f, uvx_scale = 1.f;
-    float *norm1 = nullptr, *norm2 = nullptr, *dkv_norm = nullptr;
+    float *norm1 = nullptr, *norm2 = nullptr, *dkv_norm = nullptr, *dq_norm = nullptr;
+    float* sink = nullptr;                       // times log2(e)
+    ExpertsBlock experts;
+    ScanMixer scan;
+    bool own_kv() const { return c.kv_from < 0; }
+    const PackedW& first() const { return scan.on() ? scan.in : c.q_rank ? dq : qkv; }  // the product the normed input meets
     int rope = 0;                                // index of the rotation table
     LatentCache cache_shape() const {
         LatentCache k;
@@ -31,10 +41,26 @@ struct LatentLayer {
 };
 
 struct RopeTable {
-    double base = 0;
+    double base = 0, factor = 0, original = 0, fast = 0, slow = 0;
     int dims = 0;
     float *cos = nullptr, *sin = nullptr;
+    bool serves(const nvllm_latent_layer& c) const {
+        return base == c.rot_base && dims == c.rot_dim && factor == c.yarn_factor &&
+               (factor <= 0 || (original == c.yarn_original && fast == c.yarn_fast && slow == c.yarn_slow));
+    }
+    double frequency(int i) const;
+    double magnitude() const { return factor > 0 ? 0.1 * std::log(factor) + 1.0 : 1.0; }  // of both cos and sin
 };
+// YaRN (Peng et al., "YaRN: Efficient Context Window Extension of Large Language Models"): slow pairs are divided by `factor`, fast ones
+// kept, a ramp over the pairs in between
+double RopeTable::frequency(int i) const {
+    const double f = std::pow(base, -2.0 * i / dims);
+    if (factor <= 0) return f;
+    auto pair_of = [&](double turns) { return dims * std::log(original / (2 * M_PI * turns)) / (2 * std::log(base)); };
+    const double lo = std::max(std::floor(pair_of(fast)), 0.0), hi = std::min(std::ceil(pair_of(slow)), dims - 1.0);
+    const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+    return f / factor * ramp + f * (1 - ramp);
+}
 
 struct LatentModel : DecoderImpl {
     nvllm_latent_config cfg{};
@@ -55,7 +81,11 @@ struct LatentModel : DecoderImpl {
     int *d_exp = nullptr, *d_tile_exp = nullptr, *h_exp = nullptr;
     struct Segment { int pos0, n; };
     std::vector<Segment> segments;
-    float *y1 = nullptr, *y2 = nullptr, *ctx_f = nullptr, *act_f = nullptr;                   // 32-bit mode
+    float *y1 = nullptr, *y2 = nullptr, *ctx_f = nullptr, *act_f = nullptr, *cq_f = nullptr;  // 32-bit mode
+    bf16_bits *cqh = nullptr, *cql = nullptr;                                                 // normed query latents
+    ExpertsScratch experts;
+    ScanScratch scan;
+    bool has_state = false;
 
     ~LatentModel() override;
     int load_tensor(nvllm_model* m, const char* name, const void* data, int dtype, const int64_t* shape, int ndim) override;
@@ -66,6 +96,7 @@ struct LatentModel : DecoderImpl {
     int64_t kv_bytes_per_token() const override;
     int64_t kv_read_bytes(int len) const override;
     int tile_rows(int qt) const override { return qt == 1 ? 1 : kLatentTileRows; }
+    bool recurrent() const override { return has_state; }
     int plan_chunk(nvllm_model* m, const int* pos, const int* slot, const int* seq, int R, const int* tile_row0, int n_tiles, int qt) override;
     int forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n_last, int logits_row0) override;
 };
@@ -83,11 +114,31 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
         return fail(ctx, NVLLM_EINVAL, "loop [%d, %d) outside the %d layers", c.loop_start, c.loop_stop, c.num_layers);
     for (int l = 0; l < c.num_layers; ++l) {
         const nvllm_latent_layer& k = layers[l];
-        if (k.heads < 1 || k.dim < 1 || k.rot_dim < 0 || k.vdim < 1 || k.kv_rank < 1 || k.ff < 0) return fail(ctx, NVLLM_EINVAL, "layer %d has non-positive sizes", l);
+        if (k.ff < 0 || k.experts < 0 || (k.ff && k.experts)) return fail(ctx, NVLLM_EINVAL, "layer %d: feed-forward sizes", l);
+        if (k.ff % tp || (k.experts && (k.expert_ff % tp || k.shared_ff % tp)))
+            return fail(ctx, NVLLM_EINVAL, "layer %d: feed-forward width not divisible by tp_size %d", l, tp);
+        if (k.ff && k.glu != NVLLM_GLU_CLAMPED && k.glu != NVLLM_GLU_GELU) return fail(ctx, NVLLM_EINVAL, "layer %d: feed-forward activation %d unknown", l, k.glu);
+        if (k.ff && k.glu == NVLLM_GLU_CLAMPED && k.glu_limit <= 0) return fail(ctx, NVLLM_EINVAL, "layer %d: the feed-forward's limit must be positive", l);
+        if (k.experts && (k.experts > kMaxExperts || k.top < 1 || k.top > std::min(k.experts, kMaxTop) || k.expert_ff < 1 || k.shared_ff < 0))
+            return fail(ctx, NVLLM_EINVAL, "layer %d: %d of %d experts of width %d unsupported (at most %d of %d)", l, k.top, k.experts, k.expert_ff, kMaxTop, kMaxExperts);
+        if (k.mixer == NVLLM_SELECTIVE_SCAN) {
+            if (k.inner < 1 || k.state < 1 || k.state > kMaxScanStates || k.conv_taps < 1 || k.conv_taps > 16 || k.dt_rank < 1)
+                return fail(ctx, NVLLM_EINVAL, "layer %d: scan of %d channels, %d states (at most %d), %d taps (at most 16), rank %d unsupported", l, k.inner, k.state, kMaxScanStates, k.conv_taps, k.dt_rank);
+            if (k.inner % tp) return fail(ctx, NVLLM_EINVAL, "layer %d: %d channels not divisible by tp_size %d", l, k.inner, tp);
+            continue;
+        }
+        if (k.mixer != NVLLM_LATENT_ATTENTION) return fail(ctx, NVLLM_EINVAL, "layer %d: mixer %d unknown", l, k.mixer);
+        if (k.heads < 1 || k.dim < 1 || k.rot_dim < 0 || k.vdim < 1 || k.kv_rank < 1 || k.q_rank < 0 || k.q_rank > 16384) return fail(ctx, NVLLM_EINVAL, "layer %d has non-positive sizes", l);
         if (k.rot_dim % 2) return fail(ctx, NVLLM_EINVAL, "layer %d: rot_dim %d is odd", l, k.rot_dim);
-        if (k.heads % tp || k.ff % tp) return fail(ctx, NVLLM_EINVAL, "layer %d: heads %d or feed-forward width %d not divisible by tp_size %d", l, k.heads, k.ff, tp);
+        if (k.heads % tp) return fail(ctx, NVLLM_EINVAL, "layer %d: heads %d not divisible by tp_size %d", l, k.heads, tp);
         if (up(k.kv_rank, 32) + up(k.rot_dim, 32) > 2560) return fail(ctx, NVLLM_EINVAL, "layer %d: latent of %d + %d elements unsupported (at most 2560)", l, k.kv_rank, k.rot_dim);
-        if (k.ff && k.glu_limit <= 0) return fail(ctx, NVLLM_EINVAL, "layer %d: the feed-forward's limit must be positive", l);
+        if (k.kv_from >= 0) {
+            if (k.kv_from >= l || layers[k.kv_from].mixer != NVLLM_LATENT_ATTENTION || layers[k.kv_from].kv_from >= 0)
+                return fail(ctx, NVLLM_EINVAL, "layer %d: layer %d has no latent cache of its own before it", l, k.kv_from);
+            const nvllm_latent_layer& j = layers[k.kv_from];
+            if (j.kv_rank != k.kv_rank || j.rot_dim != k.rot_dim) return fail(ctx, NVLLM_EINVAL, "layer %d reads the cache of layer %d, whose sizes differ", l, k.kv_from);
+            if (loop) return fail(ctx, NVLLM_EINVAL, "layer %d: shared caches beside looped layers are unsupported", l);
+        }
     }
     HIPCHK(ctx, hipSetDevice(ctx->device));
     nvllm_model* m = new nvllm_model();
@@ -108,20 +159,13 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
     }
     m->L = (int)L.order.size();
     for (int l = 0; l < c.num_layers; ++l) {
-        if (layers[l].window <= 0) { m->widest_window = 0; break; }
+        if (layers[l].mixer == NVLLM_LATENT_ATTENTION && layers[l].window <= 0) { m->widest_window = 0; break; }
         m->widest_window = std::max(m->widest_window, (int)layers[l].window);
     }
-    auto alloc_w = [&](PackedW& w, int N, int K) -> int {
-        w.N = N; w.K = K;
-        HIPCHK(ctx, hipMalloc((void**)&w.data, w.bytes()));
-        HIPCHK(ctx, hipMemsetAsync(w.data, 0, w.bytes(), ctx->stream));  // padding rows and columns stay zero
-        return NVLLM_OK;
-    };
-    auto alloc_v = [&](float** p, int n) -> int {
-        int rc = dmalloc(ctx, p, n);
-        if (!rc) HIPCHK(ctx, hipMemsetAsync(*p, 0, (size_t)n * 4, ctx->stream));
-        return rc;
-    };
+    auto alloc_w = [&](PackedW& w, int N, int K) { return alloc_packed(ctx, w, N, K); };
+    auto alloc_v = [&](float** p, size_t n) { return alloc_vec(ctx, p, n); };
+    // wide projections: a whole number of the prompt product's 192- or 256-feature tiles
+    auto wide = [&](int n) { return n >= 1536 && !c.f32 ? std::min(up(n, 192), up(n, 256)) : up(n, 16); };
     int rc = dmalloc(ctx, &L.embed, (size_t)c.vocab_size * L.ldr);
     if (!rc) HIPCHK(ctx, hipMemsetAsync(L.embed, 0, (size_t)c.vocab_size * L.ldr * 2, ctx->stream));
     if (!rc) rc = alloc_w(L.head, L.Vp, L.Kw);
@@ -130,31 +174,50 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
     for (int l = 0; l < c.num_layers && !rc; ++l) {
         LatentLayer& w = L.layers[l];
         w.c = layers[l];
-        w.heads = w.c.heads / tp; w.ff = w.c.ff / tp;
+        w.ff = w.c.ff / tp; w.ff_p = up(w.ff, 128);
+        rc = alloc_v(&w.norm1, L.Kw);
+        if (w.ff) {
+            if (!rc) rc = alloc_w(w.gu, 2 * w.ff_p, L.Kw);
+            if (!rc) rc = alloc_w(w.down, L.ldr, w.ff_p);
+        }
+        if (!rc && !c.one_norm && (w.ff || w.c.experts)) rc = alloc_v(&w.norm2, L.Kw);
+        w.experts.weight_in = w.c.expert_weight_in;
+        if (!rc && w.c.experts) rc = w.experts.create(ctx, w.c.experts, w.c.top, w.c.expert_ff, w.c.shared_ff, c.width, L.Kw, L.ldr);
+        if (w.c.mixer == NVLLM_SELECTIVE_SCAN) {
+            L.has_state = true;
+            if (!rc) rc = w.scan.create(ctx, w.c.inner, w.c.state, w.c.conv_taps, w.c.dt_rank, L.Kw, c.f32);
+            w.Kc = w.scan.Kc;
+            if (!rc) rc = alloc_w(w.o, L.ldr, w.Kc);
+            continue;
+        }
+        w.heads = w.c.heads / tp;
         // the expanded form has instances for the padded sizes below; layers without one keep the plain padding
         w.expands = !c.f32 && latent_prefill_dim(w.c.dim) && latent_prefill_vdim(w.c.vdim) && w.c.kv_rank <= 512 && w.c.rot_dim > 0 && w.c.rot_dim <= 64;
         w.dim_p = w.expands ? latent_prefill_dim(w.c.dim) : up(w.c.dim, 32); w.rank_p = c.f32 ? up(w.c.kv_rank, 32) : latent_rank_padded(w.c.kv_rank); w.rot_p = up(w.c.rot_dim, 32);
-        w.vdim_p = w.expands ? latent_prefill_vdim(w.c.vdim) : up(w.c.vdim, 16); w.ff_p = up(w.ff, 128);
-        w.Nq = w.heads * (w.c.dim + w.c.rot_dim) + w.c.kv_rank + w.c.rot_dim;
-        // wide projections: a whole number of the prompt product's 192- or 256-feature tiles
-        w.Nq = w.Nq >= 1536 && !c.f32 ? std::min(up(w.Nq, 192), up(w.Nq, 256)) : up(w.Nq, 16);
+        w.vdim_p = w.expands ? latent_prefill_vdim(w.c.vdim) : up(w.c.vdim, 16);
+        const int latent_rows = w.own_kv() ? w.c.kv_rank + w.c.rot_dim : 0;
+        w.Nq = wide(w.heads * (w.c.dim + w.c.rot_dim) + (w.c.q_rank ? 0 : latent_rows));
         w.Kc = up(w.heads * w.c.vdim, 128);
-        rc = alloc_w(w.qkv, w.Nq, L.Kw);
+        if (w.c.q_rank) {
+            w.Nd = wide(w.c.q_rank + latent_rows); w.Kq = up(w.c.q_rank, 128);
+            if (!rc) rc = alloc_w(w.dq, w.Nd, L.Kw);
+            if (!rc) rc = alloc_v(&w.dq_norm, w.Kq);
+        }
+        if (!rc && w.c.sink) rc = alloc_v(&w.sink, w.heads);
+        if (!rc) rc = alloc_w(w.qkv, w.Nq, w.c.q_rank ? w.Kq : L.Kw);
         if (!rc) rc = alloc_w(w.ukt, w.heads * w.rank_p, w.dim_p);
         if (!rc && w.expands) rc = alloc_w(w.ukx, w.heads * w.dim_p, w.rank_p);
         if (!rc && w.expands) rc = alloc_w(w.uvx, w.heads * w.vdim_p, w.rank_p);
         if (!rc) rc = alloc_w(w.uv, w.heads * w.vdim_p, w.rank_p);
         if (!rc) rc = alloc_w(w.o, L.ldr, w.Kc);
-        if (!rc) rc = alloc_v(&w.norm1, L.Kw);
         if (!rc) rc = alloc_v(&w.dkv_norm, w.rank_p);
-        if (!rc && w.ff) {
-            rc = alloc_w(w.gu, 2 * w.ff_p, L.Kw);
-            if (!rc) rc = alloc_w(w.down, L.ldr, w.ff_p);
-            if (!rc) rc = alloc_v(&w.norm2, L.Kw);
-        }
         int t = 0;
-        while (t < (int)L.ropes.size() && !(L.ropes[t].base == w.c.rot_base && L.ropes[t].dims == w.c.rot_dim)) ++t;
-        if (t == (int)L.ropes.size()) { RopeTable r; r.base = w.c.rot_base; r.dims = w.c.rot_dim; L.ropes.push_back(r); }
+        while (t < (int)L.ropes.size() && !L.ropes[t].serves(w.c)) ++t;
+        if (t == (int)L.ropes.size()) {
+            RopeTable r;
+            r.base = w.c.rot_base; r.dims = w.c.rot_dim; r.factor = w.c.yarn_factor; r.original = w.c.yarn_original; r.fast = w.c.yarn_fast; r.slow = w.c.yarn_slow;
+            L.ropes.push_back(r);
+        }
         w.rope = t;
     }
     if (!rc && hipStreamSynchronize(ctx->stream) != hipSuccess) rc = fail(ctx, NVLLM_EHIP, "weight allocation failed");
@@ -165,9 +228,13 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
 
 void LatentModel::free_kv() {
     LatentModel& L = *this;
-    for (void* p : L.cache) if (p) (void)hipFree(p);
+    for (size_t i = 0; i < L.cache.size(); ++i)
+        if (L.cache[i] && L.layers[L.order[i]].own_kv()) (void)hipFree(L.cache[i]);
     L.cache.clear();
-    void* ptrs[] = {L.slabs2, L.q, L.qlat, L.olat, L.part_o, L.part_ml, L.tap, L.kx, L.vx, L.d_exp, L.d_tile_exp, L.x2h, L.x2l, L.y1, L.y2, L.ctx_f, L.act_f};
+    L.experts.release();
+    L.scan.release();
+    for (LatentLayer& w : L.layers) w.scan.free_kv();
+    void* ptrs[] = {L.cq_f, L.cqh, L.cql, L.slabs2, L.q, L.qlat, L.olat, L.part_o, L.part_ml, L.tap, L.kx, L.vx, L.d_exp, L.d_tile_exp, L.x2h, L.x2l, L.y1, L.y2, L.ctx_f, L.act_f};
     for (void* p : ptrs) if (p) (void)hipFree(p);
     L.slabs2 = L.q = L.qlat = L.olat = L.part_o = L.part_ml = L.tap = nullptr;
     L.x2h = L.x2l = nullptr;
@@ -176,7 +243,8 @@ void LatentModel::free_kv() {
     if (L.h_exp) (void)hipHostFree(L.h_exp);
     L.h_exp = nullptr;
     L.exp_cap = L.exp_n = 0;
-    L.y1 = L.y2 = L.ctx_f = L.act_f = nullptr;
+    L.y1 = L.y2 = L.ctx_f = L.act_f = L.cq_f = nullptr;
+    L.cqh = L.cql = nullptr;
     for (RopeTable& r : L.ropes) {
         if (r.cos) (void)hipFree(r.cos);
         if (r.sin) (void)hipFree(r.sin);
@@ -189,7 +257,10 @@ LatentModel::~LatentModel() {
     free_kv();
     (void)hipFree(L.embed); (void)hipFree(L.head.data); (void)hipFree(L.final_norm);
     for (LatentLayer& w : L.layers) {
-        for (PackedW* p : {&w.qkv, &w.ukt, &w.ukx, &w.uv, &w.uvx, &w.o, &w.gu, &w.down}) (void)hipFree(p->data);
+        w.experts.destroy();
+        w.scan.destroy();
+        (void)hipFree(w.dq_norm); (void)hipFree(w.sink);
+        for (PackedW* p : {&w.dq, &w.qkv, &w.ukt, &w.ukx, &w.uv, &w.uvx, &w.o, &w.gu, &w.down}) (void)hipFree(p->data);
         (void)hipFree(w.norm1); (void)hipFree(w.norm2); (void)hipFree(w.dkv_norm);
     }
 }
@@ -221,8 +292,25 @@ static int put_expand(nvllm_ctx* ctx, const PackedW& w, float* unscale, const Ho
     });
 }
 
-static const char* const kMixTensors[] = {"norm1", "mix.q", "mix.dkv", "mix.dkv.norm", "mix.uk", "mix.uv", "mix.o"};
-static const char* const kMlpTensors[] = {"norm2", "mlp.gate", "mlp.up", "mlp.down"};
+// the checkpoint's tensors of a layer
+static std::vector<std::string> layer_tensors(const LatentLayer& w, bool one_norm) {
+    std::vector<std::string> t = {"norm1", "mix.o"};
+    auto add = [&](std::initializer_list<const char*> names) { t.insert(t.end(), names.begin(), names.end()); };
+    if (w.scan.on()) {
+        for (const std::string& s : ScanMixer::tensors()) t.push_back("mix." + s);
+    } else {
+        add({"mix.uk", "mix.uv"});
+        if (w.c.q_rank) add({"mix.dq", "mix.dq.norm", "mix.uq"});
+        else add({"mix.q"});
+        if (w.own_kv()) add({"mix.dkv", "mix.dkv.norm"});
+        if (w.c.sink) add({"mix.sink"});
+    }
+    if (!one_norm && (w.ff || w.experts.on())) add({"norm2"});
+    if (w.ff) add({"mlp.gate", "mlp.up", "mlp.down"});
+    if (w.experts.on())
+        for (const std::string& s : w.experts.tensors()) t.push_back("mlp." + s);
+    return t;
+}
 
 int LatentModel::load_tensor(nvllm_model* m, const char* name, const void* data, int dtype, const int64_t* shape, int ndim) {
     nvllm_ctx* ctx = m->ctx;
@@ -263,12 +351,37 @@ int LatentModel::load_tensor(nvllm_model* m, const char* name, const void* data,
         LatentLayer& w = L.layers[l];
         const int dim = w.c.dim, rot = w.c.rot_dim, vdim = w.c.vdim, kr = w.c.kv_rank, Hl = w.heads, H = w.c.heads, ff = w.c.ff;
         const int64_t h0 = (int64_t)rank * Hl, f0 = (int64_t)rank * w.ff;
+        // rotated pairs of neighbours: the rows are put in the order that pairs i with i + rot / 2 (queries and keys alike: scores do not change)
+        auto turned = [&](int i) { return !w.c.rot_pairs ? i : i < rot / 2 ? 2 * i : 2 * (i - rot / 2) + 1; };
+        auto q_row = [&](int r) { const int n = r / (dim + rot), i = r % (dim + rot); return (h0 + n) * (dim + rot) + (i < dim ? i : dim + turned(i - dim)); };
+        auto kv_row = [&](int r) { return r < kr ? r : kr + turned(r - kr); };
+        auto put_o = [&](int64_t all, int n, int64_t c0) -> int {
+            int e = want(W, all);
+            return e ? e : put_rows(ctx, w.o, 0, W, n, -1, [&](int r, int c) { return h.at(r, c0 + c); });
+        };
+        const bool latents = !w.scan.on(), own = latents && w.own_kv(), narrow = latents && w.c.q_rank > 0;
+        const int qr = w.c.q_rank, Q = H * (dim + rot);
+        const std::vector<std::string> names = layer_tensors(w, L.cfg.one_norm);
+        if (std::find(names.begin(), names.end(), s) == names.end()) return fail(ctx, NVLLM_EINVAL, "unknown tensor name '%s'", name);
         if (!strcmp(s, "norm1")) rc = vec(w.norm1, W);
-        else if (!strcmp(s, "mix.q")) {
-            if (!(rc = want((int64_t)H * (dim + rot), W)))
-                rc = put_rows(ctx, w.qkv, 0, Hl * (dim + rot), W, -1, [&](int r, int c) { return h.at(h0 * (dim + rot) + r, c); });
-        } else if (!strcmp(s, "mix.dkv")) {
-            if (!(rc = want(kr + rot, W))) rc = put_rows(ctx, w.qkv, Hl * (dim + rot), kr + rot, W, -1, [&](int r, int c) { return h.at(r, c); });
+        else if (w.scan.on() && !strcmp(s, "mix.o")) rc = put_o(w.c.inner, w.scan.n, (int64_t)rank * w.scan.n);
+        else if (w.scan.on() && !strncmp(s, "mix.", 4)) rc = w.scan.load(m, name, s + 4, h, rows, cols, W);
+        else if (w.experts.on() && !strncmp(s, "mlp.", 4)) rc = w.experts.load(m, name, s + 4, h, rows, cols);
+        else if (!strcmp(s, "mix.q") || !strcmp(s, "mix.uq")) {
+            const int K = narrow ? qr : W;
+            if (!(rc = want(Q, K))) rc = put_rows(ctx, w.qkv, 0, Hl * (dim + rot), K, -1, [&](int r, int c) { return h.at(q_row(r), c); });
+        } else if (!strcmp(s, "mix.dq")) {
+            if (!(rc = want(qr, W))) rc = put_rows(ctx, w.dq, 0, qr, W, -1, [&](int r, int c) { return h.at(r, c); });
+        } else if (!strcmp(s, "mix.dq.norm")) rc = vec(w.dq_norm, qr);
+        else if (!strcmp(s, "mix.sink")) {
+            if (!(rc = want(1, H))) {
+                std::vector<float> t(Hl);
+                for (int i = 0; i < Hl; ++i) t[i] = (float)(h.f32(h0 + i) * 1.4426950408889634);
+                HIPCHK(ctx, hipMemcpy(w.sink, t.data(), t.size() * 4, hipMemcpyHostToDevice));
+            }
+        } else if (own && !strcmp(s, "mix.dkv")) {
+            if (!(rc = want(kr + rot, W)))
+                rc = put_rows(ctx, narrow ? w.dq : w.qkv, narrow ? qr : Hl * (dim + rot), kr + rot, W, -1, [&](int r, int c) { return h.at(kv_row(r), c); });
         } else if (!strcmp(s, "mix.dkv.norm")) rc = vec(w.dkv_norm, kr);
         else if (!strcmp(s, "mix.uk")) {  // transposed per head: the query is carried into latent space
             if (!(rc = want((int64_t)H * dim, kr)))
@@ -285,8 +398,8 @@ int LatentModel::load_tensor(nvllm_model* m, const char* name, const void* data,
                 });
             if (!rc && w.expands) rc = put_expand(ctx, w.uvx, &w.uvx_scale, h, h0, Hl, vdim, w.vdim_p, kr);
         } else if (!strcmp(s, "mix.o")) {
-            if (!(rc = want(W, (int64_t)H * vdim))) rc = put_rows(ctx, w.o, 0, W, Hl * vdim, -1, [&](int r, int c) { return h.at(r, h0 * vdim + c); });
-        } else if (ff && !strcmp(s, "norm2")) rc = vec(w.norm2, W);
+            rc = put_o((int64_t)H * vdim, Hl * vdim, h0 * vdim);
+        } else if (!strcmp(s, "norm2")) rc = vec(w.norm2, W);
         else if (ff && (!strcmp(s, "mlp.gate") || !strcmp(s, "mlp.up"))) {
             if (!(rc = want(ff, W))) rc = put_rows(ctx, w.gu, 0, w.ff, W, s[4] == 'g' ? 0 : 1, [&](int r, int c) { return h.at(f0 + r, c); });
         } else if (ff && !strcmp(s, "mlp.down")) {
@@ -303,17 +416,11 @@ int LatentModel::finalize(nvllm_model* m) {
     for (const char* s : {"embed", "head", "final.norm"})
         if (!m->loaded.count(s)) return fail(ctx, NVLLM_ESTATE, "missing tensor %s", s);
     char name[96];
-    for (int l = 0; l < latent(m).cfg.num_layers; ++l) {
-        for (const char* s : kMixTensors) {
-            snprintf(name, sizeof name, "l%d.%s", l, s);
+    for (int l = 0; l < latent(m).cfg.num_layers; ++l)
+        for (const std::string& s : layer_tensors(latent(m).layers[l], latent(m).cfg.one_norm)) {
+            snprintf(name, sizeof name, "l%d.%s", l, s.c_str());
             if (!m->loaded.count(name)) return fail(ctx, NVLLM_ESTATE, "missing tensor %s", name);
         }
-        if (latent(m).layers[l].ff)
-            for (const char* s : kMlpTensors) {
-                snprintf(name, sizeof name, "l%d.%s", l, s);
-                if (!m->loaded.count(name)) return fail(ctx, NVLLM_ESTATE, "missing tensor %s", name);
-            }
-    }
     m->finalized = true;
     return NVLLM_OK;
 }
@@ -323,15 +430,17 @@ int64_t LatentModel::weight_bytes() const {
     int64_t b = (int64_t)L.head.bytes() + (int64_t)L.cfg.width * 4;
     for (int l : L.order) {
         const LatentLayer& w = L.layers[l];
+        b += (int64_t)(w.dq.bytes() + w.experts.step_bytes() + w.scan.bytes());
         b += (int64_t)(w.qkv.bytes() + w.ukt.bytes() + w.uv.bytes() + w.o.bytes() + w.gu.bytes() + w.down.bytes());
-        b += (int64_t)((w.ff ? 2 : 1) * L.cfg.width + w.c.kv_rank) * 4;
+        b += (int64_t)((w.norm2 ? 2 : 1) * L.cfg.width + w.c.kv_rank) * 4;
     }
     return b;
 }
 int64_t LatentModel::kv_bytes_per_token() const {
     const LatentModel& L = *this;
     int64_t b = 0;
-    for (int l : L.order) b += (int64_t)(L.layers[l].rank_p + L.layers[l].rot_p) * (L.cfg.f32 ? 4 : 2);
+    for (int l : L.order)
+        if (L.layers[l].own_kv()) b += (int64_t)(L.layers[l].rank_p + L.layers[l].rot_p) * (L.cfg.f32 ? 4 : 2);
     return b;
 }
 int64_t LatentModel::kv_read_bytes(int len) const {
@@ -339,6 +448,7 @@ int64_t LatentModel::kv_read_bytes(int len) const {
     int64_t b = 0;
     for (int l : L.order) {
         const LatentLayer& w = L.layers[l];
+        if (w.scan.on()) b += (int64_t)w.scan.state_bytes() * 2;  // read and written
         b += (int64_t)(w.rank_p + w.rot_p) * (L.cfg.f32 ? 4 : 2) * (w.c.window > 0 ? std::min(len, w.c.window) : len);
     }
     return b;
@@ -355,14 +465,25 @@ int LatentModel::kv_alloc(nvllm_model* m) {
     const size_t R = m->max_rows, R16 = (R + 15) / 16 * 16;
     L.cache.assign(L.order.size(), nullptr);
     for (size_t i = 0; i < L.order.size(); ++i) {
-        const LatentLayer& w = L.layers[L.order[i]];
+        LatentLayer& w = L.layers[L.order[i]];
+        if (w.scan.on()) {  // no cache; its state once, however often the layer runs
+            if (!w.scan.st) {
+                int e = w.scan.kv_alloc(m);
+                if (e) return e;
+            }
+            continue;
+        }
+        if (!w.own_kv()) { L.cache[i] = L.cache[w.c.kv_from]; continue; }  // no loop: run = layer
         const size_t bytes = (size_t)m->num_blocks * kBlockTokens * (w.rank_p + w.rot_p) * (f32 ? 4 : 2);
         HIPCHK(ctx, hipMalloc(&L.cache[i], bytes));
         HIPCHK(ctx, hipMemsetAsync(L.cache[i], 0, bytes, s));  // padding stays zero, unwritten tokens finite
     }
-    size_t nmax = L.ldr, q_row = 0, lat_row = 0, kc = 0, ffp = 0;
+    size_t nmax = L.ldr, q_row = 0, lat_row = 0, kc = 0, ffp = 0, kq = 0;
     for (const LatentLayer& w : L.layers) {
-        nmax = std::max<size_t>({nmax, (size_t)w.Nq, (size_t)2 * w.ff_p});
+        nmax = std::max<size_t>({nmax, (size_t)w.Nq, (size_t)w.Nd, (size_t)2 * w.ff_p, (size_t)w.scan.Nin, (size_t)w.scan.Nx, (size_t)w.experts.sh_p});
+        kq = std::max<size_t>(kq, w.Kq);
+        if (w.scan.on()) L.scan.reserve(w.scan, R);
+        if (w.experts.on()) L.experts.reserve(w.experts, R);
         q_row = std::max<size_t>(q_row, (size_t)w.heads * (w.dim_p + w.rot_p));
         lat_row = std::max<size_t>(lat_row, (size_t)w.heads * w.rank_p);
         kc = std::max<size_t>(kc, w.Kc);
@@ -380,6 +501,8 @@ int LatentModel::kv_alloc(nvllm_model* m) {
     if (!rc) rc = dmalloc(ctx, &L.slabs2, m->slab_floats);
     if (!rc) rc = dmalloc(ctx, &m->red, R * L.ldr);
     if (!rc) rc = dmalloc(ctx, &L.tap, R * L.ldr);
+    if (!rc) rc = L.experts.alloc(ctx, f32);
+    if (!rc) rc = L.scan.alloc(m, f32);
     if (!rc) rc = zalloc((void**)&L.q, R * q_row * 4);
     if (!rc) rc = zalloc((void**)&L.qlat, R * lat_row * 4);
     if (!rc) rc = zalloc((void**)&L.olat, R * lat_row * 4);
@@ -395,7 +518,9 @@ int LatentModel::kv_alloc(nvllm_model* m) {
         if (!rc) rc = zalloc((void**)&L.y2, R * L.Kw * 4);
         if (!rc) rc = zalloc((void**)&L.ctx_f, R * kc * 4);
         if (!rc && ffp) rc = zalloc((void**)&L.act_f, R * ffp * 4);
+        if (!rc && kq) rc = zalloc((void**)&L.cq_f, R * kq * 4);
     } else {
+        if (kq) for (bf16_bits** p : {&L.cqh, &L.cql}) if (!rc) rc = zalloc((void**)p, R16 * kq * 2);
         // activation planes are read in whole 16-row blocks; columns past a layer's own width meet zero weights
         for (bf16_bits** p : {&m->xh, &m->xl, &L.x2h, &L.x2l}) if (!rc) rc = zalloc((void**)p, R16 * L.Kw * 2);
         for (bf16_bits** p : {&m->ctxh, &m->ctxl}) if (!rc) rc = zalloc((void**)p, R16 * kc * 2);
@@ -417,16 +542,16 @@ int LatentModel::kv_alloc(nvllm_model* m) {
         if (!rc) HIPCHK(ctx, hipHostMalloc((void**)&L.h_exp, ((size_t)3 * L.exp_cap + R) * sizeof(int), hipHostMallocDefault));
     }
     if (rc) return rc;
-    // rotation tables, one per (base, dims): angle p * base^(-2i/dims)
+    // rotation tables, one per rotation: angle p * f_i
     m->rope_len = (int)std::min<int64_t>((int64_t)m->max_blocks * kBlockTokens, 1 << 20);
     for (RopeTable& t : L.ropes) {
         const int half = t.dims / 2;
         std::vector<float> hc((size_t)m->rope_len * half), hs(hc.size());
         for (int i = 0; i < half; ++i) {
-            const double f = std::pow(t.base, -2.0 * i / t.dims);
+            const double f = t.frequency(i), mag = t.magnitude();
             for (int p = 0; p < m->rope_len; ++p) {
-                hc[(size_t)p * half + i] = (float)std::cos(p * f);
-                hs[(size_t)p * half + i] = (float)std::sin(p * f);
+                hc[(size_t)p * half + i] = (float)(std::cos(p * f) * mag);
+                hs[(size_t)p * half + i] = (float)(std::sin(p * f) * mag);
             }
         }
         rc = dmalloc(ctx, &t.cos, hc.size());
@@ -446,10 +571,15 @@ int LatentModel::plan_chunk(nvllm_model* m, const int* pos, const int* slot, con
     LatentModel& L = latent(m);
     L.exp_n = 0;
     L.segments.clear();
+    if (qt != 1 && L.has_state) {
+        int rc = L.scan.plan(m, slot, seq, R);
+        if (rc) return rc;
+    }
     if (qt == 1 || !L.exp_cap || m->opt_latent_plain || m->opt_latent_absorb == 1) return NVLLM_OK;
     int widest = 0;  // <= 0: some layer sees everything
     bool all = false;
-    for (const LatentLayer& w : L.layers) { all |= w.c.window <= 0; widest = std::max(widest, w.c.window); }
+    for (const LatentLayer& w : L.layers)
+        if (!w.scan.on()) { all |= w.c.window <= 0; widest = std::max(widest, w.c.window); }
     int n = 0;
     int *h_slot = L.h_exp, *h_tile = L.h_exp + L.exp_cap, *h_pos0 = L.h_exp + 2 * L.exp_cap, *h_te = L.h_exp + 3 * L.exp_cap;
     int k = 0;  // q-tile
@@ -486,14 +616,16 @@ static bool latent_expanded_pays(const nvllm_model* m, const LatentLayer& w, int
     return expanded < absorbed;
 }
 
-static int latent_attention(nvllm_model* m, const LatentLayer& w, void* cache_data, const float* qkv, int n_slabs, int R, int n_tiles, int qt, int ctx_packed) {
+// first: slabs of the product the normed input met; with query latents the second product overwrites them
+static int latent_attention(nvllm_model* m, const LatentLayer& w, void* cache_data, float* first, int n_slabs, int R, int n_tiles, int qt, int ctx_packed) {
     nvllm_ctx* ctx = m->ctx;
     LatentModel& L = latent(m);
     hipStream_t s = ctx->stream;
     const bool f32 = L.cfg.f32 != 0;
     const int dq = w.dim_p + w.rot_p;
+    const float* qkv = first;
     LatentRowsArgs ra;
-    ra.qkv = qkv; ra.n_slabs = n_slabs; ra.ldq = w.Nq; ra.slab_stride = (int64_t)R * w.Nq;
+    ra.ldq = w.Nq; ra.slab_stride = (int64_t)R * w.Nq;
     ra.heads = w.heads; ra.dim = w.c.dim; ra.dim_p = w.dim_p;
     ra.scale = (float)(w.c.scale * 1.4426950408889634);
     ra.norm_w = w.dkv_norm; ra.eps = (float)L.cfg.norm_eps;
@@ -502,10 +634,25 @@ static int latent_attention(nvllm_model* m, const LatentLayer& w, void* cache_da
     ra.q = L.q;
     ra.cache = w.cache_shape();
     ra.cache.data = cache_data; ra.cache.f32 = f32;
+    ra.kv_slabs = n_slabs; ra.ldkv = w.c.q_rank ? w.Nd : w.Nq; ra.kv_stride = (int64_t)R * ra.ldkv;
+    if (w.own_kv()) ra.kv = first + (w.c.q_rank ? w.c.q_rank : w.heads * (w.c.dim + w.c.rot_dim));
+    if (w.c.q_rank) {
+        ProductPlan pq;
+        if (!f32) pq = plan_product(m, R, w.qkv);
+        QueryLatentArgs qa;
+        qa.in = first; qa.n_slabs = n_slabs; qa.ld = w.Nd; qa.slab_stride = ra.kv_stride; qa.rank = w.c.q_rank; qa.ldx = w.Kq; qa.norm_w = w.dq_norm; qa.eps = ra.eps;
+        qa.xh = L.cqh; qa.xl = L.cql; qa.y = L.cq_f; qa.packed = pq.packed;
+        PROF(m, PROF_QK, launch_query_latent(qa, ra, R, s));
+        ra.kv = nullptr;  // written
+        int rc = f32 ? exact_product(m, L.cq_f, w.qkv, first, R) : run_product(m, pq, L.cqh, L.cql, w.qkv, first, R, &n_slabs);
+        if (rc) return rc;
+        if (f32) n_slabs = 1;
+    }
+    ra.qkv = qkv; ra.n_slabs = n_slabs;
     const bool matrix_core = latent_attn_ok(ra.cache) && !m->opt_latent_plain;
     const bool fused = matrix_core && qt == 1 && !m->opt_no_fused && w.dim_p <= 1024;  // decode: the kernels around the attention in two launches
     const bool expanded = qt == 2 && latent_expanded_pays(m, w, R);
-    if (expanded) PROF(m, PROF_QK, launch_latent_cache(ra, R, s));
+    if (expanded) { if (ra.kv) PROF(m, PROF_QK, launch_latent_cache(ra, R, s)); }
     else if (!fused) PROF(m, PROF_QK, launch_latent_rows(ra, R, s));
     if (expanded) {
         LatentExpandArgs ea;
@@ -519,7 +666,7 @@ static int latent_attention(nvllm_model* m, const LatentLayer& w, void* cache_da
         pa.cos = ra.cos; pa.sin = ra.sin; pa.cache = ra.cache; pa.block_tables = m->d_block_tables; pa.max_blocks = m->max_blocks;
         pa.kx = L.kx; pa.vx = L.vx; pa.cap = L.exp_cap;
         pa.tile_row0 = m->d_tile_row0; pa.tile_nrows = m->d_tile_nrows; pa.tile_slot = m->d_tile_slot; pa.tile_exp = L.d_tile_exp;
-        pa.tile_order = m->d_tile_order; pa.pos = m->d_pos; pa.n_tiles = n_tiles; pa.heads = w.heads; pa.window = w.c.window;
+        pa.tile_order = m->d_tile_order; pa.pos = m->d_pos; pa.n_tiles = n_tiles; pa.heads = w.heads; pa.window = w.c.window; pa.sink = w.sink;
         pa.dim_p = w.dim_p; pa.vdim = w.c.vdim; pa.vdim_p = w.vdim_p; pa.oh = m->ctxh; pa.ol = m->ctxl; pa.ld = w.Kc; pa.packed = ctx_packed;
         PROF(m, PROF_ATTN, launch_latent_prefill(pa, s));
         ++m->latent_expanded;
@@ -541,7 +688,7 @@ static int latent_attention(nvllm_model* m, const LatentLayer& w, void* cache_da
     aa.cache = ra.cache; aa.block_tables = m->d_block_tables; aa.max_blocks = m->max_blocks;
     aa.tile_row0 = m->d_tile_row0; aa.tile_nrows = m->d_tile_nrows; aa.tile_slot = m->d_tile_slot; aa.pos = m->d_pos; aa.slot = m->d_slot;
     aa.single = qt == 1 && n_tiles == R;
-    aa.heads = w.heads; aa.window = w.c.window; aa.out = L.olat;
+    aa.heads = w.heads; aa.window = w.c.window; aa.sink = w.sink; aa.out = L.olat;
     int parts = 1;
     if (matrix_core) {
         if (fused && R <= m->max_seqs) {
@@ -581,15 +728,17 @@ int LatentModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
     const bool f32 = L.cfg.f32 != 0, tp = ctx->tp_size > 1;
     m->tap_rows = R;
     AddNormArgs base;  // the sum pending on the residual stream
+    base.center = L.cfg.norm == NVLLM_NORM_LAYER;
     base.W = L.cfg.width; base.ldr = L.ldr; base.ldx = L.Kw; base.eps = (float)L.cfg.norm_eps;
     base.ids = m->d_ids; base.embed = L.embed; base.embed_scale = (float)L.cfg.embed_scale;
     for (size_t run = 0; run < L.order.size(); ++run) {
-        const LatentLayer& w = L.layers[L.order[run]];
-        const GluSpec spec{(float)w.c.glu_limit, (float)w.c.glu_alpha, (float)w.c.glu_shift};
+        LatentLayer& w = L.layers[L.order[run]];
+        const bool gelu = w.c.glu == NVLLM_GLU_GELU;
+        const GluSpec spec{gelu ? 0.f : (float)w.c.glu_limit, (float)w.c.glu_alpha, (float)w.c.glu_shift, gelu};
         ProductPlan pq, po, pd;
         GluPlan pg;
         if (!f32) {
-            pq = plan_product(m, R, w.qkv);
+            pq = plan_product(m, R, w.first());
             po = plan_product(m, R, w.o);
             if (w.ff) {
                 pd = plan_product(m, R, w.down);
@@ -602,34 +751,47 @@ int LatentModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
         }
         AddNormArgs na = base;
         na.residual_out = m->resid;
-        na.w[0] = w.norm1; na.w[1] = w.ff ? w.norm2 : nullptr;
+        // the feed-forward's input: its own norm's output, or the mixer's where they share the norm (twice when the products want other orders)
+        const bool mlp = w.ff || w.experts.on(), same = L.cfg.one_norm && (f32 || w.experts.on() || pg.packed == pq.packed);
+        if (w.experts.on()) pg.packed = pq.packed;
+        na.w[0] = w.norm1; na.w[1] = !mlp || same ? nullptr : L.cfg.one_norm ? w.norm1 : w.norm2;
+        const float* y_ff = same ? L.y1 : L.y2;
+        const bf16_bits *ffh = same ? m->xh : L.x2h, *ffl = same ? m->xl : L.x2l;
         if (f32) { na.y[0] = L.y1; na.y[1] = L.y2; }
         else {
             na.xh[0] = m->xh; na.xl[0] = m->xl; na.packed[0] = pq.packed;
             na.xh[1] = L.x2h; na.xl[1] = L.x2l; na.packed[1] = pg.packed;
         }
         PROF(m, PROF_NORM, launch_add_norm(na, R, s));
-        int ns = 1, rc = f32 ? exact_product(m, L.y1, w.qkv, m->slabs, R) : run_product(m, pq, m->xh, m->xl, w.qkv, m->slabs, R, &ns);
-        if (!rc) rc = latent_attention(m, w, L.cache[run], m->slabs, ns, R, n_tiles, qt, po.packed);
+        int ns = 1, rc = f32 ? exact_product(m, L.y1, w.first(), m->slabs, R) : run_product(m, pq, m->xh, m->xl, w.first(), m->slabs, R, &ns);
+        if (!rc && w.scan.on()) rc = run_scan(m, w.scan, L.scan, m->slabs, ns, L.slabs2, R, qt, f32 ? L.ctx_f : nullptr, po.packed);
+        else if (!rc) rc = latent_attention(m, w, L.cache[run], m->slabs, ns, R, n_tiles, qt, po.packed);
         if (rc) return rc;
         int no = 1, nd = 1;
+        BranchSum ff;
+        if (w.experts.on()) {
+            rc = run_experts(m, w.experts, L.experts, ffh, ffl, pg.packed, f32 ? y_ff : nullptr, R, &ff);
+            if (rc) return rc;
+        }
         if (w.ff) {
             if (f32) {
-                rc = exact_product(m, L.y2, w.gu, m->slabs, R);
+                rc = exact_product(m, y_ff, w.gu, m->slabs, R);
                 if (rc) return rc;
                 PROF(m, PROF_SILU, launch_silu_mul_interleaved(m->slabs, 1, 0, R, w.ff_p, nullptr, nullptr, 0, s, spec, L.act_f));
                 rc = exact_product(m, L.act_f, w.down, L.slabs2, R);
             } else {
-                rc = run_glu(m, pg, L.x2h, L.x2l, w.gu, R, spec, m->xh2, m->xl2, pd.packed);
+                rc = run_glu(m, pg, ffh, ffl, w.gu, R, spec, m->xh2, m->xl2, pd.packed);
                 if (!rc) rc = run_product(m, pd, m->xh2, m->xl2, w.down, L.slabs2, R, &nd);
             }
             if (rc) return rc;
+            ff.in = L.slabs2; ff.n_slabs = nd; ff.slab_stride = (int64_t)R * L.ldr;
         }
         rc = f32 ? exact_product(m, L.ctx_f, w.o, m->slabs, R) : run_product(m, po, m->ctxh, m->ctxl, w.o, m->slabs, R, &no);
         if (rc) return rc;
         base.ids = nullptr;
         base.in = m->slabs; base.n_slabs = no; base.slab_stride = (int64_t)R * L.ldr;
-        base.in2 = w.ff ? L.slabs2 : nullptr; base.n_slabs2 = nd; base.slab_stride2 = (int64_t)R * L.ldr;
+        base.in2 = ff.in; base.n_slabs2 = ff.n_slabs; base.slab_stride2 = ff.slab_stride; base.in2_scale = ff.scale;
+        base.gather = ff.gather; base.gather_row = ff.gather_row; base.n_gather = ff.n_gather;
         base.residual_in = m->resid;
         if (tp) {  // both branches of the layer in one all-reduce
             AddNormArgs sum = base;
@@ -637,7 +799,7 @@ int LatentModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
             HIPCHK(ctx, launch_add_norm(sum, R, s));
             rc = comm_allreduce_sum(ctx, m->red, (size_t)R * L.ldr);
             if (rc) return rc;
-            base.in = m->red; base.n_slabs = 1; base.in2 = nullptr;
+            base.in = m->red; base.n_slabs = 1; base.in2 = nullptr; base.n_gather = 0;
         }
         if (m->taps) {  // residual stream after this run
             AddNormArgs t = base;

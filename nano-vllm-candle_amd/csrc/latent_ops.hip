@@ -8,13 +8,16 @@
 namespace nvllm {
 
 // ---------------------------------------------------------------------------------------------------
-// residual add + up to two RMSNorms of the same row; one workgroup per row, 4 columns per thread and step
+// residual add + up to two norms of the same row; one workgroup per row, 4 columns per thread and step
 // ---------------------------------------------------------------------------------------------------
 constexpr int kAddNormMax = 8192;  // widest row
 
+enum { NORM_PLAIN, NORM_POST, NORM_CENTER };
+
 // BS = 256, or 1024 for few wide rows (decode): every thread's loads are then in flight at once
-template <int BS, bool POST>
+template <int BS, int KIND>
 __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
+    constexpr bool POST = KIND == NORM_POST;
     constexpr int NV = kAddNormMax / 4 / BS;
     __shared__ float red[BS / 64];
     const int r = blockIdx.x;
@@ -33,7 +36,16 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
                                 bf16_to_f32(e.y & 0xffff) * a.embed_scale, bf16_to_f32(e.y >> 16) * a.embed_scale);
             } else {
                 if (a.in) add_slabs(s, a.in + (size_t)src * a.ldr + (size_t)i * 4, a.n_slabs, a.slab_stride);
-                if (a.in2) add_slabs(s, a.in2 + (size_t)src * a.ldr + (size_t)i * 4, a.n_slabs2, a.slab_stride2);
+                if (a.in2) {
+                    float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
+                    add_slabs(t, a.in2 + (size_t)src * a.ldr + (size_t)i * 4, a.n_slabs2, a.slab_stride2);
+                    const float f = a.in2_scale ? a.in2_scale[src] : 1.f;
+                    s.x += t.x * f; s.y += t.y * f; s.z += t.z * f; s.w += t.w * f;
+                }
+                for (int k = 0; k < a.n_gather; ++k) {
+                    const float4 t = *reinterpret_cast<const float4*>(a.gather + (size_t)a.gather_row[(size_t)src * a.n_gather + k] * a.ldr + (size_t)i * 4);
+                    s.x += t.x; s.y += t.y; s.z += t.z; s.w += t.w;
+                }
             }
             float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
             if (a.residual_in) t = *reinterpret_cast<const float4*>(a.residual_in + (size_t)src * a.ldr + (size_t)i * 4);
@@ -43,6 +55,21 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
                 if (a.residual_in) { s.x += t.x; s.y += t.y; s.z += t.z; s.w += t.w; }
                 if (a.residual_out) *reinterpret_cast<float4*>(a.residual_out + (size_t)src * a.ldr + (size_t)i * 4) = s;
             }
+            cache[c] = s;
+            ss += KIND == NORM_CENTER ? (s.x + s.y) + (s.z + s.w) : s.x * s.x + s.y * s.y + s.z * s.z + s.w * s.w;
+        }
+    }
+    if constexpr (KIND == NORM_CENTER) {
+        if (!a.w[0] && !a.w[1]) return;
+        const float mean = block_sum(ss, red, BS / 64) / (float)a.W;
+        ss = 0.f;
+#pragma unroll
+        for (int c = 0; c < NV; ++c) {
+            const int i = threadIdx.x + c * BS;
+            if (i >= nv4) continue;
+            float4 s = cache[c];
+            s.x = i * 4 < a.W ? s.x - mean : 0.f; s.y = i * 4 + 1 < a.W ? s.y - mean : 0.f;
+            s.z = i * 4 + 2 < a.W ? s.z - mean : 0.f; s.w = i * 4 + 3 < a.W ? s.w - mean : 0.f;
             cache[c] = s;
             ss += s.x * s.x + s.y * s.y + s.z * s.z + s.w * s.w;
         }
@@ -93,10 +120,11 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
 
 // prompt chunks whose outputs are planes in fragment order: one workgroup = 16 rows, lane (grp, l15) owns row l15's eight consecutive
 // columns of k-tiles wave, wave + 16, ...  Reads are whole 128-byte lines, every plane store one contiguous KiB per wave.
-template <int IT, bool POST>
+template <int IT, int KIND>
 __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, int rows) {
     constexpr int NW = 16;
-    __shared__ float red[POST ? 2 : 1][NW][16];
+    constexpr bool POST = KIND == NORM_POST;
+    __shared__ float red[KIND == NORM_PLAIN ? 1 : 2][NW][16];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, grp = lane >> 4;
     const int KT = a.ldr >> 5, row = blockIdx.x * 16 + l15, rowc = min(row, rows - 1);
     float v[IT][8];
@@ -113,13 +141,17 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
             s0 = make_float4(bf16_to_f32(e.x & 0xffff) * f, bf16_to_f32(e.x >> 16) * f, bf16_to_f32(e.y & 0xffff) * f, bf16_to_f32(e.y >> 16) * f);
             s1 = make_float4(bf16_to_f32(e.z & 0xffff) * f, bf16_to_f32(e.z >> 16) * f, bf16_to_f32(e.w & 0xffff) * f, bf16_to_f32(e.w >> 16) * f);
         } else {
-            auto add = [&](const float* p) {
+            auto add = [&](const float* p, float f = 1.f) {
                 const float4 t0 = *reinterpret_cast<const float4*>(p), t1 = *reinterpret_cast<const float4*>(p + 4);
-                s0.x += t0.x; s0.y += t0.y; s0.z += t0.z; s0.w += t0.w;
-                s1.x += t1.x; s1.y += t1.y; s1.z += t1.z; s1.w += t1.w;
+                s0.x += t0.x * f; s0.y += t0.y * f; s0.z += t0.z * f; s0.w += t0.w * f;
+                s1.x += t1.x * f; s1.y += t1.y * f; s1.z += t1.z * f; s1.w += t1.w * f;
             };
             if (a.in) for (int sl = 0; sl < a.n_slabs; ++sl) add(a.in + (size_t)sl * a.slab_stride + off);
-            if (a.in2) for (int sl = 0; sl < a.n_slabs2; ++sl) add(a.in2 + (size_t)sl * a.slab_stride2 + off);
+            if (a.in2) {
+                const float f = a.in2_scale ? a.in2_scale[rowc] : 1.f;
+                for (int sl = 0; sl < a.n_slabs2; ++sl) add(a.in2 + (size_t)sl * a.slab_stride2 + off, f);
+            }
+            for (int k = 0; k < a.n_gather; ++k) add(a.gather + (size_t)a.gather_row[(size_t)rowc * a.n_gather + k] * a.ldr + col);
             if (!POST && a.residual_in) add(a.residual_in + off);
         }
         if (!POST && a.residual_out && row < rows) {
@@ -129,9 +161,9 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
         v[i][0] = s0.x; v[i][1] = s0.y; v[i][2] = s0.z; v[i][3] = s0.w;
         v[i][4] = s1.x; v[i][5] = s1.y; v[i][6] = s1.z; v[i][7] = s1.w;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) ss += v[i][e] * v[i][e];
+        for (int e = 0; e < 8; ++e) ss += KIND == NORM_CENTER ? v[i][e] : v[i][e] * v[i][e];
     }
-    auto row_rinv = [&](float (&rd)[NW][16]) {
+    auto row_sum = [&](float (&rd)[NW][16]) {
         ss += __shfl_xor(ss, 16);
         ss += __shfl_xor(ss, 32);
         if (grp == 0) rd[wave][l15] = ss;
@@ -139,8 +171,23 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
         ss = 0.f;
 #pragma unroll
         for (int q = 0; q < NW; ++q) ss += rd[q][l15];
-        return 1.0f / sqrtf(ss / (float)a.W + a.eps);
+        return ss;
     };
+    auto row_rinv = [&](float (&rd)[NW][16]) { return 1.0f / sqrtf(row_sum(rd) / (float)a.W + a.eps); };
+    if constexpr (KIND == NORM_CENTER) {
+        const float mean = row_sum(red[1]) / (float)a.W;
+        ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < IT; ++i) {
+            const int kt = wave + i * NW;
+            if (kt >= KT) continue;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                v[i][e] = kt * 32 + grp * 8 + e < a.W ? v[i][e] - mean : 0.f;
+                ss += v[i][e] * v[i][e];
+            }
+        }
+    }
     if constexpr (POST) {
         const float f = row_rinv(red[1]) * a.post_mult;
         ss = 0.f;
@@ -195,21 +242,23 @@ hipError_t launch_add_norm(const AddNormArgs& a, int rows, hipStream_t s) {
     if (a.raw && a.w[0]) return hipErrorInvalidValue;
     bool packed = any && a.ldr == a.ldx && a.ldr % 32 == 0 && !a.row_idx && (!post || a.residual_in);
     for (int k = 0; k < 2; ++k) packed &= !(a.w[k] || (k == 0 && a.raw)) || (a.packed[k] && a.xh[k] && !a.y[k]);
+    if (a.center && (post || a.raw)) return hipErrorInvalidValue;
     auto launch = [&](auto P) {
-        constexpr bool POST = decltype(P)::value;
+        constexpr int KIND = decltype(P)::value;
         if (packed && rows >= 512 && a.ldr <= 4096) {
             const int kt = a.ldr / 32, tiles = (rows + 15) / 16;
-            if (kt <= 32) add_norm_rows16_kernel<2, POST><<<tiles, 1024, 0, s>>>(a, rows);
-            else if (kt <= 64) add_norm_rows16_kernel<4, POST><<<tiles, 1024, 0, s>>>(a, rows);
-            else add_norm_rows16_kernel<8, POST><<<tiles, 1024, 0, s>>>(a, rows);
+            if (kt <= 32) add_norm_rows16_kernel<2, KIND><<<tiles, 1024, 0, s>>>(a, rows);
+            else if (kt <= 64) add_norm_rows16_kernel<4, KIND><<<tiles, 1024, 0, s>>>(a, rows);
+            else add_norm_rows16_kernel<8, KIND><<<tiles, 1024, 0, s>>>(a, rows);
         } else if (rows <= 128 && a.ldr >= 2048) {
-            add_norm_kernel<1024, POST><<<rows, 1024, 0, s>>>(a);
+            add_norm_kernel<1024, KIND><<<rows, 1024, 0, s>>>(a);
         } else {
-            add_norm_kernel<256, POST><<<rows, 256, 0, s>>>(a);
+            add_norm_kernel<256, KIND><<<rows, 256, 0, s>>>(a);
         }
     };
-    if (post) launch(std::true_type{});
-    else launch(std::false_type{});
+    if (post) launch(std::integral_constant<int, NORM_POST>{});
+    else if (a.center) launch(std::integral_constant<int, NORM_CENTER>{});
+    else launch(std::integral_constant<int, NORM_PLAIN>{});
     return hipGetLastError();
 }
 
@@ -226,7 +275,7 @@ __device__ __forceinline__ void cache_put(const LatentCache& c, size_t block_bas
 __device__ __forceinline__ void latent_to_cache(const LatentRowsArgs& a, int row, int lane) {
     const LatentCache& c = a.cache;
     const int half = c.rot >> 1, pos = a.pos[row];
-    const float* in = a.qkv + (size_t)row * a.ldq + (size_t)a.heads * (a.dim + c.rot);
+    const float* in = a.kv + (size_t)row * a.ldkv;
     const float* cs = a.cos + (size_t)pos * half;
     const float* sn = a.sin + (size_t)pos * half;
     const int blk = a.block_tables[(size_t)a.slot[row] * a.max_blocks + (pos / kBlockTokens)];
@@ -240,16 +289,16 @@ __device__ __forceinline__ void latent_to_cache(const LatentRowsArgs& a, int row
             v[i] = in[d];
             w[i] = a.norm_w[d];
         }
-        for (int sl0 = 1; sl0 < a.n_slabs; sl0 += 4) {
+        for (int sl0 = 1; sl0 < a.kv_slabs; sl0 += 4) {
             float t[4][8];
 #pragma unroll
             for (int u = 0; u < 4; ++u)
 #pragma unroll
-                for (int i = 0; i < 8; ++i) t[u][i] = in[(size_t)min(sl0 + u, a.n_slabs - 1) * a.slab_stride + min(lane + i * 64, c.rank - 1)];
+                for (int i = 0; i < 8; ++i) t[u][i] = in[(size_t)min(sl0 + u, a.kv_slabs - 1) * a.kv_stride + min(lane + i * 64, c.rank - 1)];
 #pragma unroll
             for (int u = 0; u < 4; ++u)
 #pragma unroll
-                for (int i = 0; i < 8; ++i) v[i] += sl0 + u < a.n_slabs ? t[u][i] : 0.f;
+                for (int i = 0; i < 8; ++i) v[i] += sl0 + u < a.kv_slabs ? t[u][i] : 0.f;
         }
 #pragma unroll
         for (int i = 0; i < 8; ++i) ss += lane + i * 64 < c.rank ? v[i] * v[i] : 0.f;
@@ -260,14 +309,14 @@ __device__ __forceinline__ void latent_to_cache(const LatentRowsArgs& a, int row
     } else {
         float ss = 0.f;
         for (int d = lane; d < c.rank; d += 64) {
-            const float v = slab_elem(in + d, a.n_slabs, a.slab_stride);
+            const float v = slab_elem(in + d, a.kv_slabs, a.kv_stride);
             ss += v * v;
         }
         const float rinv = 1.0f / sqrtf(wave_sum(ss) / (float)c.rank + a.eps);
-        for (int d = lane; d < c.rank; d += 64) cache_put(c, base, t, d, slab_elem(in + d, a.n_slabs, a.slab_stride) * rinv * a.norm_w[d]);
+        for (int d = lane; d < c.rank; d += 64) cache_put(c, base, t, d, slab_elem(in + d, a.kv_slabs, a.kv_stride) * rinv * a.norm_w[d]);
     }
     for (int i = lane; i < half; i += 64) {
-        const float u = slab_elem(in + c.rank + i, a.n_slabs, a.slab_stride), v = slab_elem(in + c.rank + half + i, a.n_slabs, a.slab_stride);
+        const float u = slab_elem(in + c.rank + i, a.kv_slabs, a.kv_stride), v = slab_elem(in + c.rank + half + i, a.kv_slabs, a.kv_stride);
         cache_put(c, base, t, c.rank_p + i, u * cs[i] - v * sn[i]);
         cache_put(c, base, t, c.rank_p + half + i, v * cs[i] + u * sn[i]);
     }
@@ -276,7 +325,7 @@ __device__ __forceinline__ void latent_to_cache(const LatentRowsArgs& a, int row
 __global__ void __launch_bounds__(256) latent_rows_kernel(LatentRowsArgs a) {
     const int lane = threadIdx.x & 63;
     const int row = blockIdx.x, head = blockIdx.y * 4 + (threadIdx.x >> 6);
-    if (head > a.heads) return;
+    if (head > a.heads || (head == a.heads && !a.kv)) return;
     const LatentCache& c = a.cache;
     const int rot = c.rot, half = rot >> 1, pos = a.pos[row];
     const float* in = a.qkv + (size_t)row * a.ldq + (size_t)head * (a.dim + rot);
@@ -333,6 +382,60 @@ hipError_t launch_latent_cache(const LatentRowsArgs& a, int rows, hipStream_t s)
     if (a.cache.rot % 2 || a.cache.rank_p % 32 || a.cache.rot_p % 32) return hipErrorInvalidValue;
     if (rows <= 0) return hipSuccess;
     latent_cache_kernel<<<(rows + 3) / 4, 256, 0, s>>>(a, rows);
+    return hipGetLastError();
+}
+
+__global__ void __launch_bounds__(256) query_latent_kernel(QueryLatentArgs a, LatentRowsArgs kv) {
+    __shared__ float red[4];
+    const int row = blockIdx.x;
+    if (blockIdx.y) {
+        if (threadIdx.x < 64) latent_to_cache(kv, row, threadIdx.x);
+        return;
+    }
+    const float* in = a.in + (size_t)row * a.ld;
+    auto four = [&](int c) {
+        f32x4 v = {0.f, 0.f, 0.f, 0.f};
+        if (c + 4 <= a.rank && ((a.ld | a.slab_stride) & 3) == 0) {
+            float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
+            add_slabs(t, in + c, a.n_slabs, a.slab_stride);
+            v = f32x4{t.x, t.y, t.z, t.w};
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (c + e < a.rank) v[e] = slab_elem(in + c + e, a.n_slabs, a.slab_stride);
+        }
+        return v;
+    };
+    auto put = [&](int c, f32x4 v, float rinv) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = c + e < a.rank ? (v[e] * rinv) * a.norm_w[c + e] : 0.f;
+        if (a.y) *reinterpret_cast<float4*>(a.y + (size_t)row * a.ldx + c) = make_float4(v[0], v[1], v[2], v[3]);
+        if (a.xh) put_planes4(a.xh, a.xl, row, c, 4, a.ldx, a.packed, v);
+    };
+    constexpr int NV = 4;  // ranks up to 4096 stay in registers
+    f32x4 v[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = (threadIdx.x + i * 256) * 4;
+        v[i] = c < a.rank ? four(c) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss += v[i][e] * v[i][e];
+    }
+    for (int c = (threadIdx.x + NV * 256) * 4; c < a.rank; c += 1024) {
+        const f32x4 t = four(c);
+        ss += (t[0] * t[0] + t[1] * t[1]) + (t[2] * t[2] + t[3] * t[3]);
+    }
+    const float rinv = 1.0f / sqrtf(block_sum(ss, red, 4) / (float)a.rank + a.eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+        if ((int)(threadIdx.x + i * 256) * 4 < a.ldx) put((threadIdx.x + i * 256) * 4, v[i], rinv);
+    for (int c = (threadIdx.x + NV * 256) * 4; c < a.ldx; c += 1024) put(c, c < a.rank ? four(c) : f32x4{0.f, 0.f, 0.f, 0.f}, rinv);
+}
+hipError_t launch_query_latent(const QueryLatentArgs& a, const LatentRowsArgs& kv, int rows, hipStream_t s) {
+    if (a.rank < 1 || a.rank > a.ld || a.ldx < a.rank || a.ldx % 32 || (!a.xh && !a.y) || kv.cache.rot % 2 || kv.cache.rank_p % 32 || kv.cache.rot_p % 32) return hipErrorInvalidValue;
+    if (rows <= 0) return hipSuccess;
+    query_latent_kernel<<<dim3(rows, kv.kv ? 2 : 1), 256, 0, s>>>(a, kv);
     return hipGetLastError();
 }
 
@@ -413,11 +516,13 @@ __global__ void __launch_bounds__(256) head_gemm_kernel(HeadGemmArgs a) {
             const int row = m0 + b * 16 + l15;
             if (row >= a.M) continue;
             f32x4 v = acc[n][b];
-            if (a.decay_rate) {
+            if (a.decay_bias) {
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    if (head == 0) {
-                        const int f = min(f0 + r, a.n_valid - 1);
+                    const int f = min(f0 + r, a.n_valid - 1);
+                    if (!a.decay_rate) {
+                        v[r] = softplusf(v[r] + a.decay_bias[f]);
+                    } else if (head == 0) {
                         v[r] = expf(-a.decay_rate[f] * softplusf(v[r] + a.decay_bias[f]));
                     } else {
                         v[r] = 1.0f / (1.0f + expf(-v[r]));
@@ -501,7 +606,7 @@ __global__ void __launch_bounds__(256) latent_query_kernel(LatentRowsArgs a, con
         if (blockIdx.z) return;
         const int q = head - a.heads;
         if (q < 4) {
-            if (q * 4 + wave < nr) latent_to_cache(a, r0 + q * 4 + wave, lane);
+            if (a.kv && q * 4 + wave < nr) latent_to_cache(a, r0 + q * 4 + wave, lane);
             return;
         }
         const int half = c.rot >> 1, per = c.rot_p - half, i = (q - 4) * 256 + (int)threadIdx.x;  // one pair (or one padding zero) per thread
@@ -587,6 +692,10 @@ __global__ void __launch_bounds__(256) latent_values_kernel(LatentAttnArgs a, co
         }
 #pragma unroll
         for (int o = 1; o < 16; o <<= 1) ms = fmaxf(ms, __shfl_xor(ms, o));
+        if (a.sink) {
+            ms = fmaxf(ms, a.sink[head]);
+            if (q == 0) lt = exp2f(a.sink[head] - ms);
+        }
 #pragma unroll
         for (int i = 0; i < kLatentMaxParts / 16; ++i) lt += l[i] * exp2f(m[i] - ms);
 #pragma unroll
@@ -701,6 +810,10 @@ __global__ void __launch_bounds__(256) latent_attn_plain_kernel(LatentAttnArgs a
     __syncthreads();
     float ms = -1e30f, lt = 0.f, f[4];
     for (int w = 0; w < 4; ++w) ms = fmaxf(ms, sh[(size_t)w * (c.rank_p + 2)]);
+    if (a.sink) {
+        ms = fmaxf(ms, a.sink[head]);
+        lt = exp2f(a.sink[head] - ms);
+    }
     for (int w = 0; w < 4; ++w) {
         f[w] = exp2f(sh[(size_t)w * (c.rank_p + 2)] - ms);
         lt += f[w] * sh[(size_t)w * (c.rank_p + 2) + 1];

@@ -307,7 +307,11 @@ __global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatentPrefillArg
         l += __shfl_xor(l, 16);
         l += __shfl_xor(l, 32);
         if (my_pos[s] < 0) continue;
-        const float inv = 1.0f / l;
+        float inv = 1.0f / l;
+        if (a.sink) {
+            const float sk = a.sink[head], mn = fmaxf(m[s], sk), f = __builtin_amdgcn_exp2f(m[s] - mn);
+            inv = f / (l * f + __builtin_amdgcn_exp2f(sk - mn));
+        }
         const int row = row0 + wave * 32 + s * 16 + l15;
 #pragma unroll
         for (int d = 0; d < VT; ++d) {

@@ -1,0 +1,304 @@
+// gfx950 kernels of routed feed-forwards: choice of experts, grouping of rows, products over groups.
+#include <algorithm>
+
+#include "device_common.h"
+#include "moe.h"
+
+namespace nvllm {
+
+// ---------------------------------------------------------------------------------------------------
+// choice: one wave per row; lane l holds the logits of experts l, l + 64, ...
+// ---------------------------------------------------------------------------------------------------
+__device__ __forceinline__ float sigmoid_exact(float x) { return 1.0f / (1.0f + expf(-x)); }
+
+template <int NV>
+__device__ __forceinline__ void route_row(const RouteArgs& a, int row, int lane) {
+    const float* z = a.z + (size_t)row * a.ld;
+    float v[NV];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int e = lane + i * 64;
+        const float x = z[min(e, a.experts - 1)];
+        v[i] = e < a.experts ? x : -INFINITY;
+    }
+    if (a.gate_col >= 0 && lane == 0) a.gate[row] = sigmoid_exact(z[a.gate_col]);
+    for (int k = 0; k < a.top; ++k) {
+        float best = -INFINITY;
+        int at = kMaxExperts;  // the lowest index wins a tie
+#pragma unroll
+        for (int i = 0; i < NV; ++i)
+            if (v[i] > best) { best = v[i]; at = lane + i * 64; }
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) {
+            const float b = __shfl_xor(best, o);
+            const int c = __shfl_xor(at, o);
+            if (b > best || (b == best && c < at)) { best = b; at = c; }
+        }
+        at = min(at, a.experts - 1);  // no finite logit left
+        if (lane == 0) {
+            a.chosen[(size_t)row * a.top + k] = at;
+            a.score[(size_t)row * a.top + k] = sigmoid_exact(best);
+        }
+#pragma unroll
+        for (int i = 0; i < NV; ++i)
+            if (at == lane + i * 64) v[i] = -INFINITY;
+    }
+}
+template <int NV>
+__global__ void __launch_bounds__(256) route_kernel(RouteArgs a) {
+    const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (row < a.rows) route_row<NV>(a, row, threadIdx.x & 63);
+}
+
+// one workgroup: group sizes, starts and every row's position; NV > 0: the choice as well (few rows)
+template <int NV>
+__global__ void __launch_bounds__(1024) group_rows_kernel(RouteArgs a) {
+    __shared__ int count[kMaxExperts + 1], start[kMaxExperts + 1], wave_total[16];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int groups = a.experts + a.shared_group, n = a.rows * a.top;
+    for (int g = tid; g <= kMaxExperts; g += 1024) count[g] = 0;
+    if constexpr (NV > 0)
+        for (int row = wave; row < a.rows; row += 16) route_row<NV>(a, row, lane);
+    __syncthreads();
+    for (int i = tid; i < n; i += 1024) atomicAdd(&count[a.chosen[i]], 1);
+    if (a.shared_group && tid == 0) count[a.experts] = a.rows;
+    __syncthreads();
+    // exclusive prefix sum of the aligned sizes: two groups per thread (groups <= 1025: the last thread takes the odd one)
+    const int g0 = tid, sz = g0 < groups ? (count[g0] + a.align - 1) / a.align * a.align : 0;
+    int inc = sz;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+        const int t = __shfl_up(inc, o);
+        if (lane >= o) inc += t;
+    }
+    if (lane == 63) wave_total[wave] = inc;
+    __syncthreads();
+    int base = 0, all = 0;
+    for (int w = 0; w < 16; ++w) {
+        if (w < wave) base += wave_total[w];
+        all += wave_total[w];
+    }
+    if (g0 < groups) start[g0] = base + inc - sz;
+    if (groups > 1024 && tid == 0) start[1024] = all;  // the shared group after 1024 experts
+    __syncthreads();
+    const int end = groups > 1024 ? all + (count[1024] + a.align - 1) / a.align * a.align : all;
+    for (int g = tid; g < groups; g += 1024) {
+        const int p0 = start[g], c = count[g], p1 = p0 + (c + a.align - 1) / a.align * a.align;
+        for (int t = p0 / a.align; t < p1 / a.align; ++t) a.tile_group[t] = g;
+        for (int p = p0 + c; p < p1; ++p) { a.src[p] = -1; a.pre[p] = 0.f; a.post[p] = 0.f; }
+    }
+    for (int t = end / a.align + tid; t < a.cap / a.align; t += 1024) a.tile_group[t] = -1;
+    __syncthreads();
+    const int per = a.top + a.shared_group;
+    for (int g = tid; g <= kMaxExperts; g += 1024) count[g] = 0;
+    __syncthreads();
+    for (int i = tid; i < n; i += 1024) {
+        const int g = a.chosen[i], row = i / a.top, k = i - row * a.top, p = start[g] + atomicAdd(&count[g], 1);
+        const float sc = a.score[i];
+        a.src[p] = row;
+        a.pre[p] = a.weight_in ? sc : 1.f;
+        a.post[p] = a.weight_in ? 1.f : sc;
+        a.place[(size_t)row * per + k] = p;
+    }
+    if (a.shared_group)
+        for (int row = tid; row < a.rows; row += 1024) {
+            const int p = start[a.experts] + row;
+            a.src[p] = row;
+            a.pre[p] = 1.f;
+            a.post[p] = a.gate_col >= 0 ? a.gate[row] : 1.f;
+            a.place[(size_t)row * per + a.top] = p;
+        }
+}
+
+hipError_t launch_route(const RouteArgs& a, hipStream_t s) {
+    const int64_t need = (int64_t)a.rows * a.top + (int64_t)std::min(a.experts, a.rows * a.top) * (a.align - 1) + (a.shared_group ? a.rows + a.align - 1 : 0);
+    if (a.experts < 1 || a.experts > kMaxExperts || a.top < 1 || a.top > std::min(a.experts, kMaxTop) || a.align < 1 || a.cap % a.align || need > a.cap ||
+        a.ld < a.experts || a.gate_col >= a.ld || (a.gate_col >= 0 && !a.gate))
+        return hipErrorInvalidValue;
+    if (a.rows <= 0) return hipSuccess;
+    const bool one = a.rows <= 64;
+    const int nv = (a.experts + 63) / 64;
+#define NVLLM_RT(V_)                                                        \
+    if (one) group_rows_kernel<V_><<<1, 1024, 0, s>>>(a);                   \
+    else {                                                                  \
+        route_kernel<V_><<<(a.rows + 3) / 4, 256, 0, s>>>(a);               \
+        group_rows_kernel<0><<<1, 1024, 0, s>>>(a);                         \
+    }
+    if (nv <= 1) { NVLLM_RT(1) }
+    else if (nv <= 2) { NVLLM_RT(2) }
+    else if (nv <= 4) { NVLLM_RT(4) }
+    else if (nv <= 8) { NVLLM_RT(8) }
+    else { NVLLM_RT(16) }
+#undef NVLLM_RT
+    return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------------------------------
+// products over groups: MT m-tiles (16 positions each) of one group x NT n-tiles per wave; the four waves take other n-tiles (WK = 1)
+// or a quarter of K each, summed through LDS (WK = 4: few rows, many weight bytes)
+// ---------------------------------------------------------------------------------------------------
+template <int MT, int NT, int WK, bool EXACT>
+__global__ void __launch_bounds__(256) group_gemm_kernel(GroupGemmArgs a) {
+    __shared__ __attribute__((aligned(16))) f32x4 part[WK == 4 ? 4 * NT * MT * 64 : 1];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int l15 = lane & 15, grp = lane >> 4;
+    const int tile = blockIdx.y, g = a.tile_group ? a.tile_group[tile] : 0;
+    if (g < 0) return;
+    const bool other = g == a.last;
+    const int ntiles = (other ? a.Ns : a.N) >> 4, KT = (other ? a.Ks : a.K) >> 5;
+    const int nt0 = WK == 4 ? (int)blockIdx.x * NT : ((int)blockIdx.x * 4 + wave) * NT;
+    if (nt0 >= ntiles) return;  // WK = 4: the whole workgroup
+    const uint4* wp = other ? a.ws : a.w + (size_t)g * a.w_group;
+    const int per = WK == 4 ? (KT + 3) / 4 : KT, k0 = WK == 4 ? wave * per : 0, k1 = min(KT, k0 + per);
+    const int p0 = tile * (MT * 16);
+    // this lane's row of every m-tile (padding positions: row 0, result multiplied by 0 or never read)
+    const int KX = a.ldx >> 5;
+    size_t xo[MT], step;
+#pragma unroll
+    for (int b = 0; b < MT; ++b) {
+        const int p = p0 + b * 16 + l15;
+        int row = a.src ? a.src[p] : p;
+        row = min(max(row, 0), a.x_rows - 1);
+        if constexpr (EXACT) xo[b] = (size_t)row * a.ldx + grp * 8;
+        else xo[b] = a.x_packed ? ((size_t)(row >> 4) * KX * 64 + (grp << 4) + (row & 15)) : ((size_t)row * a.ldx >> 3) + grp;
+    }
+    step = EXACT ? 32 : a.x_packed ? 64 : 4;
+    f32x4 acc[NT][MT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+#pragma unroll
+        for (int b = 0; b < MT; ++b) acc[n][b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const uint4 *xh = reinterpret_cast<const uint4*>(a.xh), *xl = reinterpret_cast<const uint4*>(a.xl);
+    constexpr int U = EXACT ? 1 : MT == 1 ? 4 : 1;  // k-tiles in flight
+    for (int kt0 = k0; kt0 < k1; kt0 += U) {
+        uint4 wf[U][NT];
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+            for (int n = 0; n < NT; ++n) wf[u][n] = wp[((size_t)min(nt0 + n, ntiles - 1) * KT + min(kt0 + u, k1 - 1)) * 64 + lane];
+        if constexpr (EXACT) {
+            float xv[MT][8];
+#pragma unroll
+            for (int b = 0; b < MT; ++b) {
+                *reinterpret_cast<float4*>(&xv[b][0]) = *reinterpret_cast<const float4*>(a.xf + xo[b] + (size_t)kt0 * step);
+                *reinterpret_cast<float4*>(&xv[b][4]) = *reinterpret_cast<const float4*>(a.xf + xo[b] + (size_t)kt0 * step + 4);
+            }
+#pragma unroll
+            for (int n = 0; n < NT; ++n) {
+                const uint32_t wd[4] = {wf[0][n].x, wf[0][n].y, wf[0][n].z, wf[0][n].w};
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    const float wv = (j & 1) ? __builtin_bit_cast(float, wd[j >> 1] & 0xffff0000u) : __builtin_bit_cast(float, wd[j >> 1] << 16);
+#pragma unroll
+                    for (int b = 0; b < MT; ++b) acc[n][b] = __builtin_amdgcn_mfma_f32_16x16x4f32(wv, xv[b][j], acc[n][b], 0, 0, 0);
+                }
+            }
+        } else {
+            uint4 fh[U][MT], fl[U][MT];
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+#pragma unroll
+                for (int b = 0; b < MT; ++b) {
+                    const size_t o = xo[b] + (size_t)min(kt0 + u, k1 - 1) * step;
+                    fh[u][b] = xh[o];
+                    fl[u][b] = xl[o];
+                }
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+                if (kt0 + u < k1) {
+#pragma unroll
+                    for (int n = 0; n < NT; ++n) {
+                        const bf16x8 wv = __builtin_bit_cast(bf16x8, wf[u][n]);
+#pragma unroll
+                        for (int b = 0; b < MT; ++b) {
+                            acc[n][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv, __builtin_bit_cast(bf16x8, fh[u][b]), acc[n][b], 0, 0, 0);
+                            acc[n][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv, __builtin_bit_cast(bf16x8, fl[u][b]), acc[n][b], 0, 0, 0);
+                        }
+                    }
+                }
+        }
+    }
+    if constexpr (WK == 4) {
+#pragma unroll
+        for (int n = 0; n < NT; ++n)
+#pragma unroll
+            for (int b = 0; b < MT; ++b) part[((wave * NT + n) * MT + b) * 64 + lane] = acc[n][b];
+        __syncthreads();
+    }
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+        if (nt0 + n >= ntiles) continue;
+        const int f = (nt0 + n) * 16 + grp * 4;
+#pragma unroll
+        for (int b = 0; b < MT; ++b) {
+            f32x4 v = acc[n][b];
+            if constexpr (WK == 4) {
+                if ((n * MT + b) % 4 != wave) continue;
+                v = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int q = 0; q < 4; ++q) {
+                    const f32x4 t = part[((q * NT + n) * MT + b) * 64 + lane];
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) v[r] += t[r];
+                }
+            }
+            const int p = p0 + b * 16 + l15;
+            if (!a.tile_group && p >= a.x_rows) continue;
+            const float pre = a.pre ? a.pre[p] : 1.f, post = a.post ? a.post[p] : 1.f;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                v[r] *= pre;
+                if (a.relu2) v[r] = relu2(v[r]);
+                v[r] *= post;
+            }
+            if (a.out) *reinterpret_cast<float4*>(a.out + (size_t)p * a.ldo + f) = make_float4(v[0], v[1], v[2], v[3]);
+            if (a.oh) put_planes4(a.oh, a.ol, p, f, 4, a.ldo, 1, v);
+        }
+    }
+}
+
+hipError_t launch_group_gemm(const GroupGemmArgs& a, hipStream_t s) {
+    const bool exact = a.xf != nullptr;
+    const int nmax = a.last >= 0 ? std::max(a.N, a.Ns) : a.N, kmax = a.last >= 0 ? std::max(a.K, a.Ks) : a.K;
+    if (a.N % 16 || a.K % 32 || (a.last >= 0 && (a.Ns % 16 || a.Ks % 32 || !a.ws)) || a.ldx % 32 || a.ldx < kmax || (!exact && (!a.xh || !a.xl)) ||
+        (!a.out && !a.oh) || a.ldo < nmax || a.ldo % (a.oh ? 32 : 4) || a.x_rows < 1 || (a.align != 16 && a.align != 64))
+        return hipErrorInvalidValue;
+    const int tiles = a.tile_group ? a.tiles : (a.x_rows + a.align - 1) / a.align;
+    if (tiles <= 0) return hipSuccess;
+    const int nt = nmax / 16;
+#define NVLLM_GG(MT_, NT_, WK_, EX_) group_gemm_kernel<MT_, NT_, WK_, EX_><<<dim3((nt + NT_ * (WK_ == 4 ? 1 : 4) - 1) / (NT_ * (WK_ == 4 ? 1 : 4)), tiles), 256, 0, s>>>(a)
+    if (a.align == 64) {
+        if (exact) NVLLM_GG(4, 1, 1, true);
+        else NVLLM_GG(4, 2, 1, false);
+    } else {
+        if (exact) NVLLM_GG(1, 1, 4, true);
+        else NVLLM_GG(1, 2, 4, false);
+    }
+#undef NVLLM_GG
+    return hipGetLastError();
+}
+
+__global__ void __launch_bounds__(256) gather_planes_kernel(const uint4* __restrict__ xh, const uint4* __restrict__ xl, int packed, const int* __restrict__ src, int K,
+                                                            uint4* __restrict__ oh, uint4* __restrict__ ol) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, KT = K >> 5, grp = lane >> 4;
+    const int row = src[blockIdx.x * 16 + (lane & 15)];
+    const int rc = max(row, 0);
+    const size_t x0 = packed ? (size_t)(rc >> 4) * KT * 64 + (grp << 4) + (rc & 15) : ((size_t)rc * K >> 3) + grp;
+    const size_t step = packed ? 64 : 4, o0 = (size_t)blockIdx.x * KT * 64 + lane;
+    for (int kt = blockIdx.y * 4 + wave; kt < KT; kt += 4 * gridDim.y) {
+        uint4 h = xh[x0 + kt * step], l = xl[x0 + kt * step];
+        if (row < 0) h = l = make_uint4(0, 0, 0, 0);
+        oh[o0 + (size_t)kt * 64] = h;
+        ol[o0 + (size_t)kt * 64] = l;
+    }
+}
+hipError_t launch_gather_planes(const bf16_bits* xh, const bf16_bits* xl, int packed, const int* src, int positions, int K, bf16_bits* oh, bf16_bits* ol,
+                                hipStream_t s) {
+    if (K % 32 || positions % 16) return hipErrorInvalidValue;
+    if (positions <= 0) return hipSuccess;
+    gather_planes_kernel<<<dim3(positions / 16, std::max(1, std::min(K / 128, 4))), 256, 0, s>>>(reinterpret_cast<const uint4*>(xh), reinterpret_cast<const uint4*>(xl), packed, src, K,
+                                                                                              reinterpret_cast<uint4*>(oh), reinterpret_cast<uint4*>(ol));
+    return hipGetLastError();
+}
+
+}  // namespace nvllm

@@ -5,11 +5,13 @@ import os
 from .berevik import BerevikForCausalLM
 from .gopunex import GopunexForCausalLM
 from .qwen3 import Qwen3ForCausalLM
+from .tafopel import TafopelForCausalLM
 
 MODELS = {
     "Berevik": BerevikForCausalLM,
     "Gopunex": GopunexForCausalLM,
     "Qwen3ForCausalLM": Qwen3ForCausalLM,
+    "Tafopel": TafopelForCausalLM,
 }
 
 
