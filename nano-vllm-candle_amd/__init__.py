@@ -10,8 +10,10 @@ from .causal_lm import CausalLM  # noqa: F401
 from .gopunex import GopunexConfig, GopunexForCausalLM  # noqa: F401
 from .qwen3 import Qwen3Config, Qwen3ForCausalLM  # noqa: F401
 from .registry import MODELS, load_model  # noqa: F401
+from .tafopel import TafopelConfig, TafopelForCausalLM  # noqa: F401
 from .tp import TPConfig, get_tp  # noqa: F401
 
 __all__ = ["Context", "DeviceArray", "Qwen3Config", "Qwen3ForCausalLM", "Qwen3ModelRunner", "LLMEngine", "Scheduler",
            "SchedulerConfig", "SamplingParams", "Sequence", "ModelRunner", "TPConfig", "get_tp", "CausalLM", "BerevikConfig",
-           "BerevikForCausalLM", "GopunexConfig", "GopunexForCausalLM", "CausalLMRunner", "MODELS", "load_model"]
+           "BerevikForCausalLM", "GopunexConfig", "GopunexForCausalLM", "TafopelConfig",
+           "TafopelForCausalLM", "CausalLMRunner", "MODELS", "load_model"]

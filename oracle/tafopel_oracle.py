@@ -232,3 +232,14 @@ def random_weights(cfg, seed=0):
 def bf16(a):
     u = np.ascontiguousarray(a, np.float32).view(np.uint32)
     return ((u + 0x7FFF + ((u >> 16) & 1)) & 0xFFFF0000).astype(np.uint32).view(np.float32).reshape(np.shape(a))
+
+
+def greedy(cfg, w, prompt, n):
+    """(ids, logits rows) of n greedy tokens, the whole sequence run again for each"""
+    toks, ids, rows = list(prompt), [], []
+    for _ in range(n):
+        r = run(cfg, w, toks)[0][-1]
+        rows.append(r)
+        ids.append(int(len(r) - 1 - np.argmax(r[::-1])))  # the last of equal maxima
+        toks.append(ids[-1])
+    return ids, rows
