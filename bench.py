@@ -73,6 +73,12 @@ def parse():
     ap.add_argument("--berevik-window", type=int, default=1 << 20, help="attention window of the --berevik layers")
     ap.add_argument("--berevik-batch", type=int, default=64)
     ap.add_argument("--berevik-prompt", type=int, default=1024)
+    ap.add_argument("--tafopel", nargs="*", metavar="SIZE", default=None,
+                    help="instead of the headline: the Tafopel design beside the closest designs at equal size (bench_tafopel.py; sizes 1k 2k 4k, default all)")
+    ap.add_argument("--tafopel-kinds", nargs="+", default=None, help="attention, scan, experts, mixed (default all)")
+    ap.add_argument("--tafopel-batch", type=int, default=64)
+    ap.add_argument("--tafopel-prompt", type=int, default=1024)
+    ap.add_argument("--tafopel-alone", action="store_true", help="without the other designs")
     ap.add_argument("--gopunex", nargs="*", metavar="SIZE", default=None,
                     help="instead of the headline: the Gopunex design beside Qwen3 layers of equal size (bench_gopunex.py; sizes 1k 2k 4k, default all)")
     ap.add_argument("--gopunex-mixers", nargs="+", default=None, help="attention, channel_delta, lightning, mixed (default all)")
@@ -332,6 +338,11 @@ def live_traffic(a, dom_kernel):
 
 def main():
     a = parse()
+    if a.tafopel is not None:
+        import bench_tafopel
+
+        bench_tafopel.main(a.tafopel or None, batch=a.tafopel_batch, prompt=a.tafopel_prompt, kinds=a.tafopel_kinds or bench_tafopel.KINDS, with_twins=not a.tafopel_alone)
+        return
     if a.gopunex is not None:
         import bench_gopunex
 
