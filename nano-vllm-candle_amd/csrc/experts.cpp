@@ -3,10 +3,10 @@
 
 #include <algorithm>
 
-int ExpertsBlock::create(nvllm_ctx* ctx, int experts_, int top_, int ff_, int shared_, int W_, int Kw_, int ldr_) {
+int ExpertsBlock::create(nvllm_ctx* ctx, int experts_, int top_, int ff_, int shared_, int W_, int Kw_, int ldr_, bool f32) {
     const int tp = ctx->tp_size;
     experts = experts_; top = top_; ff_all = ff_; shared_all = shared_; W = W_; Kw = Kw_; ldr = ldr_;
-    ff = ff_all / tp; sh = shared_all / tp; ff_p = up(ff, 128); sh_p = sh ? up(sh, 128) : 0;
+    ff = ff_all / tp; sh = shared_all / tp; ff_p = ff >= 512 && !f32 ? up_tile(ff) : up(ff, 128); sh_p = !sh ? 0 : sh >= 512 && !f32 ? up_tile(sh) : up(sh, 128);
     Nr = up(experts + (sh ? 1 : 0), 16);
     int rc = alloc_packed(ctx, router, Nr, Kw);
     if (!rc) rc = alloc_packed(ctx, wup, experts * ff_p, Kw);
@@ -66,6 +66,7 @@ void ExpertsScratch::reserve(const ExpertsBlock& e, size_t R) {
     n_place = std::max(n_place, R * per);
     n_out = std::max<size_t>(n_out, e.ldr);
     n_in = std::max<size_t>(n_in, e.Kw);
+    n_sh = std::max<size_t>(n_sh, (R + 15) / 16 * 16 * e.sh_p);
 }
 int ExpertsScratch::alloc(nvllm_ctx* ctx, bool f32) {
     if (!cap) return NVLLM_OK;
@@ -82,18 +83,29 @@ int ExpertsScratch::alloc(nvllm_ctx* ctx, bool f32) {
         if (!rc) rc = dmalloc(ctx, &act_f, (size_t)cap * lda);
     } else {
         for (bf16_bits** p : {&ah, &al}) if (!rc) rc = dmalloc(ctx, p, (size_t)cap * lda);
+        if (n_sh) for (bf16_bits** p : {&sh, &sl}) if (!rc) rc = dmalloc(ctx, p, n_sh);
         for (bf16_bits** p : {&gh, &gl}) if (!rc) rc = dmalloc(ctx, p, (size_t)cap * n_in);
     }
     return rc;
 }
 void ExpertsScratch::release() {
     for (void* p : {(void*)z, (void*)score, (void*)gate, (void*)pre, (void*)post, (void*)out, (void*)act_f, (void*)chosen, (void*)place, (void*)src, (void*)tile_group, (void*)ah,
-                    (void*)al, (void*)gh, (void*)gl})
+                    (void*)al, (void*)gh, (void*)gl, (void*)sh, (void*)sl})
         if (p) (void)hipFree(p);
     *this = ExpertsScratch();
 }
 
-int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_bits* xh, const bf16_bits* xl, int packed, const float* y, int R, BranchSum* out) {
+// prompt chunks with enough rows per expert: groups of whole blocks of the prompt product
+static int tile_align(const nvllm_model* m, const ExpertsBlock& e, int R) {
+    const int rows = R * e.top / e.experts;  // of an expert, on average
+    if (m->opt_tile_min_wgs <= 0 || R <= kFusedMaxRows || rows < (m->opt_tile_min_wgs == 1 ? 1 : 48)) return 0;
+    for (int align : {rows >= 320 ? 256 : 128, 256})
+        if (gemm_tile_group_ok(e.ff_p, e.Kw, align) && gemm_tile_group_ok(e.ldr, e.ff_p, align)) return align;
+    return 0;
+}
+int experts_packed(const nvllm_model* m, const ExpertsBlock& e, int R, int otherwise) { return e.sh && tile_align(m, e, R) ? plan_product(m, R, e.sup).packed : otherwise; }
+
+int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_bits* xh, const bf16_bits* xl, int packed, const float* y, int R, float* slabs2, BranchSum* out) {
     nvllm_ctx* ctx = m->ctx;
     hipStream_t s = ctx->stream;
     const bool f32 = y != nullptr;
@@ -105,12 +117,36 @@ int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_b
     RouteArgs ra;
     ra.z = x.z; ra.ld = e.Nr; ra.rows = R; ra.experts = e.experts; ra.top = e.top; ra.weight_in = e.weight_in;
     ra.gate_col = e.sh ? e.experts : -1;
-    ra.shared_group = e.sh > 0;
-    ra.align = R * e.top >= 32 * e.experts ? 64 : 16;
+    const int tile = f32 ? 0 : tile_align(m, e, R);
+    ra.shared_group = e.sh > 0 && !tile;
+    ra.align = tile ? tile : R * e.top >= 32 * e.experts ? 64 : 16;
     ra.cap = x.cap;
     ra.chosen = x.chosen; ra.score = x.score; ra.gate = x.gate; ra.place = x.place; ra.src = x.src; ra.pre = x.pre; ra.post = x.post; ra.tile_group = x.tile_group;
     PROF(m, PROF_QK, launch_route(ra, s));
     const int64_t longest = (int64_t)R * e.top + (int64_t)std::min(e.experts, R * e.top) * (ra.align - 1) + (ra.shared_group ? R + ra.align - 1 : 0);
+    out->gather = x.out; out->gather_row = x.place; out->n_gather = e.top + ra.shared_group;
+    if (tile) {
+        const int n = (int)(longest / tile) * tile;
+        PROF(m, PROF_QK, launch_gather_planes(xh, xl, packed, R, x.src, x.tile_group, tile, n, e.Kw, x.gh, x.gl, s));
+        TileGroups tg;
+        tg.tile_group = x.tile_group; tg.align = tile; tg.w_group = (int64_t)e.ff_p * e.Kw / 8; tg.pre = x.pre; tg.post = x.post;
+        PackedW w = e.wup;
+        w.N = e.ff_p;
+        PROF(m, PROF_GEMM, launch_gemm_tile_group(x.gh, x.gl, w, n, tg, nullptr, x.ah, x.al, s));
+        w = e.down;
+        w.N = e.ldr;
+        tg.w_group = (int64_t)e.ldr * e.ff_p / 8;
+        PROF(m, PROF_GEMM, launch_gemm_tile_group(x.ah, x.al, w, n, tg, x.out, nullptr, nullptr, s));
+        m->tile_launches += 2;
+        if (e.sh) {
+            const ProductPlan pu = plan_product(m, R, e.sup), pd = plan_product(m, R, e.sdown);
+            int rc = run_relu2(m, pu, xh, xl, e.sup, R, x.sh, x.sl, pd.packed);
+            if (!rc) rc = run_product(m, pd, x.sh, x.sl, e.sdown, slabs2, R, &out->n_slabs);
+            if (rc) return rc;
+            out->in = slabs2; out->slab_stride = (int64_t)R * e.ldr; out->scale = x.gate;
+        }
+        return NVLLM_OK;
+    }
     GroupGemmArgs ga = in;
     ga.src = x.src; ga.w = e.wup.data; ga.w_group = (int64_t)e.ff_p * e.Kw / 8; ga.N = e.ff_p; ga.K = e.Kw;
     if (ra.shared_group) { ga.ws = e.sup.data; ga.last = e.experts; ga.Ns = e.sh_p; ga.Ks = e.Kw; }
@@ -125,6 +161,5 @@ int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_b
     if (ra.shared_group) { gd.ws = e.sdown.data; gd.last = e.experts; gd.Ns = e.ldr; gd.Ks = e.sh_p; }
     gd.tile_group = x.tile_group; gd.align = ra.align; gd.tiles = ga.tiles; gd.out = x.out; gd.ldo = e.ldr;
     PROF(m, PROF_GEMM, launch_group_gemm(gd, s));
-    out->gather = x.out; out->gather_row = x.place; out->n_gather = e.top + ra.shared_group;
     return NVLLM_OK;
 }

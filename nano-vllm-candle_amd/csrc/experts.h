@@ -22,7 +22,7 @@ struct ExpertsBlock {
     PackedW router;                                        // a row per expert, then the shared gate's
     PackedW wup, down, sup, sdown;                         // wup [experts * ff_p x Kw], down [experts * ldr x ff_p]
     bool on() const { return experts > 0; }
-    int create(nvllm_ctx* ctx, int experts, int top, int ff, int shared, int W, int Kw, int ldr);
+    int create(nvllm_ctx* ctx, int experts, int top, int ff, int shared, int W, int Kw, int ldr, bool f32);
     void destroy();
     // `s`: the name behind "mlp."; 1: not a tensor of this block
     int load(nvllm_model* m, const char* name, const char* s, const HostMat& h, int64_t rows, int64_t cols);
@@ -35,14 +35,16 @@ struct ExpertsScratch {
     int cap = 0, lda = 0;
     float *z = nullptr, *score = nullptr, *gate = nullptr, *pre = nullptr, *post = nullptr, *out = nullptr, *act_f = nullptr;
     int *chosen = nullptr, *place = nullptr, *src = nullptr, *tile_group = nullptr;
-    bf16_bits *ah = nullptr, *al = nullptr, *gh = nullptr, *gl = nullptr;
+    bf16_bits *ah = nullptr, *al = nullptr, *gh = nullptr, *gl = nullptr, *sh = nullptr, *sl = nullptr;
     void reserve(const ExpertsBlock& e, size_t rows);       // sizes first, for every block, ...
     int alloc(nvllm_ctx* ctx, bool f32);                    // ... then the buffers
     void release();
 private:
-    size_t n_z = 0, n_top = 0, n_place = 0, n_rows = 0, n_out = 0, n_in = 0;
+    size_t n_z = 0, n_top = 0, n_place = 0, n_rows = 0, n_out = 0, n_in = 0, n_sh = 0;
     friend struct ExpertsBlock;
 };
 
-// the branch of R normed rows: planes xh / xl (ld Kw), or f32 rows y (32-bit mode)
-int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_bits* xh, const bf16_bits* xl, int packed, const float* y, int R, BranchSum* out);
+// the order the planes are wanted in: prompt chunks run the shared expert as an ordinary product
+int experts_packed(const nvllm_model* m, const ExpertsBlock& e, int R, int otherwise);
+// the branch of R normed rows: planes xh / xl (ld Kw), or f32 rows y (32-bit mode); slabs2: scratch of slab_floats
+int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_bits* xh, const bf16_bits* xl, int packed, const float* y, int R, float* slabs2, BranchSum* out);

@@ -184,7 +184,7 @@ struct DeltaRowsArgs {
 };
 constexpr float kUnitNormEps = 1e-6f;
 hipError_t launch_delta_rows(const DeltaRowsArgs& a, int rows, hipStream_t s);
-// gate_in -> decays and output gates (HeadGemmArgs with decay_rate set)
+// gate_in -> decays and output gates (HeadGemmArgs with decay_rate set), or step sizes alone (decay_bias without it)
 hipError_t launch_delta_gates(const HeadGemmArgs& a, hipStream_t s);
 // the history half of it for chunks with longer segments (after launch_delta_rows)
 hipError_t launch_delta_history(const DeltaRowsArgs& a, hipStream_t s);

@@ -698,17 +698,13 @@ int HybridModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
         if (!rc) rc = product(m, po, ctx_f, m->ctxh, m->ctxl, w.o, R, &ns);
         if (!rc) rc = add(ns, w.norm1, w.ff ? &pu : last ? nullptr : &pnext);
         if (!rc && w.ff) {
-            if (pu.kind == P_TILE && gemm_tile_ok(R, w.ff_p, Kw, 4, m->opt_tile_min_wgs)) {
-                PROF(m, PROF_GEMM, launch_gemm_tile(m->xh, m->xl, w.up, R, 4, nullptr, m->xh2, m->xl2, pd.packed, m->opt_tile_min_wgs, 1, nullptr, s));
-                ++m->tile_launches;
-            } else if (pu.kind == P_ROW && gemm_rowdir_ok(w.ff_p, Kw, 3, R)) {
-                RowParArgs ua;
-                ua.xh = m->xh; ua.xl = m->xl; ua.ldx = Kw; ua.oh = m->xh2; ua.ol = m->xl2; ua.M = R; ua.x_packed = pu.packed; ua.o_packed = pd.packed;
-                PROF(m, PROF_GEMM, launch_gemm_rowpar(ua, w.up, 3, s));
-            } else {
-                rc = product(m, pu, y, m->xh, m->xl, w.up, R, &ns);
+            if (f32) {
+                rc = exact_product(m, y, w.up, m->slabs, R);
                 if (rc) return rc;
-                PROF(m, PROF_SILU, launch_relu2(m->slabs, ns, (int64_t)R * w.ff_p, R, w.ff_p, f32 ? nullptr : m->xh2, f32 ? nullptr : m->xl2, pd.packed, f32 ? act_f : nullptr, s));
+                PROF(m, PROF_SILU, launch_relu2(m->slabs, 1, 0, R, w.ff_p, nullptr, nullptr, 0, act_f, s));
+            } else {
+                rc = run_relu2(m, pu, m->xh, m->xl, w.up, R, m->xh2, m->xl2, pd.packed);
+                if (rc) return rc;
             }
             rc = product(m, pd, act_f, m->xh2, m->xl2, w.down, R, &ns);
             if (!rc) rc = add(ns, w.norm2, last ? nullptr : &pnext);

@@ -560,7 +560,8 @@ __device__ __forceinline__ float softplus_fast(float z) {
 }
 __device__ __forceinline__ float sigmoid_fast(float x) { return __builtin_amdgcn_rcpf(1.0f + exp_fast(-x)); }
 
-template <int KT>
+// STEP: one head of softplus(v + bias) alone (step sizes of a scan)
+template <int KT, bool STEP>
 __global__ void __launch_bounds__(256) delta_gates_kernel(HeadGemmArgs a) {
     __shared__ __attribute__((aligned(16))) uint4 xs[2 * 4 * KT * 64];  // [plane][row tile][k-tile][lane]
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, grp = lane >> 4;
@@ -607,8 +608,8 @@ __global__ void __launch_bounds__(256) delta_gates_kernel(HeadGemmArgs a) {
         }
         const int f0 = nt * 16 + grp * 4;
         float4 rate = make_float4(0.f, 0.f, 0.f, 0.f), dt = rate;
-        if (head == 0) {
-            rate = *reinterpret_cast<const float4*>(a.decay_rate + f0);
+        if (STEP || head == 0) {
+            if constexpr (!STEP) rate = *reinterpret_cast<const float4*>(a.decay_rate + f0);
             dt = *reinterpret_cast<const float4*>(a.decay_bias + f0);
         }
 #pragma unroll
@@ -616,7 +617,8 @@ __global__ void __launch_bounds__(256) delta_gates_kernel(HeadGemmArgs a) {
             const int row = row0 + b * 16 + l15;
             const f32x4 v = acc[b];
             float4 o;
-            if (head == 0) o = make_float4(exp_fast(-rate.x * softplus_fast(v[0] + dt.x)), exp_fast(-rate.y * softplus_fast(v[1] + dt.y)),
+            if constexpr (STEP) o = make_float4(softplus_fast(v[0] + dt.x), softplus_fast(v[1] + dt.y), softplus_fast(v[2] + dt.z), softplus_fast(v[3] + dt.w));
+            else if (head == 0) o = make_float4(exp_fast(-rate.x * softplus_fast(v[0] + dt.x)), exp_fast(-rate.y * softplus_fast(v[1] + dt.y)),
                                            exp_fast(-rate.z * softplus_fast(v[2] + dt.z)), exp_fast(-rate.w * softplus_fast(v[3] + dt.w)));
             else o = make_float4(sigmoid_fast(v[0]), sigmoid_fast(v[1]), sigmoid_fast(v[2]), sigmoid_fast(v[3]));
             if (row < a.M) *reinterpret_cast<float4*>(a.y + (size_t)row * a.y_row + (size_t)head * a.y_head + f0) = o;
@@ -625,16 +627,23 @@ __global__ void __launch_bounds__(256) delta_gates_kernel(HeadGemmArgs a) {
 }
 hipError_t launch_delta_gates(const HeadGemmArgs& a, hipStream_t s) {
     const int kt = a.K / 32;
-    if (a.exact || kt > 4 || a.N % 16 || a.K % 32 || a.x_row % 4 || a.x_head % 4 || a.y_row % 4 || a.y_head % 4 || a.n_valid != a.N || !a.decay_rate)
+    const bool step = a.decay_bias && !a.decay_rate && a.heads == 1;
+    if (a.exact || kt > 4 + 4 * step || a.N % 16 || a.K % 32 || a.x_row % 4 || a.x_head % 4 || a.y_row % 4 || a.y_head % 4 || a.n_valid != a.N || (!a.decay_rate && !step))
         return launch_head_gemm(a, s);
     if (a.M <= 0) return hipSuccess;
     // eight slices per row block for prompt chunks, for few rows one tile per wave
     const int blocks = (a.M + 63) / 64, tiles = a.N / 16;
     const dim3 grid(blocks, a.heads, std::max(1, std::min((tiles + 3) / 4, std::max(8, 256 / (blocks * a.heads)))));
-    if (kt == 1) delta_gates_kernel<1><<<grid, 256, 0, s>>>(a);
-    else if (kt == 2) delta_gates_kernel<2><<<grid, 256, 0, s>>>(a);
-    else if (kt == 3) delta_gates_kernel<3><<<grid, 256, 0, s>>>(a);
-    else delta_gates_kernel<4><<<grid, 256, 0, s>>>(a);
+    switch (step ? kt + 8 : kt) {
+        case 1: delta_gates_kernel<1, false><<<grid, 256, 0, s>>>(a); break;
+        case 2: delta_gates_kernel<2, false><<<grid, 256, 0, s>>>(a); break;
+        case 3: delta_gates_kernel<3, false><<<grid, 256, 0, s>>>(a); break;
+        case 4: delta_gates_kernel<4, false><<<grid, 256, 0, s>>>(a); break;
+#define NVLLM_ST(K_) case K_ + 8: delta_gates_kernel<K_, true><<<grid, 256, 0, s>>>(a); break;
+        NVLLM_ST(1) NVLLM_ST(2) NVLLM_ST(3) NVLLM_ST(4) NVLLM_ST(5) NVLLM_ST(6) NVLLM_ST(7) NVLLM_ST(8)
+#undef NVLLM_ST
+        default: return hipErrorInvalidValue;
+    }
     return hipGetLastError();
 }
 

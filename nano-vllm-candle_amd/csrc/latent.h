@@ -30,6 +30,7 @@ struct AddNormArgs {
     float* residual_out = nullptr;
     const int* row_idx = nullptr;      // input row of output row r (outputs are compact)
     int W = 0, ldr = 0, ldx = 0;
+    int ld_in = 0;                     // row stride of `in` where it is not ldr (16-row form only)
     float eps = 0.f;
     const float* post_w = nullptr;
     float post_mult = 1.f;

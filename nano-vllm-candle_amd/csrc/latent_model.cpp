@@ -165,7 +165,7 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
     auto alloc_w = [&](PackedW& w, int N, int K) { return alloc_packed(ctx, w, N, K); };
     auto alloc_v = [&](float** p, size_t n) { return alloc_vec(ctx, p, n); };
     // wide projections: a whole number of the prompt product's 192- or 256-feature tiles
-    auto wide = [&](int n) { return n >= 1536 && !c.f32 ? std::min(up(n, 192), up(n, 256)) : up(n, 16); };
+    auto wide = [&](int n) { return n >= 1536 && !c.f32 ? up_tile(n) : up(n, 16); };
     int rc = dmalloc(ctx, &L.embed, (size_t)c.vocab_size * L.ldr);
     if (!rc) HIPCHK(ctx, hipMemsetAsync(L.embed, 0, (size_t)c.vocab_size * L.ldr * 2, ctx->stream));
     if (!rc) rc = alloc_w(L.head, L.Vp, L.Kw);
@@ -182,7 +182,7 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
         }
         if (!rc && !c.one_norm && (w.ff || w.c.experts)) rc = alloc_v(&w.norm2, L.Kw);
         w.experts.weight_in = w.c.expert_weight_in;
-        if (!rc && w.c.experts) rc = w.experts.create(ctx, w.c.experts, w.c.top, w.c.expert_ff, w.c.shared_ff, c.width, L.Kw, L.ldr);
+        if (!rc && w.c.experts) rc = w.experts.create(ctx, w.c.experts, w.c.top, w.c.expert_ff, w.c.shared_ff, c.width, L.Kw, L.ldr, c.f32);
         if (w.c.mixer == NVLLM_SELECTIVE_SCAN) {
             L.has_state = true;
             if (!rc) rc = w.scan.create(ctx, w.c.inner, w.c.state, w.c.conv_taps, w.c.dt_rank, L.Kw, c.f32);
@@ -752,8 +752,8 @@ int LatentModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
         AddNormArgs na = base;
         na.residual_out = m->resid;
         // the feed-forward's input: its own norm's output, or the mixer's where they share the norm (twice when the products want other orders)
-        const bool mlp = w.ff || w.experts.on(), same = L.cfg.one_norm && (f32 || w.experts.on() || pg.packed == pq.packed);
-        if (w.experts.on()) pg.packed = pq.packed;
+        if (w.experts.on() && !f32) pg.packed = experts_packed(m, w.experts, R, pq.packed);
+        const bool mlp = w.ff || w.experts.on(), same = L.cfg.one_norm && (f32 || pg.packed == pq.packed);
         na.w[0] = w.norm1; na.w[1] = !mlp || same ? nullptr : L.cfg.one_norm ? w.norm1 : w.norm2;
         const float* y_ff = same ? L.y1 : L.y2;
         const bf16_bits *ffh = same ? m->xh : L.x2h, *ffl = same ? m->xl : L.x2l;
@@ -770,7 +770,7 @@ int LatentModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
         int no = 1, nd = 1;
         BranchSum ff;
         if (w.experts.on()) {
-            rc = run_experts(m, w.experts, L.experts, ffh, ffl, pg.packed, f32 ? y_ff : nullptr, R, &ff);
+            rc = run_experts(m, w.experts, L.experts, ffh, ffl, pg.packed, f32 ? y_ff : nullptr, R, L.slabs2, &ff);
             if (rc) return rc;
         }
         if (w.ff) {

@@ -146,7 +146,8 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
                 s0.x += t0.x * f; s0.y += t0.y * f; s0.z += t0.z * f; s0.w += t0.w * f;
                 s1.x += t1.x * f; s1.y += t1.y * f; s1.z += t1.z * f; s1.w += t1.w * f;
             };
-            if (a.in) for (int sl = 0; sl < a.n_slabs; ++sl) add(a.in + (size_t)sl * a.slab_stride + off);
+            const size_t off_in = a.ld_in ? (size_t)rowc * a.ld_in + col : off;
+            if (a.in) for (int sl = 0; sl < a.n_slabs; ++sl) add(a.in + (size_t)sl * a.slab_stride + off_in);
             if (a.in2) {
                 const float f = a.in2_scale ? a.in2_scale[rowc] : 1.f;
                 for (int sl = 0; sl < a.n_slabs2; ++sl) add(a.in2 + (size_t)sl * a.slab_stride2 + off, f);
@@ -242,10 +243,10 @@ hipError_t launch_add_norm(const AddNormArgs& a, int rows, hipStream_t s) {
     if (a.raw && a.w[0]) return hipErrorInvalidValue;
     bool packed = any && a.ldr == a.ldx && a.ldr % 32 == 0 && !a.row_idx && (!post || a.residual_in);
     for (int k = 0; k < 2; ++k) packed &= !(a.w[k] || (k == 0 && a.raw)) || (a.packed[k] && a.xh[k] && !a.y[k]);
-    if (a.center && (post || a.raw)) return hipErrorInvalidValue;
+    if ((a.center && (post || a.raw)) || (a.ld_in && (!packed || a.ldr > 4096 || a.ld_in % 4 || a.slab_stride % 4))) return hipErrorInvalidValue;
     auto launch = [&](auto P) {
         constexpr int KIND = decltype(P)::value;
-        if (packed && rows >= 512 && a.ldr <= 4096) {
+        if (packed && (rows >= 512 || a.ld_in) && a.ldr <= 4096) {
             const int kt = a.ldr / 32, tiles = (rows + 15) / 16;
             if (kt <= 32) add_norm_rows16_kernel<2, KIND><<<tiles, 1024, 0, s>>>(a, rows);
             else if (kt <= 64) add_norm_rows16_kernel<4, KIND><<<tiles, 1024, 0, s>>>(a, rows);
@@ -435,6 +436,14 @@ __global__ void __launch_bounds__(256) query_latent_kernel(QueryLatentArgs a, La
 hipError_t launch_query_latent(const QueryLatentArgs& a, const LatentRowsArgs& kv, int rows, hipStream_t s) {
     if (a.rank < 1 || a.rank > a.ld || a.ldx < a.rank || a.ldx % 32 || (!a.xh && !a.y) || kv.cache.rot % 2 || kv.cache.rank_p % 32 || kv.cache.rot_p % 32) return hipErrorInvalidValue;
     if (rows <= 0) return hipSuccess;
+    if (rows >= 512 && a.packed && a.xh && !a.y && a.rank == a.ldx && a.rank <= 4096 && a.ld % 4 == 0 && a.slab_stride % 4 == 0) {
+        AddNormArgs n;
+        n.in = a.in; n.n_slabs = a.n_slabs; n.slab_stride = a.slab_stride; n.ld_in = a.ld; n.W = n.ldr = n.ldx = a.rank; n.eps = a.eps;
+        n.w[0] = a.norm_w; n.xh[0] = a.xh; n.xl[0] = a.xl; n.packed[0] = 1;
+        hipError_t e = launch_add_norm(n, rows, s);
+        if (e != hipSuccess || !kv.kv) return e;
+        return launch_latent_cache(kv, rows, s);
+    }
     query_latent_kernel<<<dim3(rows, kv.kv ? 2 : 1), 256, 0, s>>>(a, kv);
     return hipGetLastError();
 }

@@ -278,11 +278,12 @@ hipError_t launch_group_gemm(const GroupGemmArgs& a, hipStream_t s) {
     return hipGetLastError();
 }
 
-__global__ void __launch_bounds__(256) gather_planes_kernel(const uint4* __restrict__ xh, const uint4* __restrict__ xl, int packed, const int* __restrict__ src, int K,
-                                                            uint4* __restrict__ oh, uint4* __restrict__ ol) {
+__global__ void __launch_bounds__(256) gather_planes_kernel(const uint4* __restrict__ xh, const uint4* __restrict__ xl, int packed, int rows, const int* __restrict__ src,
+                                                            const int* __restrict__ tile_group, int align, int K, uint4* __restrict__ oh, uint4* __restrict__ ol) {
+    if (tile_group[blockIdx.x * 16 / align] < 0) return;  // src is not set there
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, KT = K >> 5, grp = lane >> 4;
     const int row = src[blockIdx.x * 16 + (lane & 15)];
-    const int rc = max(row, 0);
+    const int rc = min(max(row, 0), rows - 1);
     const size_t x0 = packed ? (size_t)(rc >> 4) * KT * 64 + (grp << 4) + (rc & 15) : ((size_t)rc * K >> 3) + grp;
     const size_t step = packed ? 64 : 4, o0 = (size_t)blockIdx.x * KT * 64 + lane;
     for (int kt = blockIdx.y * 4 + wave; kt < KT; kt += 4 * gridDim.y) {
@@ -292,11 +293,11 @@ __global__ void __launch_bounds__(256) gather_planes_kernel(const uint4* __restr
         ol[o0 + (size_t)kt * 64] = l;
     }
 }
-hipError_t launch_gather_planes(const bf16_bits* xh, const bf16_bits* xl, int packed, const int* src, int positions, int K, bf16_bits* oh, bf16_bits* ol,
-                                hipStream_t s) {
-    if (K % 32 || positions % 16) return hipErrorInvalidValue;
+hipError_t launch_gather_planes(const bf16_bits* xh, const bf16_bits* xl, int packed, int rows, const int* src, const int* tile_group, int align, int positions, int K,
+                                bf16_bits* oh, bf16_bits* ol, hipStream_t s) {
+    if (K % 32 || positions % 16 || align < 16 || align % 16 || rows < 1) return hipErrorInvalidValue;
     if (positions <= 0) return hipSuccess;
-    gather_planes_kernel<<<dim3(positions / 16, std::max(1, std::min(K / 128, 4))), 256, 0, s>>>(reinterpret_cast<const uint4*>(xh), reinterpret_cast<const uint4*>(xl), packed, src, K,
+    gather_planes_kernel<<<dim3(positions / 16, std::max(1, std::min(K / 128, 4))), 256, 0, s>>>(reinterpret_cast<const uint4*>(xh), reinterpret_cast<const uint4*>(xl), packed, rows, src, tile_group, align, K,
                                                                                               reinterpret_cast<uint4*>(oh), reinterpret_cast<uint4*>(ol));
     return hipGetLastError();
 }

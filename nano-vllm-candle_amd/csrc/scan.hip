@@ -282,20 +282,34 @@ __global__ void __launch_bounds__(256) scan_prompt_kernel(ScanArgs a) {
         __syncthreads();
         if (t0 + TB < n) fetch(t0 + TB);
         const int m = min(TB, n - t0);
-        for (int t = 0; t < m; ++t) {
-            const float dt = dts[t * CH + lc], x = xs[t * CH + lc], dx = dt * x;
-            float B[NS], C[NS], y = 0.f;
-            load_states(B, bcs + t * 2 * ST + q * NS);
-            if constexpr (!CARRY) load_states(C, bcs + t * 2 * ST + ST + q * NS);
+        // U tokens at a time: everything but the state's own chain is independent.  Tokens past the end have dt = 0: the state stays.
+        constexpr int U = NS == 4 ? 4 : 1;
+        for (int t = 0; t < m; t += U) {
+            float dt[U], dx[U], B[U][NS], C[U][NS], y[U];
 #pragma unroll
-            for (int i = 0; i < NS; ++i) {
-                S[i] = S[i] * __builtin_amdgcn_exp2f(dt * A[i]) + dx * B[i];
-                if constexpr (!CARRY) y += S[i] * C[i];
+            for (int u = 0; u < U; ++u) {
+                const int tt = t + u;
+                dt[u] = tt < m ? dts[tt * CH + lc] : 0.f;
+                dx[u] = dt[u] * xs[tt * CH + lc];
+                load_states(B[u], bcs + tt * 2 * ST + q * NS);
+                if constexpr (!CARRY) load_states(C[u], bcs + tt * 2 * ST + ST + q * NS);
             }
-            if constexpr (CARRY) total += dt;
-            else {
-                y = lanes_sum<NL>(y);
-                if (q == 0) xs[t * CH + lc] = y;  // this channel's x at t has been read by its lanes' wave
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                y[u] = 0.f;
+#pragma unroll
+                for (int i = 0; i < NS; ++i) {
+                    S[i] = S[i] * __builtin_amdgcn_exp2f(dt[u] * A[i]) + dx[u] * B[u][i];
+                    if constexpr (!CARRY) y[u] += S[i] * C[u][i];
+                }
+                if constexpr (CARRY) total += dt[u];
+            }
+            if constexpr (!CARRY) {
+#pragma unroll
+                for (int u = 0; u < U; ++u) {
+                    y[u] = lanes_sum<NL>(y[u]);
+                    if (q == 0) xs[(t + u) * CH + lc] = y[u];  // this channel's x there has been read by its lanes' wave
+                }
             }
         }
         if constexpr (!CARRY) {

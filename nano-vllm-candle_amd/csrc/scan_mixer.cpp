@@ -8,8 +8,8 @@ int ScanMixer::create(nvllm_ctx* ctx, int inner_, int state_, int taps_, int ran
     inner = inner_; state = state_; taps = taps_; rank = rank_;
     n = inner / ctx->tp_size; S = scan_states(state); n_p = up(n, scan_channels(S)); rank_p = up(rank, 32); Kc = up(n, 128);
     // wide projections: a whole number of the prompt product's 192- or 256-feature tiles
-    Nin = 2 * n >= 1536 && !f32 ? std::min(up(2 * n, 192), up(2 * n, 256)) : up(2 * n, 16);
-    Nx = up(rank_p + 2 * S, 16);
+    Nin = 2 * n >= 1536 && !f32 ? up_tile(2 * n) : up(2 * n, 16);
+    Nx = n >= 1536 && !f32 ? up_tile(rank_p + 2 * S) : up(rank_p + 2 * S, 16);
     int rc = alloc_packed(ctx, in, Nin, Kw);
     if (!rc) rc = alloc_packed(ctx, x, Nx, Kc);
     if (!rc) rc = alloc_packed(ctx, dt, n_p, rank_p);
@@ -181,7 +181,7 @@ int run_scan(nvllm_model* m, ScanMixer& w, ScanScratch& x, const float* in, int 
     HeadGemmArgs ga;
     ga.x = dbc; ga.x_row = w.Nx; ga.w = w.dt.data; ga.N = ga.n_valid = w.n_p; ga.K = w.rank_p; ga.M = R; ga.exact = f32;
     ga.y = x.dt; ga.y_row = w.n_p; ga.decay_bias = w.dt_b;
-    PROF(m, PROF_GEMM, launch_head_gemm(ga, s));
+    PROF(m, PROF_GEMM, launch_delta_gates(ga, s));
     ScanArgs sa;
     sa.x = x.x; sa.ldx = w.Kc; sa.dt = x.dt; sa.bc = dbc; sa.ldbc = w.Nx; sa.b0 = w.rank_p; sa.c0 = w.rank_p + w.S;
     sa.z = in + w.n; sa.z_slabs = n_slabs; sa.ldz = w.Nin; sa.z_stride = ca.slab_stride;

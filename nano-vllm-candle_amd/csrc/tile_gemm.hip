@@ -19,6 +19,7 @@
 // MODE 0: f32 [M][N].  MODE 2: W is the gate/up matrix interleaved in 16-row tiles; the epilogue writes
 // silu(gate)*up as hi/lo planes [M][N/2] (row-major or xpack_off order) -- SiluAndMul, activation.rs:13-18.
 // MODE 4: squared ReLU of every feature as hi/lo planes [M][N].
+// MODE 5, 6: every row block belongs to a group with weights of its own (routed experts): post relu2(pre x.W^T) as planes, plain f32.
 // MODE 3 (NTW = 8, head_dim 128): W is the fused QKV matrix, so a wave's 64 rows x 128 features are 64 tokens of ONE
 // head and the epilogue is the whole of qwen3.rs:208-234 on registers: RMS norm over the head (q_norm / k_norm BEFORE
 // RoPE), half-split RoPE (rotary_embedding.rs:82-107: features d and d+64 sit in the same lane, accumulators j and j+4),
@@ -45,6 +46,7 @@ struct TileArgs {
     int MB = 0, NB = 0;         // row blocks, feature blocks
     int map = 0;                // 0: id -> (nb fastest); 1: blocks of one XCD share rows; 2: share features
     QkvArgs q;                  // MODE 3
+    TileGroups g;               // MODE 5, 6
 #ifdef NVLLM_STAMPS
     unsigned long long* stamps = nullptr;  // diagnostic build: [workgroup][16 waves][8 points] of s_memrealtime
 #endif
@@ -86,6 +88,12 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
         if (mb >= a.MB || nb >= a.NB) return;  // whole workgroup, before any barrier
     }
     const int mtiles = (a.M + 15) >> 4;
+    const uint4* wbase = a.wp;
+    if constexpr (MODE >= 5) {
+        const int g = a.g.tile_group[mb * (WM * 64) / a.g.align];
+        if (g < 0) return;  // whole workgroup, before any barrier
+        wbase += (size_t)g * a.g.w_group;
+    }
     NVLLM_STAMP(a, 0);
     // MODE 3: position and cache block of this lane's four tokens, fetched NOW (two dependent loads each) so that they
     // land under the K loop; in the epilogue they were 8 us of latency chain per workgroup (stamps)
@@ -113,7 +121,7 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
             // MODE 3: the block's two heads are nb and NB + nb, not neighbours: a V head (whose epilogue is scattered
             // 2-byte cache stores) then always shares its workgroup with a q head, and the V tail spreads over twice the CUs
             const int ntile = MODE == 3 ? (f < NTW ? nb : a.NB + nb) * NTW + f % NTW : nb * FRW + f;
-            src[i] = a.wp + ((size_t)ntile * a.KT + kt0) * 64;
+            src[i] = wbase + ((size_t)ntile * a.KT + kt0) * 64;
         } else {
             const int g = f - FRW, plane = g / XT, mt = min(mb * XT + (g % XT), mtiles - 1);
             src[i] = (plane ? a.xl : a.xh) + ((size_t)mt * a.KT + kt0) * 64;
@@ -225,7 +233,7 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
     // D[feature 4*grp + r][token l15]
     const int nt0 = nb * FRW + wn * NTW;
     const int row0 = mb * (WM * 64) + wm * 64;
-    if constexpr (MODE == 0) {
+    if constexpr (MODE == 0 || MODE == 6) {
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
             const int row = row0 + b * 16 + l15;
@@ -377,17 +385,19 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
                 }
             }
         }
-    } else if constexpr (MODE == 4) {
+    } else if constexpr (MODE == 4 || MODE == 5) {
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
             const int row = row0 + b * 16 + l15;
             if (row < a.M) {
+                [[maybe_unused]] float pre = 1.f, post = 1.f;
+                if constexpr (MODE == 5) { pre = a.g.pre[row]; post = a.g.post[row]; }
 #pragma unroll
                 for (int j = 0; j < NTW; ++j) {
                     const int f0 = (nt0 + j) * 16 + grp * 4;
                     uint16_t h[4], l[4];
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) split_bf16(relu2(acc[j][b][r]), h[r], l[r]);
+                    for (int r = 0; r < 4; ++r) split_bf16(MODE == 5 ? relu2(acc[j][b][r] * pre) * post : relu2(acc[j][b][r]), h[r], l[r]);
                     const size_t xo = a.act_packed ? xpack_off(row, f0, a.N >> 5) : (size_t)row * a.N + f0;
                     *reinterpret_cast<uint2*>(a.act_hi + xo) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
                     *reinterpret_cast<uint2*>(a.act_lo + xo) = make_uint2(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16));
@@ -516,6 +526,31 @@ hipError_t launch_gemm_tile_qkv(const bf16_bits* xh, const bf16_bits* xl, const 
     a.xh = reinterpret_cast<const uint4*>(xh); a.xl = reinterpret_cast<const uint4*>(xl); a.wp = w.data;
     a.M = M; a.N = w.N; a.KT = w.K / 32; a.q = qa;
     return tile_launch_t<8, 2, 3>(a, 1, s);
+}
+
+// rows of a block, features of a block: 256 x 256, 256 x 192 or 128 x 256 (few rows per group)
+static TileShape group_shape(int N, int K, int align) {
+    TileShape t;
+    if (K % 64 || K < 128) return t;
+    if (align == 128) { if (N % 256 == 0) { t.ntw = 4; t.wn = 4; } }
+    else if (align == 256) { t.ntw = N % 256 == 0 ? 8 : N % 192 == 0 ? 6 : 0; t.wn = 2; }
+    return t;
+}
+bool gemm_tile_group_ok(int N, int K, int align) { return group_shape(N, K, align).ntw != 0; }
+hipError_t launch_gemm_tile_group(const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int positions, const TileGroups& g, float* out, bf16_bits* act_hi,
+                                  bf16_bits* act_lo, hipStream_t s) {
+    const TileShape t = group_shape(w.N, w.K, g.align);
+    if (!t.ntw || positions % g.align || !g.tile_group || (act_hi && (!g.pre || !g.post))) return hipErrorNotSupported;
+    if (positions <= 0) return hipSuccess;
+    TileArgs a;
+    a.xh = reinterpret_cast<const uint4*>(xh); a.xl = reinterpret_cast<const uint4*>(xl); a.wp = w.data;
+    a.out = out; a.act_hi = act_hi; a.act_lo = act_lo; a.act_packed = 1; a.M = positions; a.N = w.N; a.KT = w.K / 32; a.g = g;
+    if (act_hi) {
+        if (t.wn == 4) return tile_launch_t<4, 4, 5>(a, 1, s);
+        return t.ntw == 8 ? tile_launch_t<8, 2, 5>(a, 1, s) : tile_launch_t<6, 2, 5>(a, 1, s);
+    }
+    if (t.wn == 4) return tile_launch_t<4, 4, 6>(a, 1, s);
+    return t.ntw == 8 ? tile_launch_t<8, 2, 6>(a, 1, s) : tile_launch_t<6, 2, 6>(a, 1, s);
 }
 
 // row-major plane [M][K] -> xpack_off order (tests and the tuning bench; the product's producers write the order directly)
