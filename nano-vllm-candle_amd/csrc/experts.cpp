@@ -65,7 +65,6 @@ void ExpertsScratch::reserve(const ExpertsBlock& e, size_t R) {
     n_top = std::max(n_top, R * e.top);
     n_place = std::max(n_place, R * per);
     n_out = std::max<size_t>(n_out, e.ldr);
-    n_in = std::max<size_t>(n_in, e.Kw);
     n_sh = std::max<size_t>(n_sh, (R + 15) / 16 * 16 * e.sh_p);
 }
 int ExpertsScratch::alloc(nvllm_ctx* ctx, bool f32) {
@@ -84,13 +83,12 @@ int ExpertsScratch::alloc(nvllm_ctx* ctx, bool f32) {
     } else {
         for (bf16_bits** p : {&ah, &al}) if (!rc) rc = dmalloc(ctx, p, (size_t)cap * lda);
         if (n_sh) for (bf16_bits** p : {&sh, &sl}) if (!rc) rc = dmalloc(ctx, p, n_sh);
-        for (bf16_bits** p : {&gh, &gl}) if (!rc) rc = dmalloc(ctx, p, (size_t)cap * n_in);
     }
     return rc;
 }
 void ExpertsScratch::release() {
     for (void* p : {(void*)z, (void*)score, (void*)gate, (void*)pre, (void*)post, (void*)out, (void*)act_f, (void*)chosen, (void*)place, (void*)src, (void*)tile_group, (void*)ah,
-                    (void*)al, (void*)gh, (void*)gl, (void*)sh, (void*)sl})
+                    (void*)al, (void*)sh, (void*)sl})
         if (p) (void)hipFree(p);
     *this = ExpertsScratch();
 }
@@ -103,16 +101,17 @@ static int tile_align(const nvllm_model* m, const ExpertsBlock& e, int R) {
         if (gemm_tile_group_ok(e.ff_p, e.Kw, align) && gemm_tile_group_ok(e.ldr, e.ff_p, align)) return align;
     return 0;
 }
-int experts_packed(const nvllm_model* m, const ExpertsBlock& e, int R, int otherwise) { return e.sh && tile_align(m, e, R) ? plan_product(m, R, e.sup).packed : otherwise; }
+bool experts_gather(const nvllm_model* m, const ExpertsBlock& e, int R) { return tile_align(m, e, R) > 0; }
 
-int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_bits* xh, const bf16_bits* xl, int packed, const float* y, int R, float* slabs2, BranchSum* out) {
+int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_bits* xh, const bf16_bits* xl, int packed, const bf16_bits* rh, const bf16_bits* rl,
+                const float* y, int R, float* slabs2, BranchSum* out) {
     nvllm_ctx* ctx = m->ctx;
     hipStream_t s = ctx->stream;
     const bool f32 = y != nullptr;
     GroupGemmArgs in;  // of rows
     in.xh = xh; in.xl = xl; in.xf = y; in.ldx = e.Kw; in.x_packed = packed; in.x_rows = R;
     GroupGemmArgs rg = in;
-    rg.w = e.router.data; rg.N = e.Nr; rg.K = e.Kw; rg.align = R > 64 ? 64 : 16; rg.out = x.z; rg.ldo = e.Nr;
+    rg.w = e.router.data; rg.N = e.Nr; rg.K = e.Kw; rg.align = R > 64 && e.Nr > 128 ? 64 : 16; rg.out = x.z; rg.ldo = e.Nr;
     PROF(m, PROF_GEMM, launch_group_gemm(rg, s));
     RouteArgs ra;
     ra.z = x.z; ra.ld = e.Nr; ra.rows = R; ra.experts = e.experts; ra.top = e.top; ra.weight_in = e.weight_in;
@@ -127,20 +126,21 @@ int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_b
     out->gather = x.out; out->gather_row = x.place; out->n_gather = e.top + ra.shared_group;
     if (tile) {
         const int n = (int)(longest / tile) * tile;
-        PROF(m, PROF_QK, launch_gather_planes(xh, xl, packed, R, x.src, x.tile_group, tile, n, e.Kw, x.gh, x.gl, s));
         TileGroups tg;
-        tg.tile_group = x.tile_group; tg.align = tile; tg.w_group = (int64_t)e.ff_p * e.Kw / 8; tg.pre = x.pre; tg.post = x.post;
+        tg.tile_group = x.tile_group; tg.align = tile; tg.w_group = (int64_t)e.ff_p * e.Kw / 8; tg.src = x.src; tg.x_rows = R; tg.pre = x.pre; tg.post = x.post;
         PackedW w = e.wup;
         w.N = e.ff_p;
-        PROF(m, PROF_GEMM, launch_gemm_tile_group(x.gh, x.gl, w, n, tg, nullptr, x.ah, x.al, s));
+        PROF(m, PROF_GEMM, launch_gemm_tile_group(rh, rl, w, n, tg, nullptr, x.ah, x.al, s));
         w = e.down;
         w.N = e.ldr;
         tg.w_group = (int64_t)e.ldr * e.ff_p / 8;
         PROF(m, PROF_GEMM, launch_gemm_tile_group(x.ah, x.al, w, n, tg, x.out, nullptr, nullptr, s));
         m->tile_launches += 2;
         if (e.sh) {
-            const ProductPlan pu = plan_product(m, R, e.sup), pd = plan_product(m, R, e.sdown);
-            int rc = run_relu2(m, pu, xh, xl, e.sup, R, x.sh, x.sl, pd.packed);
+            ProductPlan pu = plan_product(m, R, e.sup), pd = plan_product(m, R, e.sdown);
+            const bool ours = pu.packed == packed;  // else the row-major planes and a kernel that takes them
+            if (!ours && pu.packed) pu = ProductPlan{P_GENERIC, 0, pu.max_split};
+            int rc = run_relu2(m, pu, ours ? xh : rh, ours ? xl : rl, e.sup, R, x.sh, x.sl, pd.packed);
             if (!rc) rc = run_product(m, pd, x.sh, x.sl, e.sdown, slabs2, R, &out->n_slabs);
             if (rc) return rc;
             out->in = slabs2; out->slab_stride = (int64_t)R * e.ldr; out->scale = x.gate;

@@ -35,16 +35,18 @@ struct ExpertsScratch {
     int cap = 0, lda = 0;
     float *z = nullptr, *score = nullptr, *gate = nullptr, *pre = nullptr, *post = nullptr, *out = nullptr, *act_f = nullptr;
     int *chosen = nullptr, *place = nullptr, *src = nullptr, *tile_group = nullptr;
-    bf16_bits *ah = nullptr, *al = nullptr, *gh = nullptr, *gl = nullptr, *sh = nullptr, *sl = nullptr;
+    bf16_bits *ah = nullptr, *al = nullptr, *sh = nullptr, *sl = nullptr;
     void reserve(const ExpertsBlock& e, size_t rows);       // sizes first, for every block, ...
     int alloc(nvllm_ctx* ctx, bool f32);                    // ... then the buffers
     void release();
 private:
-    size_t n_z = 0, n_top = 0, n_place = 0, n_rows = 0, n_out = 0, n_in = 0, n_sh = 0;
+    size_t n_z = 0, n_top = 0, n_place = 0, n_rows = 0, n_out = 0, n_sh = 0;
     friend struct ExpertsBlock;
 };
 
-// the order the planes are wanted in: prompt chunks run the shared expert as an ordinary product
-int experts_packed(const nvllm_model* m, const ExpertsBlock& e, int R, int otherwise);
-// the branch of R normed rows: planes xh / xl (ld Kw), or f32 rows y (32-bit mode); slabs2: scratch of slab_floats
-int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_bits* xh, const bf16_bits* xl, int packed, const float* y, int R, float* slabs2, BranchSum* out);
+// long prompt chunks gather the experts' rows from row-major planes, beside those of the shared expert (an ordinary product) and the router
+bool experts_gather(const nvllm_model* m, const ExpertsBlock& e, int R);
+// the branch of R normed rows: planes xh / xl (ld Kw), and rh / rl row-major where experts_gather says so, or f32 rows y (32-bit mode); slabs2:
+// scratch of slab_floats
+int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_bits* xh, const bf16_bits* xl, int packed, const bf16_bits* rh, const bf16_bits* rl,
+                const float* y, int R, float* slabs2, BranchSum* out);

@@ -203,11 +203,14 @@ bool gemm_tile_qkv_ok(int M, int N, int K, int hd, int min_wgs);
 hipError_t launch_gemm_tile_qkv(const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int M, const QkvArgs& qa, int min_wgs,
                                 hipStream_t s);
 // rows in groups that start at multiples of `align` (128 or 256), every group with weights [N x K] of its own, group g's w_group uint4 behind
-// the first: post relu2(pre x.W_g^T) as planes in xpack_off order, or plain f32 [positions][N].  w.N, w.K: sizes of one group.
+// the first: post relu2(pre x.W_g^T) as planes in xpack_off order (x: row-major planes [x_rows][K], position p is row src[p]), or plain f32
+// [positions][N] (x: planes of positions in xpack_off order).  w.N, w.K: sizes of one group.
 struct TileGroups {
     const int* tile_group = nullptr;  // group of every `align` positions, -1: unused
     int align = 256;
     int64_t w_group = 0;
+    const int* src = nullptr;         // [positions], with planes; -1: padding
+    int x_rows = 0;
     const float* pre = nullptr;       // [positions], with planes
     const float* post = nullptr;
 };

@@ -752,8 +752,9 @@ int LatentModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
         AddNormArgs na = base;
         na.residual_out = m->resid;
         // the feed-forward's input: its own norm's output, or the mixer's where they share the norm (twice when the products want other orders)
-        if (w.experts.on() && !f32) pg.packed = experts_packed(m, w.experts, R, pq.packed);
-        const bool mlp = w.ff || w.experts.on(), same = L.cfg.one_norm && (f32 || pg.packed == pq.packed);
+        const bool mlp = w.ff || w.experts.on(), gathers = w.experts.on() && !f32 && experts_gather(m, w.experts, R);
+        if (w.experts.on()) pg.packed = gathers ? 0 : pq.packed;
+        const bool same = L.cfg.one_norm && (f32 || pg.packed == pq.packed);
         na.w[0] = w.norm1; na.w[1] = !mlp || same ? nullptr : L.cfg.one_norm ? w.norm1 : w.norm2;
         const float* y_ff = same ? L.y1 : L.y2;
         const bf16_bits *ffh = same ? m->xh : L.x2h, *ffl = same ? m->xl : L.x2l;
@@ -770,7 +771,8 @@ int LatentModel::forward_chunk(nvllm_model* m, int R, int n_tiles, int qt, int n
         int no = 1, nd = 1;
         BranchSum ff;
         if (w.experts.on()) {
-            rc = run_experts(m, w.experts, L.experts, ffh, ffl, pg.packed, f32 ? y_ff : nullptr, R, L.slabs2, &ff);
+            const bool two = gathers && L.cfg.one_norm && !same;  // the mixer's planes serve the shared expert and the router
+            rc = run_experts(m, w.experts, L.experts, two ? m->xh : ffh, two ? m->xl : ffl, two ? pq.packed : pg.packed, ffh, ffl, f32 ? y_ff : nullptr, R, L.slabs2, &ff);
             if (rc) return rc;
         }
         if (w.ff) {

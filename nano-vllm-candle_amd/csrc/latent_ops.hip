@@ -228,7 +228,8 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
             uint16_t h[8], l[8];
 #pragma unroll
             for (int e = 0; e < 8; ++e) split_bf16(raw ? v[i][e] : (v[i][e] * rinv) * wv[e], h[e], l[e]);
-            const size_t o = ((size_t)blockIdx.x * KT + kt) * 64 + lane;
+            if (!a.packed[k] && row >= rows) continue;
+            const size_t o = a.packed[k] ? ((size_t)blockIdx.x * KT + kt) * 64 + lane : (((size_t)row * a.ldx) >> 3) + kt * 4 + grp;
             reinterpret_cast<uint4*>(a.xh[k])[o] = make_uint4(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16), h[4] | ((uint32_t)h[5] << 16), h[6] | ((uint32_t)h[7] << 16));
             reinterpret_cast<uint4*>(a.xl[k])[o] = make_uint4(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16), l[4] | ((uint32_t)l[5] << 16), l[6] | ((uint32_t)l[7] << 16));
         }
@@ -242,7 +243,7 @@ hipError_t launch_add_norm(const AddNormArgs& a, int rows, hipStream_t s) {
     const bool post = a.post_w != nullptr, any = a.w[0] || a.w[1] || a.raw;
     if (a.raw && a.w[0]) return hipErrorInvalidValue;
     bool packed = any && a.ldr == a.ldx && a.ldr % 32 == 0 && !a.row_idx && (!post || a.residual_in);
-    for (int k = 0; k < 2; ++k) packed &= !(a.w[k] || (k == 0 && a.raw)) || (a.packed[k] && a.xh[k] && !a.y[k]);
+    for (int k = 0; k < 2; ++k) packed &= !(a.w[k] || (k == 0 && a.raw)) || ((a.packed[k] || (k == 1 && a.w[0])) && a.xh[k] && !a.y[k]);
     if ((a.center && (post || a.raw)) || (a.ld_in && (!packed || a.ldr > 4096 || a.ld_in % 4 || a.slab_stride % 4))) return hipErrorInvalidValue;
     auto launch = [&](auto P) {
         constexpr int KIND = decltype(P)::value;

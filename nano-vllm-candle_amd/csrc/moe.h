@@ -49,9 +49,5 @@ struct GroupGemmArgs {
     int ldo = 0;
 };
 hipError_t launch_group_gemm(const GroupGemmArgs& a, hipStream_t s);
-// planes of the rows src[p] in position order, fragment order (the source in fragment order or row-major as told; K % 32 == 0); padding
-// positions of a group: zeros, unused tiles: not written
-hipError_t launch_gather_planes(const bf16_bits* xh, const bf16_bits* xl, int packed, int rows, const int* src, const int* tile_group, int align, int positions, int K,
-                                bf16_bits* oh, bf16_bits* ol, hipStream_t s);
 
 }  // namespace nvllm

@@ -7,60 +7,70 @@
 namespace nvllm {
 
 // ---------------------------------------------------------------------------------------------------
-// choice: one wave per row; lane l holds the logits of experts l, l + 64, ...
+// choice: NL lanes per row (16, 32 or a wave); lane l of them holds the logits of experts l, l + NL, ...
 // ---------------------------------------------------------------------------------------------------
 __device__ __forceinline__ float sigmoid_exact(float x) { return 1.0f / (1.0f + expf(-x)); }
 
-template <int NV>
+template <int NV, int NL>
 __device__ __forceinline__ void route_row(const RouteArgs& a, int row, int lane) {
-    const float* z = a.z + (size_t)row * a.ld;
+    const bool in = row < a.rows;  // lanes past the last row take part in the exchanges
+    const float* z = a.z + (size_t)min(row, a.rows - 1) * a.ld;
     float v[NV];
+    float gate = 0.f;
+    if (a.gate_col >= 0) gate = z[a.gate_col];
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-        const int e = lane + i * 64;
+        const int e = lane + i * NL;
         const float x = z[min(e, a.experts - 1)];
         v[i] = e < a.experts ? x : -INFINITY;
     }
-    if (a.gate_col >= 0 && lane == 0) a.gate[row] = sigmoid_exact(z[a.gate_col]);
+    if (a.gate_col >= 0 && lane == 0 && in) a.gate[row] = sigmoid_exact(gate);
     for (int k = 0; k < a.top; ++k) {
         float best = -INFINITY;
         int at = kMaxExperts;  // the lowest index wins a tie
 #pragma unroll
         for (int i = 0; i < NV; ++i)
-            if (v[i] > best) { best = v[i]; at = lane + i * 64; }
+            if (v[i] > best) { best = v[i]; at = lane + i * NL; }
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
+        for (int o = NL / 2; o > 0; o >>= 1) {
             const float b = __shfl_xor(best, o);
             const int c = __shfl_xor(at, o);
             if (b > best || (b == best && c < at)) { best = b; at = c; }
         }
         at = min(at, a.experts - 1);  // no finite logit left
-        if (lane == 0) {
+        if (lane == 0 && in) {
             a.chosen[(size_t)row * a.top + k] = at;
             a.score[(size_t)row * a.top + k] = sigmoid_exact(best);
         }
 #pragma unroll
         for (int i = 0; i < NV; ++i)
-            if (at == lane + i * 64) v[i] = -INFINITY;
+            if (at == lane + i * NL) v[i] = -INFINITY;
     }
 }
-template <int NV>
+template <int NV, int NL>
 __global__ void __launch_bounds__(256) route_kernel(RouteArgs a) {
-    const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (row < a.rows) route_row<NV>(a, row, threadIdx.x & 63);
+    route_row<NV, NL>(a, blockIdx.x * (256 / NL) + threadIdx.x / NL, threadIdx.x % NL);
 }
 
 // one workgroup: group sizes, starts and every row's position; NV > 0: the choice as well (few rows)
-template <int NV>
+template <int NV, int NL>
 __global__ void __launch_bounds__(1024) group_rows_kernel(RouteArgs a) {
     __shared__ int count[kMaxExperts + 1], start[kMaxExperts + 1], wave_total[16];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int groups = a.experts + a.shared_group, n = a.rows * a.top;
     for (int g = tid; g <= kMaxExperts; g += 1024) count[g] = 0;
     if constexpr (NV > 0)
-        for (int row = wave; row < a.rows; row += 16) route_row<NV>(a, row, lane);
+        for (int r0 = 0; r0 < a.rows; r0 += 1024 / NL) route_row<NV, NL>(a, r0 + tid / NL, tid % NL);
     __syncthreads();
-    for (int i = tid; i < n; i += 1024) atomicAdd(&count[a.chosen[i]], 1);
+    constexpr int U = 8;  // loads in flight
+    for (int i0 = tid; i0 < n; i0 += 1024 * U) {
+        int g[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) g[u] = a.chosen[min(i0 + u * 1024, n - 1)];
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+            if (i0 + u * 1024 < n) atomicAdd(&count[g[u]], 1);
+    }
     if (a.shared_group && tid == 0) count[a.experts] = a.rows;
     __syncthreads();
     // exclusive prefix sum of the aligned sizes: two groups per thread (groups <= 1025: the last thread takes the odd one)
@@ -92,13 +102,24 @@ __global__ void __launch_bounds__(1024) group_rows_kernel(RouteArgs a) {
     const int per = a.top + a.shared_group;
     for (int g = tid; g <= kMaxExperts; g += 1024) count[g] = 0;
     __syncthreads();
-    for (int i = tid; i < n; i += 1024) {
-        const int g = a.chosen[i], row = i / a.top, k = i - row * a.top, p = start[g] + atomicAdd(&count[g], 1);
-        const float sc = a.score[i];
-        a.src[p] = row;
-        a.pre[p] = a.weight_in ? sc : 1.f;
-        a.post[p] = a.weight_in ? 1.f : sc;
-        a.place[(size_t)row * per + k] = p;
+    for (int i0 = tid; i0 < n; i0 += 1024 * U) {
+        int g[U];
+        float sc[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            g[u] = a.chosen[min(i0 + u * 1024, n - 1)];
+            sc[u] = a.score[min(i0 + u * 1024, n - 1)];
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int i = i0 + u * 1024;
+            if (i >= n) continue;
+            const int row = i / a.top, k = i - row * a.top, p = start[g[u]] + atomicAdd(&count[g[u]], 1);
+            a.src[p] = row;
+            a.pre[p] = a.weight_in ? sc[u] : 1.f;
+            a.post[p] = a.weight_in ? 1.f : sc[u];
+            a.place[(size_t)row * per + k] = p;
+        }
     }
     if (a.shared_group)
         for (int row = tid; row < a.rows; row += 1024) {
@@ -118,17 +139,19 @@ hipError_t launch_route(const RouteArgs& a, hipStream_t s) {
     if (a.rows <= 0) return hipSuccess;
     const bool one = a.rows <= 64;
     const int nv = (a.experts + 63) / 64;
-#define NVLLM_RT(V_)                                                        \
-    if (one) group_rows_kernel<V_><<<1, 1024, 0, s>>>(a);                   \
-    else {                                                                  \
-        route_kernel<V_><<<(a.rows + 3) / 4, 256, 0, s>>>(a);               \
-        group_rows_kernel<0><<<1, 1024, 0, s>>>(a);                         \
+#define NVLLM_RT(V_, L_)                                                                   \
+    if (one) group_rows_kernel<V_, L_><<<1, 1024, 0, s>>>(a);                              \
+    else {                                                                                 \
+        route_kernel<V_, L_><<<(a.rows + 256 / L_ - 1) / (256 / L_), 256, 0, s>>>(a);      \
+        group_rows_kernel<0, 64><<<1, 1024, 0, s>>>(a);                                    \
     }
-    if (nv <= 1) { NVLLM_RT(1) }
-    else if (nv <= 2) { NVLLM_RT(2) }
-    else if (nv <= 4) { NVLLM_RT(4) }
-    else if (nv <= 8) { NVLLM_RT(8) }
-    else { NVLLM_RT(16) }
+    if (a.experts <= 16) { NVLLM_RT(1, 16) }
+    else if (a.experts <= 32) { NVLLM_RT(1, 32) }
+    else if (nv <= 1) { NVLLM_RT(1, 64) }
+    else if (nv <= 2) { NVLLM_RT(2, 64) }
+    else if (nv <= 4) { NVLLM_RT(4, 64) }
+    else if (nv <= 8) { NVLLM_RT(8, 64) }
+    else { NVLLM_RT(16, 64) }
 #undef NVLLM_RT
     return hipGetLastError();
 }
@@ -275,30 +298,6 @@ hipError_t launch_group_gemm(const GroupGemmArgs& a, hipStream_t s) {
         else NVLLM_GG(1, 2, 4, false);
     }
 #undef NVLLM_GG
-    return hipGetLastError();
-}
-
-__global__ void __launch_bounds__(256) gather_planes_kernel(const uint4* __restrict__ xh, const uint4* __restrict__ xl, int packed, int rows, const int* __restrict__ src,
-                                                            const int* __restrict__ tile_group, int align, int K, uint4* __restrict__ oh, uint4* __restrict__ ol) {
-    if (tile_group[blockIdx.x * 16 / align] < 0) return;  // src is not set there
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, KT = K >> 5, grp = lane >> 4;
-    const int row = src[blockIdx.x * 16 + (lane & 15)];
-    const int rc = min(max(row, 0), rows - 1);
-    const size_t x0 = packed ? (size_t)(rc >> 4) * KT * 64 + (grp << 4) + (rc & 15) : ((size_t)rc * K >> 3) + grp;
-    const size_t step = packed ? 64 : 4, o0 = (size_t)blockIdx.x * KT * 64 + lane;
-    for (int kt = blockIdx.y * 4 + wave; kt < KT; kt += 4 * gridDim.y) {
-        uint4 h = xh[x0 + kt * step], l = xl[x0 + kt * step];
-        if (row < 0) h = l = make_uint4(0, 0, 0, 0);
-        oh[o0 + (size_t)kt * 64] = h;
-        ol[o0 + (size_t)kt * 64] = l;
-    }
-}
-hipError_t launch_gather_planes(const bf16_bits* xh, const bf16_bits* xl, int packed, int rows, const int* src, const int* tile_group, int align, int positions, int K,
-                                bf16_bits* oh, bf16_bits* ol, hipStream_t s) {
-    if (K % 32 || positions % 16 || align < 16 || align % 16 || rows < 1) return hipErrorInvalidValue;
-    if (positions <= 0) return hipSuccess;
-    gather_planes_kernel<<<dim3(positions / 16, std::max(1, std::min(K / 128, 4))), 256, 0, s>>>(reinterpret_cast<const uint4*>(xh), reinterpret_cast<const uint4*>(xl), packed, rows, src, tile_group, align, K,
-                                                                                              reinterpret_cast<uint4*>(oh), reinterpret_cast<uint4*>(ol));
     return hipGetLastError();
 }
 

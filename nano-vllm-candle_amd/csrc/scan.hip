@@ -7,7 +7,8 @@
 
 namespace nvllm {
 
-__device__ __forceinline__ float silu_exact(float x) { return x / (1.0f + expf(-x)); }
+// x / (1 + e^-x) with the hardware exponential and reciprocal (an ulp each): the argument's rounding costs |x| 2^-24 of e^-x
+__device__ __forceinline__ float silu_fast(float x) { return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * -1.4426950408889634f)); }
 
 // ---------------------------------------------------------------------------------------------------
 // convolution rows: four channels per thread
@@ -34,7 +35,7 @@ __device__ __forceinline__ float4 row4(const float* p, int c, int channels) {
 }
 __device__ __forceinline__ void fma4(float4& y, const float4& x, const float4& w) { y.x += x.x * w.x; y.y += x.y * w.y; y.z += x.z * w.z; y.w += x.w * w.w; }
 __device__ __forceinline__ void conv_out(const ConvRowsArgs& a, int row, int c, const float4& y) {
-    const f32x4 v = {silu_exact(y.x), silu_exact(y.y), silu_exact(y.z), silu_exact(y.w)};
+    const f32x4 v = {silu_fast(y.x), silu_fast(y.y), silu_fast(y.z), silu_fast(y.w)};
     const int left = a.channels - c;
     float* o = a.x + (size_t)row * a.ldx + c;
     if (left >= 4) *reinterpret_cast<float4*>(o) = make_float4(v[0], v[1], v[2], v[3]);
@@ -86,38 +87,66 @@ __global__ void __launch_bounds__(256) conv_decode_kernel(ConvRowsArgs a) {
     fma4(y, cur, row4(a.conv + (size_t)H * a.channels, c, a.channels));
     conv_out(a, row, c, y);
 }
-// prompt chunks: 16 rows per workgroup, the window in registers
+// prompt chunks: a wave owns 16 rows x 32 channels, lane (grp, l15) row l15's eight consecutive channels: its plane stores in fragment
+// order are one contiguous KiB
 template <int TAPS>
 __global__ void __launch_bounds__(256) conv_rows16_kernel(ConvRowsArgs a, int rows) {
-    const int row0 = blockIdx.y * 16, row1 = min(row0 + 16, rows), c = (blockIdx.x * 256 + threadIdx.x) * 4;
-    if (c >= a.channels) return;
-    float4 w[TAPS], x[TAPS];
-#pragma unroll
-    for (int i = 0; i < TAPS; ++i) w[i] = row4(a.conv + (size_t)i * a.channels, c, a.channels);
-    const float4 bias = row4(a.bias, c, a.channels);
-    float4 ahead = conv_input4(a, row0, c);
-    for (int row = row0; row < row1; ++row) {
-        const bool start = row == 0 || a.slot[row - 1] != a.slot[row];
-        if (row == row0 || start) {
-            const RowPast p = row_past(a, row);
-#pragma unroll
-            for (int j = 1; j < TAPS; ++j) {
-                float t[4];
-#pragma unroll
-                for (int e = 0; e < 4; ++e) t[e] = c + e < a.channels ? past_input(a, p, row, j, c + e, a.channels) : 0.f;
-                x[TAPS - 1 - j] = make_float4(t[0], t[1], t[2], t[3]);
-            }
+    const int lane = threadIdx.x & 63, l15 = lane & 15, grp = lane >> 4;
+    const int row0 = blockIdx.y * 16, row = min(row0 + l15, rows - 1), kt = blockIdx.x * 4 + (threadIdx.x >> 6), c = kt * 32 + grp * 8;
+    if (kt * 32 >= a.channels) return;
+    float y[8], w[8];
+    auto eight = [&](float (&v)[8], const float* p, bool whole) {
+        if (whole) {
+            *reinterpret_cast<float4*>(&v[0]) = *reinterpret_cast<const float4*>(p);
+            *reinterpret_cast<float4*>(&v[4]) = *reinterpret_cast<const float4*>(p + 4);
         } else {
 #pragma unroll
-            for (int i = 0; i < TAPS - 1; ++i) x[i] = x[i + 1];
+            for (int e = 0; e < 8; ++e) v[e] = c + e < a.channels ? p[e] : 0.f;
         }
-        x[TAPS - 1] = ahead;
-        ahead = conv_input4(a, min(row + 1, rows - 1), c);
-        float4 y = bias;
+    };
+    const bool whole = (a.channels & 7) == 0 && c < a.channels;
+    eight(y, a.bias + c, whole);
+    // the window of every row of the wave inside this chunk (a sequence's rows are consecutive)
+    const int far = row - (TAPS - 1);
+    const bool inside = far >= 0 && a.slot[max(far, 0)] == a.slot[row];
+    if (__all(inside) && a.n_slabs == 1 && whole && (a.ld & 3) == 0) {
+        float x[TAPS][8];
 #pragma unroll
-        for (int i = 0; i < TAPS; ++i) fma4(y, x[i], w[i]);
-        conv_out(a, row, c, y);
+        for (int i = 0; i < TAPS; ++i) eight(x[i], a.in + (size_t)(far + i) * a.ld + c, true);
+#pragma unroll
+        for (int i = 0; i < TAPS; ++i) {
+            eight(w, a.conv + (size_t)i * a.channels + c, true);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) y[e] += x[i][e] * w[e];
+        }
+    } else {
+        const RowPast p = row_past(a, row);
+        for (int i = 0; i < TAPS; ++i) {
+            eight(w, a.conv + (size_t)i * a.channels + c, whole);
+#pragma unroll
+            for (int e = 0; e < 8; ++e)
+                if (c + e < a.channels) y[e] += past_input(a, p, row, TAPS - 1 - i, c + e, a.channels) * w[e];
+        }
     }
+    if (row0 + l15 >= rows) return;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) y[e] = silu_fast(y[e]);
+    float* o = a.x + (size_t)row * a.ldx + c;
+    if (whole) {
+        *reinterpret_cast<float4*>(o) = make_float4(y[0], y[1], y[2], y[3]);
+        *reinterpret_cast<float4*>(o + 4) = make_float4(y[4], y[5], y[6], y[7]);
+    } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+            if (c + e < a.channels) o[e] = y[e];
+    }
+    if (!a.xh) return;
+    uint16_t h[8], l[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) split_bf16(c + e < a.channels ? y[e] : 0.f, h[e], l[e]);
+    const size_t at = a.packed ? xpack_off(row, c, a.ldx >> 5) : (size_t)row * a.ldx + c;  // ldx is a multiple of 32: padding columns exist
+    *reinterpret_cast<uint4*>(a.xh + at) = make_uint4(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16), h[4] | ((uint32_t)h[5] << 16), h[6] | ((uint32_t)h[7] << 16));
+    *reinterpret_cast<uint4*>(a.xl + at) = make_uint4(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16), l[4] | ((uint32_t)l[5] << 16), l[6] | ((uint32_t)l[7] << 16));
 }
 hipError_t launch_conv_rows(const ConvRowsArgs& a, int rows, hipStream_t s) {
     if (a.taps < 1 || a.taps > kMaxTaps || a.channels > a.ld || a.channels > a.ldx || a.ldx % 32 || (a.taps > 1 && !a.history)) return hipErrorInvalidValue;
@@ -127,7 +156,7 @@ hipError_t launch_conv_rows(const ConvRowsArgs& a, int rows, hipStream_t s) {
         conv_decode_kernel<<<dim3(bx, rows), 256, 0, s>>>(a);
         return hipGetLastError();
     }
-    const dim3 grid(bx, (rows + 15) / 16);
+    const dim3 grid((a.channels + 127) / 128, (rows + 15) / 16);
     if (rows >= 64 && a.taps == 4) conv_rows16_kernel<4><<<grid, 256, 0, s>>>(a, rows);
     else if (rows >= 64 && a.taps == 3) conv_rows16_kernel<3><<<grid, 256, 0, s>>>(a, rows);
     else if (rows >= 64 && a.taps == 2) conv_rows16_kernel<2><<<grid, 256, 0, s>>>(a, rows);
@@ -203,7 +232,7 @@ __global__ void __launch_bounds__(256) scan_decode_kernel(ScanArgs a) {
     }
     store_states(st, S);
     y = lanes_sum<NL>(y);
-    if (q == 0) ys[lc] = (y + a.D[c] * x) * silu_exact(z);
+    if (q == 0) ys[lc] = (y + a.D[c] * x) * silu_fast(z);
     __syncthreads();
     if ((int)threadIdx.x * 4 < CH) put_row4(a, row, blockIdx.x * CH + threadIdx.x * 4, f32x4{ys[threadIdx.x * 4], ys[threadIdx.x * 4 + 1], ys[threadIdx.x * 4 + 2], ys[threadIdx.x * 4 + 3]});
 }
@@ -230,6 +259,8 @@ __global__ void __launch_bounds__(256) scan_prompt_kernel(ScanArgs a) {
     }
     if (CARRY && k == of - 1) return;
     load_states(A, a.A + at);
+    [[maybe_unused]] float D = 0.f;
+    if constexpr (!CARRY) D = a.D[c];
 #pragma unroll
     for (int i = 0; i < NS; ++i) S[i] = 0.f;
     float total = 0.f;
@@ -285,12 +316,13 @@ __global__ void __launch_bounds__(256) scan_prompt_kernel(ScanArgs a) {
         // U tokens at a time: everything but the state's own chain is independent.  Tokens past the end have dt = 0: the state stays.
         constexpr int U = NS == 4 ? 4 : 1;
         for (int t = 0; t < m; t += U) {
-            float dt[U], dx[U], B[U][NS], C[U][NS], y[U];
+            float dt[U], x[U], dx[U], B[U][NS], C[U][NS], y[U];
 #pragma unroll
             for (int u = 0; u < U; ++u) {
                 const int tt = t + u;
                 dt[u] = tt < m ? dts[tt * CH + lc] : 0.f;
-                dx[u] = dt[u] * xs[tt * CH + lc];
+                x[u] = xs[tt * CH + lc];
+                dx[u] = dt[u] * x[u];
                 load_states(B[u], bcs + tt * 2 * ST + q * NS);
                 if constexpr (!CARRY) load_states(C[u], bcs + tt * 2 * ST + ST + q * NS);
             }
@@ -308,7 +340,7 @@ __global__ void __launch_bounds__(256) scan_prompt_kernel(ScanArgs a) {
 #pragma unroll
                 for (int u = 0; u < U; ++u) {
                     y[u] = lanes_sum<NL>(y[u]);
-                    if (q == 0) xs[(t + u) * CH + lc] = y[u];  // this channel's x there has been read by its lanes' wave
+                    if (q == 0) xs[(t + u) * CH + lc] = y[u] + D * x[u];  // this channel's x there has been read by its lanes' wave
                 }
             }
         }
@@ -319,10 +351,7 @@ __global__ void __launch_bounds__(256) scan_prompt_kernel(ScanArgs a) {
                 const size_t row = row0 + t0 + t;
                 f32x4 v;
 #pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    const int cr = min(c0 + ch + r, a.channels - 1);
-                    v[r] = (xs[e + r] + a.D[cr] * a.x[row * a.ldx + cr]) * silu_exact(zs[e + r]);
-                }
+                for (int r = 0; r < 4; ++r) v[r] = xs[e + r] * silu_fast(zs[e + r]);
                 put_row4(a, (int)row, c0 + ch, v);
             }
         }

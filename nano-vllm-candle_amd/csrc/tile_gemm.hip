@@ -114,9 +114,21 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
     // DMA sources of this wave's copies at k-tile 0, without the lane part (advance: 64 uint4 per k-tile).  Row tiles
     // past the end are clamped to the last one: their products land in columns of D that are never stored.
     const uint4* src[NI];
+    [[maybe_unused]] uint32_t voff[NI], kstep[NI];  // MODE 5: x is row-major and its rows are gathered: lane part, uint4 per k-tile
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
         const int f = min(wave + 8 * i, FR - 1);
+        if constexpr (MODE == 5) {
+            voff[i] = lane;
+            kstep[i] = 64;
+            if (f >= FRW) {
+                const int g = f - FRW, row = a.g.src[mb * (WM * 64) + (g % XT) * 16 + l15];
+                src[i] = g >= XT ? a.xl : a.xh;
+                voff[i] = (uint32_t)min(max(row, 0), a.g.x_rows - 1) * (uint32_t)(a.KT * 4) + grp;  // padding: any row, its factors are 0
+                kstep[i] = 4;
+                continue;
+            }
+        }
         if (f < FRW) {
             // MODE 3: the block's two heads are nb and NB + nb, not neighbours: a V head (whose epilogue is scattered
             // 2-byte cache stores) then always shares its workgroup with a q head, and the V tail spreads over twice the CUs
@@ -134,7 +146,10 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
 #pragma unroll
         for (int i = 0; i < NI; ++i) {
             const int f = wave + 8 * i;
-            if (FR % 8 == 0 || f < FR)
+            if constexpr (MODE == 5) {
+                if (FR % 8 == 0 || f < FR)
+                    __builtin_amdgcn_global_load_lds((gptr_t)(src[i] + (size_t)min(s, KT - 1) * kstep[i] + voff[i]), (lptr_t)(lds + (size_t)(buf * FR + f) * 64), 16, 0, 0);
+            } else if (FR % 8 == 0 || f < FR)
                 __builtin_amdgcn_global_load_lds((gptr_t)(src[i] + koff + lane), (lptr_t)(lds + (size_t)(buf * FR + f) * 64), 16, 0, 0);
         }
     };
@@ -540,7 +555,7 @@ bool gemm_tile_group_ok(int N, int K, int align) { return group_shape(N, K, alig
 hipError_t launch_gemm_tile_group(const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int positions, const TileGroups& g, float* out, bf16_bits* act_hi,
                                   bf16_bits* act_lo, hipStream_t s) {
     const TileShape t = group_shape(w.N, w.K, g.align);
-    if (!t.ntw || positions % g.align || !g.tile_group || (act_hi && (!g.pre || !g.post))) return hipErrorNotSupported;
+    if (!t.ntw || positions % g.align || !g.tile_group || (act_hi && (!g.pre || !g.post || !g.src || g.x_rows < 1 || (int64_t)g.x_rows * w.K / 8 > INT32_MAX))) return hipErrorNotSupported;
     if (positions <= 0) return hipSuccess;
     TileArgs a;
     a.xh = reinterpret_cast<const uint4*>(xh); a.xl = reinterpret_cast<const uint4*>(xl); a.wp = w.data;
