@@ -76,6 +76,7 @@ int ExpertsScratch::alloc(nvllm_ctx* ctx, bool f32) {
     if (!rc) rc = dmalloc(ctx, &place, n_place);
     for (float** p : {&pre, &post}) if (!rc) rc = dmalloc(ctx, p, cap);
     if (!rc) rc = dmalloc(ctx, &src, cap);
+    if (!rc) rc = dmalloc(ctx, &cursor, kMaxExperts + 1);
     if (!rc) rc = dmalloc(ctx, &tile_group, cap / 16);
     if (!rc) rc = dmalloc(ctx, &out, (size_t)cap * n_out);
     if (f32) {
@@ -87,7 +88,7 @@ int ExpertsScratch::alloc(nvllm_ctx* ctx, bool f32) {
     return rc;
 }
 void ExpertsScratch::release() {
-    for (void* p : {(void*)z, (void*)score, (void*)gate, (void*)pre, (void*)post, (void*)out, (void*)act_f, (void*)chosen, (void*)place, (void*)src, (void*)tile_group, (void*)ah,
+    for (void* p : {(void*)z, (void*)score, (void*)gate, (void*)pre, (void*)post, (void*)out, (void*)act_f, (void*)chosen, (void*)place, (void*)src, (void*)tile_group, (void*)cursor, (void*)ah,
                     (void*)al, (void*)sh, (void*)sl})
         if (p) (void)hipFree(p);
     *this = ExpertsScratch();
@@ -120,7 +121,7 @@ int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_b
     ra.shared_group = e.sh > 0 && !tile;
     ra.align = tile ? tile : R * e.top >= 32 * e.experts ? 64 : 16;
     ra.cap = x.cap;
-    ra.chosen = x.chosen; ra.score = x.score; ra.gate = x.gate; ra.place = x.place; ra.src = x.src; ra.pre = x.pre; ra.post = x.post; ra.tile_group = x.tile_group;
+    ra.chosen = x.chosen; ra.score = x.score; ra.gate = x.gate; ra.place = x.place; ra.src = x.src; ra.pre = x.pre; ra.post = x.post; ra.tile_group = x.tile_group; ra.cursor = x.cursor;
     PROF(m, PROF_QK, launch_route(ra, s));
     const int64_t longest = (int64_t)R * e.top + (int64_t)std::min(e.experts, R * e.top) * (ra.align - 1) + (ra.shared_group ? R + ra.align - 1 : 0);
     out->gather = x.out; out->gather_row = x.place; out->n_gather = e.top + ra.shared_group;

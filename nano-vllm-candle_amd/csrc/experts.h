@@ -34,7 +34,7 @@ struct ExpertsBlock {
 struct ExpertsScratch {
     int cap = 0, lda = 0;
     float *z = nullptr, *score = nullptr, *gate = nullptr, *pre = nullptr, *post = nullptr, *out = nullptr, *act_f = nullptr;
-    int *chosen = nullptr, *place = nullptr, *src = nullptr, *tile_group = nullptr;
+    int *chosen = nullptr, *place = nullptr, *src = nullptr, *tile_group = nullptr, *cursor = nullptr;
     bf16_bits *ah = nullptr, *al = nullptr, *sh = nullptr, *sl = nullptr;
     void reserve(const ExpertsBlock& e, size_t rows);       // sizes first, for every block, ...
     int alloc(nvllm_ctx* ctx, bool f32);                    // ... then the buffers

@@ -23,6 +23,7 @@ struct RouteArgs {
     float* pre = nullptr;        // [cap] factor of the expert's input
     float* post = nullptr;       // [cap] factor of its output
     int* tile_group = nullptr;   // [cap / align] group of a tile, -1: unused
+    int* cursor = nullptr;       // [experts + 1] scratch
 };
 hipError_t launch_route(const RouteArgs& a, hipStream_t s);
 

@@ -52,7 +52,23 @@ __global__ void __launch_bounds__(256) route_kernel(RouteArgs a) {
     route_row<NV, NL>(a, blockIdx.x * (256 / NL) + threadIdx.x / NL, threadIdx.x % NL);
 }
 
-// one workgroup: group sizes, starts and every row's position; NV > 0: the choice as well (few rows)
+// a member's entries
+__device__ __forceinline__ void place_row(const RouteArgs& a, int i, int p, float score) {
+    const int row = i / a.top, k = i - row * a.top;
+    a.src[p] = row;
+    a.pre[p] = a.weight_in ? score : 1.f;
+    a.post[p] = a.weight_in ? 1.f : score;
+    a.place[(size_t)row * (a.top + a.shared_group) + k] = p;
+}
+__device__ __forceinline__ void place_shared(const RouteArgs& a, int row, int p) {
+    a.src[p] = row;
+    a.pre[p] = 1.f;
+    a.post[p] = a.gate_col >= 0 ? a.gate[row] : 1.f;
+    a.place[(size_t)row * (a.top + 1) + a.top] = p;
+}
+
+// one workgroup: group sizes, starts, tiles and padding.  NV > 0 (few rows): the choice and every row's position as well; else the positions
+// are left to place_rows_kernel, which starts from cursor.
 template <int NV, int NL>
 __global__ void __launch_bounds__(1024) group_rows_kernel(RouteArgs a) {
     __shared__ int count[kMaxExperts + 1], start[kMaxExperts + 1], wave_total[16];
@@ -62,7 +78,7 @@ __global__ void __launch_bounds__(1024) group_rows_kernel(RouteArgs a) {
     if constexpr (NV > 0)
         for (int r0 = 0; r0 < a.rows; r0 += 1024 / NL) route_row<NV, NL>(a, r0 + tid / NL, tid % NL);
     __syncthreads();
-    constexpr int U = 8;  // loads in flight
+    constexpr int U = NV > 0 ? 1 : 8;  // loads in flight
     for (int i0 = tid; i0 < n; i0 += 1024 * U) {
         int g[U];
 #pragma unroll
@@ -73,8 +89,8 @@ __global__ void __launch_bounds__(1024) group_rows_kernel(RouteArgs a) {
     }
     if (a.shared_group && tid == 0) count[a.experts] = a.rows;
     __syncthreads();
-    // exclusive prefix sum of the aligned sizes: two groups per thread (groups <= 1025: the last thread takes the odd one)
-    const int g0 = tid, sz = g0 < groups ? (count[g0] + a.align - 1) / a.align * a.align : 0;
+    // exclusive prefix sum of the aligned sizes, one group per thread (a shared group after 1024 experts: the first thread again)
+    const int sz = tid < groups ? (count[tid] + a.align - 1) / a.align * a.align : 0;
     int inc = sz;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
@@ -88,53 +104,48 @@ __global__ void __launch_bounds__(1024) group_rows_kernel(RouteArgs a) {
         if (w < wave) base += wave_total[w];
         all += wave_total[w];
     }
-    if (g0 < groups) start[g0] = base + inc - sz;
-    if (groups > 1024 && tid == 0) start[1024] = all;  // the shared group after 1024 experts
+    if (tid < groups) start[tid] = base + inc - sz;
+    if (groups > 1024 && tid == 0) start[1024] = all;
     __syncthreads();
     const int end = groups > 1024 ? all + (count[1024] + a.align - 1) / a.align * a.align : all;
-    for (int g = tid; g < groups; g += 1024) {
+    for (int g = wave; g < groups; g += 16) {
         const int p0 = start[g], c = count[g], p1 = p0 + (c + a.align - 1) / a.align * a.align;
-        for (int t = p0 / a.align; t < p1 / a.align; ++t) a.tile_group[t] = g;
-        for (int p = p0 + c; p < p1; ++p) { a.src[p] = -1; a.pre[p] = 0.f; a.post[p] = 0.f; }
+        for (int t = p0 / a.align + lane; t < p1 / a.align; t += 64) a.tile_group[t] = g;
+        for (int p = p0 + c + lane; p < p1; p += 64) { a.src[p] = -1; a.pre[p] = 0.f; a.post[p] = 0.f; }
     }
     for (int t = end / a.align + tid; t < a.cap / a.align; t += 1024) a.tile_group[t] = -1;
-    __syncthreads();
-    const int per = a.top + a.shared_group;
-    for (int g = tid; g <= kMaxExperts; g += 1024) count[g] = 0;
-    __syncthreads();
-    for (int i0 = tid; i0 < n; i0 += 1024 * U) {
-        int g[U];
-        float sc[U];
-#pragma unroll
-        for (int u = 0; u < U; ++u) {
-            g[u] = a.chosen[min(i0 + u * 1024, n - 1)];
-            sc[u] = a.score[min(i0 + u * 1024, n - 1)];
-        }
-#pragma unroll
-        for (int u = 0; u < U; ++u) {
-            const int i = i0 + u * 1024;
-            if (i >= n) continue;
-            const int row = i / a.top, k = i - row * a.top, p = start[g[u]] + atomicAdd(&count[g[u]], 1);
-            a.src[p] = row;
-            a.pre[p] = a.weight_in ? sc[u] : 1.f;
-            a.post[p] = a.weight_in ? 1.f : sc[u];
-            a.place[(size_t)row * per + k] = p;
+    if constexpr (NV == 0) {
+        for (int g = tid; g < groups; g += 1024) a.cursor[g] = start[g];
+    } else {
+        __syncthreads();
+        for (int i = tid; i < n; i += 1024) place_row(a, i, atomicAdd(&start[a.chosen[i]], 1), a.score[i]);
+        if (a.shared_group) {
+            __syncthreads();
+            for (int row = tid; row < a.rows; row += 1024) place_shared(a, row, start[a.experts] + row);
         }
     }
-    if (a.shared_group)
-        for (int row = tid; row < a.rows; row += 1024) {
-            const int p = start[a.experts] + row;
-            a.src[p] = row;
-            a.pre[p] = 1.f;
-            a.post[p] = a.gate_col >= 0 ? a.gate[row] : 1.f;
-            a.place[(size_t)row * per + a.top] = p;
-        }
+}
+// many rows: a workgroup reserves a range of every group for its share of them.  The order of a group's members does not matter: every
+// position is computed alone.
+__global__ void __launch_bounds__(1024) place_rows_kernel(RouteArgs a) {
+    __shared__ int count[kMaxExperts], base[kMaxExperts];
+    const int tid = threadIdx.x, n = a.rows * a.top, i = blockIdx.x * 1024 + tid;
+    for (int g = tid; g < a.experts; g += 1024) count[g] = 0;
+    __syncthreads();
+    const int g = i < n ? a.chosen[i] : 0;
+    const float score = i < n ? a.score[i] : 0.f;
+    const int at = i < n ? atomicAdd(&count[g], 1) : 0;
+    __syncthreads();
+    for (int e = tid; e < a.experts; e += 1024) base[e] = count[e] ? atomicAdd(&a.cursor[e], count[e]) : 0;
+    __syncthreads();
+    if (i < n) place_row(a, i, base[g] + at, score);
+    if (a.shared_group && i < a.rows) place_shared(a, i, a.cursor[a.experts] + i);
 }
 
 hipError_t launch_route(const RouteArgs& a, hipStream_t s) {
     const int64_t need = (int64_t)a.rows * a.top + (int64_t)std::min(a.experts, a.rows * a.top) * (a.align - 1) + (a.shared_group ? a.rows + a.align - 1 : 0);
     if (a.experts < 1 || a.experts > kMaxExperts || a.top < 1 || a.top > std::min(a.experts, kMaxTop) || a.align < 1 || a.cap % a.align || need > a.cap ||
-        a.ld < a.experts || a.gate_col >= a.ld || (a.gate_col >= 0 && !a.gate))
+        a.ld < a.experts || a.gate_col >= a.ld || (a.gate_col >= 0 && !a.gate) || !a.cursor)
         return hipErrorInvalidValue;
     if (a.rows <= 0) return hipSuccess;
     const bool one = a.rows <= 64;
@@ -144,6 +155,7 @@ hipError_t launch_route(const RouteArgs& a, hipStream_t s) {
     else {                                                                                 \
         route_kernel<V_, L_><<<(a.rows + 256 / L_ - 1) / (256 / L_), 256, 0, s>>>(a);      \
         group_rows_kernel<0, 64><<<1, 1024, 0, s>>>(a);                                    \
+        place_rows_kernel<<<(a.rows * a.top + 1023) / 1024, 1024, 0, s>>>(a);              \
     }
     if (a.experts <= 16) { NVLLM_RT(1, 16) }
     else if (a.experts <= 32) { NVLLM_RT(1, 32) }
