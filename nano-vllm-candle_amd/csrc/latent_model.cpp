@@ -199,7 +199,8 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
         w.Nq = wide(w.heads * (w.c.dim + w.c.rot_dim) + (w.c.q_rank ? 0 : latent_rows));
         w.Kc = up(w.heads * w.c.vdim, 128);
         if (w.c.q_rank) {
-            w.Nd = wide(w.c.q_rank + latent_rows); w.Kq = up(w.c.q_rank, 128);
+            const int rows = w.c.q_rank + latent_rows;
+            w.Nd = rows >= 512 && rows < 1536 && !c.f32 ? up(rows, 256) : wide(rows); w.Kq = up(w.c.q_rank, 128);
             if (!rc) rc = alloc_w(w.dq, w.Nd, L.Kw);
             if (!rc) rc = alloc_v(&w.dq_norm, w.Kq);
         }
