@@ -91,7 +91,7 @@ void ScanMixer::free_kv() {
     }
 }
 
-constexpr int kShortestPiece = 64, kScanWaves = 2048;  // rows of a piece at least; waves the pieces of a chunk aim at
+constexpr int kShortestPiece = 64, kScanWaves = 1024;  // rows of a piece at least; waves the pieces of a chunk aim at
 
 void ScanScratch::reserve(const ScanMixer& w, size_t R) {
     n_x = std::max(n_x, R * w.Kc);
