@@ -73,7 +73,7 @@ def test_missing_library_raises(monkeypatch, tmp_path):
 def _kernel_resources():
     out = {}
     for name in ("kernel_resources.txt", "kernel_resources_tile.txt", "kernel_resources_latent.txt", "kernel_resources_latent_prefill.txt", "kernel_resources_bias_attn.txt",
-                 "kernel_resources_recurrent.txt", "kernel_resources_recurrent_chunk.txt"):
+                 "kernel_resources_recurrent.txt", "kernel_resources_recurrent_chunk.txt", "kernel_resources_scan.txt", "kernel_resources_moe.txt"):
         path = os.path.join(ROOT, "nano-vllm-candle_amd", name)
         if not os.path.exists(path):
             pytest.skip(name + " missing: rebuild the library (make -C nano-vllm-candle_amd/csrc)")
@@ -139,3 +139,15 @@ def test_bias_attention_and_recurrence_kernels_stay_in_registers():
             assert r["Occupancy [waves/SIMD]"] >= 2, (n, r)
         if "recurrence_decode_kernelILi2" in n:
             assert r["Occupancy [waves/SIMD]"] >= 4 and r["ScratchSize [bytes/lane]"] == 0, (n, r)
+
+
+def test_scan_and_expert_kernels_stay_in_registers():
+    res = _kernel_resources()
+    for part, count in (("scan_prompt_kernel", 18), ("scan_decode_kernel", 9), ("conv_rows16_kernel", 3), ("group_gemm_kernel", 4), ("gemm_tile_kernelILi8ELi2ELi5", 1), ("gemm_tile_kernelILi8ELi2ELi6", 1)):
+        hits = {n: r for n, r in res.items() if part in n and "piece_scan" not in n}
+        assert len(hits) == count, (part, len(hits))
+        for n, r in hits.items():
+            assert r["ScratchSize [bytes/lane]"] == 0, (n, r)
+    for n, r in res.items():
+        if "scan_prompt_kernelILi4ELi4E" in n or "scan_decode_kernelILi4ELi4E" in n:
+            assert r["Occupancy [waves/SIMD]"] >= 4, (n, r)
