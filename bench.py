@@ -527,7 +527,7 @@ def main():
     # an event pair around nothing, recorded between busy kernels: what every bracket adds to a launch's duration
     # A bracket around a launch adds less than a whole empty bracket (the second event's processing overlaps the
     # kernel's tail).  Calibration against rocprofv3 --kernel-trace of this command, compared on the SAME step window
-    # (round 1 compared a bracketed figure of the later, longer-context profile steps with rocprof's all-step average and
+    # (an earlier version compared a bracketed figure of the later, longer-context profile steps with rocprof's all-step average and
     # took 0.8): bracketed 26.79 us on the profile steps (95.9 MB per launch), empty bracket 5.89 us, rocprof 22.70 us over
     # all steps (87.1 MB) = 24.3 us scaled to the profile steps' bytes (7 us fixed + a part proportional to the bytes):
     # excess 2.5 us = 0.42 of the empty bracket.  0.4 keeps the figure conservative (a slightly longer kernel).

@@ -383,7 +383,7 @@ def test_full_size_batch64_properties(pkg, ctx):
         _, l1 = m2.step([0], [prompts[i]], True, want_logits=True)
         # not bit-equal: a different batch shape picks a different split-K / chunking (f32 sum order), and an f16
         # rounding flip in a cached K/V element moves logits by ~1e-4; the bound is half the parity tolerance and must
-        # not drift: the measured value is printed (round 1: 9.0e-5)
+        # not drift: the measured value is printed (9.0e-5)
         e = rel_err(l1[0], lg[i])
         print(f"[parity] sequence {i} alone vs inside the batch of 64: {e:.3e} (bound 5e-4)")
         assert e < 5e-4

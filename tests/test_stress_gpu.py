@@ -17,7 +17,7 @@ from tests.util import oracle_config
 pytestmark = pytest.mark.gpu
 
 HEAVY = 1
-# Measured (round 3, MI355X; tools/numerics_study.py reproduces the shares on the CPU): with the default 16-bit cache the heavy
+# Measured (MI355X; tools/numerics_study.py reproduces the shares on the CPU): with the default 16-bit cache the heavy
 # profile lands at 0.5e-3 .. 1.2e-3 -- the f16 rounding of V (not normalised, heavy-tailed through the layernorm weights) is the
 # largest single term (6e-4 of ~7e-4), K 2..5e-4, P 1.5e-4.  The opt-in 24-bit V (kv_v_bits = 24: f16 + an e5m2 residual
 # byte, V bytes x1.5) removes that term.  Bars: 24-bit V must hold the 1e-3 parity tolerance; the default must stay under

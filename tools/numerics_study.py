@@ -20,7 +20,7 @@ ap.add_argument("--seeds", type=int, default=2)
 a = ap.parse_args()
 cfg = O.make_config(vocab_size=a.vocab, hidden_size=1024, head_dim=128, num_hidden_layers=a.layers, num_attention_heads=16,
                     num_key_value_heads=8, intermediate_size=3072)
-VARIANTS = [("K f16", 1), ("V f16", 2), ("P f16", 4), ("K+V+P f16 (shipped round 2)", 7), ("K bf16", 8), ("V bf16", 16),
+VARIANTS = [("K f16", 1), ("V f16", 2), ("P f16", 4), ("K+V+P f16 (the former default)", 7), ("K bf16", 8), ("V bf16", 16),
             ("K f16x2", 32), ("K f16x2 + V f16 + P f16", 32 | 2 | 4), ("K f16 + V f16 + P bf16x2", 1 | 2 | 128),
             ("K f16x2 + V f16 + P bf16x2", 32 | 2 | 128), ("K f16 + V f16x2 + P bf16x2", 1 | 64 | 128),
             ("V f16 + e5m2 lo", 256), ("K f16 + V f16+e5m2 + P f16", 1 | 256 | 4),
