@@ -150,36 +150,65 @@ typedef struct nvllm_latent_config {
  * D, o}, and l<i>.mlp.{gate, up, down} or l<i>.mlp.{router, e<k>.up, e<k>.down, shared.up, shared.down, shared.sg}. */
 int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_config* cfg, const nvllm_latent_layer* layers, nvllm_model** out);
 
-/* ---- hybrid decoders: every layer has one of three token mixers and optionally a squared-ReLU feed-forward; sublayers read the
- * residual stream itself and are normed on their output, x += residual_mult * norm(sublayer(x)).  Norm weights of layers and of the
- * output are stored minus norm_offset.  Loading, pool, step, sampling and decode are the same API as the Qwen3 model's; recurrent
- * state lives in the sequence's slot, and a step that asks for a sequence shorter than what was processed starts it again. */
-#define NVLLM_MIXER_ATTENTION 0 /* grouped-query attention, distance bias instead of positions */
+/* ---- hybrid decoders: every layer has a token mixer, or two side by side, and optionally a feed-forward (plain or routed).  Sublayers
+ * are normed on their output, x += residual_mult * norm(sublayer(x)), with pre_norm on their input too, and a range of layers may be
+ * passed through several times.  Norm weights of layers and of the output are stored minus norm_offset.  Loading, pool, step, sampling
+ * and decode are the same API as the Qwen3 model's; recurrent state lives in the sequence's slot, and a step that asks for a sequence
+ * shorter than what was processed starts it again. */
+#define NVLLM_MIXER_ATTENTION 0 /* grouped-query attention: distance bias, rotation, window, sink, short convolutions as configured */
 #define NVLLM_MIXER_LINEAR 1    /* S = decay_h S + k v^T, o = S^T q; silu inputs, one output norm over all heads, output gate */
-#define NVLLM_MIXER_DELTA 2     /* gated delta rule with a decay per key channel, short convolutions, output norm per head, output gate */
-typedef struct nvllm_hybrid_layer {
+#define NVLLM_MIXER_DELTA 2     /* gated delta rule, short convolutions, output norm per head, output gate */
+#define NVLLM_QK_NORM_ALL 0     /* RMS norm over the whole query (key) projection, with weights */
+#define NVLLM_QK_NORM_HEAD 1    /* RMS norm over each head after the rotation, no weights */
+#define NVLLM_SINK_NONE 0
+#define NVLLM_SINK_ONE 1        /* the softmax denominator has one more term exp(0) */
+#define NVLLM_SINK_HEAD 2       /* ... exp(sink_h), learned */
+#define NVLLM_ACT_RELU2 0
+#define NVLLM_ACT_GELU 1        /* x / 2 (1 + erf(x / sqrt 2)) */
+typedef struct nvllm_hybrid_mixer {
     int32_t mixer;
     int32_t heads, kv_heads, dim, vdim; /* per head: query/key and value size; kv_heads divides heads */
-    int32_t ff;                         /* feed-forward width, 0 = the layer has none */
     /* attention */
-    double scale;                       /* of q . k; q and k are RMS-normed over the whole projection before */
+    double scale;                       /* of q . k */
     int32_t bias_rows;                  /* rows of the distance table (0: no bias): half of them exact, the rest logarithmic up to bias_max */
     double bias_max;
-    int32_t sink;                       /* 1: the softmax denominator has one more term exp(0) */
+    int32_t sink;                       /* NVLLM_SINK_* */
     int32_t v_mix;                      /* 1: values are mixed with those of the first layer that has this set */
+    int32_t qk_norm;                    /* NVLLM_QK_NORM_*; convolutions and rotation go with NVLLM_QK_NORM_HEAD */
+    int32_t window;                     /* visible positions including the token itself; <= 0: all earlier ones */
+    int32_t rot_dim;                    /* the first dimensions of a head turn, 2 i with 2 i + 1 (0: none) */
+    double rot_base, yarn_factor, yarn_original, yarn_fast, yarn_slow; /* yarn_factor <= 0: no scaling */
+    int32_t out_bias;                   /* 1: the output projection has a bias */
     /* NVLLM_MIXER_LINEAR */
     const double* decay;                /* [heads], read by the create call only */
+    /* attention (0: no convolutions) and NVLLM_MIXER_DELTA */
+    int32_t conv_taps;
     /* NVLLM_MIXER_DELTA */
-    int32_t conv_taps, decay_rank, gate_rank;
+    int32_t decay_rank;                 /* > 0: a decay per head and key channel, projected in two steps; 0: one decay per head */
+    int32_t gate_rank;                  /* > 0: sigmoid of a projection in two steps; 0: silu of one projection */
+} nvllm_hybrid_mixer;
+typedef struct nvllm_hybrid_layer {
+    nvllm_hybrid_mixer mix;
+    int32_t branches;                   /* 2: `side` reads the same input, the result is half the sum of both outputs, each normed; else 1 */
+    nvllm_hybrid_mixer side;
+    int32_t ff;                         /* feed-forward width, 0 = the layer has none */
+    int32_t act;                        /* NVLLM_ACT_* */
+    int32_t experts, top, expert_ff;    /* routed feed-forward (ff = 0): silu-gated experts, softmax scores over all of them on the output; 0: none */
+    int32_t groups, groups_kept;        /* equal groups of neighbouring experts; only the best `groups_kept` by their largest score are open */
 } nvllm_hybrid_layer;
 typedef struct nvllm_hybrid_config {
     int32_t vocab_size, width, num_layers;
     double norm_eps, embed_scale, residual_mult, norm_offset;
     int32_t f32;                        /* 0: bf16 weights, hi + lo planes, f16 cache; 1: every product and the cache in f32 */
+    int32_t pre_norm;                   /* 1: the sublayers read norm1 (norm2) of the stream, their outputs are normed with norm1b (norm2b) */
+    int32_t loop_start, loop_stop, loop_times; /* layers [start, stop) are passed through loop_times times, each pass with a cache and state of
+                                           its own; the embedding output is added to the stream before every pass but the first; <= 1: no loop */
 } nvllm_hybrid_config;
-/* Tensor names for nvllm_model_load_tensor: embed, head, final.norm and, per layer, l<i>.norm1, l<i>.norm2, l<i>.mlp.{up, down},
- * l<i>.mix.o and by mixer: attention l<i>.mix.{q, k, v} with .b, .{q, k}.norm, .rel, .vmix (a scalar); linear l<i>.mix.{q, k, v, g,
- * norm}; delta l<i>.mix.{q, k, v} with .conv, .{b, A_log, a1, a2, dt_bias, g1, g2, norm}. */
+/* Tensor names for nvllm_model_load_tensor: embed, head, final.norm and, per layer, l<i>.norm1, l<i>.norm2 (with pre_norm .norm1b, .norm2b),
+ * l<i>.mlp.{up, down} or l<i>.mlp.{router, e<k>.gate, e<k>.up, e<k>.down}, and the mixer's under l<i>.mix (two mixers: l<i>.mix.left and
+ * l<i>.mix.right, each with the norm .out of its output): .o and by mixer: attention .{q, k, v} with .b (and .conv), .o.b, .{q, k}.norm,
+ * .rel, .vmix (a scalar), .sink; linear .{q, k, v, g, norm}; delta .{q, k, v} with .conv, .{b, A_log, dt_bias, norm}, .{a1, a2} or .a,
+ * .{g1, g2} or .g. */
 int nvllm_model_create_hybrid(nvllm_ctx* ctx, const nvllm_hybrid_config* cfg, const nvllm_hybrid_layer* layers, nvllm_model** out);
 
 /* ---- KV block pool (the real allocation the reference's stub BlockManager lacks,

@@ -8,6 +8,7 @@ from .engine import (LLMEngine, ModelRunner, CausalLMRunner, Qwen3ModelRunner, S
 from .berevik import BerevikConfig, BerevikForCausalLM  # noqa: F401
 from .causal_lm import CausalLM  # noqa: F401
 from .gopunex import GopunexConfig, GopunexForCausalLM  # noqa: F401
+from .lefalix import LefalixConfig, LefalixForCausalLM  # noqa: F401
 from .qwen3 import Qwen3Config, Qwen3ForCausalLM  # noqa: F401
 from .registry import MODELS, load_model  # noqa: F401
 from .tafopel import TafopelConfig, TafopelForCausalLM  # noqa: F401
@@ -15,5 +16,5 @@ from .tp import TPConfig, get_tp  # noqa: F401
 
 __all__ = ["Context", "DeviceArray", "Qwen3Config", "Qwen3ForCausalLM", "Qwen3ModelRunner", "LLMEngine", "Scheduler",
            "SchedulerConfig", "SamplingParams", "Sequence", "ModelRunner", "TPConfig", "get_tp", "CausalLM", "BerevikConfig",
-           "BerevikForCausalLM", "GopunexConfig", "GopunexForCausalLM", "TafopelConfig",
+           "BerevikForCausalLM", "GopunexConfig", "GopunexForCausalLM", "LefalixConfig", "LefalixForCausalLM", "TafopelConfig",
            "TafopelForCausalLM", "CausalLMRunner", "MODELS", "load_model"]

@@ -54,26 +54,39 @@ class LatentConfigC(C.Structure):
         (n, C.c_double) for n in ("norm_eps", "embed_scale", "logit_softcap")] + [(n, C.c_int32) for n in ("norm", "one_norm", "f32")]
 
 
-class HybridLayerC(C.Structure):
-    """nvllm_hybrid_layer"""
+class HybridMixerC(C.Structure):
+    """nvllm_hybrid_mixer"""
 
-    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "vdim", "ff")] + [
-        ("scale", C.c_double), ("bias_rows", C.c_int32), ("bias_max", C.c_double), ("sink", C.c_int32), ("v_mix", C.c_int32),
-        ("decay", C.POINTER(C.c_double)), ("conv_taps", C.c_int32), ("decay_rank", C.c_int32), ("gate_rank", C.c_int32),
-    ]
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "vdim")] + [
+        ("scale", C.c_double), ("bias_rows", C.c_int32), ("bias_max", C.c_double)] + [
+        (n, C.c_int32) for n in ("sink", "v_mix", "qk_norm", "window", "rot_dim")] + [
+        (n, C.c_double) for n in ("rot_base", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow")] + [
+        ("out_bias", C.c_int32), ("decay", C.POINTER(C.c_double)), ("conv_taps", C.c_int32), ("decay_rank", C.c_int32), ("gate_rank", C.c_int32)]
+
+
+class HybridLayerC(C.Structure):
+    """nvllm_hybrid_layer; the fields of `mix` are the layer's own names too"""
+
+    _anonymous_ = ("mix",)
+    _fields_ = [("mix", HybridMixerC), ("branches", C.c_int32), ("side", HybridMixerC)] + [
+        (n, C.c_int32) for n in ("ff", "act", "experts", "top", "expert_ff", "groups", "groups_kept")]
 
 
 class HybridConfigC(C.Structure):
     """nvllm_hybrid_config"""
 
     _fields_ = [(n, C.c_int32) for n in ("vocab_size", "width", "num_layers")] + [
-        (n, C.c_double) for n in ("norm_eps", "embed_scale", "residual_mult", "norm_offset")] + [("f32", C.c_int32)]
+        (n, C.c_double) for n in ("norm_eps", "embed_scale", "residual_mult", "norm_offset")] + [
+        (n, C.c_int32) for n in ("f32", "pre_norm", "loop_start", "loop_stop", "loop_times")]
 
 
 LATENT_ATTENTION, SELECTIVE_SCAN = 0, 1
 GLU_CLAMPED, GLU_GELU = 0, 1
 NORM_RMS, NORM_LAYER = 0, 1
 MIXER_ATTENTION, MIXER_LINEAR, MIXER_DELTA = 0, 1, 2  # NVLLM_MIXER_*
+QK_NORM_ALL, QK_NORM_HEAD = 0, 1
+SINK_NONE, SINK_ONE, SINK_HEAD = 0, 1, 2
+ACT_RELU2, ACT_GELU = 0, 1
 
 _vp, _fp = C.c_void_p, C.c_void_p  # device pointers travel as integers
 _SIGS = {

@@ -5,6 +5,7 @@ import ctypes as C
 import json
 import os
 import struct
+from dataclasses import dataclass
 
 import numpy as np
 
@@ -273,3 +274,16 @@ def random_matrix(shape, rng):
     """bf16 bits of unit output variance: random sign and mantissa, exponent of 1 / sqrt(fan-in)"""
     e = 127 - max(1, int(round(0.5 * np.log2(shape[1]))))
     return (rng.integers(0, 1 << 16, shape, dtype=np.uint16) & np.uint16(0x807F)) | np.uint16(e << 7)
+
+
+@dataclass
+class Yarn:
+    """YaRN scaling of a rotation"""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+    @classmethod
+    def from_dict(cls, d):
+        return cls(*(float(d[k]) for k in ("factor", "original", "fast", "slow"))) if d else None

@@ -1,5 +1,5 @@
-// gfx950 grouped-query attention over the paged cache with a distance bias and an optional sink term in the denominator:
-//   s = q . k (scaled) + bias[head][min(i - j, n_bias - 1)],  p_j = exp(s_j) / ([sink] + sum exp(s_j)),  j <= i.
+// gfx950 grouped-query attention over the paged cache with an optional distance bias, window and sink term in the denominator:
+//   s = q . k (scaled) + bias[head][min(i - j, n_bias - 1)],  p_j = exp(s_j) / ([exp(sink_h)] + sum exp(s_j)),  i - window < j <= i.
 // Scores, weights and sums are f32, in units of log2.  Query rows are (token, head of the group) pairs, so one cached key serves every
 // head of its group.  Matrix-core kernels (f16 cache): A = K (or V) fragment as stored, B = q (or P) as f16 hi + lo, the accumulator
 // layout of the scores is the B-fragment order of P.
@@ -9,6 +9,8 @@
 #include "hybrid.h"
 
 namespace nvllm {
+
+__device__ __forceinline__ int first_seen(int pos, int window) { return window > 0 ? max(0, pos - window + 1) : 0; }
 
 static const int kDimChunks[] = {1, 2, 3, 4, 8};   // of 32
 static const int kVdimTiles[] = {2, 4, 8, 16};     // of 16
@@ -53,12 +55,14 @@ __global__ void __launch_bounds__(256) bias_attn_plain_kernel(BiasAttnArgs a) {
     float o[NE], m = -1e30f, l = 0.f;
 #pragma unroll
     for (int e = 0; e < NE; ++e) o[e] = 0.f;
-    for (int j0 = wave * 64; j0 <= pos; j0 += 256) {
+    const int first = first_seen(pos, a.window);
+    for (int j0 = (first & ~63) + wave * 64; j0 <= pos; j0 += 256) {
         const int j = j0 + lane;
         const size_t blk = (size_t)bt[j0 / kBlockTokens] * c.kv + kvh;
         const T* kp = reinterpret_cast<const T*>(c.k) + blk * kBlockTokens * c.dim_p + k_packed_offset(j & (kBlockTokens - 1), 0, c.dim_p);
         float s = -1e30f;
-        if (j <= pos) {
+        const bool seen = j >= first && j <= pos;
+        if (seen) {
             s = 0.f;
             for (int d = 0; d < c.dim_p; d += 8) {
                 float k[8];
@@ -71,7 +75,7 @@ __global__ void __launch_bounds__(256) bias_attn_plain_kernel(BiasAttnArgs a) {
         float mt = s;
 #pragma unroll
         for (int x = 32; x > 0; x >>= 1) mt = fmaxf(mt, __shfl_xor(mt, x));
-        const float mn = fmaxf(m, mt), al = exp2f(m - mn), p = j <= pos ? exp2f(s - mn) : 0.f;
+        const float mn = fmaxf(m, mt), al = exp2f(m - mn), p = seen ? exp2f(s - mn) : 0.f;
         m = mn;
         l = l * al + wave_sum(p);
         pw[wave][lane] = p;  // read by this wave alone
@@ -99,9 +103,10 @@ __global__ void __launch_bounds__(256) bias_attn_plain_kernel(BiasAttnArgs a) {
     for (int e = 0; e < NE; ++e)
         if (lane + e * 64 < c.vdim_p) mine[2 + lane + e * 64] = o[e];
     __syncthreads();
-    float ms = a.sink ? 0.f : -1e30f, f[4];
+    const float sink = a.sink ? a.sink[head] : 0.f;
+    float ms = a.sink ? sink : -1e30f, f[4];
     for (int w = 0; w < 4; ++w) ms = fmaxf(ms, acc[(size_t)w * (c.vdim_p + 2)]);
-    float lt = a.sink ? exp2f(-ms) : 0.f;
+    float lt = a.sink ? exp2f(sink - ms) : 0.f;
     for (int w = 0; w < 4; ++w) {
         f[w] = exp2f(acc[(size_t)w * (c.vdim_p + 2)] - ms);
         lt += f[w] * acc[(size_t)w * (c.vdim_p + 2) + 1];
@@ -180,7 +185,8 @@ __global__ void __launch_bounds__(256) bias_decode_kernel(BiasAttnArgs a) {
     const int gqa = a.heads / a.kv.kv, hb = (gqa + 15) / 16, kvh = blockIdx.y / hb, h0 = (blockIdx.y % hb) * 16;
     const bool valid = h0 + l15 < gqa;
     const int head = kvh * gqa + min(h0 + l15, gqa - 1);
-    const int t_hi = (pos >> 5) + 1, t_begin = a.part_tiles ? (int)blockIdx.z * a.part_tiles : 0;
+    const int first = first_seen(pos, a.window), t_lo = first >> 5;
+    const int t_hi = (pos >> 5) + 1, t_begin = t_lo + (a.part_tiles ? (int)blockIdx.z * a.part_tiles : 0);
     const int t_end = a.part_tiles ? min(t_hi, t_begin + a.part_tiles) : t_hi;
     if (t_begin >= t_hi) return;
     const int* bt = a.block_tables + (size_t)a.slot[row] * a.max_blocks;
@@ -239,11 +245,12 @@ __global__ void __launch_bounds__(256) bias_decode_kernel(BiasAttnArgs a) {
 #pragma unroll
             for (int i = 0; i < 2 * DC; ++i) kf[i] = ld_stream16(p + i * 512);
         }
+        auto seen = [&](int j) { return j <= pos && j >= first; };
         float mt = -1e30f;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            if (tokA + r <= pos) mt = fmaxf(mt, sa[r]);
-            if (tokB + r <= pos) mt = fmaxf(mt, sb[r]);
+            if (seen(tokA + r)) mt = fmaxf(mt, sa[r]);
+            if (seen(tokB + r)) mt = fmaxf(mt, sb[r]);
         }
         mt = fmaxf(mt, __shfl_xor(mt, 16));
         mt = fmaxf(mt, __shfl_xor(mt, 32));
@@ -253,8 +260,8 @@ __global__ void __launch_bounds__(256) bias_decode_kernel(BiasAttnArgs a) {
         float ps = 0.f, pa[4], pb[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            pa[r] = tokA + r <= pos ? __builtin_amdgcn_exp2f(sa[r] - mn) : 0.f;
-            pb[r] = tokB + r <= pos ? __builtin_amdgcn_exp2f(sb[r] - mn) : 0.f;
+            pa[r] = seen(tokA + r) ? __builtin_amdgcn_exp2f(sa[r] - mn) : 0.f;
+            pb[r] = seen(tokB + r) ? __builtin_amdgcn_exp2f(sb[r] - mn) : 0.f;
             ps += pa[r] + pb[r];
         }
         split_weights(pa, pb, P, Pl);
@@ -274,11 +281,13 @@ __global__ void __launch_bounds__(256) bias_decode_kernel(BiasAttnArgs a) {
     lsum += __shfl_xor(lsum, 32);
     if (grp == 0) { ml[wave][0][l15] = m; ml[wave][1][l15] = lsum; }
     __syncthreads();
-    const int n_parts = a.part_tiles ? (t_hi + a.part_tiles - 1) / a.part_tiles : 1;
-    float ms = a.sink && n_parts == 1 ? 0.f : -1e30f;
+    const int n_parts = a.part_tiles ? (t_hi - t_lo + a.part_tiles - 1) / a.part_tiles : 1;
+    const bool sinks = a.sink && n_parts == 1;
+    const float sink = sinks ? a.sink[head] : 0.f;
+    float ms = sinks ? sink : -1e30f;
 #pragma unroll
     for (int w = 0; w < 4; ++w) ms = fmaxf(ms, ml[w][0][l15]);
-    float lt = a.sink && n_parts == 1 ? __builtin_amdgcn_exp2f(-ms) : 0.f;
+    float lt = sinks ? __builtin_amdgcn_exp2f(sink - ms) : 0.f;
 #pragma unroll
     for (int w = 0; w < 4; ++w) lt += ml[w][1][l15] * __builtin_amdgcn_exp2f(ml[w][0][l15] - ms);
     const float f = __builtin_amdgcn_exp2f(m - ms), scale = n_parts > 1 ? 1.0f : 1.0f / lt;
@@ -313,16 +322,17 @@ __global__ void __launch_bounds__(256) bias_combine_kernel(BiasAttnArgs a, int i
     const int lane = threadIdx.x & 63, it = blockIdx.x * 4 + (threadIdx.x >> 6);
     if (it >= items) return;
     const int row = it / a.heads, head = it % a.heads;
-    const int n = ((a.pos[row] >> 5) + 1 + a.part_tiles - 1) / a.part_tiles;
+    const int pos = a.pos[row], n = ((pos >> 5) + 1 - (first_seen(pos, a.window) >> 5) + a.part_tiles - 1) / a.part_tiles;
     if (n <= 1) return;  // written by the attention kernel
     const float* pm = a.part_ml + (size_t)it * a.max_parts * 2;
-    float ms = a.sink ? 0.f : -1e30f, mine = -1e30f, l = 0.f;
+    const float sink = a.sink ? a.sink[head] : 0.f;
+    float ms = a.sink ? sink : -1e30f, mine = -1e30f, l = 0.f;
     if (lane < n) { mine = pm[2 * lane]; l = pm[2 * lane + 1]; }  // at most kBiasMaxParts = 64 parts
     ms = fmaxf(ms, mine);
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) ms = fmaxf(ms, __shfl_xor(ms, o));
     const float w = lane < n ? exp2f(mine - ms) : 0.f;
-    const float inv = 1.0f / (wave_sum(w * l) + (a.sink ? exp2f(-ms) : 0.f));
+    const float inv = 1.0f / (wave_sum(w * l) + (a.sink ? exp2f(sink - ms) : 0.f));
     for (int e0 = 0; e0 < a.kv.vdim_p; e0 += 256) {  // every lane stays for the shuffles
         const int e = e0 + lane * 4;
         const float* po = a.part_o + (size_t)it * a.max_parts * a.kv.vdim_p + min(e, a.kv.vdim_p - 4);
@@ -386,7 +396,8 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
     if (f0 >= total) return;
     const int pos0 = a.pos[row0];
     const int pmin = pos0 + f0 / gqa, pmax = pos0 + min(f0 + RW - 1, total - 1) / gqa;
-    const int nt = (pmax >> 5) + 1;
+    const int nt = (pmax >> 5) + 1, t0 = first_seen(pmin, a.window) >> 5;
+    const int low = a.window > 0 ? pmax - a.window + 1 : 0;  // some row does not see the tokens before
     const int* bt = a.block_tables + (size_t)slot * a.max_blocks;
     const _Float16* kd = reinterpret_cast<const _Float16*>(a.kv.k);
     const _Float16* vd = reinterpret_cast<const _Float16*>(a.kv.v);
@@ -402,7 +413,7 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
             if (F % 4 == 0 || f < F) __builtin_amdgcn_global_load_lds((gptr_t)((f < 2 * DC ? kp : vp) + f * 64 + lane), (lptr_t)(b + f * 64), 16, 0, 0);
         }
     };
-    stage(0, buf[0]);
+    stage(t0, buf[t0 & 1]);
     if (bias_lds)
         for (int i = threadIdx.x; i < gqa * a.n_bias; i += 256) tab[i] = a.bias[(size_t)kvh * gqa * a.n_bias + i];
     int my_pos[MT];
@@ -436,7 +447,7 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
     }
     dma_publish_barrier();
     const uint32_t tab0 = lds_address(tab);
-    for (int t = 0; t < nt; ++t) {
+    for (int t = t0; t < nt; ++t) {
         const uint32_t b = lds_address(buf[t & 1]) + lane * 16;
         if (t + 1 < nt) stage(t + 1, buf[(t + 1) & 1]);  // its last readers have passed the barrier of the previous tile
         const int tokA = (t << 5) + grp * 4, tokB = tokA + 16;
@@ -499,15 +510,18 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
             for (int d = 0; d < VG; ++d) NVLLM_LDS_READ128(vf[d], b + d0 * 1024, (2 * DC + d) * 1024);
         };
         read_v(0);
-        const bool edge = (t << 5) + 31 > pmin;  // some row does not see the whole tile
+        const bool edge = (t << 5) + 31 > pmin || (t << 5) < low;  // some row does not see the whole tile
         f16x8 P[MT], Pl[MT];
 #pragma unroll
         for (int u = 0; u < MT; ++u) {
+            // distances 0 .. span - 1 are seen
+            const uint32_t span = a.window > 0 ? (uint32_t)a.window : 0x7fffffffu;
+            auto hidden = [&](int j) { return (uint32_t)(my_pos[u] - j) >= span; };
             if (edge) {
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    if (tokA + r > my_pos[u]) sa[u][r] = -1e30f;
-                    if (tokB + r > my_pos[u]) sb[u][r] = -1e30f;
+                    if (hidden(tokA + r)) sa[u][r] = -1e30f;
+                    if (hidden(tokB + r)) sb[u][r] = -1e30f;
                 }
             }
             float mt = fmaxf(max3_raw(sa[u][0], sa[u][1], sa[u][2]), max3_raw(sa[u][3], sb[u][0], sb[u][1]));
@@ -520,8 +534,8 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 // a row that sees nothing of any tile so far has mn = -1e30: its masked scores would count as exp2(0)
-                pa[r] = edge && tokA + r > my_pos[u] ? 0.f : __builtin_amdgcn_exp2f(sa[u][r] - mn);
-                pb[r] = edge && tokB + r > my_pos[u] ? 0.f : __builtin_amdgcn_exp2f(sb[u][r] - mn);
+                pa[r] = edge && hidden(tokA + r) ? 0.f : __builtin_amdgcn_exp2f(sa[u][r] - mn);
+                pb[r] = edge && hidden(tokB + r) ? 0.f : __builtin_amdgcn_exp2f(sb[u][r] - mn);
                 ps += pa[r] + pb[r];
             }
             split_weights(pa, pb, P[u], Pl[u]);
@@ -553,9 +567,9 @@ __global__ void __launch_bounds__(256, 2) bias_prefill_kernel(BiasAttnArgs a, in
         float l = lsum[u];
         l += __shfl_xor(l, 16);
         l += __shfl_xor(l, 32);
-        const float ms = a.sink ? fmaxf(m[u], 0.f) : m[u];
+        const float sink = a.sink ? a.sink[kvh * gqa + hd[u]] : 0.f, ms = a.sink ? fmaxf(m[u], sink) : m[u];
         float f = __builtin_amdgcn_exp2f(m[u] - ms);
-        f = f / (l * f + (a.sink ? __builtin_amdgcn_exp2f(-ms) : 0.f));
+        f = f / (l * f + (a.sink ? __builtin_amdgcn_exp2f(sink - ms) : 0.f));
         if (!valid[u]) continue;
         const int col = (kvh * gqa + hd[u]) * a.kv.vdim;
 #pragma unroll

@@ -84,19 +84,19 @@ int run_glu(nvllm_model* m, const GluPlan& g, const bf16_bits* xh, const bf16_bi
     return NVLLM_OK;
 }
 
-int run_relu2(nvllm_model* m, const ProductPlan& p, const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int R, bf16_bits* oh, bf16_bits* ol, int out_packed) {
+int run_act(nvllm_model* m, const ProductPlan& p, nvllm::Act act, const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int R, bf16_bits* oh, bf16_bits* ol, int out_packed) {
     hipStream_t s = m->ctx->stream;
-    if (p.kind == P_TILE && gemm_tile_ok(R, w.N, w.K, 4, m->opt_tile_min_wgs)) {
-        PROF(m, PROF_GEMM, launch_gemm_tile(xh, xl, w, R, 4, nullptr, oh, ol, out_packed, m->opt_tile_min_wgs, 1, nullptr, s));
+    if (p.kind == P_TILE && gemm_tile_ok(R, w.N, w.K, 4 + act, m->opt_tile_min_wgs)) {
+        PROF(m, PROF_GEMM, launch_gemm_tile(xh, xl, w, R, 4 + act, nullptr, oh, ol, out_packed, m->opt_tile_min_wgs, 1, nullptr, s));
         ++m->tile_launches;
-    } else if (p.kind == P_ROW && gemm_rowdir_ok(w.N, w.K, 3, R)) {
+    } else if (p.kind == P_ROW && gemm_rowdir_ok(w.N, w.K, 3 + act, R)) {
         RowParArgs a;
         a.xh = xh; a.xl = xl; a.ldx = w.K; a.oh = oh; a.ol = ol; a.M = R; a.x_packed = p.packed; a.o_packed = out_packed;
-        PROF(m, PROF_GEMM, launch_gemm_rowpar(a, w, 3, s));
+        PROF(m, PROF_GEMM, launch_gemm_rowpar(a, w, 3 + act, s));
     } else {
         int ns = 1, rc = run_product(m, p, xh, xl, w, m->slabs, R, &ns);
         if (rc) return rc;
-        PROF(m, PROF_SILU, launch_relu2(m->slabs, ns, (int64_t)R * w.N, R, w.N, oh, ol, out_packed, nullptr, s));
+        PROF(m, PROF_SILU, launch_act(act, m->slabs, ns, (int64_t)R * w.N, R, w.N, oh, ol, out_packed, nullptr, s));
     }
     return NVLLM_OK;
 }

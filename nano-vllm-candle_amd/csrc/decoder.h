@@ -98,8 +98,8 @@ int run_product(nvllm_model* m, const ProductPlan& p, const bf16_bits* xh, const
 GluPlan plan_glu(const nvllm_model* m, int R, const PackedW& w, bool want_packed_out);
 int run_glu(nvllm_model* m, const GluPlan& g, const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int R, const GluSpec& spec,
             bf16_bits* oh, bf16_bits* ol, int out_packed);
-// squared ReLU of x.W^T as hi/lo planes oh / ol on the plan of the product, through m->slabs where no epilogue fits
-int run_relu2(nvllm_model* m, const ProductPlan& p, const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int R, bf16_bits* oh, bf16_bits* ol, int out_packed);
+// activation of x.W^T as hi/lo planes oh / ol on the plan of the product, through m->slabs where no epilogue fits
+int run_act(nvllm_model* m, const ProductPlan& p, nvllm::Act act, const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int R, bf16_bits* oh, bf16_bits* ol, int out_packed);
 // 32-bit product of row-major f32 rows
 int exact_product(nvllm_model* m, const float* x, const PackedW& w, float* out, int R);
 

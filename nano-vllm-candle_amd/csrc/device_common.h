@@ -49,6 +49,19 @@ __device__ __forceinline__ float relu2(float x) {
     return x * x;
 }
 
+// x / 2 (1 + erf(x / sqrt 2)) with erfc by formula 7.1.26 of Abramowitz and Stegun, "Handbook of Mathematical Functions" (absolute error
+// 1.5e-7): for f16 and bf16 hi + lo consumers
+__device__ __forceinline__ float gelu_erf_fast(float x) {
+    const float z = fabsf(x) * 0.7071067811865476f, t = __builtin_amdgcn_rcpf(1.0f + 0.3275911f * z);
+    const float p = ((((1.061405429f * t - 1.453152027f) * t + 1.421413741f) * t - 0.284496736f) * t + 0.254829592f) * t;
+    const float c = p * __expf(-z * z);  // erfc(z)
+    return 0.5f * x * (x < 0.f ? c : 2.0f - c);
+}
+template <int ACT>
+__device__ __forceinline__ float act_of(float x) {
+    return ACT == ACT_GELU ? gelu_erf_fast(x) : relu2(x);
+}
+
 // 1 / 2 (1 + tanh a) = 1 / (1 + e^-2a): -2a of the tanh form of GELU
 __device__ __forceinline__ float gelu_arg(float g) { return -1.5957691216057308f * (g + 0.044715f * g * g * g); }
 

@@ -9,7 +9,7 @@ int ExpertsBlock::create(nvllm_ctx* ctx, int experts_, int top_, int ff_, int sh
     ff = ff_all / tp; sh = shared_all / tp; ff_p = ff >= 512 && !f32 ? up_tile(ff) : up(ff, 128); sh_p = !sh ? 0 : sh >= 512 && !f32 ? up_tile(sh) : up(sh, 128);
     Nr = up(experts + (sh ? 1 : 0), 16);
     int rc = alloc_packed(ctx, router, Nr, Kw);
-    if (!rc) rc = alloc_packed(ctx, wup, experts * ff_p, Kw);
+    if (!rc) rc = alloc_packed(ctx, wup, experts * up_rows(), Kw);
     if (!rc) rc = alloc_packed(ctx, down, experts * ldr, ff_p);
     if (!rc && sh) rc = alloc_packed(ctx, sup, sh_p, Kw);
     if (!rc && sh) rc = alloc_packed(ctx, sdown, ldr, sh_p);
@@ -26,9 +26,9 @@ int ExpertsBlock::load(nvllm_model* m, const char* name, const char* s, const Ho
         if (rows == r && cols == c) return NVLLM_OK;
         return fail(ctx, NVLLM_EINVAL, "tensor '%s': shape mismatch (got %lld x %lld, want %lld x %lld)", name, (long long)rows, (long long)cols, (long long)r, (long long)c);
     };
-    auto put_up = [&](const PackedW& w, int row0, int64_t all, int n, int64_t r0) -> int {
+    auto put_up = [&](const PackedW& w, int row0, int64_t all, int n, int64_t r0, int ileave = -1) -> int {
         int rc = want(all, W);
-        return rc ? rc : put_rows(ctx, w, row0, n, W, -1, [&](int r, int c) { return h.at(r0 + r, c); });
+        return rc ? rc : put_rows(ctx, w, row0, n, W, ileave, [&](int r, int c) { return h.at(r0 + r, c); });
     };
     auto put_down = [&](const PackedW& w, int row0, int64_t all, int n, int64_t c0) -> int {
         int rc = want(W, all);
@@ -40,7 +40,8 @@ int ExpertsBlock::load(nvllm_model* m, const char* name, const char* s, const Ho
     if (sh && !strcmp(s, "shared.down")) return put_down(sdown, 0, shared_all, sh, s0);
     int e = -1, off = 0;
     if (sscanf(s, "e%d.%n", &e, &off) == 1 && off && e >= 0 && e < experts) {
-        if (!strcmp(s + off, "up")) return put_up(wup, e * ff_p, ff_all, ff, f0);
+        if (gated && !strcmp(s + off, "gate")) return put_up(wup, e * up_rows(), ff_all, ff, f0, 0);
+        if (!strcmp(s + off, "up")) return put_up(wup, e * up_rows(), ff_all, ff, f0, gated ? 1 : -1);
         if (!strcmp(s + off, "down")) return put_down(down, e * ldr, ff_all, ff, f0);
     }
     return 1;
@@ -48,7 +49,8 @@ int ExpertsBlock::load(nvllm_model* m, const char* name, const char* s, const Ho
 std::vector<std::string> ExpertsBlock::tensors() const {
     std::vector<std::string> t = {"router"};
     for (int e = 0; e < experts; ++e)
-        for (const char* s : {".up", ".down"}) t.push_back("e" + std::to_string(e) + s);
+        for (const char* s : {".gate", ".up", ".down"})
+            if (gated || s[1] != 'g') t.push_back("e" + std::to_string(e) + s);
     if (sh) for (const char* s : {"shared.up", "shared.down", "shared.sg"}) t.push_back(s);
     return t;
 }
@@ -99,7 +101,7 @@ static int tile_align(const nvllm_model* m, const ExpertsBlock& e, int R) {
     const int rows = R * e.top / e.experts;  // of an expert, on average
     if (m->opt_tile_min_wgs <= 0 || R <= kFusedMaxRows || rows < (m->opt_tile_min_wgs == 1 ? 1 : 48)) return 0;
     for (int align : {rows >= 320 ? 256 : 128, 256})
-        if (gemm_tile_group_ok(e.ff_p, e.Kw, align) && gemm_tile_group_ok(e.ldr, e.ff_p, align)) return align;
+        if (gemm_tile_group_ok(e.up_rows(), e.Kw, align) && gemm_tile_group_ok(e.ldr, e.ff_p, align)) return align;
     return 0;
 }
 bool experts_gather(const nvllm_model* m, const ExpertsBlock& e, int R) { return tile_align(m, e, R) > 0; }
@@ -116,6 +118,7 @@ int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_b
     PROF(m, PROF_GEMM, launch_group_gemm(rg, s));
     RouteArgs ra;
     ra.z = x.z; ra.ld = e.Nr; ra.rows = R; ra.experts = e.experts; ra.top = e.top; ra.weight_in = e.weight_in;
+    ra.softmax = e.softmax; ra.groups = e.groups; ra.keep = e.keep;
     ra.gate_col = e.sh ? e.experts : -1;
     const int tile = f32 ? 0 : tile_align(m, e, R);
     ra.shared_group = e.sh > 0 && !tile;
@@ -128,9 +131,9 @@ int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_b
     if (tile) {
         const int n = (int)(longest / tile) * tile;
         TileGroups tg;
-        tg.tile_group = x.tile_group; tg.align = tile; tg.w_group = (int64_t)e.ff_p * e.Kw / 8; tg.src = x.src; tg.x_rows = R; tg.pre = x.pre; tg.post = x.post;
+        tg.tile_group = x.tile_group; tg.align = tile; tg.w_group = (int64_t)e.up_rows() * e.Kw / 8; tg.src = x.src; tg.x_rows = R; tg.pre = x.pre; tg.post = x.post; tg.gated = e.gated;
         PackedW w = e.wup;
-        w.N = e.ff_p;
+        w.N = e.up_rows();
         PROF(m, PROF_GEMM, launch_gemm_tile_group(rh, rl, w, n, tg, nullptr, x.ah, x.al, s));
         w = e.down;
         w.N = e.ldr;
@@ -141,7 +144,7 @@ int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_b
             ProductPlan pu = plan_product(m, R, e.sup), pd = plan_product(m, R, e.sdown);
             const bool ours = pu.packed == packed;  // else the row-major planes and a kernel that takes them
             if (!ours && pu.packed) pu = ProductPlan{P_GENERIC, 0, pu.max_split};
-            int rc = run_relu2(m, pu, ours ? xh : rh, ours ? xl : rl, e.sup, R, x.sh, x.sl, pd.packed);
+            int rc = run_act(m, pu, ACT_RELU2, ours ? xh : rh, ours ? xl : rl, e.sup, R, x.sh, x.sl, pd.packed);
             if (!rc) rc = run_product(m, pd, x.sh, x.sl, e.sdown, slabs2, R, &out->n_slabs);
             if (rc) return rc;
             out->in = slabs2; out->slab_stride = (int64_t)R * e.ldr; out->scale = x.gate;
@@ -149,9 +152,11 @@ int run_experts(nvllm_model* m, ExpertsBlock& e, ExpertsScratch& x, const bf16_b
         return NVLLM_OK;
     }
     GroupGemmArgs ga = in;
-    ga.src = x.src; ga.w = e.wup.data; ga.w_group = (int64_t)e.ff_p * e.Kw / 8; ga.N = e.ff_p; ga.K = e.Kw;
+    ga.src = x.src; ga.w = e.wup.data; ga.w_group = (int64_t)e.up_rows() * e.Kw / 8; ga.N = e.up_rows(); ga.K = e.Kw;
     if (ra.shared_group) { ga.ws = e.sup.data; ga.last = e.experts; ga.Ns = e.sh_p; ga.Ks = e.Kw; }
-    ga.tile_group = x.tile_group; ga.align = ra.align; ga.tiles = (int)(longest / ra.align); ga.pre = x.pre; ga.post = x.post; ga.relu2 = 1;
+    ga.tile_group = x.tile_group; ga.align = ra.align; ga.tiles = (int)(longest / ra.align); ga.post = x.post;
+    if (e.gated) ga.glu = 1;
+    else { ga.pre = x.pre; ga.relu2 = 1; }
     ga.ldo = x.lda;
     if (f32) ga.out = x.act_f;
     else { ga.oh = x.ah; ga.ol = x.al; }

@@ -18,9 +18,11 @@ struct ExpertsBlock {
     int experts = 0, top = 0, ff_all = 0, shared_all = 0;  // widths of the whole model (shared_all 0: no shared expert)
     int ff = 0, ff_p = 0, sh = 0, sh_p = 0;                // this rank's share, padded
     int weight_in = 1;
+    int gated = 0, softmax = 0, groups = 1, keep = 1;      // set before create: experts silu(gate) up (else squared ReLU; no shared one beside), scores and groups as in RouteArgs
+    int up_rows() const { return gated ? 2 * ff_p : ff_p; }
     int W = 0, Kw = 0, ldr = 0, Nr = 0;
     PackedW router;                                        // a row per expert, then the shared gate's
-    PackedW wup, down, sup, sdown;                         // wup [experts * ff_p x Kw], down [experts * ldr x ff_p]
+    PackedW wup, down, sup, sdown;                         // wup [experts * up_rows x Kw], down [experts * ldr x ff_p]
     bool on() const { return experts > 0; }
     int create(nvllm_ctx* ctx, int experts, int top, int ff, int shared, int W, int Kw, int ldr, bool f32);
     void destroy();

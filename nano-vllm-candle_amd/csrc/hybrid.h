@@ -14,11 +14,11 @@ struct Segments {
     int single = 0;             // decode: segment i is row i, its slot is slot[i] (row0, n unused)
 };
 
-// ---- feed-forward activation: y = max(x, 0)^2 over the summed slabs, as bf16 hi/lo planes [rows][F] or f32 ------------------------
-hipError_t launch_relu2(const float* in, int n_slabs, int64_t slab_stride, int rows, int F, bf16_bits* hi, bf16_bits* lo, int packed, float* y,
-                        hipStream_t s);
+// ---- feed-forward activation of the summed slabs, as bf16 hi/lo planes [rows][F] or f32 -------------------------------------------
+hipError_t launch_act(Act act, const float* in, int n_slabs, int64_t slab_stride, int rows, int F, bf16_bits* hi, bf16_bits* lo, int packed, float* y,
+                      hipStream_t s);
 
-// ---- attention with a distance bias ------------------------------------------------------------------------------------------------
+// ---- grouped-query attention ------------------------------------------------------------------------------------------------
 // K in QK^T fragment order with dim_p, V in PV fragment order with vdim_p (device_common.h), blocks of kBlockTokens tokens per kv head:
 // [block][kv][kBlockTokens * dim_p] / [block][kv][kBlockTokens * vdim_p]; f16 or f32; padding zero.
 struct PagedKV {
@@ -61,7 +61,8 @@ struct BiasAttnArgs {
     int heads = 0;
     const float* bias = nullptr;     // [heads][n_bias] by distance, times log2(e); distances from n_bias - 1 on share the last entry
     int n_bias = 0;                  // 0: no bias
-    int sink = 0;                    // one more term exp(0) in the denominator
+    int window = 0;                  // > 0: a token sees itself and the window - 1 before it
+    const float* sink = nullptr;     // [heads] one more term 2^sink in the denominator; nullptr: none
     const int* block_tables = nullptr;
     int max_blocks = 0;
     const int* tile_row0 = nullptr;
@@ -99,9 +100,10 @@ struct RecurArgs {
     const float* k = nullptr;
     const float* v = nullptr;        // [rows][heads][vdim_p]
     int heads = 0, q_heads = 0, dim_p = 0, vdim = 0, vdim_p = 0;
-    // delta rule: decays per key channel and write strengths; nullptr: constant decays per head
+    // delta rule: decays per key channel (g) or per head (gh) and write strengths; nullptr: constant decays per head
     const float* g = nullptr;        // rows of stride g_row, head * dim_p
     int64_t g_row = 0;
+    const float* gh = nullptr;       // [rows][heads] one decay per head instead
     const float* beta = nullptr;     // [rows][heads]
     const float* decay = nullptr;    // [heads]
     float* state = nullptr;
@@ -112,9 +114,9 @@ struct RecurArgs {
 // RMS norm of o over one head or over all heads, times weight and gate, as context planes / f32 rows [rows][ld], column head * vdim
 struct GatedNormArgs {
     const float* o = nullptr;        // [rows][heads][vdim_p]
-    const float* gate = nullptr;     // sigmoid already applied; rows of stride gate_row, heads of stride gate_head
-    int64_t gate_row = 0;
-    int gate_head = 0;
+    const float* gate = nullptr;     // the factor itself, or with gate_slabs > 0 the slabs of a projection z, the factor being silu(z)
+    int64_t gate_row = 0, gate_stride = 0;  // rows, slabs
+    int gate_head = 0, gate_slabs = 0;      // heads
     int heads = 0, vdim = 0, vdim_p = 0;
     int whole = 0;                   // 1: one norm over all heads, weight [heads * vdim]; 0: per head, weight [vdim]
     const float* ssq = nullptr;      // whole: [rows][2], entry 0 the sum of squares over every rank's heads
@@ -163,10 +165,13 @@ hipError_t launch_linear_rows(const LinearRowsArgs& a, int rows, hipStream_t s);
 // rows after the projection of the delta rule: causal convolution + silu of q, k, v (history in the sequence's slot), unit q and k,
 // beta, and the inputs of the two-step gate projections
 struct DeltaRowsArgs {
-    const float* in = nullptr;       // columns: kv * dim query, kv * dim key, heads * vdim value, heads beta, rank_p decay, rank_p gate inputs
+    // columns: kv * dim query, kv * dim key, heads * vdim value, heads beta, then rank_p decay and rank_p gate inputs (two-step gates), or
+    // heads decay inputs (rate set)
+    const float* in = nullptr;
     int n_slabs = 1, ld = 0;
     int64_t slab_stride = 0;
     int heads = 0, kv = 0, dim = 0, dim_p = 0, vdim = 0, vdim_p = 0, rank_p = 0, taps = 1;
+    const float* in_bias = nullptr;  // unused (short_conv.h)
     const float* conv = nullptr;     // [taps][channels], channels = 2 kv dim + heads vdim in column order
     float q_scale = 1.f;
     // history: raw projections of the last taps - 1 tokens, [2][slots][taps - 1][channels]; a segment that starts at position p reads
@@ -180,10 +185,46 @@ struct DeltaRowsArgs {
     float* k = nullptr;
     float* v = nullptr;              // [rows][heads][vdim_p]
     float* beta = nullptr;           // [rows][heads]
-    float* gate_in = nullptr;        // [rows][2][rank_p]
+    float* gate_in = nullptr;        // two-step gates: [rows][2][rank_p]
+    // one decay per head: exp(-rate softplus(decay input + dt))
+    const float* rate = nullptr;     // [heads]
+    const float* dt = nullptr;       // [heads]
+    float* decay = nullptr;          // [rows][heads]
+    __host__ __device__ int channels() const { return 2 * kv * dim + heads * vdim; }
+    __host__ __device__ int extras() const { return heads + (rate ? heads : 2 * rank_p); }  // columns behind the channels
 };
 constexpr float kUnitNormEps = 1e-6f;
 hipError_t launch_delta_rows(const DeltaRowsArgs& a, int rows, hipStream_t s);
+// rows after the q / k / v projection of attention with short convolutions: bias, causal convolution, rotation of neighbouring dimensions,
+// RMS norm per head (no weight), cache write; history as in DeltaRowsArgs (biased projections)
+struct ConvAttnRowsArgs {
+    const float* in = nullptr;       // columns: heads * dim query, kv * dim key, kv * vdim value
+    int n_slabs = 1, ld = 0;
+    int64_t slab_stride = 0;
+    const float* in_bias = nullptr;  // [channels], nullptr: none
+    int heads = 0, taps = 1;
+    const float* conv = nullptr;     // [taps][channels]
+    int rot = 0;                     // rotated dimensions (even)
+    const float* cos = nullptr;      // [positions][rot / 2]
+    const float* sin = nullptr;
+    float eps = 0.f, q_scale = 1.f;  // q_scale: score scale * log2(e)
+    float* history = nullptr;
+    int slots = 0;
+    Segments seg;
+    const int* pos = nullptr;
+    const int* slot = nullptr;
+    const int* block_tables = nullptr;
+    int max_blocks = 0;
+    float* q = nullptr;              // [rows][heads][dim_p], scaled, padding zero
+    PagedKV kv;
+    __host__ __device__ int channels() const { return (heads + kv.kv) * kv.dim + kv.kv * kv.vdim; }
+    __host__ __device__ int units() const { return heads + 2 * kv.kv; }  // waves per row
+};
+constexpr int kConvAttnDim = 512;    // widest head
+hipError_t launch_conv_attn_rows(const ConvAttnRowsArgs& a, int rows, hipStream_t s);
+// the history half of it for chunks with longer segments (after launch_conv_attn_rows)
+hipError_t launch_conv_attn_history(const ConvAttnRowsArgs& a, hipStream_t s);
+
 // gate_in -> decays and output gates (HeadGemmArgs with decay_rate set), or step sizes alone (decay_bias without it)
 hipError_t launch_delta_gates(const HeadGemmArgs& a, hipStream_t s);
 // the history half of it for chunks with longer segments (after launch_delta_rows)

@@ -1,4 +1,4 @@
-// gfx950 row kernels of the hybrid decoders: squared-ReLU activation, the steps between a mixer's input projection and its attention or
+// gfx950 row kernels of the hybrid decoders: activations, the steps between a mixer's input projection and its attention or
 // recurrence (biases, norms, value mixing, cache write; convolution, unit norms, gates), the gated output norm.
 #include <algorithm>
 
@@ -11,26 +11,31 @@ namespace nvllm {
 __device__ __forceinline__ float sigmoidf(float x) { return 1.0f / (1.0f + expf(-x)); }
 
 // ---------------------------------------------------------------------------------------------------
-// squared ReLU
+// activation of summed slabs
 // ---------------------------------------------------------------------------------------------------
-__global__ void __launch_bounds__(256) relu2_kernel(const float* __restrict__ in, int n_slabs, int64_t slab_stride, int rows, int F,
+template <int ACT>
+__global__ void __launch_bounds__(256) act_kernel(const float* __restrict__ in, int n_slabs, int64_t slab_stride, int rows, int F,
                                                     uint16_t* __restrict__ hi, uint16_t* __restrict__ lo, int packed, float* __restrict__ y) {
     const int64_t total = (int64_t)rows * (F >> 2);
     for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (int64_t)gridDim.x * 256) {
         const int r = (int)(i / (F >> 2)), c = (int)(i % (F >> 2)) * 4;
         float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
         add_slabs(s, in + (size_t)r * F + c, n_slabs, slab_stride);
-        const f32x4 v = {relu2(s.x), relu2(s.y), relu2(s.z), relu2(s.w)};
+        const float x[4] = {s.x, s.y, s.z, s.w};
+        f32x4 v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = ACT == ACT_GELU ? 0.5f * x[e] * (1.0f + erff(x[e] * 0.7071067811865476f)) : relu2(x[e]);
         if (y) *reinterpret_cast<float4*>(y + (size_t)r * F + c) = make_float4(v[0], v[1], v[2], v[3]);
         if (hi) put_planes4(hi, lo, r, c, 4, F, packed, v);
     }
 }
-hipError_t launch_relu2(const float* in, int n_slabs, int64_t slab_stride, int rows, int F, bf16_bits* hi, bf16_bits* lo, int packed, float* y,
-                        hipStream_t s) {
+hipError_t launch_act(Act act, const float* in, int n_slabs, int64_t slab_stride, int rows, int F, bf16_bits* hi, bf16_bits* lo, int packed, float* y,
+                      hipStream_t s) {
     if (F % 32 || n_slabs < 1) return hipErrorInvalidValue;
     if (rows <= 0) return hipSuccess;
     const int64_t wgs = ((int64_t)rows * (F / 4) + 255) / 256;
-    relu2_kernel<<<(int)std::min<int64_t>(wgs, 8192), 256, 0, s>>>(in, n_slabs, slab_stride, rows, F, hi, lo, packed, y);
+    auto* const kernel = act == ACT_GELU ? act_kernel<ACT_GELU> : act_kernel<ACT_RELU2>;
+    kernel<<<(int)std::min<int64_t>(wgs, 8192), 256, 0, s>>>(in, n_slabs, slab_stride, rows, F, hi, lo, packed, y);
     return hipGetLastError();
 }
 
@@ -302,13 +307,20 @@ hipError_t launch_linear_rows(const LinearRowsArgs& a, int rows, hipStream_t s) 
 }
 
 // ---------------------------------------------------------------------------------------------------
-// delta rule: one wave per (row, unit); units = q heads, k heads, v heads, then one for beta and the gate inputs.  The form for any
-// size of prompt chunk first, then those of decode and of long chunks.
+// delta rule: one wave per (row, unit); units = q heads, k heads, v heads, then those of delta_extra.  The form for any size of prompt
+// chunk first, then those of decode and of long chunks.
 // ---------------------------------------------------------------------------------------------------
 __device__ __forceinline__ float conv_silu(const DeltaRowsArgs& a, const RowPast& p, int row, int c, int channels) {
     float y = 0.f;
     for (int i = 0; i < a.taps; ++i) y += past_input(a, p, row, a.taps - 1 - i, c, channels) * a.conv[(size_t)i * channels + c];
     return y * sigmoidf(y);
+}
+
+// column i behind the convolved ones: write strengths, then what the decays come from, or the decays of the heads
+__device__ __forceinline__ void delta_extra(const DeltaRowsArgs& a, int row, int i, float x) {
+    if (i < a.heads) a.beta[(size_t)row * a.heads + i] = sigmoidf(x);
+    else if (a.rate) a.decay[(size_t)row * a.heads + i - a.heads] = expf(-a.rate[i - a.heads] * softplusf(x + a.dt[i - a.heads]));
+    else a.gate_in[(size_t)row * 2 * a.rank_p + i - a.heads] = x;
 }
 
 template <int NE>
@@ -336,9 +348,7 @@ __global__ void __launch_bounds__(256) delta_rows_kernel(DeltaRowsArgs a) {
         float* o = a.v + ((size_t)row * a.heads + h) * a.vdim_p;
         for (int d = lane; d < a.vdim_p; d += 64) o[d] = d < a.vdim ? conv_silu(a, p, row, c0 + d, channels) : 0.f;
     } else {
-        const float* in = a.in + (size_t)row * a.ld + channels;
-        for (int h = lane; h < a.heads; h += 64) a.beta[(size_t)row * a.heads + h] = sigmoidf(slab_elem(in + h, a.n_slabs, a.slab_stride));
-        for (int i = lane; i < 2 * a.rank_p; i += 64) a.gate_in[(size_t)row * 2 * a.rank_p + i] = slab_elem(in + a.heads + i, a.n_slabs, a.slab_stride);
+        for (int i = lane; i < a.extras(); i += 64) delta_extra(a, row, i, slab_elem(a.in + (size_t)row * a.ld + channels + i, a.n_slabs, a.slab_stride));
     }
 }
 
@@ -349,12 +359,7 @@ __global__ void __launch_bounds__(256) delta_rows_decode_kernel(DeltaRowsArgs a)
     const int channels = 2 * a.kv * a.dim + a.heads * a.vdim;
     if (unit > 2 * a.kv + a.heads) return;
     if (unit == 2 * a.kv + a.heads) {
-        const float* in = a.in + (size_t)row * a.ld + channels;
-        for (int i = lane; i < a.heads + 2 * a.rank_p; i += 64) {
-            const float x = slab_elem(in + i, a.n_slabs, a.slab_stride);
-            if (i < a.heads) a.beta[(size_t)row * a.heads + i] = sigmoidf(x);
-            else a.gate_in[(size_t)row * 2 * a.rank_p + i - a.heads] = x;
-        }
+        for (int i = lane; i < a.extras(); i += 64) delta_extra(a, row, i, slab_elem(a.in + (size_t)row * a.ld + channels + i, a.n_slabs, a.slab_stride));
         return;
     }
     const int slot = a.slot[row], pos = a.pos[row];
@@ -417,12 +422,17 @@ __global__ void __launch_bounds__(256) delta_rows16_kernel(DeltaRowsArgs a, int 
     const int channels = 2 * a.kv * a.dim + a.heads * a.vdim;
     if (unit > 2 * a.kv + a.heads) return;
     if (unit == 2 * a.kv + a.heads) {
-        const int per = a.heads + 2 * a.rank_p;
-        for (int i = lane; i < (row1 - row0) * per; i += 64) {
-            const int row = row0 + i / per, c = i % per;
-            const float x = slab_elem(a.in + (size_t)row * a.ld + channels + c, a.n_slabs, a.slab_stride);
-            if (c < a.heads) a.beta[(size_t)row * a.heads + c] = sigmoidf(x);
-            else a.gate_in[(size_t)row * 2 * a.rank_p + c - a.heads] = x;
+        const int per = a.extras(), n = (row1 - row0) * per;
+        for (int i0 = lane; i0 < n; i0 += 256) {  // four loads in flight
+            float x[4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const int i = min(i0 + u * 64, n - 1);
+                x[u] = slab_elem(a.in + (size_t)(row0 + i / per) * a.ld + channels + i % per, a.n_slabs, a.slab_stride);
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+                if (i0 + u * 64 < n) delta_extra(a, row0 + (i0 + u * 64) / per, (i0 + u * 64) % per, x[u]);
         }
         return;
     }
@@ -518,7 +528,7 @@ static bool delta_rows16(const DeltaRowsArgs& a, int rows, hipStream_t s) {
     return true;
 }
 hipError_t launch_delta_rows(const DeltaRowsArgs& a, int rows, hipStream_t s) {
-    if (a.dim_p % 64 || a.vdim_p % 4 || a.taps < 1 || 2 * a.kv * a.dim + a.heads * (a.vdim + 1) + 2 * a.rank_p > a.ld) return hipErrorInvalidValue;
+    if (a.dim_p % 64 || a.vdim_p % 4 || a.taps < 1 || a.channels() + a.extras() > a.ld || (a.rate ? !a.dt || !a.decay : !a.gate_in)) return hipErrorInvalidValue;
     if (a.dim_p > 512) return hipErrorNotSupported;
     if (rows <= 0) return hipSuccess;
     if (!a.seg.single && rows >= 64) {
@@ -650,6 +660,11 @@ hipError_t launch_delta_gates(const HeadGemmArgs& a, hipStream_t s) {
 // ---------------------------------------------------------------------------------------------------
 // gated output norm: one wave per (row, head), or one workgroup per row when the norm runs over all heads
 // ---------------------------------------------------------------------------------------------------
+__device__ __forceinline__ float gate_factor(const GatedNormArgs& a, const float* p) {
+    if (!a.gate_slabs) return *p;
+    const float z = slab_elem(p, a.gate_slabs, a.gate_stride);
+    return z * sigmoidf(z);
+}
 template <bool WHOLE>
 __global__ void __launch_bounds__(256) gated_norm_kernel(GatedNormArgs a, int rows) {
     __shared__ float red[4];
@@ -661,7 +676,7 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(GatedNormArgs a, int ro
     constexpr int step = WHOLE ? 256 : 64;
     const int t0 = WHOLE ? threadIdx.x : lane;
     const float n = WHOLE ? (float)a.all : (float)a.vdim;
-    if ((a.vdim & 3) == 0) {  // four values of one head per thread; padding columns of o are zero
+    if ((a.vdim & 3) == 0 && ((a.gate_head | a.gate_row | a.gate_stride) & 3) == 0 && (reinterpret_cast<uintptr_t>(a.gate) & 15) == 0) {  // four values of one head per thread; padding columns of o are zero
         const int n4 = WHOLE ? a.heads * (a.vdim_p >> 2) : a.vdim_p >> 2;
         float ss = 0.f;
         if (WHOLE && a.ssq) {
@@ -677,7 +692,10 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(GatedNormArgs a, int ro
         for (int i = t0; i < n4; i += step) {
             const int h = WHOLE ? i * 4 / a.vdim_p : 0, e = i * 4 - h * a.vdim_p, col = (head0 + h) * a.vdim + e;
             if (e >= a.vdim) continue;
-            const float4 x = reinterpret_cast<const float4*>(o)[i], g = *reinterpret_cast<const float4*>(gate + (size_t)h * a.gate_head + e);
+            const float4 x = reinterpret_cast<const float4*>(o)[i];
+            float4 g = make_float4(0.f, 0.f, 0.f, 0.f);
+            add_slabs(g, gate + (size_t)h * a.gate_head + e, max(a.gate_slabs, 1), a.gate_stride);
+            if (a.gate_slabs) g = make_float4(g.x * sigmoidf(g.x), g.y * sigmoidf(g.y), g.z * sigmoidf(g.z), g.w * sigmoidf(g.w));
             const float4 w = *reinterpret_cast<const float4*>(a.weight + (WHOLE ? col : e));
             const f32x4 v = {(x.x * rinv) * w.x * g.x, (x.y * rinv) * w.y * g.y, (x.z * rinv) * w.z * g.z, (x.w * rinv) * w.w * g.w};
             if (a.of) *reinterpret_cast<float4*>(a.of + (size_t)row * a.ld + col) = make_float4(v[0], v[1], v[2], v[3]);
@@ -700,7 +718,7 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(GatedNormArgs a, int ro
     const float rinv = 1.0f / sqrtf(ss / n + a.eps);
     for (int i = t0; i < cnt; i += step) {
         const int h = WHOLE ? i / a.vdim : 0, e = i - h * a.vdim, col = (head0 + h) * a.vdim + e;
-        const float v = (o[h * a.vdim_p + e] * rinv) * a.weight[i] * gate[h * a.gate_head + e];
+        const float v = (o[h * a.vdim_p + e] * rinv) * a.weight[i] * gate_factor(a, gate + (size_t)h * a.gate_head + e);
         if (a.of) a.of[(size_t)row * a.ld + col] = v;
         if (a.oh) {
             const size_t x = a.packed ? xpack_off(row, col, a.ld >> 5) : (size_t)row * a.ld + col;
@@ -709,7 +727,7 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(GatedNormArgs a, int ro
     }
 }
 hipError_t launch_gated_norm(const GatedNormArgs& a, int rows, hipStream_t s) {
-    if (a.heads * a.vdim > a.ld || (!a.oh && !a.of) || (a.whole && a.all < 1) || a.vdim_p % 4 || a.gate_head % 4 || a.gate_row % 4) return hipErrorInvalidValue;
+    if (a.heads * a.vdim > a.ld || (!a.oh && !a.of) || (a.whole && a.all < 1) || a.vdim_p % 4) return hipErrorInvalidValue;
     if (rows <= 0) return hipSuccess;
     if (a.whole) gated_norm_kernel<true><<<rows, 256, 0, s>>>(a, rows);
     else gated_norm_kernel<false><<<(rows * a.heads + 3) / 4, 256, 0, s>>>(a, rows);

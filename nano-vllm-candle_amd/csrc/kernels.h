@@ -23,7 +23,7 @@ struct PackedW {
 };
 
 // pack rows [row0, row0+rows) of dst from a row-major bf16 source (ld = elements between rows)
-// ileave: -1 = rows land at row0.. ; 0/1 = gate(0)/up(1) rows interleaved in 16-row tiles (SwiGLU epilogue layout)
+// ileave: -1 = rows land at row0.. ; 0/1 = gate(0)/up(1) rows interleaved in 16-row tiles from row0 on (SwiGLU epilogue layout)
 hipError_t launch_pack_rows(const PackedW& dst, int row0, int rows, const bf16_bits* src, int64_t ld, int ileave,
                             hipStream_t s);
 // generate rows [row0,row0+rows) of dst from the synthetic tensor `spec` (synth_device.h): logical element
@@ -75,6 +75,9 @@ struct GluSpec {
     float limit = 0.f, alpha = 1.f, shift = 0.f;
     int gelu = 0;
 };
+
+// activation of a feed-forward without a gate
+enum Act { ACT_RELU2 = 0, ACT_GELU = 1 };  // max(x, 0)^2; the exact GELU, x / 2 (1 + erf(x / sqrt 2))
 
 // ---- GEMM: out[ks][M][N] = x[M][K-slice ks] . W[N][K-slice ks]^T  (f32 slabs, ks < n_split) ------
 struct GemmPlan {
@@ -189,7 +192,7 @@ hipError_t launch_qk_norm_rope_kvwrite(const QkvArgs& a, int rows, hipStream_t s
 
 // ---- prefill GEMM (tile_gemm.hip): 256 x 256/192 output tile, both operands in fragment order -------------------
 // x planes in xpack_off order; mode 0: out f32 [M][N]; mode 2: w = interleaved gate/up, act hi/lo [M][N/2] (row-major or
-// xpack_off order); mode 4: squared ReLU as hi/lo planes [M][N].  min_wgs: smallest grid the kernel is used for (a 256-row tile needs many rows to fill 256 CUs).
+// xpack_off order); mode 4 + act: the activation of every feature as hi/lo planes [M][N].  min_wgs: smallest grid the kernel is used for (a 256-row tile needs many rows to fill 256 CUs).
 // hipErrorNotSupported = shape not covered.
 bool gemm_tile_ok(int M, int N, int K, int mode, int min_wgs);
 // mode 0 with n_slabs != nullptr may split K (narrow outputs, 128-row blocks): out = [*n_slabs][M][N], up to max_split slabs
@@ -203,8 +206,9 @@ bool gemm_tile_qkv_ok(int M, int N, int K, int hd, int min_wgs);
 hipError_t launch_gemm_tile_qkv(const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int M, const QkvArgs& qa, int min_wgs,
                                 hipStream_t s);
 // rows in groups that start at multiples of `align` (128 or 256), every group with weights [N x K] of its own, group g's w_group uint4 behind
-// the first: post relu2(pre x.W_g^T) as planes in xpack_off order (x: row-major planes [x_rows][K], position p is row src[p]), or plain f32
-// [positions][N] (x: planes of positions in xpack_off order).  w.N, w.K: sizes of one group.
+// the first: post relu2(pre x.W_g^T), or gated the post silu(g) u of interleaved gate / up features, as planes in xpack_off order (x: row-major
+// planes [x_rows][K], position p is row src[p]), or plain f32 [positions][N] (x: planes of positions in xpack_off order).  w.N, w.K: sizes of
+// one group.
 struct TileGroups {
     const int* tile_group = nullptr;  // group of every `align` positions, -1: unused
     int align = 256;
@@ -213,6 +217,7 @@ struct TileGroups {
     int x_rows = 0;
     const float* pre = nullptr;       // [positions], with planes
     const float* post = nullptr;
+    int gated = 0;                    // with planes
 };
 bool gemm_tile_group_ok(int N, int K, int align);
 hipError_t launch_gemm_tile_group(const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int positions, const TileGroups& g, float* out, bf16_bits* act_hi,
@@ -319,7 +324,7 @@ bool gemm_rowdir_ok(int N, int K, int epi, int M);
 bool gemm_rowpar_ok(int N, int K, int epi, int M);
 int gemm_rowpar_splits(int N, int K, int epi, int M);  // f32 slabs the plain epilogue leaves (1 = complete sums)
 int gemm_rowpar_groups(int N, int K);
-// epi: 0 residual + next-norm prep, 1 SwiGLU, 2 plain f32 output, 3 squared ReLU as planes oh / ol (register-direct kernel only)
+// epi: 0 residual + next-norm prep, 1 SwiGLU, 2 plain f32 output, 3 + act: the activation as planes oh / ol (register-direct kernel only)
 hipError_t launch_gemm_rowpar(const RowParArgs& a, const PackedW& w, int epi, hipStream_t s);
 
 // ---- SwiGLU -----------------------------------------------------------------------------------------

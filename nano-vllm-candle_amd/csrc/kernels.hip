@@ -22,7 +22,7 @@ namespace nvllm {
 // ileave >= 0: destination rows are interleaved in 16-row tiles, source row r -> ((r/16)*2 + ileave)*16 + r%16
 // (gate_up: tile 2t = gate features 16t.., tile 2t+1 = up features 16t.. so one wave holds both of a feature)
 __device__ __forceinline__ int dest_row(int row0, int rl, int ileave) {
-    return ileave < 0 ? row0 + rl : (((rl >> 4) * 2 + ileave) << 4) + (rl & 15);
+    return row0 + (ileave < 0 ? rl : (((rl >> 4) * 2 + ileave) << 4) + (rl & 15));
 }
 
 __global__ void __launch_bounds__(256) pack_rows_kernel(uint4* __restrict__ dst, int KT, int row0, int rows,
@@ -1157,11 +1157,11 @@ __global__ void __launch_bounds__(NWK * 64) gemm_rowdir_kernel(RowParArgs a, con
             *reinterpret_cast<uint2*>(a.oh + o) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
             *reinterpret_cast<uint2*>(a.ol + o) = make_uint2(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16));
         }
-    } else if constexpr (EPI == 3) {
+    } else if constexpr (EPI >= 3) {
         if (fin && row < M) {
             uint16_t h[4], l[4];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) split_bf16(relu2(sum[r]), h[r], l[r]);
+            for (int r = 0; r < 4; ++r) split_bf16(act_of<EPI - 3>(sum[r]), h[r], l[r]);
             const int f0 = ntile * 16 + grp * 4;
             const size_t o = a.o_packed ? xpack_off(row, f0, N >> 5) : (size_t)row * N + f0;
             *reinterpret_cast<uint2*>(a.oh + o) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
@@ -1210,7 +1210,7 @@ struct RowParShape { int mt, nwn, nwk, tpw, ph, ns; };
 //   big matrices (>= 24 MB): all rows (up to 64) in one workgroup so every weight byte crosses L2 once, K sliced
 //   into <= 1024-deep pieces over blockIdx.y (plain epilogue only: the slices leave f32 slabs).
 static bool rowpar_shape(int N, int K, int epi, int M, RowParShape& sh) {
-    if (N % 16 || K % 32 || epi == 3) return false;
+    if (N % 16 || K % 32 || epi >= 3) return false;
     const int KT = K / 32, ntiles = N / 16;
     const bool big = (size_t)N * K * 2 >= (size_t)24 << 20 && M > 16;
     static const int tpws[] = {8, 12, 16};
@@ -1320,7 +1320,7 @@ hipError_t launch_gemm_rowpar(const RowParArgs& a, const PackedW& w, int epi, hi
         if (epi == 0) return rowdir_dispatch<0>(d, a, w, s);
         if (epi == 1) return rowdir_dispatch<1>(d, a, w, s);
         if (epi == 2) return rowdir_dispatch<2>(d, a, w, s);
-        if (epi == 3 && a.oh && (!a.o_packed || w.N % 32 == 0)) return rowdir_dispatch<3>(d, a, w, s);
+        if ((epi == 3 || epi == 4) && a.oh && (!a.o_packed || w.N % 32 == 0)) return epi == 3 ? rowdir_dispatch<3>(d, a, w, s) : rowdir_dispatch<4>(d, a, w, s);
         return hipErrorInvalidValue;
     }
     if (a.x_packed || a.o_packed) return hipErrorNotSupported;  // packed planes: register-direct kernel only

@@ -9,7 +9,7 @@ constexpr int kLatentTileRows = 128;  // rows of one q-tile of a prompt chunk (a
 constexpr int kLatentMaxParts = 64;   // split-KV partitions per row
 
 // ---- residual add + up to two norms of the same row ---------------------------------------------------------------------
-// s = sum of the partial sums in / in2 (or embed[id] * embed_scale) (+ residual); residual_out = s;
+// s = sum of the partial sums in / in2 (or embed[id] * embed_scale) (+ residual); residual_out = s; post_w: s = residual + post_mult * norm(sum) instead;
 // output k = s / sqrt(mean(s^2) + eps) * w[k], as bf16 hi/lo planes and/or f32.  Rows are W wide, stored with stride ldr
 // (multiple of 16, zeros beyond W); planes / y have stride ldx (zeros beyond W).
 struct AddNormArgs {
@@ -32,8 +32,11 @@ struct AddNormArgs {
     int W = 0, ldr = 0, ldx = 0;
     int ld_in = 0;                     // row stride of `in` where it is not ldr (16-row form only)
     float eps = 0.f;
+    const float* in_bias = nullptr;    // [ldr] added to the sum of `in`
     const float* post_w = nullptr;
     float post_mult = 1.f;
+    const float* branch_w[2] = {nullptr, nullptr};  // both set, with post_w: half the sum of `in` and `in2`, each RMS-normed with its weight first
+    int again = 0;                     // with post_w: the new residual takes embed[id] * embed_scale on top (`in` is read beside ids)
     const float* w[2] = {nullptr, nullptr};  // nullptr: output k absent
     int center = 0;                    // layer norm: the mean is taken off before the root mean square and the weight
     int raw = 0;                       // output 0 is s itself (w[0] unused)

@@ -13,6 +13,7 @@
 
 #include "decoder.h"
 #include "experts.h"
+#include "rope.h"
 #include "scan_mixer.h"
 
 struct LatentLayer {
@@ -39,28 +40,6 @@ struct LatentLayer {
         return k;
     }
 };
-
-struct RopeTable {
-    double base = 0, factor = 0, original = 0, fast = 0, slow = 0;
-    int dims = 0;
-    float *cos = nullptr, *sin = nullptr;
-    bool serves(const nvllm_latent_layer& c) const {
-        return base == c.rot_base && dims == c.rot_dim && factor == c.yarn_factor &&
-               (factor <= 0 || (original == c.yarn_original && fast == c.yarn_fast && slow == c.yarn_slow));
-    }
-    double frequency(int i) const;
-    double magnitude() const { return factor > 0 ? 0.1 * std::log(factor) + 1.0 : 1.0; }  // of both cos and sin
-};
-// YaRN (Peng et al., "YaRN: Efficient Context Window Extension of Large Language Models"): slow pairs are divided by `factor`, fast ones
-// kept, a ramp over the pairs in between
-double RopeTable::frequency(int i) const {
-    const double f = std::pow(base, -2.0 * i / dims);
-    if (factor <= 0) return f;
-    auto pair_of = [&](double turns) { return dims * std::log(original / (2 * M_PI * turns)) / (2 * std::log(base)); };
-    const double lo = std::max(std::floor(pair_of(fast)), 0.0), hi = std::min(std::ceil(pair_of(slow)), dims - 1.0);
-    const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
-    return f / factor * ramp + f * (1 - ramp);
-}
 
 struct LatentModel : DecoderImpl {
     nvllm_latent_config cfg{};
@@ -212,14 +191,7 @@ extern "C" int nvllm_model_create_latent(nvllm_ctx* ctx, const nvllm_latent_conf
         if (!rc) rc = alloc_w(w.uv, w.heads * w.vdim_p, w.rank_p);
         if (!rc) rc = alloc_w(w.o, L.ldr, w.Kc);
         if (!rc) rc = alloc_v(&w.dkv_norm, w.rank_p);
-        int t = 0;
-        while (t < (int)L.ropes.size() && !L.ropes[t].serves(w.c)) ++t;
-        if (t == (int)L.ropes.size()) {
-            RopeTable r;
-            r.base = w.c.rot_base; r.dims = w.c.rot_dim; r.factor = w.c.yarn_factor; r.original = w.c.yarn_original; r.fast = w.c.yarn_fast; r.slow = w.c.yarn_slow;
-            L.ropes.push_back(r);
-        }
-        w.rope = t;
+        w.rope = rope_index(L.ropes, RopeTable{w.c.rot_base, w.c.yarn_factor, w.c.yarn_original, w.c.yarn_fast, w.c.yarn_slow, w.c.rot_dim});
     }
     if (!rc && hipStreamSynchronize(ctx->stream) != hipSuccess) rc = fail(ctx, NVLLM_EHIP, "weight allocation failed");
     if (rc) { nvllm_model_destroy(m); return rc; }
@@ -246,11 +218,7 @@ void LatentModel::free_kv() {
     L.exp_cap = L.exp_n = 0;
     L.y1 = L.y2 = L.ctx_f = L.act_f = L.cq_f = nullptr;
     L.cqh = L.cql = nullptr;
-    for (RopeTable& r : L.ropes) {
-        if (r.cos) (void)hipFree(r.cos);
-        if (r.sin) (void)hipFree(r.sin);
-        r.cos = r.sin = nullptr;
-    }
+    for (RopeTable& r : L.ropes) r.release();
 }
 
 LatentModel::~LatentModel() {
@@ -546,20 +514,8 @@ int LatentModel::kv_alloc(nvllm_model* m) {
     // rotation tables, one per rotation: angle p * f_i
     m->rope_len = (int)std::min<int64_t>((int64_t)m->max_blocks * kBlockTokens, 1 << 20);
     for (RopeTable& t : L.ropes) {
-        const int half = t.dims / 2;
-        std::vector<float> hc((size_t)m->rope_len * half), hs(hc.size());
-        for (int i = 0; i < half; ++i) {
-            const double f = t.frequency(i), mag = t.magnitude();
-            for (int p = 0; p < m->rope_len; ++p) {
-                hc[(size_t)p * half + i] = (float)(std::cos(p * f) * mag);
-                hs[(size_t)p * half + i] = (float)(std::sin(p * f) * mag);
-            }
-        }
-        rc = dmalloc(ctx, &t.cos, hc.size());
-        if (!rc) rc = dmalloc(ctx, &t.sin, hs.size());
+        rc = t.upload(ctx, m->rope_len);
         if (rc) return rc;
-        HIPCHK(ctx, hipMemcpy(t.cos, hc.data(), hc.size() * 4, hipMemcpyHostToDevice));
-        HIPCHK(ctx, hipMemcpy(t.sin, hs.data(), hs.size() * 4, hipMemcpyHostToDevice));
     }
     return NVLLM_OK;
 }

@@ -12,14 +12,16 @@ namespace nvllm {
 // ---------------------------------------------------------------------------------------------------
 constexpr int kAddNormMax = 8192;  // widest row
 
-enum { NORM_PLAIN, NORM_POST, NORM_CENTER };
+enum { NORM_PLAIN, NORM_POST, NORM_CENTER, NORM_BRANCH };  // NORM_BRANCH: two normed branches, then as NORM_POST
 
 // BS = 256, or 1024 for few wide rows (decode): every thread's loads are then in flight at once
 template <int BS, int KIND>
 __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
-    constexpr bool POST = KIND == NORM_POST;
+    constexpr bool POST = KIND == NORM_POST || KIND == NORM_BRANCH;
     constexpr int NV = kAddNormMax / 4 / BS;
     __shared__ float red[BS / 64];
+    float4 other[KIND == NORM_BRANCH ? NV : 1];
+    float so = 0.f;
     const int r = blockIdx.x;
     const int src = a.row_idx ? a.row_idx[r] : r;
     const int nv4 = a.ldr >> 2;
@@ -30,13 +32,22 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
         const int i = threadIdx.x + c * BS;
         if (i < nv4) {
             float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (a.ids) {
+            if (!POST && a.ids) {
                 const uint2 e = *reinterpret_cast<const uint2*>(a.embed + (size_t)a.ids[src] * a.ldr + (size_t)i * 4);
                 s = make_float4(bf16_to_f32(e.x & 0xffff) * a.embed_scale, bf16_to_f32(e.x >> 16) * a.embed_scale,
                                 bf16_to_f32(e.y & 0xffff) * a.embed_scale, bf16_to_f32(e.y >> 16) * a.embed_scale);
             } else {
                 if (a.in) add_slabs(s, a.in + (size_t)src * a.ldr + (size_t)i * 4, a.n_slabs, a.slab_stride);
-                if (a.in2) {
+                if (POST && a.in_bias) {
+                    const float4 b = *reinterpret_cast<const float4*>(a.in_bias + (size_t)i * 4);
+                    s.x += b.x; s.y += b.y; s.z += b.z; s.w += b.w;
+                }
+                if constexpr (KIND == NORM_BRANCH) {
+                    float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
+                    add_slabs(t, a.in2 + (size_t)src * a.ldr + (size_t)i * 4, a.n_slabs2, a.slab_stride2);
+                    other[c] = t;
+                    so += t.x * t.x + t.y * t.y + t.z * t.z + t.w * t.w;
+                } else if (a.in2) {
                     float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
                     add_slabs(t, a.in2 + (size_t)src * a.ldr + (size_t)i * 4, a.n_slabs2, a.slab_stride2);
                     const float f = a.in2_scale ? a.in2_scale[src] : 1.f;
@@ -74,6 +85,22 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
             ss += s.x * s.x + s.y * s.y + s.z * s.z + s.w * s.w;
         }
     }
+    if constexpr (KIND == NORM_BRANCH) {
+        const float f = 0.5f / sqrtf(block_sum(ss, red, BS / 64) / (float)a.W + a.eps), fo = 0.5f / sqrtf(block_sum(so, red, BS / 64) / (float)a.W + a.eps);
+        ss = 0.f;
+#pragma unroll
+        for (int c = 0; c < NV; ++c) {
+            const int i = threadIdx.x + c * BS;
+            if (i >= nv4) continue;
+            const float4 w = *reinterpret_cast<const float4*>(a.branch_w[0] + (size_t)i * 4), v = *reinterpret_cast<const float4*>(a.branch_w[1] + (size_t)i * 4);
+            float4 s = cache[c];
+            const float4 t = other[c];
+            s.x = (s.x * f) * w.x + (t.x * fo) * v.x; s.y = (s.y * f) * w.y + (t.y * fo) * v.y;
+            s.z = (s.z * f) * w.z + (t.z * fo) * v.z; s.w = (s.w * f) * w.w + (t.w * fo) * v.w;
+            cache[c] = s;
+            ss += s.x * s.x + s.y * s.y + s.z * s.z + s.w * s.w;
+        }
+    }
     if constexpr (POST) {
         const float f = a.post_mult / sqrtf(block_sum(ss, red, BS / 64) / (float)a.W + a.eps);
         ss = 0.f;
@@ -84,6 +111,11 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
             const float4 w = *reinterpret_cast<const float4*>(a.post_w + (size_t)i * 4);
             float4 s = cache[c];
             s.x = res[c].x + (s.x * f) * w.x; s.y = res[c].y + (s.y * f) * w.y; s.z = res[c].z + (s.z * f) * w.z; s.w = res[c].w + (s.w * f) * w.w;
+            if (a.again) {
+                const uint2 e = *reinterpret_cast<const uint2*>(a.embed + (size_t)a.ids[src] * a.ldr + (size_t)i * 4);
+                s.x += bf16_to_f32(e.x & 0xffff) * a.embed_scale; s.y += bf16_to_f32(e.x >> 16) * a.embed_scale;
+                s.z += bf16_to_f32(e.y & 0xffff) * a.embed_scale; s.w += bf16_to_f32(e.y >> 16) * a.embed_scale;
+            }
             if (a.residual_out) *reinterpret_cast<float4*>(a.residual_out + (size_t)src * a.ldr + (size_t)i * 4) = s;
             cache[c] = s;
             ss += s.x * s.x + s.y * s.y + s.z * s.z + s.w * s.w;
@@ -123,8 +155,10 @@ __global__ void __launch_bounds__(BS) add_norm_kernel(AddNormArgs a) {
 template <int IT, int KIND>
 __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, int rows) {
     constexpr int NW = 16;
-    constexpr bool POST = KIND == NORM_POST;
-    __shared__ float red[KIND == NORM_PLAIN ? 1 : 2][NW][16];
+    constexpr bool POST = KIND == NORM_POST || KIND == NORM_BRANCH;
+    __shared__ float red[KIND == NORM_PLAIN ? 1 : KIND == NORM_BRANCH ? 4 : 2][NW][16];
+    float o[KIND == NORM_BRANCH ? IT : 1][8];
+    float so = 0.f;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, grp = lane >> 4;
     const int KT = a.ldr >> 5, row = blockIdx.x * 16 + l15, rowc = min(row, rows - 1);
     float v[IT][8];
@@ -135,7 +169,7 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
         if (kt >= KT) continue;
         const size_t col = (size_t)kt * 32 + grp * 8, off = (size_t)rowc * a.ldr + col;
         float4 s0 = make_float4(0.f, 0.f, 0.f, 0.f), s1 = s0;
-        if (a.ids) {
+        if (!POST && a.ids) {
             const uint4 e = *reinterpret_cast<const uint4*>(a.embed + (size_t)a.ids[rowc] * a.ldr + col);
             const float f = a.embed_scale;
             s0 = make_float4(bf16_to_f32(e.x & 0xffff) * f, bf16_to_f32(e.x >> 16) * f, bf16_to_f32(e.y & 0xffff) * f, bf16_to_f32(e.y >> 16) * f);
@@ -148,7 +182,17 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
             };
             const size_t off_in = a.ld_in ? (size_t)rowc * a.ld_in + col : off;
             if (a.in) for (int sl = 0; sl < a.n_slabs; ++sl) add(a.in + (size_t)sl * a.slab_stride + off_in);
-            if (a.in2) {
+            if (POST && a.in_bias) add(a.in_bias + col);
+            if constexpr (KIND == NORM_BRANCH) {
+                const float4 k0 = s0, k1 = s1;
+                s0 = s1 = make_float4(0.f, 0.f, 0.f, 0.f);
+                for (int sl = 0; sl < a.n_slabs2; ++sl) add(a.in2 + (size_t)sl * a.slab_stride2 + off);
+                o[i][0] = s0.x; o[i][1] = s0.y; o[i][2] = s0.z; o[i][3] = s0.w;
+                o[i][4] = s1.x; o[i][5] = s1.y; o[i][6] = s1.z; o[i][7] = s1.w;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) so += o[i][e] * o[i][e];
+                s0 = k0; s1 = k1;
+            } else if (a.in2) {
                 const float f = a.in2_scale ? a.in2_scale[rowc] : 1.f;
                 for (int sl = 0; sl < a.n_slabs2; ++sl) add(a.in2 + (size_t)sl * a.slab_stride2 + off, f);
             }
@@ -189,6 +233,23 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
             }
         }
     }
+    if constexpr (KIND == NORM_BRANCH) {
+        const float f = 0.5f * row_rinv(red[2]);
+        ss = so;
+        const float fo = 0.5f * row_rinv(red[3]);
+        ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < IT; ++i) {
+            const int kt = wave + i * NW;
+            if (kt >= KT) continue;
+            const float *w = a.branch_w[0] + kt * 32 + grp * 8, *u = a.branch_w[1] + kt * 32 + grp * 8;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                v[i][e] = (v[i][e] * f) * w[e] + (o[i][e] * fo) * u[e];
+                ss += v[i][e] * v[i][e];
+            }
+        }
+    }
     if constexpr (POST) {
         const float f = row_rinv(red[1]) * a.post_mult;
         ss = 0.f;
@@ -201,6 +262,12 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
             const float4 w0 = *reinterpret_cast<const float4*>(a.post_w + col), w1 = *reinterpret_cast<const float4*>(a.post_w + col + 4);
             s0.x += (v[i][0] * f) * w0.x; s0.y += (v[i][1] * f) * w0.y; s0.z += (v[i][2] * f) * w0.z; s0.w += (v[i][3] * f) * w0.w;
             s1.x += (v[i][4] * f) * w1.x; s1.y += (v[i][5] * f) * w1.y; s1.z += (v[i][6] * f) * w1.z; s1.w += (v[i][7] * f) * w1.w;
+            if (a.again) {
+                const uint4 e = *reinterpret_cast<const uint4*>(a.embed + (size_t)a.ids[rowc] * a.ldr + col);
+                const float fe = a.embed_scale;
+                s0.x += bf16_to_f32(e.x & 0xffff) * fe; s0.y += bf16_to_f32(e.x >> 16) * fe; s0.z += bf16_to_f32(e.y & 0xffff) * fe; s0.w += bf16_to_f32(e.y >> 16) * fe;
+                s1.x += bf16_to_f32(e.z & 0xffff) * fe; s1.y += bf16_to_f32(e.z >> 16) * fe; s1.z += bf16_to_f32(e.w & 0xffff) * fe; s1.w += bf16_to_f32(e.w >> 16) * fe;
+            }
             if (a.residual_out && row < rows) {
                 *reinterpret_cast<float4*>(a.residual_out + off) = s0;
                 *reinterpret_cast<float4*>(a.residual_out + off + 4) = s1;
@@ -241,7 +308,9 @@ hipError_t launch_add_norm(const AddNormArgs& a, int rows, hipStream_t s) {
         return hipErrorInvalidValue;
     if (rows <= 0) return hipSuccess;
     const bool post = a.post_w != nullptr, any = a.w[0] || a.w[1] || a.raw;
+    const bool branch = a.branch_w[0] != nullptr;
     if (a.raw && a.w[0]) return hipErrorInvalidValue;
+    if ((a.again && (!post || !a.ids || !a.embed)) || (a.in_bias && !post) || (branch && (!post || !a.branch_w[1] || !a.in || !a.in2 || a.in2_scale || a.n_gather))) return hipErrorInvalidValue;
     bool packed = any && a.ldr == a.ldx && a.ldr % 32 == 0 && !a.row_idx && (!post || a.residual_in);
     for (int k = 0; k < 2; ++k) packed &= !(a.w[k] || (k == 0 && a.raw)) || ((a.packed[k] || (k == 1 && a.w[0])) && a.xh[k] && !a.y[k]);
     if ((a.center && (post || a.raw)) || (a.ld_in && (!packed || a.ldr > 4096 || a.ld_in % 4 || a.slab_stride % 4))) return hipErrorInvalidValue;
@@ -258,7 +327,8 @@ hipError_t launch_add_norm(const AddNormArgs& a, int rows, hipStream_t s) {
             add_norm_kernel<256, KIND><<<rows, 256, 0, s>>>(a);
         }
     };
-    if (post) launch(std::integral_constant<int, NORM_POST>{});
+    if (branch) launch(std::integral_constant<int, NORM_BRANCH>{});
+    else if (post) launch(std::integral_constant<int, NORM_POST>{});
     else if (a.center) launch(std::integral_constant<int, NORM_CENTER>{});
     else launch(std::integral_constant<int, NORM_PLAIN>{});
     return hipGetLastError();

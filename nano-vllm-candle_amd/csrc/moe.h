@@ -14,9 +14,11 @@ struct RouteArgs {
     int gate_col = -1;           // column of the shared gate (-1: none)
     int shared_group = 0;        // every row is a member of group `experts` too
     int weight_in = 1;           // the score multiplies the expert's input (else its output)
+    int softmax = 0;             // scores: softmax over all experts (else the sigmoid of each logit)
+    int groups = 1, keep = 1;    // equal groups of neighbours; only experts of the `keep` groups with the largest logits can be chosen
     int align = 16, cap = 0;     // cap: positions allocated (a multiple of align)
     int* chosen = nullptr;       // [rows][top]
-    float* score = nullptr;      // [rows][top] sigmoid of the chosen logits
+    float* score = nullptr;      // [rows][top] scores of the chosen
     float* gate = nullptr;       // [rows] sigmoid of the shared gate's logit
     int* place = nullptr;        // [rows][top + shared_group] position of the row in each of its groups
     int* src = nullptr;          // [cap] row of a position (padding: -1)
@@ -44,6 +46,7 @@ struct GroupGemmArgs {
     const float* pre = nullptr;
     const float* post = nullptr;
     int relu2 = 0;                   // act: squared ReLU (else none)
+    int glu = 0;                     // silu(gate) up of features in interleaved 16-row tiles (N, ldo: of the weights, of the result); no pre
     float* out = nullptr;            // f32 [positions][ldo], or
     bf16_bits* oh = nullptr;         // planes of positions in fragment order, ldo columns
     bf16_bits* ol = nullptr;

@@ -25,12 +25,13 @@ __device__ __forceinline__ void route_row(const RouteArgs& a, int row, int lane)
         v[i] = e < a.experts ? x : -INFINITY;
     }
     if (a.gate_col >= 0 && lane == 0 && in) a.gate[row] = sigmoid_exact(gate);
-    for (int k = 0; k < a.top; ++k) {
-        float best = -INFINITY;
-        int at = kMaxExperts;  // the lowest index wins a tie
+    // the largest of the row and its expert, lowest index on a tie
+    auto largest = [&](const float (&x)[NV], float& best, int& at) {
+        best = -INFINITY;
+        at = kMaxExperts;
 #pragma unroll
         for (int i = 0; i < NV; ++i)
-            if (v[i] > best) { best = v[i]; at = lane + i * NL; }
+            if (x[i] > best) { best = x[i]; at = lane + i * NL; }
 #pragma unroll
         for (int o = NL / 2; o > 0; o >>= 1) {
             const float b = __shfl_xor(best, o);
@@ -38,9 +39,45 @@ __device__ __forceinline__ void route_row(const RouteArgs& a, int row, int lane)
             if (b > best || (b == best && c < at)) { best = b; at = c; }
         }
         at = min(at, a.experts - 1);  // no finite logit left
+    };
+    float top_z = 0.f, total = 1.f;
+    if (a.softmax) {
+        top_z = v[0];
+#pragma unroll
+        for (int i = 1; i < NV; ++i) top_z = fmaxf(top_z, v[i]);
+#pragma unroll
+        for (int o = NL / 2; o > 0; o >>= 1) top_z = fmaxf(top_z, __shfl_xor(top_z, o));
+        total = 0.f;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) total += expf(v[i] - top_z);
+#pragma unroll
+        for (int o = NL / 2; o > 0; o >>= 1) total += __shfl_xor(total, o);
+    }
+    if (a.keep < a.groups) {  // the best group left holds the largest logit of the groups left
+        const int per = a.experts / a.groups;
+        float left[NV];
+        bool kept[NV];
+#pragma unroll
+        for (int i = 0; i < NV; ++i) { left[i] = v[i]; kept[i] = false; }
+        for (int k = 0; k < a.keep; ++k) {
+            float best;
+            int at;
+            largest(left, best, at);
+            const int g = at / per;
+#pragma unroll
+            for (int i = 0; i < NV; ++i)
+                if ((lane + i * NL) / per == g) { left[i] = -INFINITY; kept[i] = true; }
+        }
+#pragma unroll
+        for (int i = 0; i < NV; ++i) v[i] = kept[i] ? v[i] : -INFINITY;
+    }
+    for (int k = 0; k < a.top; ++k) {
+        float best;
+        int at;
+        largest(v, best, at);
         if (lane == 0 && in) {
             a.chosen[(size_t)row * a.top + k] = at;
-            a.score[(size_t)row * a.top + k] = sigmoid_exact(best);
+            a.score[(size_t)row * a.top + k] = a.softmax ? expf(best - top_z) / total : sigmoid_exact(best);
         }
 #pragma unroll
         for (int i = 0; i < NV; ++i)
@@ -145,7 +182,7 @@ __global__ void __launch_bounds__(1024) place_rows_kernel(RouteArgs a) {
 hipError_t launch_route(const RouteArgs& a, hipStream_t s) {
     const int64_t need = (int64_t)a.rows * a.top + (int64_t)std::min(a.experts, a.rows * a.top) * (a.align - 1) + (a.shared_group ? a.rows + a.align - 1 : 0);
     if (a.experts < 1 || a.experts > kMaxExperts || a.top < 1 || a.top > std::min(a.experts, kMaxTop) || a.align < 1 || a.cap % a.align || need > a.cap ||
-        a.ld < a.experts || a.gate_col >= a.ld || (a.gate_col >= 0 && !a.gate) || !a.cursor)
+        a.groups < 1 || a.experts % a.groups || a.keep < 1 || (a.keep < a.groups && a.top > a.keep * (a.experts / a.groups)) || a.ld < a.experts || a.gate_col >= a.ld || (a.gate_col >= 0 && !a.gate) || !a.cursor)
         return hipErrorInvalidValue;
     if (a.rows <= 0) return hipSuccess;
     const bool one = a.rows <= 64;
@@ -170,9 +207,9 @@ hipError_t launch_route(const RouteArgs& a, hipStream_t s) {
 
 // ---------------------------------------------------------------------------------------------------
 // products over groups: MT m-tiles (16 positions each) of one group x NT n-tiles per wave; the four waves take other n-tiles (WK = 1)
-// or a quarter of K each, summed through LDS (WK = 4: few rows, many weight bytes)
+// or a quarter of K each, summed through LDS (WK = 4: few rows, many weight bytes).  GLU: n-tiles are pairs of a gate and an up tile.
 // ---------------------------------------------------------------------------------------------------
-template <int MT, int NT, int WK, bool EXACT>
+template <int MT, int NT, int WK, bool EXACT, bool GLU>
 __global__ void __launch_bounds__(256) group_gemm_kernel(GroupGemmArgs a) {
     __shared__ __attribute__((aligned(16))) f32x4 part[WK == 4 ? 4 * NT * MT * 64 : 1];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -260,23 +297,44 @@ __global__ void __launch_bounds__(256) group_gemm_kernel(GroupGemmArgs a) {
             for (int b = 0; b < MT; ++b) part[((wave * NT + n) * MT + b) * 64 + lane] = acc[n][b];
         __syncthreads();
     }
+    auto whole = [&](int n, int b) {  // the finished sum
+        f32x4 v = acc[n][b];
+        if constexpr (WK == 4) {
+            v = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int q = 0; q < 4; ++q) {
+                const f32x4 t = part[((q * NT + n) * MT + b) * 64 + lane];
+#pragma unroll
+                for (int r = 0; r < 4; ++r) v[r] += t[r];
+            }
+        }
+        return v;
+    };
+    if constexpr (GLU) {
+        static_assert(!GLU || NT == 2, "a gate tile and its up tile");
+        const int f = (nt0 >> 1) * 16 + grp * 4;
+#pragma unroll
+        for (int b = 0; b < MT; ++b) {
+            if (WK == 4 && b % 4 != wave) continue;
+            const f32x4 gate = whole(0, b), up = whole(1, b);
+            const int p = p0 + b * 16 + l15;
+            const float post = a.post ? a.post[p] : 1.f;
+            f32x4 v;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] = (EXACT ? gate[r] / (1.0f + expf(-gate[r])) * up[r] : silu_mul(gate[r], up[r])) * post;
+            if (a.out) *reinterpret_cast<float4*>(a.out + (size_t)p * a.ldo + f) = make_float4(v[0], v[1], v[2], v[3]);
+            if (a.oh) put_planes4(a.oh, a.ol, p, f, 4, a.ldo, 1, v);
+        }
+        return;
+    }
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
         if (nt0 + n >= ntiles) continue;
         const int f = (nt0 + n) * 16 + grp * 4;
 #pragma unroll
         for (int b = 0; b < MT; ++b) {
-            f32x4 v = acc[n][b];
-            if constexpr (WK == 4) {
-                if ((n * MT + b) % 4 != wave) continue;
-                v = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int q = 0; q < 4; ++q) {
-                    const f32x4 t = part[((q * NT + n) * MT + b) * 64 + lane];
-#pragma unroll
-                    for (int r = 0; r < 4; ++r) v[r] += t[r];
-                }
-            }
+            if (WK == 4 && (n * MT + b) % 4 != wave) continue;
+            f32x4 v = whole(n, b);
             const int p = p0 + b * 16 + l15;
             if (!a.tile_group && p >= a.x_rows) continue;
             const float pre = a.pre ? a.pre[p] : 1.f, post = a.post ? a.post[p] : 1.f;
@@ -296,18 +354,22 @@ hipError_t launch_group_gemm(const GroupGemmArgs& a, hipStream_t s) {
     const bool exact = a.xf != nullptr;
     const int nmax = a.last >= 0 ? std::max(a.N, a.Ns) : a.N, kmax = a.last >= 0 ? std::max(a.K, a.Ks) : a.K;
     if (a.N % 16 || a.K % 32 || (a.last >= 0 && (a.Ns % 16 || a.Ks % 32 || !a.ws)) || a.ldx % 32 || a.ldx < kmax || (!exact && (!a.xh || !a.xl)) ||
-        (!a.out && !a.oh) || a.ldo < nmax || a.ldo % (a.oh ? 32 : 4) || a.x_rows < 1 || (a.align != 16 && a.align != 64))
+        (!a.out && !a.oh) || a.ldo < (a.glu ? nmax / 2 : nmax) || (a.glu && (a.N % 32 || a.last >= 0 || a.relu2 || a.pre || !a.tile_group)) || a.ldo % (a.oh ? 32 : 4) || a.x_rows < 1 || (a.align != 16 && a.align != 64))
         return hipErrorInvalidValue;
     const int tiles = a.tile_group ? a.tiles : (a.x_rows + a.align - 1) / a.align;
     if (tiles <= 0) return hipSuccess;
     const int nt = nmax / 16;
-#define NVLLM_GG(MT_, NT_, WK_, EX_) group_gemm_kernel<MT_, NT_, WK_, EX_><<<dim3((nt + NT_ * (WK_ == 4 ? 1 : 4) - 1) / (NT_ * (WK_ == 4 ? 1 : 4)), tiles), 256, 0, s>>>(a)
+#define NVLLM_GG(MT_, NT_, WK_, EX_, GLU_) group_gemm_kernel<MT_, NT_, WK_, EX_, GLU_><<<dim3((nt + NT_ * (WK_ == 4 ? 1 : 4) - 1) / (NT_ * (WK_ == 4 ? 1 : 4)), tiles), 256, 0, s>>>(a)
     if (a.align == 64) {
-        if (exact) NVLLM_GG(4, 1, 1, true);
-        else NVLLM_GG(4, 2, 1, false);
+        if (a.glu && exact) NVLLM_GG(4, 2, 1, true, true);
+        else if (a.glu) NVLLM_GG(4, 2, 1, false, true);
+        else if (exact) NVLLM_GG(4, 1, 1, true, false);
+        else NVLLM_GG(4, 2, 1, false, false);
     } else {
-        if (exact) NVLLM_GG(1, 1, 4, true);
-        else NVLLM_GG(1, 2, 4, false);
+        if (a.glu && exact) NVLLM_GG(1, 2, 4, true, true);
+        else if (a.glu) NVLLM_GG(1, 2, 4, false, true);
+        else if (exact) NVLLM_GG(1, 1, 4, true, false);
+        else NVLLM_GG(1, 2, 4, false, false);
     }
 #undef NVLLM_GG
     return hipGetLastError();

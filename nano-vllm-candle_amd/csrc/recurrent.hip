@@ -12,9 +12,11 @@
 namespace nvllm {
 
 // one token on the wave's registers
-template <int R4, bool DELTA>
+enum { DECAY_CONST, DECAY_CHANNEL, DECAY_HEAD };  // constant decays; delta rule with a decay per key channel, per head
+template <int R4, int KIND>
 __device__ __forceinline__ float2 recur_token(float (&S)[R4][2][4], const float4 (&k)[R4], const float4 (&q)[R4], const float4 (&g)[R4], float decay,
                                               float2 v, float beta) {
+    constexpr bool DELTA = KIND != DECAY_CONST;
     float dk[2] = {0.f, 0.f}, dq[2] = {0.f, 0.f}, kq = 0.f;
 #pragma unroll
     for (int r = 0; r < R4; ++r) {
@@ -25,7 +27,7 @@ __device__ __forceinline__ float2 recur_token(float (&S)[R4][2][4], const float4
             kq += kv[i] * qv[i];
 #pragma unroll
             for (int c = 0; c < 2; ++c) {
-                S[r][c][i] *= DELTA ? gv[i] : decay;
+                S[r][c][i] *= KIND == DECAY_CHANNEL ? gv[i] : decay;
                 if (DELTA) dk[c] += S[r][c][i] * kv[i];
                 dq[c] += S[r][c][i] * qv[i];
             }
@@ -65,10 +67,11 @@ __device__ __forceinline__ void state_io(float (&S)[R4][2][4], float* st, int la
 }
 
 // one workgroup = 32 columns of one head of one segment, tokens in pieces of TT staged through LDS (two buffers)
-template <int R4, bool DELTA>
+template <int R4, int KIND>
 __global__ void __launch_bounds__(256) recurrence_kernel(RecurArgs a) {
-    constexpr int DP = R4 * 64, TT = R4 <= 2 ? 16 : 8, NV = DELTA ? 3 : 2;
-    constexpr int W4 = NV * DP / 4 + 9;             // float4 per token: k, q, (g), 32 values, beta
+    constexpr bool DELTA = KIND != DECAY_CONST, CHANNEL = KIND == DECAY_CHANNEL;
+    constexpr int DP = R4 * 64, TT = R4 <= 2 ? 16 : 8, NV = CHANNEL ? 3 : 2;
+    constexpr int W4 = NV * DP / 4 + 9;             // float4 per token: k, q, (g), 32 values, beta and decay
     constexpr int NL = (TT * W4 + 255) / 256;
     __shared__ __attribute__((aligned(16))) float4 buf[2][TT * W4];
     __shared__ float obuf[TT][32];
@@ -88,16 +91,16 @@ __global__ void __launch_bounds__(256) recurrence_kernel(RecurArgs a) {
 #pragma unroll
                 for (int i = 0; i < 4; ++i) S[r][c][i] = 0.f;
     }
-    const float decay = DELTA ? 1.f : a.decay[head];
+    const float decay = DELTA ? 1.f : a.decay[head];  // of every token
     // slot w of token t
     auto fetch = [&](int t, int w) -> float4 {
         const size_t row = row0 + min(t, n - 1);
         if (w < DP / 4) return reinterpret_cast<const float4*>(a.k + (row * a.q_heads + qh) * DP)[w];
         if (w < 2 * (DP / 4)) return reinterpret_cast<const float4*>(a.q + (row * a.q_heads + qh) * DP)[w - DP / 4];
-        if (DELTA && w < 3 * (DP / 4)) return reinterpret_cast<const float4*>(a.g + row * a.g_row + (size_t)head * DP)[w - 2 * (DP / 4)];
+        if (CHANNEL && w < 3 * (DP / 4)) return reinterpret_cast<const float4*>(a.g + row * a.g_row + (size_t)head * DP)[w - 2 * (DP / 4)];
         const int x = w - NV * (DP / 4);
         if (x < 8) return reinterpret_cast<const float4*>(a.v + (row * a.heads + head) * a.vdim_p + cb * 32)[x];
-        return make_float4(DELTA ? a.beta[row * a.heads + head] : 0.f, 0.f, 0.f, 0.f);
+        return make_float4(DELTA ? a.beta[row * a.heads + head] : 0.f, KIND == DECAY_HEAD ? a.gh[row * a.heads + head] : 0.f, 0.f, 0.f);
     };
     float4 pre[NL];
     auto load = [&](int t0) {
@@ -126,12 +129,12 @@ __global__ void __launch_bounds__(256) recurrence_kernel(RecurArgs a) {
             for (int r = 0; r < R4; ++r) {
                 k[r] = b[r * 16 + p];
                 q[r] = b[DP / 4 + r * 16 + p];
-                if (DELTA) g[r] = b[2 * (DP / 4) + r * 16 + p];
+                if (CHANNEL) g[r] = b[2 * (DP / 4) + r * 16 + p];
                 else g[r] = make_float4(0.f, 0.f, 0.f, 0.f);
             }
             const float* bv = reinterpret_cast<const float*>(b + NV * (DP / 4));
             const float2 v = *reinterpret_cast<const float2*>(bv + wave * 8 + cg * 2);
-            const float2 o = recur_token<R4, DELTA>(S, k, q, g, decay, v, bv[32]);
+            const float2 o = recur_token<R4, KIND>(S, k, q, g, KIND == DECAY_HEAD ? bv[33] : decay, v, bv[32]);
             if (p == 0) *reinterpret_cast<float2*>(&obuf[t][wave * 8 + cg * 2]) = o;
         }
         if (t0 + TT < n) park(buf[cur ^ 1]);
@@ -148,8 +151,9 @@ __global__ void __launch_bounds__(256) recurrence_kernel(RecurArgs a) {
 // decode: one workgroup = one (row, head); a wave takes every fourth block of eight columns, four blocks' state in flight.  With
 // NORM (per-head norms) the gated output norm follows in the same launch.
 // ---------------------------------------------------------------------------------------------------
-template <int R4, bool DELTA, bool NORM>
+template <int R4, int KIND, bool NORM>
 __global__ void __launch_bounds__(256) recurrence_decode_kernel(RecurArgs a, GatedNormArgs n) {
+    constexpr bool DELTA = KIND != DECAY_CONST, CHANNEL = KIND == DECAY_CHANNEL;
     constexpr int DP = R4 * 64, NB = R4 <= 2 ? 4 : 1;
     extern __shared__ float o_lds[];  // [vdim_p], NORM
     __shared__ float red[4];
@@ -160,15 +164,15 @@ __global__ void __launch_bounds__(256) recurrence_decode_kernel(RecurArgs a, Gat
     float4 k[R4], q[R4], g[R4];
     const float4* kp = reinterpret_cast<const float4*>(a.k + ((size_t)row * a.q_heads + qh) * DP) + p;
     const float4* qp = reinterpret_cast<const float4*>(a.q + ((size_t)row * a.q_heads + qh) * DP) + p;
-    const float4* gp = reinterpret_cast<const float4*>(DELTA ? a.g + (size_t)row * a.g_row + (size_t)head * DP : a.k) + p;
+    const float4* gp = reinterpret_cast<const float4*>(CHANNEL ? a.g + (size_t)row * a.g_row + (size_t)head * DP : a.k) + p;
     const float* vp = a.v + ((size_t)row * a.heads + head) * a.vdim_p + cg * 2;
 #pragma unroll
     for (int r = 0; r < R4; ++r) {
         k[r] = kp[r * 16];
         q[r] = qp[r * 16];
-        g[r] = DELTA ? gp[r * 16] : make_float4(0.f, 0.f, 0.f, 0.f);
+        g[r] = CHANNEL ? gp[r * 16] : make_float4(0.f, 0.f, 0.f, 0.f);
     }
-    const float decay = DELTA ? 1.f : a.decay[head], beta = DELTA ? a.beta[(size_t)row * a.heads + head] : 0.f;
+    const float decay = KIND == DECAY_HEAD ? a.gh[(size_t)row * a.heads + head] : DELTA ? 1.f : a.decay[head], beta = DELTA ? a.beta[(size_t)row * a.heads + head] : 0.f;
     for (int b0 = wave; b0 < blocks; b0 += 4 * NB) {
         float S[NB][R4][2][4];
         float2 v[NB];
@@ -190,7 +194,7 @@ __global__ void __launch_bounds__(256) recurrence_decode_kernel(RecurArgs a, Gat
 #pragma unroll
                         for (int i = 0; i < 4; ++i) S[u][r][c][i] = 0.f;
             }
-            const float2 o = recur_token<R4, DELTA>(S[u], k, q, g, decay, v[u], beta);
+            const float2 o = recur_token<R4, KIND>(S[u], k, q, g, decay, v[u], beta);
             state_io<R4>(S[u], st + (size_t)b * 8 * DP, lane, true);
             if (p == 0) {
                 if (NORM) *reinterpret_cast<float2*>(o_lds + b * 8 + cg * 2) = o;
@@ -205,7 +209,12 @@ __global__ void __launch_bounds__(256) recurrence_decode_kernel(RecurArgs a, Gat
         const float rinv = 1.0f / sqrtf(block_sum(ss, red, 4) / (float)n.vdim + n.eps);
         const float* gate = n.gate + (size_t)row * n.gate_row + (size_t)head * n.gate_head;
         for (int e = threadIdx.x; e < n.vdim; e += 256) {
-            const float x = (o_lds[e] * rinv) * n.weight[e] * gate[e];
+            float f = gate[e];
+            if (n.gate_slabs) {
+                f = slab_elem(gate + e, n.gate_slabs, n.gate_stride);
+                f = f / (1.0f + expf(-f));
+            }
+            const float x = (o_lds[e] * rinv) * n.weight[e] * f;
             const int col = head * n.vdim + e;
             if (n.of) n.of[(size_t)row * n.ld + col] = x;
             if (n.oh) {
@@ -218,16 +227,16 @@ __global__ void __launch_bounds__(256) recurrence_decode_kernel(RecurArgs a, Gat
 
 bool recur_ok(int dim, int vdim) { return dim >= 1 && dim <= 512 && vdim >= 1 && vdim <= 8192; }
 
-template <int R4, bool DELTA>
+template <int R4, int KIND>
 static void recurrence_t(const RecurArgs& a, const GatedNormArgs* norm, hipStream_t s) {
-    if (!a.seg.single) recurrence_kernel<R4, DELTA><<<dim3(a.heads * (a.vdim_p / 32), a.seg.count), 256, 0, s>>>(a);
-    else if (norm) recurrence_decode_kernel<R4, DELTA, true><<<dim3(a.heads, a.seg.count), 256, (size_t)a.vdim_p * 4, s>>>(a, *norm);
-    else recurrence_decode_kernel<R4, DELTA, false><<<dim3(a.heads, a.seg.count), 256, 0, s>>>(a, GatedNormArgs());
+    if (!a.seg.single) recurrence_kernel<R4, KIND><<<dim3(a.heads * (a.vdim_p / 32), a.seg.count), 256, 0, s>>>(a);
+    else if (norm) recurrence_decode_kernel<R4, KIND, true><<<dim3(a.heads, a.seg.count), 256, (size_t)a.vdim_p * 4, s>>>(a, *norm);
+    else recurrence_decode_kernel<R4, KIND, false><<<dim3(a.heads, a.seg.count), 256, 0, s>>>(a, GatedNormArgs());
 }
-template <bool DELTA>
+template <int KIND>
 static hipError_t recurrence_launch(const RecurArgs& a, const GatedNormArgs* norm, hipStream_t s) {
     switch (a.dim_p / 64) {
-#define NVLLM_RC(R_) case R_: recurrence_t<R_, DELTA>(a, norm, s); break;
+#define NVLLM_RC(R_) case R_: recurrence_t<R_, KIND>(a, norm, s); break;
         NVLLM_RC(1) NVLLM_RC(2) NVLLM_RC(3) NVLLM_RC(4) NVLLM_RC(5) NVLLM_RC(6) NVLLM_RC(7) NVLLM_RC(8)
 #undef NVLLM_RC
         default: return hipErrorNotSupported;
@@ -235,10 +244,11 @@ static hipError_t recurrence_launch(const RecurArgs& a, const GatedNormArgs* nor
     return hipGetLastError();
 }
 hipError_t launch_recurrence(const RecurArgs& a, const GatedNormArgs* norm, hipStream_t s) {
-    if (a.dim_p % 64 || a.vdim_p % 32 || a.q_heads < 1 || a.heads % a.q_heads || (a.g && !a.beta) || (!a.g && !a.decay) || (a.g_row & 3)) return hipErrorInvalidValue;
+    if (a.dim_p % 64 || a.vdim_p % 32 || a.q_heads < 1 || a.heads % a.q_heads || ((a.g || a.gh) && !a.beta) || (a.g && a.gh) || (!a.g && !a.gh && !a.decay) || (a.g_row & 3)) return hipErrorInvalidValue;
     if (norm && (!a.seg.single || norm->whole || norm->heads != a.heads || norm->vdim_p != a.vdim_p || norm->heads * norm->vdim > norm->ld)) return hipErrorInvalidValue;
     if (a.seg.count <= 0) return hipSuccess;
-    return a.g ? recurrence_launch<true>(a, norm, s) : recurrence_launch<false>(a, norm, s);
+    if (a.gh) return recurrence_launch<DECAY_HEAD>(a, norm, s);
+    return a.g ? recurrence_launch<DECAY_CHANNEL>(a, norm, s) : recurrence_launch<DECAY_CONST>(a, norm, s);
 }
 
 }  // namespace nvllm

@@ -23,7 +23,8 @@ __device__ __forceinline__ int token_slot(int j) { return ((j & 3) << 2) | (j >>
 // ---------------------------------------------------------------------------------------------------
 // one wave per (piece, head)
 // ---------------------------------------------------------------------------------------------------
-template <int R4>
+// HEAD: one decay per head and token, so the pair products are two plain products on the matrix cores with factors on their results
+template <int R4, bool HEAD>
 __global__ void __launch_bounds__(64) delta_pieces_kernel(RecurArgs a, PieceArgs c) {
     constexpr int DP = R4 * 64;
     __shared__ __attribute__((aligned(16))) float A[16 * 16];
@@ -33,10 +34,48 @@ __global__ void __launch_bounds__(64) delta_pieces_kernel(RecurArgs a, PieceArgs
     // rows past the piece's last one hold something finite that is masked
     const float* kb = a.k + ((size_t)row0 * a.q_heads + qh) * DP;
     const float* qb = a.q + ((size_t)row0 * a.q_heads + qh) * DP;
-    const float* gb = a.g + (size_t)row0 * a.g_row + (size_t)head * DP;
-    const int ks = a.q_heads * DP, gs = (int)a.g_row;
-    // A and B: lane (jg, dg) carries t_j of tokens j = 4 s + jg for the channels 64 r + 4 dg + e
-    {
+    const float* gb = HEAD ? a.gh + (size_t)row0 * a.heads + head : a.g + (size_t)row0 * a.g_row + (size_t)head * DP;
+    const int ks = a.q_heads * DP, gs = HEAD ? a.heads : (int)a.g_row;
+    [[maybe_unused]] float gh[16];
+    if constexpr (HEAD) {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) gh[i] = i < n ? gb[i * gs] : 1.f;
+        // products of decays from token j + 1 on, j = dg: to tokens i = 4 jg + r and to the piece's end
+        float f = 1.f, upto[4] = {0.f, 0.f, 0.f, 0.f}, all = 1.f;
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            if (i > dg) f *= gh[i];
+            all *= gh[i];
+            if ((i >> 2) == jg && i >= dg) upto[i & 3] = f;
+        }
+        const float end = dg < n ? f : 0.f;
+        const float* q = qb + min(dg, n - 1) * ks + jg * 4;
+        const float* k = kb + min(dg, n - 1) * ks + jg * 4;
+        float* kt = c.kt + ph * (16 * DP) + token_slot(dg);
+        f32x4 kk[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}}, qk[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+        for (int t = 0; t < R4 * 4; ++t) {
+            const float4 x = *reinterpret_cast<const float4*>(q + t * 16), y = *reinterpret_cast<const float4*>(k + t * 16);
+            const float xv[4] = {x.x, x.y, x.z, x.w}, yv[4] = {y.x, y.y, y.z, y.w};
+            float* o = kt + (t * 16 + jg * 4) * 16;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                kk[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(yv[e], yv[e], kk[t & 1], 0, 0, 0);
+                qk[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(xv[e], yv[e], qk[t & 1], 0, 0, 0);
+                o[e * 16] = yv[e] * end;
+            }
+        }
+        float* pair = c.pair + ph * 256;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int i = jg * 4 + r, at = i * 16 + token_slot(dg);
+            const float p = i < n ? upto[r] : 0.f;  // 0 for i < j too
+            A[at] = (kk[0][r] + kk[1][r]) * p;
+            pair[at] = (qk[0][r] + qk[1][r]) * p;
+        }
+        for (int d = lane; d < DP; d += 64) c.decay[ph * DP + d] = all;
+    } else {
+        // A and B: lane (jg, dg) carries t_j of tokens j = 4 s + jg for the channels 64 r + 4 dg + e
         float t[4][R4 * 4], all[R4 * 4];
 #pragma unroll
         for (int x = 0; x < R4 * 4; ++x) {
@@ -131,7 +170,7 @@ __global__ void __launch_bounds__(64) delta_pieces_kernel(RecurArgs a, PieceArgs
         float y[16], f = 1.f;
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
-            const float g = gb[i * gs + d], k = kb[i * ks + d], q = qb[i * ks + d];
+            const float g = HEAD ? gh[i] : gb[i * gs + d], k = kb[i * ks + d], q = qb[i * ks + d];
             f *= i < n ? g : 1.f;
             y[i] = i < n ? k * f : 0.f;
             c.qt[(ph * 16 + i) * DP + d] = i < n ? q * f : 0.f;
@@ -395,7 +434,8 @@ bool piece_scan_ok(int dim_p) { return dim_p % 64 == 0 && dim_p <= 256; }
 
 template <int R4, bool DELTA>
 static void piece_scan_t(const RecurArgs& a, const PieceArgs& c, hipStream_t s) {
-    if (DELTA) delta_pieces_kernel<R4><<<dim3(a.heads, c.count), 64, 0, s>>>(a, c);
+    if (DELTA && a.gh) delta_pieces_kernel<R4, true><<<dim3(a.heads, c.count), 64, 0, s>>>(a, c);
+    else if (DELTA) delta_pieces_kernel<R4, false><<<dim3(a.heads, c.count), 64, 0, s>>>(a, c);
     else linear_pieces_kernel<R4><<<dim3(a.heads, c.count), 64, 0, s>>>(a, c);
     // four waves share a stage when that still fills the chip
     const int tiles = a.vdim_p / 16, base = a.heads * a.seg.count;
@@ -406,11 +446,11 @@ static void piece_scan_t(const RecurArgs& a, const PieceArgs& c, hipStream_t s) 
     else piece_scan_kernel<R4, DELTA, 1><<<grid, 64, 0, s>>>(a, c);
 }
 hipError_t launch_piece_scan(const RecurArgs& a, const PieceArgs& c, hipStream_t s) {
-    if (!piece_scan_ok(a.dim_p) || a.vdim_p % 16 || a.seg.single || !c.pair || !c.kt || (a.g && (!c.qt || !c.wt || !c.decay || !a.beta)) || (!a.g && !a.decay)) return hipErrorInvalidValue;
+    if (!piece_scan_ok(a.dim_p) || a.vdim_p % 16 || a.seg.single || !c.pair || !c.kt || ((a.g || a.gh) && (!c.qt || !c.wt || !c.decay || !a.beta)) || (a.g && a.gh) || (!a.g && !a.gh && !a.decay)) return hipErrorInvalidValue;
     if (c.count > 65535) return hipErrorNotSupported;
     if (a.seg.count <= 0 || c.count <= 0) return hipSuccess;
     switch (a.dim_p / 64) {
-#define NVLLM_PS(R_) case R_: if (a.g) piece_scan_t<R_, true>(a, c, s); else piece_scan_t<R_, false>(a, c, s); break;
+#define NVLLM_PS(R_) case R_: if (a.g || a.gh) piece_scan_t<R_, true>(a, c, s); else piece_scan_t<R_, false>(a, c, s); break;
         NVLLM_PS(1) NVLLM_PS(2) NVLLM_PS(3) NVLLM_PS(4)
 #undef NVLLM_PS
     }

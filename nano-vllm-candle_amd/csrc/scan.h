@@ -12,6 +12,7 @@ struct ConvRowsArgs {
     int n_slabs = 1, ld = 0;
     int64_t slab_stride = 0;
     int channels = 0, taps = 1;
+    const float* in_bias = nullptr;  // [channels] added to the input (nullable)
     const float* conv = nullptr;     // [taps][channels]
     const float* bias = nullptr;     // [channels]
     float* history = nullptr;        // [2][slots][taps - 1][channels]

@@ -1,5 +1,5 @@
 // Causal short convolutions over the rows of a chunk (device code): what a row sees of earlier tokens, and the history a segment leaves.
-// A: any argument structure with in, n_slabs, slab_stride, ld (channel c of a row is column c), taps, history, slots, seg, pos, slot as in
+// A: any argument structure with in, n_slabs, slab_stride, ld (channel c of a row is column c), in_bias, taps, history, slots, seg, pos, slot as in
 // DeltaRowsArgs (hybrid.h).
 #pragma once
 #include "device_common.h"
@@ -22,10 +22,15 @@ __device__ __forceinline__ RowPast row_past(const A& a, int row) {
     p.pos0 = pos - p.in_chunk;
     return p;
 }
-// raw input of channel c, j tokens before the row
+// input of channel c
+template <class A>
+__device__ __forceinline__ float conv_input(const A& a, int row, int c) {
+    return slab_elem(a.in + (size_t)row * a.ld + c, a.n_slabs, a.slab_stride) + (a.in_bias ? a.in_bias[c] : 0.f);
+}
+// input of channel c, j tokens before the row
 template <class A>
 __device__ __forceinline__ float past_input(const A& a, const RowPast& p, int row, int j, int c, int channels) {
-    if (j <= p.in_chunk) return slab_elem(a.in + (size_t)(row - j) * a.ld + c, a.n_slabs, a.slab_stride);
+    if (j <= p.in_chunk) return conv_input(a, row - j, c);
     const int back = j - p.in_chunk;  // tokens before the segment
     if (back > p.pos0) return 0.f;
     return a.history[((((size_t)(p.pos0 & 1) * a.slots + p.slot) * (a.taps - 1)) + (a.taps - 1 - back)) * channels + c];

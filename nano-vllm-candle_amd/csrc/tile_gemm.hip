@@ -18,8 +18,9 @@
 //     operand re-reads hit that XCD's L2.
 // MODE 0: f32 [M][N].  MODE 2: W is the gate/up matrix interleaved in 16-row tiles; the epilogue writes
 // silu(gate)*up as hi/lo planes [M][N/2] (row-major or xpack_off order) -- SiluAndMul, activation.rs:13-18.
-// MODE 4: squared ReLU of every feature as hi/lo planes [M][N].
-// MODE 5, 6: every row block belongs to a group with weights of its own (routed experts): post relu2(pre x.W^T) as planes, plain f32.
+// MODE 4, 8: squared ReLU, exact GELU of every feature as hi/lo planes [M][N].
+// MODE 5, 7, 6: every row block belongs to a group with weights of its own (routed experts): post relu2(pre x.W^T) as planes, post silu(g) u
+// of interleaved gate / up features as planes, plain f32.
 // MODE 3 (NTW = 8, head_dim 128): W is the fused QKV matrix, so a wave's 64 rows x 128 features are 64 tokens of ONE
 // head and the epilogue is the whole of qwen3.rs:208-234 on registers: RMS norm over the head (q_norm / k_norm BEFORE
 // RoPE), half-split RoPE (rotary_embedding.rs:82-107: features d and d+64 sit in the same lane, accumulators j and j+4),
@@ -64,6 +65,7 @@ int tile_gemm_stamps_count() { return g_tile_stamp_launch; }
 // N = hidden size, where 256-row tiles cannot fill the chip)
 template <int NTW, int WN, int MODE>
 __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
+    constexpr bool GROUPS = MODE == 5 || MODE == 6 || MODE == 7, GATHER = MODE == 5 || MODE == 7;
     constexpr int WM = 8 / WN;             // waves along the rows, 4 row tiles (64 rows) each
     constexpr int XT = WM * 4;             // row tiles per workgroup
     constexpr int FRW = WN * NTW;          // 1 KiB fragments per stage: W ...
@@ -89,7 +91,7 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
     }
     const int mtiles = (a.M + 15) >> 4;
     const uint4* wbase = a.wp;
-    if constexpr (MODE >= 5) {
+    if constexpr (GROUPS) {
         const int g = a.g.tile_group[mb * (WM * 64) / a.g.align];
         if (g < 0) return;  // whole workgroup, before any barrier
         wbase += (size_t)g * a.g.w_group;
@@ -114,11 +116,11 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
     // DMA sources of this wave's copies at k-tile 0, without the lane part (advance: 64 uint4 per k-tile).  Row tiles
     // past the end are clamped to the last one: their products land in columns of D that are never stored.
     const uint4* src[NI];
-    [[maybe_unused]] uint32_t voff[NI], kstep[NI];  // MODE 5: x is row-major and its rows are gathered: lane part, uint4 per k-tile
+    [[maybe_unused]] uint32_t voff[NI], kstep[NI];  // GATHER: x is row-major and its rows are gathered: lane part, uint4 per k-tile
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
         const int f = min(wave + 8 * i, FR - 1);
-        if constexpr (MODE == 5) {
+        if constexpr (GATHER) {
             voff[i] = lane;
             kstep[i] = 64;
             if (f >= FRW) {
@@ -146,7 +148,7 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
 #pragma unroll
         for (int i = 0; i < NI; ++i) {
             const int f = wave + 8 * i;
-            if constexpr (MODE == 5) {
+            if constexpr (GATHER) {
                 if (FR % 8 == 0 || f < FR)
                     __builtin_amdgcn_global_load_lds((gptr_t)(src[i] + (size_t)min(s, KT - 1) * kstep[i] + voff[i]), (lptr_t)(lds + (size_t)(buf * FR + f) * 64), 16, 0, 0);
             } else if (FR % 8 == 0 || f < FR)
@@ -400,7 +402,7 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
                 }
             }
         }
-    } else if constexpr (MODE == 4 || MODE == 5) {
+    } else if constexpr (MODE == 4 || MODE == 5 || MODE == 8) {
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
             const int row = row0 + b * 16 + l15;
@@ -412,7 +414,7 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
                     const int f0 = (nt0 + j) * 16 + grp * 4;
                     uint16_t h[4], l[4];
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) split_bf16(MODE == 5 ? relu2(acc[j][b][r] * pre) * post : relu2(acc[j][b][r]), h[r], l[r]);
+                    for (int r = 0; r < 4; ++r) split_bf16(MODE == 5 ? relu2(acc[j][b][r] * pre) * post : act_of<MODE == 8 ? ACT_GELU : ACT_RELU2>(acc[j][b][r]), h[r], l[r]);
                     const size_t xo = a.act_packed ? xpack_off(row, f0, a.N >> 5) : (size_t)row * a.N + f0;
                     *reinterpret_cast<uint2*>(a.act_hi + xo) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
                     *reinterpret_cast<uint2*>(a.act_lo + xo) = make_uint2(l[0] | ((uint32_t)l[1] << 16), l[2] | ((uint32_t)l[3] << 16));
@@ -420,12 +422,14 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
             }
         }
     } else {
-        static_assert(MODE != 2 || NTW % 2 == 0, "gate and up tiles of a feature live in one wave");
+        static_assert((MODE != 2 && MODE != 7) || NTW % 2 == 0, "gate and up tiles of a feature live in one wave");
         const int I = a.N >> 1;
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
             const int row = row0 + b * 16 + l15;
             if (row < a.M) {
+                [[maybe_unused]] float post = 1.f;
+                if constexpr (MODE == 7) post = a.g.post[row];
 #pragma unroll
                 for (int pr = 0; pr < NTW / 2; ++pr) {
                     const int f0 = ((nt0 >> 1) + pr) * 16 + grp * 4;
@@ -433,7 +437,7 @@ __global__ void __launch_bounds__(512) gemm_tile_kernel(TileArgs a) {
 #pragma unroll
                     for (int r = 0; r < 4; ++r) {
                         const float g = acc[2 * pr][b][r], u = acc[2 * pr + 1][b][r];
-                        split_bf16(glu_mul(g, u, a.glu), h[r], l[r]);
+                        split_bf16(MODE == 7 ? silu_mul(g, u) * post : glu_mul(g, u, a.glu), h[r], l[r]);
                     }
                     const size_t xo = a.act_packed ? xpack_off(row, f0, I >> 5) : (size_t)row * I + f0;
                     *reinterpret_cast<uint2*>(a.act_hi + xo) = make_uint2(h[0] | ((uint32_t)h[1] << 16), h[2] | ((uint32_t)h[3] << 16));
@@ -507,7 +511,7 @@ hipError_t launch_gemm_tile(const bf16_bits* xh, const bf16_bits* xl, const Pack
     const TileShape t = tile_shape(M, w.N, w.K, mode, min_wgs, n_slabs ? max_split : 1);
     if (!t.ntw) return hipErrorNotSupported;
     if (mode == 2 && act_packed && (w.N / 2) % 32 != 0) return hipErrorNotSupported;
-    if (mode == 4 && act_packed && w.N % 32 != 0) return hipErrorNotSupported;
+    if (mode >= 4 && act_packed && w.N % 32 != 0) return hipErrorNotSupported;
     TileArgs a;
     a.xh = reinterpret_cast<const uint4*>(xh); a.xl = reinterpret_cast<const uint4*>(xl); a.wp = w.data;
     a.out = out; a.act_hi = act_hi; a.act_lo = act_lo; a.act_packed = act_packed; a.glu = glu;
@@ -524,6 +528,10 @@ hipError_t launch_gemm_tile(const bf16_bits* xh, const bf16_bits* xl, const Pack
     if (mode == 4) {
         if (t.wn == 4) return tile_launch_t<4, 4, 4>(a, 1, s);
         return t.ntw == 8 ? tile_launch_t<8, 2, 4>(a, 1, s) : tile_launch_t<6, 2, 4>(a, 1, s);
+    }
+    if (mode == 4 + ACT_GELU) {
+        if (t.wn == 4) return tile_launch_t<4, 4, 8>(a, 1, s);
+        return t.ntw == 8 ? tile_launch_t<8, 2, 8>(a, 1, s) : tile_launch_t<6, 2, 8>(a, 1, s);
     }
     return hipErrorInvalidValue;
 }
@@ -555,11 +563,15 @@ bool gemm_tile_group_ok(int N, int K, int align) { return group_shape(N, K, alig
 hipError_t launch_gemm_tile_group(const bf16_bits* xh, const bf16_bits* xl, const PackedW& w, int positions, const TileGroups& g, float* out, bf16_bits* act_hi,
                                   bf16_bits* act_lo, hipStream_t s) {
     const TileShape t = group_shape(w.N, w.K, g.align);
-    if (!t.ntw || positions % g.align || !g.tile_group || (act_hi && (!g.pre || !g.post || !g.src || g.x_rows < 1 || (int64_t)g.x_rows * w.K / 8 > INT32_MAX))) return hipErrorNotSupported;
+    if (!t.ntw || positions % g.align || !g.tile_group || (act_hi && ((!g.gated && !g.pre) || !g.post || !g.src || g.x_rows < 1 || (int64_t)g.x_rows * w.K / 8 > INT32_MAX))) return hipErrorNotSupported;
     if (positions <= 0) return hipSuccess;
     TileArgs a;
     a.xh = reinterpret_cast<const uint4*>(xh); a.xl = reinterpret_cast<const uint4*>(xl); a.wp = w.data;
     a.out = out; a.act_hi = act_hi; a.act_lo = act_lo; a.act_packed = 1; a.M = positions; a.N = w.N; a.KT = w.K / 32; a.g = g;
+    if (act_hi && g.gated) {
+        if (t.wn == 4) return tile_launch_t<4, 4, 7>(a, 1, s);
+        return t.ntw == 8 ? tile_launch_t<8, 2, 7>(a, 1, s) : tile_launch_t<6, 2, 7>(a, 1, s);
+    }
     if (act_hi) {
         if (t.wn == 4) return tile_launch_t<4, 4, 5>(a, 1, s);
         return t.ntw == 8 ? tile_launch_t<8, 2, 5>(a, 1, s) : tile_launch_t<6, 2, 5>(a, 1, s);

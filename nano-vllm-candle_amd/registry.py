@@ -4,12 +4,14 @@ import os
 
 from .berevik import BerevikForCausalLM
 from .gopunex import GopunexForCausalLM
+from .lefalix import LefalixForCausalLM
 from .qwen3 import Qwen3ForCausalLM
 from .tafopel import TafopelForCausalLM
 
 MODELS = {
     "Berevik": BerevikForCausalLM,
     "Gopunex": GopunexForCausalLM,
+    "Lefalix": LefalixForCausalLM,
     "Qwen3ForCausalLM": Qwen3ForCausalLM,
     "Tafopel": TafopelForCausalLM,
 }

@@ -9,15 +9,7 @@ from dataclasses import dataclass, field
 import numpy as np
 
 from . import _lib
-from .causal_lm import LayeredCausalLM, random_matrix
-
-
-@dataclass
-class Yarn:
-    factor: float
-    original: float
-    fast: float
-    slow: float
+from .causal_lm import LayeredCausalLM, Yarn, random_matrix
 
 
 @dataclass
@@ -78,8 +70,7 @@ class TafopelConfig:
                     rot = m["rot"]
                     if rot["dims"] != m["rot_dim"]:
                         raise RuntimeError(f"layer {i}: rot.dims {rot['dims']} differs from rot_dim {m['rot_dim']}")
-                    sc = rot.get("scaling")
-                    yarn = Yarn(*(float(sc[k]) for k in ("factor", "original", "fast", "slow"))) if sc else None
+                    yarn = Yarn.from_dict(rot.get("scaling"))
                     mix = LatentMixerConfig(m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"], m["q_rank"], float(rot["base"]), float(m["scale"]), yarn,
                                             m.get("kv_from"))
                 elif e["type"] == "mamba1":
