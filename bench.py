@@ -73,6 +73,12 @@ def parse():
     ap.add_argument("--berevik-window", type=int, default=1 << 20, help="attention window of the --berevik layers")
     ap.add_argument("--berevik-batch", type=int, default=64)
     ap.add_argument("--berevik-prompt", type=int, default=1024)
+    ap.add_argument("--lefalix", nargs="*", metavar="SIZE", default=None,
+                    help="instead of the headline: the Lefalix design beside the closest designs at equal size (bench_lefalix.py; sizes 1k 2k 4k, default all)")
+    ap.add_argument("--lefalix-kinds", nargs="+", default=None, help="parallel, window, channel_delta, experts, mixed (default all)")
+    ap.add_argument("--lefalix-batch", type=int, default=64)
+    ap.add_argument("--lefalix-prompt", type=int, default=1024)
+    ap.add_argument("--lefalix-alone", action="store_true", help="without the other designs")
     ap.add_argument("--tafopel", nargs="*", metavar="SIZE", default=None,
                     help="instead of the headline: the Tafopel design beside the closest designs at equal size (bench_tafopel.py; sizes 1k 2k 4k, default all)")
     ap.add_argument("--tafopel-kinds", nargs="+", default=None, help="attention, scan, experts, mixed (default all)")
@@ -338,6 +344,11 @@ def live_traffic(a, dom_kernel):
 
 def main():
     a = parse()
+    if a.lefalix is not None:
+        import bench_lefalix
+
+        bench_lefalix.main(a.lefalix or None, batch=a.lefalix_batch, prompt=a.lefalix_prompt, kinds=a.lefalix_kinds or bench_lefalix.KINDS, with_twins=not a.lefalix_alone)
+        return
     if a.tafopel is not None:
         import bench_tafopel
 

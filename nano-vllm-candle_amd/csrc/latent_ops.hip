@@ -157,7 +157,8 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
     constexpr int NW = 16;
     constexpr bool POST = KIND == NORM_POST || KIND == NORM_BRANCH;
     __shared__ float red[KIND == NORM_PLAIN ? 1 : KIND == NORM_BRANCH ? 4 : 2][NW][16];
-    float o[KIND == NORM_BRANCH ? IT : 1][8];
+    constexpr bool HOLD = KIND == NORM_BRANCH && IT <= 4;  // the second branch in registers; the widest rows read it again
+    float o[HOLD ? IT : 1][8];
     float so = 0.f;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, grp = lane >> 4;
     const int KT = a.ldr >> 5, row = blockIdx.x * 16 + l15, rowc = min(row, rows - 1);
@@ -187,10 +188,11 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
                 const float4 k0 = s0, k1 = s1;
                 s0 = s1 = make_float4(0.f, 0.f, 0.f, 0.f);
                 for (int sl = 0; sl < a.n_slabs2; ++sl) add(a.in2 + (size_t)sl * a.slab_stride2 + off);
-                o[i][0] = s0.x; o[i][1] = s0.y; o[i][2] = s0.z; o[i][3] = s0.w;
-                o[i][4] = s1.x; o[i][5] = s1.y; o[i][6] = s1.z; o[i][7] = s1.w;
-#pragma unroll
-                for (int e = 0; e < 8; ++e) so += o[i][e] * o[i][e];
+                so += s0.x * s0.x + s0.y * s0.y + s0.z * s0.z + s0.w * s0.w + s1.x * s1.x + s1.y * s1.y + s1.z * s1.z + s1.w * s1.w;
+                if constexpr (HOLD) {
+                    o[i][0] = s0.x; o[i][1] = s0.y; o[i][2] = s0.z; o[i][3] = s0.w;
+                    o[i][4] = s1.x; o[i][5] = s1.y; o[i][6] = s1.z; o[i][7] = s1.w;
+                }
                 s0 = k0; s1 = k1;
             } else if (a.in2) {
                 const float f = a.in2_scale ? a.in2_scale[rowc] : 1.f;
@@ -243,9 +245,19 @@ __global__ void __launch_bounds__(1024) add_norm_rows16_kernel(AddNormArgs a, in
             const int kt = wave + i * NW;
             if (kt >= KT) continue;
             const float *w = a.branch_w[0] + kt * 32 + grp * 8, *u = a.branch_w[1] + kt * 32 + grp * 8;
+            float4 x0 = make_float4(0.f, 0.f, 0.f, 0.f), x1 = x0;
+            if constexpr (HOLD) {
+                x0 = make_float4(o[i][0], o[i][1], o[i][2], o[i][3]);
+                x1 = make_float4(o[i][4], o[i][5], o[i][6], o[i][7]);
+            } else {
+                const float* p = a.in2 + (size_t)rowc * a.ldr + kt * 32 + grp * 8;
+                add_slabs(x0, p, a.n_slabs2, a.slab_stride2);
+                add_slabs(x1, p + 4, a.n_slabs2, a.slab_stride2);
+            }
+            const float x[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
-                v[i][e] = (v[i][e] * f) * w[e] + (o[i][e] * fo) * u[e];
+                v[i][e] = (v[i][e] * f) * w[e] + (x[e] * fo) * u[e];
                 ss += v[i][e] * v[i][e];
             }
         }

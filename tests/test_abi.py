@@ -73,7 +73,8 @@ def test_missing_library_raises(monkeypatch, tmp_path):
 def _kernel_resources():
     out = {}
     for name in ("kernel_resources.txt", "kernel_resources_tile.txt", "kernel_resources_latent.txt", "kernel_resources_latent_prefill.txt", "kernel_resources_bias_attn.txt",
-                 "kernel_resources_recurrent.txt", "kernel_resources_recurrent_chunk.txt", "kernel_resources_scan.txt", "kernel_resources_moe.txt"):
+                 "kernel_resources_recurrent.txt", "kernel_resources_recurrent_chunk.txt", "kernel_resources_scan.txt", "kernel_resources_moe.txt",
+                 "kernel_resources_conv_attn.txt"):
         path = os.path.join(ROOT, "nano-vllm-candle_amd", name)
         if not os.path.exists(path):
             pytest.skip(name + " missing: rebuild the library (make -C nano-vllm-candle_amd/csrc)")
@@ -143,7 +144,8 @@ def test_bias_attention_and_recurrence_kernels_stay_in_registers():
 
 def test_scan_and_expert_kernels_stay_in_registers():
     res = _kernel_resources()
-    for part, count in (("scan_prompt_kernel", 18), ("scan_decode_kernel", 9), ("conv_rows16_kernel", 3), ("group_gemm_kernel", 8), ("gemm_tile_kernelILi8ELi2ELi5", 1), ("gemm_tile_kernelILi8ELi2ELi6", 1)):
+    for part, count in (("scan_prompt_kernel", 18), ("scan_decode_kernel", 9), ("conv_rows16_kernel", 3), ("group_gemm_kernel", 8), ("gemm_tile_kernelILi8ELi2ELi5", 1), ("gemm_tile_kernelILi8ELi2ELi6", 1),
+                        ("gemm_tile_kernelILi8ELi2ELi7", 1), ("gemm_tile_kernelILi6ELi2ELi8", 1), ("conv_attn_rows16_kernel", 12), ("conv_attn_decode_kernel", 12)):
         hits = {n: r for n, r in res.items() if part in n and "piece_scan" not in n}
         assert len(hits) == count, (part, len(hits))
         for n, r in hits.items():

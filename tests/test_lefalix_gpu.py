@@ -507,3 +507,15 @@ def test_what_the_library_refuses():
     for name in ("l0.mix.nope", "l0.mix.left.rel", "l0.mix.q", "l1.mix.left.q", "l1.mix.a", "l0.mlp.gate", "l1.mlp.e6.up"):
         with pytest.raises(pkg._lib.NvllmError, match="unknown tensor"):
             pkg.LefalixForCausalLM.from_state_dict(c, dict(w, **{name: w["l0.norm1"]}))
+
+
+@pytest.mark.parametrize("width", [1024, 2048, 4096])
+def test_wide_rows_of_long_prompts(width):
+    # the two-branch norm of every width it has a form for, over whole and partly filled blocks of rows
+    cfg = config([par(win(heads=2, kv=1, dim=16, vdim=16, rot=8), rule(heads=2, kv=1, dim=16, vdim=16), dense(64)), par(win(heads=2, kv=2), rule(heads=2, kv=2))], width=width, vocab=64, loop=(0, 1, 2))
+    w = weights(cfg, 6)
+    m = make(cfg, w, "bfloat16", rows=1024)
+    for n in (528, 601):
+        toks = tokens(n, 64, n)
+        ask = [0, 15, 16, 300, n - 1]
+        assert row_err(m.step_score([n], [toks], True, [ask]), logits(cfg, w, toks, ask)) < TOL["bfloat16"]
