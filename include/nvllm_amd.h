@@ -189,7 +189,7 @@ typedef struct nvllm_hybrid_mixer {
 } nvllm_hybrid_mixer;
 typedef struct nvllm_hybrid_layer {
     nvllm_hybrid_mixer mix;
-    int32_t branches;                   /* 2: `side` reads the same input, the result is half the sum of both outputs, each normed; else 1 */
+    int32_t branches;                   /* 2: `side` reads the same input, result (norm(mix) + norm(side)) / 2; else 1 */
     nvllm_hybrid_mixer side;
     int32_t ff;                         /* feed-forward width, 0 = the layer has none */
     int32_t act;                        /* NVLLM_ACT_* */
@@ -202,7 +202,7 @@ typedef struct nvllm_hybrid_config {
     int32_t f32;                        /* 0: bf16 weights, hi + lo planes, f16 cache; 1: every product and the cache in f32 */
     int32_t pre_norm;                   /* 1: the sublayers read norm1 (norm2) of the stream, their outputs are normed with norm1b (norm2b) */
     int32_t loop_start, loop_stop, loop_times; /* layers [start, stop) are passed through loop_times times, each pass with a cache and state of
-                                           its own; the embedding output is added to the stream before every pass but the first; <= 1: no loop */
+                                           its own; a second or later pass starts from the stream plus the embeddings; <= 1: no loop */
 } nvllm_hybrid_config;
 /* Tensor names for nvllm_model_load_tensor: embed, head, final.norm and, per layer, l<i>.norm1, l<i>.norm2 (with pre_norm .norm1b, .norm2b),
  * l<i>.mlp.{up, down} or l<i>.mlp.{router, e<k>.gate, e<k>.up, e<k>.down}, and the mixer's under l<i>.mix (two mixers: l<i>.mix.left and

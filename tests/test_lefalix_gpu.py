@@ -519,3 +519,14 @@ def test_wide_rows_of_long_prompts(width):
         toks = tokens(n, 64, n)
         ask = [0, 15, 16, 300, n - 1]
         assert row_err(m.step_score([n], [toks], True, [ask]), logits(cfg, w, toks, ask)) < TOL["bfloat16"]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("rank", [1, 33, 150])
+def test_ranks_of_the_two_step_gates(rank, dtype):
+    cfg = config([delta(heads=3, kv=3, dim=40, vdim=24), par()], vocab=64)
+    w = {k: L.bf16(v).astype(np.float64) for k, v in L.random_weights(cfg, 3, rank=rank).items()}
+    toks = tokens(100, 64, 1)
+    ref = logits(cfg, w, toks)
+    m = make(cfg, w, dtype)
+    assert row_err(portions(m, 0, toks, [70, 1, 1, 28]), ref) < TOL[dtype]
