@@ -1,5 +1,5 @@
-// Decoders whose layers mix tokens by recurrence or by attention with a distance bias (hybrid_model.cpp): launchers of
-// hybrid_ops.hip (row kernels), recurrent.hip (carried-state scans) and bias_attn.hip (grouped-query attention).
+// Decoders whose layers mix tokens by recurrence, by grouped-query attention or by two mixers side by side (hybrid_model.cpp): launchers of
+// hybrid_ops.hip and conv_attn.hip (row kernels), recurrent.hip and recurrent_chunk.hip (carried-state scans) and bias_attn.hip (attention).
 #pragma once
 #include "latent.h"
 

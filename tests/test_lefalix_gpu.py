@@ -146,14 +146,11 @@ def test_small_row_buffers_cut_prompts_inside(rows, dtype):
     assert row_err(got, np.concatenate([logits(MIXED, w, a, want[0]), logits(MIXED, w, b, want[1])])) < TOL[dtype]
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("plain", [0, 1])
+@pytest.mark.parametrize("dtype, plain", [("bfloat16", 0), ("bfloat16", 1), ("float32", 0)])  # 32-bit mode has the plain kernel alone
 @pytest.mark.parametrize("window", [1, 2, 31, 32, 33, 64, 100, 256, 300])
 def test_a_key_just_inside_and_just_outside_the_window(window, plain, dtype):
     # one token outweighs every other while it is seen: right at the query, at the window's last place, one behind it; in prompts (a query
     # at every place of a tile and of a block), in portions, decoded one by one
-    if plain and dtype == "float32":
-        pytest.skip("32-bit mode has the plain kernel alone")
     cfg = beacon_config(window)
     w = beacon_weights(cfg, 63)
     m = make(cfg, w, dtype, rows=700)
